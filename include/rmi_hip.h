@@ -37,10 +37,12 @@ extern "C" {
 #define RMI_HIP_E_NOT_INIT (-3)  /* rmi_hip_init has not succeeded           */
 #define RMI_HIP_E_NO_DEVICE (-4) /* no gfx950 device visible                 */
 
+#define RMI_HIP_DTYPE_F32 0
 #define RMI_HIP_DTYPE_Q4_0 2
 #define RMI_HIP_DTYPE_Q8_0 8
 #define RMI_HIP_DTYPE_Q4_K 12
 #define RMI_HIP_DTYPE_Q6_K 14
+#define RMI_HIP_DTYPE_BF16 30
 
 /* Activation rounding of quantize_q8_0_into: the reference picks it per host
  * architecture (src/ops/quant/q8_0.rs:3-24). */
@@ -519,6 +521,40 @@ int rmi_hip_gguf_qwen3_config(const rmi_hip_gguf *g, uint32_t capacity, int roun
 /* Qwen3Model::from_source + Qwen3Session::new over the file (tensor names, shapes and types of
  * src/models/qwen3.rs:262-349; "Missing tensor: .." / "Invalid tensor ..: .." as checked_tensor, :1350-1380). */
 rmi_hip_qwen3 *rmi_hip_qwen3_create_from_gguf(const rmi_hip_gguf *g, uint32_t capacity, int rounding);
+
+/* ------------------------------------------------------------------ model folders
+ * A folder with config.json and model.safetensors (bf16, f16 or f32 weights).  The architecture that config.json
+ * names decides the session: its length, and the name in buf (up to cap - 1 bytes and a terminator); -1 on error. */
+int64_t rmi_hip_model_folder_architecture(const char *dir, char *buf, size_t cap);
+
+/* ------------------------------------------------------------------ Ruvenex decoder
+ * Parallel layers: one RMS norm read by a softmax-attention mixer (short causal convolution, partial interleaved
+ * rotation, value norm, per-head output gate), an HGRN2 mixer beside it (gated linear recurrence) and a gelu
+ * feed-forward, each sublayer's result gated element by element.  Sizes, constants and the order of layers come
+ * from config.json.  No counterpart in the reference.
+ *
+ * dtype: RMI_HIP_DTYPE_BF16 (matrix operands, keys and values in bf16, f32 accumulation; residual, norms, scores,
+ * gates and recurrent state f32) or RMI_HIP_DTYPE_F32 (everything true f32).  capacity: most tokens of a sequence.
+ * A session holds one sequence at a time. */
+typedef struct rmi_hip_ruvenex rmi_hip_ruvenex;
+rmi_hip_ruvenex *rmi_hip_ruvenex_open(const char *dir, int dtype, uint32_t capacity); /* NULL on error */
+void rmi_hip_ruvenex_destroy(rmi_hip_ruvenex *s);
+int rmi_hip_ruvenex_sizes(const rmi_hip_ruvenex *s, uint32_t *vocab, uint32_t *width, uint32_t *n_layer, uint32_t *capacity);
+/* The next tokens of the sequence from the cache and state the earlier ones left; any portions give the same
+ * result within rounding.  logits[i * vocab ..] = those of place want[i] among these tokens.  layers (NULL, or
+ * [n_layer][n_tokens][width]): the residual stream behind every layer, for comparisons. */
+int rmi_hip_ruvenex_step(rmi_hip_ruvenex *s, const uint32_t *tokens, uint32_t n_tokens, const uint32_t *want, uint32_t n_want,
+                         float *logits, float *layers);
+uint32_t rmi_hip_ruvenex_position(const rmi_hip_ruvenex *s); /* tokens of the sequence so far */
+int rmi_hip_ruvenex_reset(rmi_hip_ruvenex *s);               /* the sequence is over; a new one begins */
+/* As the rmi_hip_qwen3_* calls of the same names (greedy; a new sequence).  A prompt pass takes up to 2048 positions
+ * and computes logits only where they are read: step_argmax and step_top2 of a prompt position that is neither the
+ * prompt's last nor listed in dump_steps are left as they were, unless prompt passes are off. */
+int rmi_hip_ruvenex_set_stop_ids(rmi_hip_ruvenex *s, const uint32_t *ids, uint32_t n_ids);
+int rmi_hip_ruvenex_set_prompt_passes(rmi_hip_ruvenex *s, int enabled);
+int rmi_hip_ruvenex_generate(rmi_hip_ruvenex *s, const uint32_t *prompt, uint32_t n_prompt, uint32_t max_new,
+                             uint32_t *generated, uint32_t *step_argmax, float *step_top2, const uint32_t *dump_steps,
+                             uint32_t n_dump, float *dump_logits, double *seconds);
 
 #ifdef __cplusplus
 }

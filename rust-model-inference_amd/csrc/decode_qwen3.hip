@@ -22,29 +22,21 @@
 // and that flips the f32 rounding of the mean (about 2^-29 per norm).  A rounded
 // int8 quant that flips would move logits by 1e-2, so the step is held to
 // bit-identical logits against the CPU path, not to a tolerance.
-#include <chrono>
 #include <cmath>
 #include <utility>
 #include <vector>
 
 #include "device_math.h"
 #include "device_quant.h"
+#include "device_sample.h"
 #include "rmi_internal.h"
+#include "session.h"
 
 #include "device_common.h"
 
 namespace {
 
 __device__ __forceinline__ uint16_t f2h(float v) { return rmi_f2h(v); }
-
-// The step counter in HBM: the embedding kernel reads its token through it and the argmax kernel advances it,
-// so the next token never visits the host.  The kernels in between get the position as a launch argument:
-// reading it from HBM first would put one more memory round trip in front of their loads.  (Replaying a whole step as a HIP graph with the counter read everywhere was
-// measured: 676 vs 678 token-steps/s, no gain, so the launches stay eager.)
-struct StepParams {
-    uint32_t step;      // position of the token being processed = row of the KV cache
-    uint32_t n_prompt;  // steps below n_prompt - 1 read their token from the prompt
-};
 
 __device__ __forceinline__ double wave_sum(double v) { return wave_sum_f64(v); }
 
@@ -1199,75 +1191,14 @@ __global__ __launch_bounds__(256) void expf_kernel(const float *__restrict__ x, 
     for (size_t i = blockIdx.x * size_t(256) + threadIdx.x; i < n; i += size_t(gridDim.x) * 256) y[i] = rmi_expf(x[i]);
 }
 
-// greedy_token: the first strict maximum, the second largest value, and whether every logit is finite
-struct Top {
-    float best, second;
-    uint32_t id, finite;
+// the embedding of the next token, the argmax kernels' last act
+struct EmbedQ8 {
+    const uint8_t *w;
+    uint32_t n_oct, vocab;
+    float *x;
+    uint32_t n_embd;
+    __device__ __forceinline__ void operator()(uint32_t token) const { embed_row(w, n_oct, token, vocab, x, n_embd); }
 };
-__device__ __forceinline__ Top top_merge(const Top &a, const Top &b) {
-    Top r;
-    const bool a_first = a.best > b.best || (a.best == b.best && a.id < b.id);
-    const Top &hi = a_first ? a : b, &lo = a_first ? b : a;
-    r.best = hi.best;
-    r.id = hi.id;
-    r.second = fmaxf(fmaxf(hi.second, lo.second), lo.best);
-    r.finite = a.finite & b.finite;
-    return r;
-}
-__device__ __forceinline__ Top top_block_reduce(Top t, Top *sm) {
-    sm[threadIdx.x] = t;
-    __syncthreads();
-    for (uint32_t s = blockDim.x >> 1; s > 0; s >>= 1) {
-        if (threadIdx.x < s) sm[threadIdx.x] = top_merge(sm[threadIdx.x], sm[threadIdx.x + s]);
-        __syncthreads();
-    }
-    return sm[0];
-}
-__global__ __launch_bounds__(256) void argmax_partial_kernel(const float *__restrict__ logits, uint32_t n,
-                                                             Top *__restrict__ partial) {
-    __shared__ Top sm[256];
-    logits += size_t(blockIdx.y) * n;  // token blockIdx.y of a launch over several: its logits, its partial results
-    partial += size_t(blockIdx.y) * gridDim.x;
-    Top t{-INFINITY, -INFINITY, 0xffffffffu, 1u};
-    for (uint32_t i = blockIdx.x * 256 + threadIdx.x; i < n; i += gridDim.x * 256) {
-        const float l = logits[i];
-        if (!(fabsf(l) <= 3.4028234663852886e38f)) t.finite = 0;  // NaN or inf
-        if (l > t.best) {
-            t.second = t.best;
-            t.best = l;
-            t.id = i;
-        } else if (l > t.second) {
-            t.second = l;
-        }
-    }
-    const Top r = top_block_reduce(t, sm);
-    if (threadIdx.x == 0) partial[blockIdx.x] = r;
-}
-__global__ __launch_bounds__(256) void argmax_final_kernel(const Top *__restrict__ partial, uint32_t n_partial,
-                                                           StepParams *__restrict__ sp,
-                                                           uint32_t *__restrict__ tok, uint32_t *__restrict__ step_argmax,
-                                                           float *__restrict__ step_top2,
-                                                           uint32_t *__restrict__ nonfinite_steps,
-                                                           const uint8_t *__restrict__ w_embd, uint32_t n_oct,
-                                                           uint32_t vocab, float *__restrict__ x, uint32_t n_embd) {
-    __shared__ Top sm[256];
-    __shared__ uint32_t next_token;
-    Top t{-INFINITY, -INFINITY, 0xffffffffu, 1u};
-    for (uint32_t i = threadIdx.x; i < n_partial; i += 256) t = top_merge(t, partial[i]);
-    const Top r = top_block_reduce(t, sm);
-    if (threadIdx.x == 0) {
-        const uint32_t step = sp->step, n_prompt = sp->n_prompt;
-        step_argmax[step] = r.id;
-        step_top2[2 * step] = r.best;
-        step_top2[2 * step + 1] = r.second;
-        if (!r.finite) atomicAdd(nonfinite_steps, 1u);
-        if (step + 1 >= n_prompt) tok[step + 1] = r.id;  // the next step's token
-        next_token = step + 1 >= n_prompt ? r.id : tok[step + 1];
-        sp->step = step + 1;  // last kernel of the step: the next one sees the new position
-    }
-    __syncthreads();
-    embed_row(w_embd, n_oct, next_token, vocab, x, n_embd);  // the next step starts from its token's embedding
-}
 
 // ---- several prompt positions in one pass (rmi_hip_qwen3_generate while the tokens are known in advance)
 // the embeddings of the prompt tokens step0 .. step0 + gridDim.x - 1, n_embd apart
@@ -1276,42 +1207,11 @@ __global__ __launch_bounds__(256) void embed_batch_kernel(const uint8_t *__restr
                                                           float *__restrict__ x, uint32_t n_embd) {
     embed_row(w, n_oct, tok[step0 + blockIdx.x], vocab, x + size_t(blockIdx.x) * n_embd, n_embd);
 }
-// argmax_final_kernel for position step0 + blockIdx.x of such a pass; the workgroup of the pass's last position also
-// advances the step counter and leaves the next token's embedding where a single step starts from
-__global__ __launch_bounds__(256) void argmax_final_batch_kernel(const Top *__restrict__ partial, uint32_t n_partial,
-                                                                 StepParams *__restrict__ sp, uint32_t step0,
-                                                                 uint32_t *__restrict__ tok, uint32_t *__restrict__ step_argmax,
-                                                                 float *__restrict__ step_top2,
-                                                                 uint32_t *__restrict__ nonfinite_steps,
-                                                                 const uint8_t *__restrict__ w_embd, uint32_t n_oct,
-                                                                 uint32_t vocab, float *__restrict__ x, uint32_t n_embd) {
-    __shared__ Top sm[256];
-    __shared__ uint32_t next_token;
-    partial += size_t(blockIdx.x) * n_partial;
-    Top t{-INFINITY, -INFINITY, 0xffffffffu, 1u};
-    for (uint32_t i = threadIdx.x; i < n_partial; i += 256) t = top_merge(t, partial[i]);
-    const Top r = top_block_reduce(t, sm);
-    const uint32_t step = step0 + blockIdx.x;
-    if (threadIdx.x == 0) {
-        const uint32_t n_prompt = sp->n_prompt;
-        step_argmax[step] = r.id;
-        step_top2[2 * step] = r.best;
-        step_top2[2 * step + 1] = r.second;
-        if (!r.finite) atomicAdd(nonfinite_steps, 1u);
-        if (step + 1 >= n_prompt) tok[step + 1] = r.id;  // the next step's token
-        next_token = step + 1 >= n_prompt ? r.id : tok[step + 1];
-    }
-    if (blockIdx.x + 1 != gridDim.x) return;
-    if (threadIdx.x == 0) sp->step = step + 1;
-    __syncthreads();
-    embed_row(w_embd, n_oct, next_token, vocab, x, n_embd);
-}
-
 }  // namespace
 
 // ------------------------------------------------------------------ session
 
-struct rmi_hip_qwen3 {
+struct rmi_hip_qwen3 : RmiSession {
     rmi_hip_qwen3_config cfg{};
     uint32_t n_q = 0, n_k = 0, n_v = 0, n_attn = 0, kv_stride = 0, max_n_in = 0;
     rmi_hip_weight *embd = nullptr, *head = nullptr;  // head == embd when tied
@@ -1322,47 +1222,32 @@ struct rmi_hip_qwen3 {
     uint16_t *k_cache = nullptr, *v_cache = nullptr, *q16 = nullptr;
     float *x = nullptr, *x2 = nullptr, *resid = nullptr, *qkv = nullptr, *gu = nullptr, *logits = nullptr, *act_scales = nullptr;
     int8_t *act_q8 = nullptr;
-    uint32_t *tok = nullptr, *step_argmax = nullptr, *nonfinite = nullptr;
-    float *step_top2 = nullptr;
-    void *partial = nullptr;
     // the same buffers for kPromptBatch positions at once (prompt passes), token-major
     float *xb = nullptr, *residb = nullptr, *qkvb = nullptr, *gub = nullptr, *logitsb = nullptr, *act_scalesb = nullptr;
     uint16_t *q16b = nullptr;
     int8_t *act_q8b = nullptr;
     void *partialb = nullptr;
     void *attn_split = nullptr;          // scratch of the split attention launches (head dimension 128)
-    void *params = nullptr;              // StepParams in HBM
-    std::vector<void *> owned;  // every other device allocation, freed with the session
-    std::vector<uint32_t> stop_ids;  // generation ends before the first of these (EOS, im_end)
-    uint32_t prompt_pass = 128;      // prompt positions per pass, 0 = every position its own step (rmi_hip_qwen3_set_prompt_passes)
+
+    ~rmi_hip_qwen3() override;
+    int enqueue_step(uint32_t step, hipStream_t st) override;
+    const float *step_logits() const override { return logits; }
+    bool pass_possible(uint32_t step0, uint32_t n) const override;
+    // every position's logits, whichever are asked for
+    int enqueue_pass(uint32_t step0, uint32_t n, const uint32_t *want, uint32_t n_want, bool sample, hipStream_t st) override;
+    const float *pass_logits(uint32_t offset, uint32_t) const override { return logitsb + size_t(offset) * cfg.vocab; }
 };
 
 namespace {
 
-constexpr uint32_t kArgmaxGroups = 256;
 constexpr uint32_t kPromptBatch = 128;  // most positions a prompt pass takes (the buffers' size); kPromptPassDefault is what it takes
 constexpr uint32_t kPromptPassDefault = 128;
 
 template <typename T>
 T *dev_alloc(rmi_hip_qwen3 *s, size_t count, bool zero = false) {
-    void *p = nullptr;
-    if (hipMalloc(&p, count * sizeof(T) ? count * sizeof(T) : sizeof(T)) != hipSuccess) {
-        rmi_set_error("hipMalloc of %zu bytes failed", count * sizeof(T));
-        return nullptr;
-    }
-    s->owned.push_back(p);
-    if (zero && hipMemset(p, 0, count * sizeof(T)) != hipSuccess) return nullptr;
-    return static_cast<T *>(p);
+    return s->alloc<T>(count, zero);
 }
-
-float *upload_f32(rmi_hip_qwen3 *s, const float *host, size_t n) {
-    float *d = dev_alloc<float>(s, n);
-    if (d && hipMemcpy(d, host, n * 4, hipMemcpyHostToDevice) != hipSuccess) {
-        rmi_set_error("hipMemcpy of a norm weight failed");
-        return nullptr;
-    }
-    return d;
-}
+float *upload_f32(rmi_hip_qwen3 *s, const float *host, size_t n) { return s->upload(host, n); }
 
 rmi_hip_weight *upload_stack(const uint8_t *const *parts, const uint32_t *rows, int n_parts, uint32_t n_in) {
     // the session's constructor waits once, after the last weight
@@ -1475,9 +1360,9 @@ int enqueue_step(rmi_hip_qwen3 *s, uint32_t step, hipStream_t st) {
     if (rc != RMI_HIP_OK) return rc;
     hipLaunchKernelGGL(argmax_partial_kernel, dim3(kArgmaxGroups), dim3(256), 0, st, s->logits, c.vocab,
                        static_cast<Top *>(s->partial));
-    hipLaunchKernelGGL(argmax_final_kernel, dim3(1), dim3(256), 0, st, static_cast<const Top *>(s->partial),
-                       kArgmaxGroups, sp, s->tok, s->step_argmax, s->step_top2, s->nonfinite, s->embd->data,
-                       s->embd->n_units, c.vocab, s->x, c.n_embd);
+    hipLaunchKernelGGL(argmax_final_kernel<EmbedQ8>, dim3(1), dim3(256), 0, st, static_cast<const Top *>(s->partial),
+                       kArgmaxGroups, sp, s->tok, s->step_argmax, s->step_top2, s->nonfinite,
+                       EmbedQ8{s->embd->data, s->embd->n_units, c.vocab, s->x, c.n_embd});
     RMI_HIP_CHECK(hipGetLastError());
     return RMI_HIP_OK;
 }
@@ -1541,14 +1426,28 @@ int enqueue_prompt_pass(rmi_hip_qwen3 *s, uint32_t step0, uint32_t n, hipStream_
     if (rc != RMI_HIP_OK) return rc;
     hipLaunchKernelGGL(argmax_partial_kernel, dim3(kArgmaxGroups, n), dim3(256), 0, st, s->logitsb, c.vocab,
                        static_cast<Top *>(s->partialb));
-    hipLaunchKernelGGL(argmax_final_batch_kernel, dim3(n), dim3(256), 0, st, static_cast<const Top *>(s->partialb), kArgmaxGroups,
-                       sp, step0, s->tok, s->step_argmax, s->step_top2, s->nonfinite, s->embd->data, s->embd->n_units, c.vocab,
-                       s->x, c.n_embd);
+    hipLaunchKernelGGL(argmax_final_batch_kernel<EmbedQ8>, dim3(n), dim3(256), 0, st, static_cast<const Top *>(s->partialb), kArgmaxGroups,
+                       sp, step0, static_cast<const uint32_t *>(nullptr), s->tok, s->step_argmax, s->step_top2, s->nonfinite,
+                       EmbedQ8{s->embd->data, s->embd->n_units, c.vocab, s->x, c.n_embd});
     RMI_HIP_CHECK(hipGetLastError());
     return RMI_HIP_OK;
 }
 
 }  // namespace
+
+int rmi_hip_qwen3::enqueue_step(uint32_t step, hipStream_t st) { return ::enqueue_step(this, step, st); }
+bool rmi_hip_qwen3::pass_possible(uint32_t step0, uint32_t n) const { return prompt_pass_possible(this, step0, n); }
+int rmi_hip_qwen3::enqueue_pass(uint32_t step0, uint32_t n, const uint32_t *, uint32_t, bool, hipStream_t st) {
+    return enqueue_prompt_pass(this, step0, n, st);
+}
+rmi_hip_qwen3::~rmi_hip_qwen3() {
+    if (head && head != embd) rmi_hip_free_weight(head);
+    if (embd) rmi_hip_free_weight(embd);
+    for (auto *w : w_qkv) rmi_hip_free_weight(w);
+    for (auto *w : w_o) rmi_hip_free_weight(w);
+    for (auto *w : w_gu) rmi_hip_free_weight(w);
+    for (auto *w : w_down) rmi_hip_free_weight(w);
+}
 
 extern "C" {
 
@@ -1726,17 +1625,7 @@ int rmi_hip_qkv_attention_f16_quantize_q8_0_dev(const float *qkv, const float *q
     return RMI_HIP_OK;
 }
 
-void rmi_hip_qwen3_destroy(rmi_hip_qwen3 *s) {
-    if (!s) return;
-    if (s->head && s->head != s->embd) rmi_hip_free_weight(s->head);
-    if (s->embd) rmi_hip_free_weight(s->embd);
-    for (auto *w : s->w_qkv) rmi_hip_free_weight(w);
-    for (auto *w : s->w_o) rmi_hip_free_weight(w);
-    for (auto *w : s->w_gu) rmi_hip_free_weight(w);
-    for (auto *w : s->w_down) rmi_hip_free_weight(w);
-    for (void *p : s->owned) (void)hipFree(p);
-    delete s;
-}
+void rmi_hip_qwen3_destroy(rmi_hip_qwen3 *s) { delete s; }
 
 rmi_hip_qwen3 *rmi_hip_qwen3_create(const rmi_hip_qwen3_config *cfg, const rmi_hip_qwen3_weights *wt) {
     if (!rmi_ready()) {
@@ -1786,6 +1675,9 @@ rmi_hip_qwen3 *rmi_hip_qwen3_create(const rmi_hip_qwen3_config *cfg, const rmi_h
     if (!rmi_thread_ctx()) return nullptr;
     rmi_hip_qwen3 *s = new rmi_hip_qwen3();
     s->cfg = c;
+    s->vocab = c.vocab;
+    s->capacity = c.capacity;
+    s->prompt_pass = kPromptPassDefault;
     s->n_q = c.n_head * c.head_dim_k;
     s->n_k = c.n_head_kv * c.head_dim_k;
     s->n_v = c.n_head_kv * c.head_dim_v;
@@ -1855,11 +1747,7 @@ rmi_hip_qwen3 *rmi_hip_qwen3_create(const rmi_hip_qwen3_config *cfg, const rmi_h
          (s->resid = dev_alloc<float>(s, c.n_embd)) && (s->qkv = dev_alloc<float>(s, size_t(s->n_q) + s->n_k + s->n_v)) &&
          (s->gu = dev_alloc<float>(s, size_t(2) * c.n_ff)) && (s->logits = dev_alloc<float>(s, c.vocab)) &&
          (s->act_q8 = dev_alloc<int8_t>(s, s->max_n_in)) && (s->act_scales = dev_alloc<float>(s, s->max_n_in / 32)) &&
-         (s->tok = dev_alloc<uint32_t>(s, size_t(c.capacity) + 1, true)) &&
-         (s->step_argmax = dev_alloc<uint32_t>(s, c.capacity, true)) &&
-         (s->step_top2 = dev_alloc<float>(s, size_t(2) * c.capacity, true)) &&
-         (s->nonfinite = dev_alloc<uint32_t>(s, 1, true)) && (s->partial = dev_alloc<Top>(s, kArgmaxGroups)) &&
-         (s->params = dev_alloc<StepParams>(s, 1, true));
+         s->alloc_sampling();
     if (ok && c.head_dim_k == 128 && c.head_dim_v == 128)  // prompt passes of kPromptBatch positions (head dimension 128)
         ok = (s->xb = dev_alloc<float>(s, size_t(kPromptBatch) * c.n_embd)) &&
              (s->residb = dev_alloc<float>(s, size_t(kPromptBatch) * c.n_embd)) &&
@@ -1886,95 +1774,7 @@ rmi_hip_qwen3 *rmi_hip_qwen3_create(const rmi_hip_qwen3_config *cfg, const rmi_h
 int rmi_hip_qwen3_generate(rmi_hip_qwen3 *s, const uint32_t *prompt, uint32_t n_prompt, uint32_t max_new,
                            uint32_t *generated, uint32_t *step_argmax, float *step_top2, const uint32_t *dump_steps,
                            uint32_t n_dump, float *dump_logits, double *seconds) {
-    RMI_REQUIRE_INIT();
-    if (!s || !prompt || n_prompt == 0 || (max_new && !generated))
-        return rmi_fail(RMI_HIP_E_INVALID, "null session, prompt or output");
-    const rmi_hip_qwen3_config &c = s->cfg;
-    if (size_t(n_prompt) + max_new > c.capacity)
-        return rmi_fail(RMI_HIP_E_INVALID, "%u prompt + %u new tokens exceed the capacity %u", n_prompt, max_new,
-                        c.capacity);
-    for (uint32_t i = 0; i < n_prompt; i++)
-        if (prompt[i] >= c.vocab) return rmi_fail(RMI_HIP_E_INVALID, "token id %u outside the vocabulary", prompt[i]);
-    RmiThreadCtx *ctx = rmi_thread_ctx();
-    if (!ctx) return RMI_HIP_E_RUNTIME;
-    hipStream_t st = ctx->stream;
-    const uint32_t steps = n_prompt + max_new - 1;
-    float *d_dump = nullptr;
-    if (n_dump) {
-        if (!dump_steps || !dump_logits) return rmi_fail(RMI_HIP_E_INVALID, "null dump arrays");
-        RMI_HIP_CHECK(hipMalloc(reinterpret_cast<void **>(&d_dump), size_t(n_dump) * c.vocab * 4));
-    }
-    int rc = RMI_HIP_OK;
-    const StepParams start{0u, n_prompt};
-    hipError_t e = hipMemcpyAsync(s->tok, prompt, size_t(n_prompt) * 4, hipMemcpyHostToDevice, st);
-    if (e == hipSuccess) e = hipMemcpyAsync(s->params, &start, sizeof start, hipMemcpyHostToDevice, st);
-    if (e == hipSuccess) e = hipMemsetAsync(s->nonfinite, 0, 4, st);
-    if (e == hipSuccess) e = hipStreamSynchronize(st);
-    const auto t0 = std::chrono::steady_clock::now();
-    // Without stop ids every step is enqueued at once.  With them the host looks at the tokens every
-    // kStopCheck generated steps (one small copy) and ends the run at the first stop id, which is not part of
-    // the result (src/models/qwen3.rs:1123-1130: the loop breaks before the token is pushed).
-    constexpr uint32_t kStopCheck = 32;
-    const bool stops = !s->stop_ids.empty() && max_new > 0;
-    uint32_t n_valid = max_new, steps_done = 0, checked = 0;
-    std::vector<uint32_t> seen(stops ? max_new : 0);
-    while (e == hipSuccess && rc == RMI_HIP_OK && steps_done < steps) {
-        uint32_t until = steps;
-        if (stops) {
-            const uint32_t base = steps_done < n_prompt - 1 ? n_prompt - 1 : steps_done;
-            until = steps - base > kStopCheck ? base + kStopCheck : steps;
-        }
-        for (uint32_t step = steps_done; e == hipSuccess && rc == RMI_HIP_OK && step < until;) {
-            // prompt positions go eight to a pass while they can (their tokens are known); the rest step by step
-            uint32_t n = step < n_prompt ? n_prompt - step : 0;
-            if (n > s->prompt_pass) n = s->prompt_pass;
-            if (n > until - step) n = until - step;
-            if (n > 1 && prompt_pass_possible(s, step, n)) {
-                rc = enqueue_prompt_pass(s, step, n, st);
-                for (uint32_t d = 0; rc == RMI_HIP_OK && d < n_dump; d++)
-                    if (dump_steps[d] >= step && dump_steps[d] < step + n)
-                        e = hipMemcpyAsync(d_dump + size_t(d) * c.vocab, s->logitsb + size_t(dump_steps[d] - step) * c.vocab,
-                                           size_t(c.vocab) * 4, hipMemcpyDeviceToDevice, st);
-                step += n;
-                continue;
-            }
-            rc = enqueue_step(s, step, st);
-            for (uint32_t d = 0; rc == RMI_HIP_OK && d < n_dump; d++)
-                if (dump_steps[d] == step)
-                    e = hipMemcpyAsync(d_dump + size_t(d) * c.vocab, s->logits, size_t(c.vocab) * 4, hipMemcpyDeviceToDevice, st);
-            step++;
-        }
-        steps_done = until;
-        if (!stops || e != hipSuccess || rc != RMI_HIP_OK) continue;
-        const uint32_t have = steps_done - (n_prompt - 1);  // tokens sampled so far
-        e = hipStreamSynchronize(st);
-        if (e == hipSuccess && have > checked)
-            e = hipMemcpy(seen.data() + checked, s->tok + n_prompt + checked, size_t(have - checked) * 4, hipMemcpyDeviceToHost);
-        bool hit = false;
-        for (; e == hipSuccess && checked < have && !hit; checked++)
-            for (uint32_t id : s->stop_ids)
-                if (seen[checked] == id) {
-                    n_valid = checked;
-                    hit = true;
-                    break;
-                }
-        if (hit) break;
-    }
-    if (e == hipSuccess) e = hipStreamSynchronize(st);
-    if (seconds) *seconds = std::chrono::duration<double>(std::chrono::steady_clock::now() - t0).count();
-    uint32_t nonfinite = 0;
-    if (e == hipSuccess && rc == RMI_HIP_OK) {
-        if (n_valid) e = hipMemcpy(generated, s->tok + n_prompt, size_t(n_valid) * 4, hipMemcpyDeviceToHost);
-        if (e == hipSuccess && step_argmax) e = hipMemcpy(step_argmax, s->step_argmax, size_t(steps_done) * 4, hipMemcpyDeviceToHost);
-        if (e == hipSuccess && step_top2) e = hipMemcpy(step_top2, s->step_top2, size_t(steps_done) * 8, hipMemcpyDeviceToHost);
-        if (e == hipSuccess && n_dump) e = hipMemcpy(dump_logits, d_dump, size_t(n_dump) * c.vocab * 4, hipMemcpyDeviceToHost);
-        if (e == hipSuccess) e = hipMemcpy(&nonfinite, s->nonfinite, 4, hipMemcpyDeviceToHost);
-    }
-    if (d_dump) (void)hipFree(d_dump);
-    if (rc != RMI_HIP_OK) return rc;
-    if (e != hipSuccess) return rmi_fail(RMI_HIP_E_RUNTIME, "decode failed: %s", hipGetErrorString(e));
-    if (nonfinite) return rmi_fail(RMI_HIP_E_RUNTIME, "non-finite logits in %u steps", nonfinite);
-    return int(n_valid);
+    return rmi_session_generate(s, prompt, n_prompt, max_new, generated, step_argmax, step_top2, dump_steps, n_dump, dump_logits, seconds);
 }
 
 int rmi_hip_qwen3_set_prompt_passes(rmi_hip_qwen3 *s, int enabled) {
@@ -1985,10 +1785,7 @@ int rmi_hip_qwen3_set_prompt_passes(rmi_hip_qwen3 *s, int enabled) {
 }
 
 int rmi_hip_qwen3_set_stop_ids(rmi_hip_qwen3 *s, const uint32_t *ids, uint32_t n_ids) {
-    if (!s || (n_ids && !ids)) return rmi_fail(RMI_HIP_E_INVALID, "null session or ids");
-    if (n_ids > 16) return rmi_fail(RMI_HIP_E_INVALID, "at most 16 stop ids");
-    s->stop_ids.assign(ids, ids + n_ids);
-    return RMI_HIP_OK;
+    return rmi_session_set_stop_ids(s, ids, n_ids);
 }
 
 }  // extern "C"

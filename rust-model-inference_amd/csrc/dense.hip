@@ -1,0 +1,479 @@
+// Products on dense bf16 / f32 weights: a tiled matrix-core GEMM for several tokens, a GEMV for one, each with the
+// layer's elementwise work in its epilogue (activations, forget gates, gated residual) and, in the GEMV, the RMS
+// norm in its prologue.
+#include "device_dense.h"
+
+namespace {
+
+template <typename T>
+__global__ __launch_bounds__(256) void norm_kernel(const float *__restrict__ x, const uint32_t *__restrict__ rows,
+                                                   const float *__restrict__ weight, float eps, T *__restrict__ h, uint32_t n,
+                                                   uint32_t k_pad) {
+    __shared__ float red[4];
+    const uint32_t tid = threadIdx.x;
+    x += size_t(rows ? rows[blockIdx.x] : blockIdx.x) * n;
+    h += size_t(blockIdx.x) * k_pad;
+    float sq = 0.0f;
+    for (uint32_t i = tid; i < n; i += 256) sq = __builtin_fmaf(x[i], x[i], sq);
+    sq = wave_sum_f32(sq);
+    if ((tid & 63) == 0) red[tid >> 6] = sq;
+    __syncthreads();
+    const float r = 1.0f / sqrtf(((red[0] + red[1]) + (red[2] + red[3])) / float(n) + eps);
+    for (uint32_t i = tid; i < k_pad; i += 256) h[i] = from_f32<T>(i < n ? x[i] * r * weight[i] : 0.0f);
+}
+
+template <typename T>
+__global__ __launch_bounds__(256) void embed_kernel(const T *__restrict__ table, uint32_t k_pad, const uint32_t *__restrict__ tok,
+                                                    uint32_t vocab, float scale, float *__restrict__ x, uint32_t n) {
+    uint32_t t = tok[blockIdx.x];
+    if (t >= vocab) t = vocab - 1;  // ids are validated on the host; never read outside the table
+    for (uint32_t i = threadIdx.x; i < n; i += 256) x[size_t(blockIdx.x) * n + i] = to_f32(table[size_t(t) * k_pad + i]) * scale;
+}
+
+// ------------------------------------------------------------------ GEMM
+// One workgroup of four waves: BN weight rows x BT tokens, k in steps of 128 bytes a row through two LDS buffers; the
+// pieces of the next step are loaded into registers while this one is multiplied.  A row of a buffer is eight
+// 16-byte pieces, piece p at slot p ^ (row & 7), so that the sixteen rows of a fragment spread over the banks.
+// Weights are the A operand: a lane ends with four consecutive rows of one token.
+constexpr uint32_t kStepBytes = 128;
+
+template <typename T, int BN, int BT, int WN, int WT, bool RESIDUAL>
+__global__ __launch_bounds__(256) void dense_gemm_kernel(const T *__restrict__ w, const T *__restrict__ a, uint32_t n_rows,
+                                                         uint32_t k_pad, uint32_t n_tokens, uint32_t grid_n, uint32_t grid_t,
+                                                         RmiRowSegs rs, RmiColSegs cs, float *__restrict__ x, uint32_t width) {
+    static_assert((BN / WN) * (BT / WT) == 4, "four waves");
+    constexpr int NN = WN / 16, NT = WT / 16;
+    constexpr int PW = BN * 8 / 256, PA = (BT * 8 + 255) / 256;  // pieces a thread loads per step
+    __shared__ u32x4 lds[2][(BN + BT) * 8];
+    const uint32_t tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
+    uint32_t n_tile, t_tile;
+    rmi_gemm_tile_of(blockIdx.x, grid_n, grid_t, 1u, 0u, n_tile, t_tile);
+    const uint32_t row0 = n_tile * BN, tok0 = t_tile * BT;
+    const uint32_t wn = (wave % (BN / WN)) * WN, wt = (wave / (BN / WN)) * WT;
+    const size_t stride = size_t(k_pad) * sizeof(T);
+
+    const uint8_t *wsrc[PW], *asrc[PA];
+    uint32_t wdst[PW], adst[PA];
+#pragma unroll
+    for (int i = 0; i < PW; i++) {
+        const uint32_t e = tid + i * 256, r = e >> 3, p = e & 7;
+        const uint32_t row = row0 + r < n_rows ? row0 + r : n_rows - 1;  // rows past the end are read again and not stored
+        wsrc[i] = reinterpret_cast<const uint8_t *>(w) + row * stride + p * 16;
+        wdst[i] = r * 8 + (p ^ (r & 7));
+    }
+#pragma unroll
+    for (int i = 0; i < PA; i++) {
+        const uint32_t e = tid + i * 256, r = (e >> 3) % BT, p = e & 7;  // (fewer pieces than threads: some load twice)
+        const uint32_t tok = tok0 + r < n_tokens ? tok0 + r : n_tokens - 1;
+        asrc[i] = reinterpret_cast<const uint8_t *>(a) + tok * stride + p * 16;
+        adst[i] = BN * 8 + r * 8 + (p ^ (r & 7));
+    }
+    f32x4 acc[NN][NT];
+    f32x4 tot[RESIDUAL ? NN : 1][RESIDUAL ? NT : 1];
+#pragma unroll
+    for (int i = 0; i < NN; i++)
+#pragma unroll
+        for (int j = 0; j < NT; j++) {
+            acc[i][j] = f32x4{0.f, 0.f, 0.f, 0.f};
+            if (RESIDUAL) tot[i][j] = f32x4{0.f, 0.f, 0.f, 0.f};
+        }
+    u32x4 rw[PW], ra[PA];
+    auto load = [&](uint32_t step) {
+#pragma unroll
+        for (int i = 0; i < PW; i++) rw[i] = *reinterpret_cast<const u32x4 *>(wsrc[i] + size_t(step) * kStepBytes);
+#pragma unroll
+        for (int i = 0; i < PA; i++) ra[i] = *reinterpret_cast<const u32x4 *>(asrc[i] + size_t(step) * kStepBytes);
+    };
+    auto park = [&](uint32_t buf) {
+#pragma unroll
+        for (int i = 0; i < PW; i++) lds[buf][wdst[i]] = rw[i];
+#pragma unroll
+        for (int i = 0; i < PA; i++) lds[buf][adst[i]] = ra[i];
+    };
+    const uint32_t fr = lane & 15, g = lane >> 4;
+    // the gated sum of a finished column segment
+    auto fold = [&](const RmiColSeg &s) {
+        if constexpr (RESIDUAL) {
+#pragma unroll
+            for (int j = 0; j < NT; j++) {
+                const uint32_t tok = tok0 + wt + j * 16 + fr;
+                const bool live = tok < n_tokens;
+#pragma unroll
+                for (int i = 0; i < NN; i++) {
+                    const uint32_t row = row0 + wn + i * 16 + g * 4;
+#pragma unroll
+                    for (int r = 0; r < 4; r++) {
+                        const float gate = s.gate && live && row + r < width ? s.gate[size_t(tok) * width + row + r] : 1.0f;
+                        tot[i][j][r] = __builtin_fmaf(gate, acc[i][j][r] * s.scale, tot[i][j][r]);
+                    }
+                    acc[i][j] = f32x4{0.f, 0.f, 0.f, 0.f};
+                }
+            }
+        }
+    };
+    constexpr uint32_t kStepElems = kStepBytes / sizeof(T);
+    const uint32_t n_steps = k_pad / kStepElems;
+    uint32_t seg = 0;
+    load(0);
+    park(0);
+    __syncthreads();
+    for (uint32_t step = 0; step < n_steps; step++) {
+        const uint32_t buf = step & 1;
+        if (step + 1 < n_steps) load(step + 1);
+#pragma unroll
+        for (int c = 0; c < 2; c++) {
+            u32x4 fw[NN], fa[NT];
+#pragma unroll
+            for (int i = 0; i < NN; i++) {
+                const uint32_t r = wn + i * 16 + fr;
+                fw[i] = lds[buf][r * 8 + ((c * 4 + g) ^ (r & 7))];
+            }
+#pragma unroll
+            for (int j = 0; j < NT; j++) {
+                const uint32_t r = wt + j * 16 + fr;
+                fa[j] = lds[buf][BN * 8 + r * 8 + ((c * 4 + g) ^ (r & 7))];
+            }
+#pragma unroll
+            for (int i = 0; i < NN; i++)
+#pragma unroll
+                for (int j = 0; j < NT; j++) acc[i][j] = mma16<T>(fw[i], fa[j], acc[i][j]);
+        }
+        if (step + 1 < n_steps) park(buf ^ 1);
+        if (RESIDUAL && (step + 1) * kStepElems == cs.s[seg].k_end) {
+            fold(cs.s[seg]);
+            seg++;
+        }
+        __syncthreads();
+    }
+
+    if constexpr (RESIDUAL) {
+#pragma unroll
+        for (int j = 0; j < NT; j++) {
+            const uint32_t tok = tok0 + wt + j * 16 + fr;
+            if (tok >= n_tokens) continue;
+#pragma unroll
+            for (int i = 0; i < NN; i++) {
+                const uint32_t row = row0 + wn + i * 16 + g * 4;
+                float *dst = x + size_t(tok) * width + row;
+                if (row + 3 < width && (width & 3) == 0)
+                    *reinterpret_cast<f32x4 *>(dst) += tot[i][j];
+                else
+#pragma unroll
+                    for (int r = 0; r < 4; r++)
+                        if (row + r < width) dst[r] += tot[i][j][r];
+            }
+        }
+    } else {
+#pragma unroll
+        for (int i = 0; i < NN; i++) {
+            const uint32_t tile_row = row0 + wn + i * 16;  // a tile of sixteen rows lies in one segment
+            if (tile_row >= n_rows) continue;
+            uint32_t si = 0;
+            while (si + 1 < rs.n_segs && tile_row >= rs.s[si + 1].row0) si++;
+            const RmiRowSeg &s = rs.s[si];
+            const uint32_t r0 = tile_row - s.row0 + g * 4;
+            float bias[4], lower[4];
+#pragma unroll
+            for (int r = 0; r < 4; r++) {
+                bias[r] = s.bias && r0 + r < s.n ? s.bias[r0 + r] : 0.0f;
+                lower[r] = s.lower && r0 + r < s.n ? s.lower[r0 + r] : 0.0f;
+            }
+#pragma unroll
+            for (int j = 0; j < NT; j++) {
+                const uint32_t tok = tok0 + wt + j * 16 + fr;
+                f32x4 o;
+#pragma unroll
+                for (int r = 0; r < 4; r++) o[r] = apply_act<T>(s.act, acc[i][j][r], bias[r], lower[r]);
+                if (tok >= n_tokens) continue;
+                const size_t at = size_t(tok) * s.ld + r0;
+                if (r0 + 3 < s.n && (s.ld & 3) == 0) {
+                    if (s.out_elem)
+                        store4(static_cast<T *>(s.y) + at, o);
+                    else
+                        store4(static_cast<float *>(s.y) + at, o);
+                } else {
+#pragma unroll
+                    for (int r = 0; r < 4; r++)
+                        if (r0 + r < s.n) {
+                            if (s.out_elem)
+                                static_cast<T *>(s.y)[at + r] = from_f32<T>(o[r]);
+                            else
+                                static_cast<float *>(s.y)[at + r] = o[r];
+                        }
+                }
+            }
+        }
+    }
+}
+
+template <typename T, bool RESIDUAL>
+int launch_gemm(const RmiDense &w, const void *a, const RmiRowSegs &rs, const RmiColSegs &cs, float *x, uint32_t width,
+                uint32_t n_tokens, hipStream_t st) {
+    const uint32_t n_rows = RESIDUAL ? width : w.n_rows;
+    auto go = [&](auto kernel, uint32_t bn, uint32_t bt) {
+        const uint32_t gn = (n_rows + bn - 1) / bn, gt = (n_tokens + bt - 1) / bt;
+        hipLaunchKernelGGL(kernel, dim3(gn * gt), dim3(256), 0, st, static_cast<const T *>(w.data), static_cast<const T *>(a), n_rows,
+                           w.k_pad, n_tokens, gn, gt, rs, cs, x, width);
+    };
+    const uint64_t big = uint64_t((n_rows + 127) / 128) * ((n_tokens + 127) / 128);
+    if (n_tokens <= 16)
+        go(dense_gemm_kernel<T, 64, 16, 16, 16, RESIDUAL>, 64, 16);
+    else if (big >= uint64_t(rmi_device_cus()))
+        go(dense_gemm_kernel<T, 128, 128, 64, 64, RESIDUAL>, 128, 128);
+    else
+        go(dense_gemm_kernel<T, 64, 64, 32, 32, RESIDUAL>, 64, 64);
+    RMI_HIP_CHECK(hipGetLastError());
+    return RMI_HIP_OK;
+}
+
+// ------------------------------------------------------------------ GEMV
+// A wave takes ROWS weight rows, its lanes the 16-byte pieces of a row; two rounds of pieces are in flight.  The
+// activation sits in LDS, zero past its end, so that a piece past the end of a row (the last one is read again)
+// counts for nothing.
+constexpr uint32_t kGemvLdsMax = 144 * 1024;
+template <typename T>
+__host__ __device__ inline uint32_t gemv_lds_pieces(uint32_t k_pad) {
+    const uint32_t pieces = k_pad / (16 / sizeof(T));
+    return (pieces + 127) / 128 * 128;
+}
+
+template <typename T, int ROWS>
+__global__ __launch_bounds__(256) void norm_gemv_kernel(const T *__restrict__ w, uint32_t k_pad, const float *__restrict__ x,
+                                                        const float *__restrict__ weight, float eps, uint32_t n, RmiRowSegs rs) {
+    extern __shared__ u32x4 act[];
+    __shared__ float red[4];
+    const uint32_t tid = threadIdx.x, lane = tid & 63;
+    const uint32_t row0 = (blockIdx.x * 4 + (tid >> 6)) * ROWS;
+    const uint32_t pieces = k_pad / kPieceElems<T>, padded = gemv_lds_pieces<T>(k_pad);
+    const u32x4 *src[ROWS];
+#pragma unroll
+    for (int r = 0; r < ROWS; r++) {
+        const uint32_t row = row0 + r < rs.n_rows ? row0 + r : rs.n_rows - 1;
+        src[r] = reinterpret_cast<const u32x4 *>(w + size_t(row) * k_pad);
+    }
+    u32x4 cur[2][ROWS];
+    auto load = [&](uint32_t p0) {
+#pragma unroll
+        for (int u = 0; u < 2; u++) {
+            const uint32_t p = p0 + u * 64 + lane;
+#pragma unroll
+            for (int r = 0; r < ROWS; r++) cur[u][r] = src[r][p < pieces ? p : pieces - 1];
+        }
+    };
+    load(0);  // the weights are under way while the norm is computed
+    float sq = 0.0f;
+    for (uint32_t i = tid; i < n; i += 256) sq = __builtin_fmaf(x[i], x[i], sq);
+    sq = wave_sum_f32(sq);
+    if (lane == 0) red[tid >> 6] = sq;
+    __syncthreads();
+    const float scale = 1.0f / sqrtf(((red[0] + red[1]) + (red[2] + red[3])) / float(n) + eps);
+    T *h = reinterpret_cast<T *>(act);
+    for (uint32_t i = tid; i < padded * kPieceElems<T>; i += 256) h[i] = from_f32<T>(i < n ? x[i] * scale * weight[i] : 0.0f);
+    __syncthreads();
+    float acc[ROWS];
+#pragma unroll
+    for (int r = 0; r < ROWS; r++) acc[r] = 0.0f;
+    for (uint32_t p0 = 0; p0 < padded; p0 += 128) {
+        u32x4 now[2][ROWS];
+#pragma unroll
+        for (int u = 0; u < 2; u++)
+#pragma unroll
+            for (int r = 0; r < ROWS; r++) now[u][r] = cur[u][r];
+        if (p0 + 128 < padded) load(p0 + 128);
+#pragma unroll
+        for (int u = 0; u < 2; u++) {
+            const u32x4 hv = act[p0 + u * 64 + lane];
+#pragma unroll
+            for (int r = 0; r < ROWS; r++) acc[r] = dot_piece<T>(now[u][r], hv, acc[r]);
+        }
+    }
+    float mine = 0.0f;
+#pragma unroll
+    for (int r = 0; r < ROWS; r++) {
+        const float s = wave_sum_f32(acc[r]);
+        if (lane == uint32_t(r)) mine = s;
+    }
+    const uint32_t row = row0 + lane;
+    if (lane >= ROWS || row >= rs.n_rows) return;
+    uint32_t si = 0;
+    while (si + 1 < rs.n_segs && row0 >= rs.s[si + 1].row0) si++;
+    const RmiRowSeg &s = rs.s[si];
+    const uint32_t at = row - s.row0;
+    if (at >= s.n) return;
+    const float o = apply_act<T>(s.act, mine, s.bias ? s.bias[at] : 0.0f, s.lower ? s.lower[at] : 0.0f);
+    if (s.out_elem)
+        static_cast<T *>(s.y)[at] = from_f32<T>(o);
+    else
+        static_cast<float *>(s.y)[at] = o;
+}
+
+template <typename T, int ROWS>
+__global__ __launch_bounds__(256) void gemv_residual_kernel(const T *__restrict__ w, uint32_t k_pad, const T *__restrict__ a,
+                                                            RmiColSegs cs, float *__restrict__ x, uint32_t width) {
+    extern __shared__ u32x4 act[];
+    const uint32_t tid = threadIdx.x, lane = tid & 63;
+    const uint32_t row0 = (blockIdx.x * 4 + (tid >> 6)) * ROWS;
+    const uint32_t pieces = k_pad / kPieceElems<T>, padded = gemv_lds_pieces<T>(k_pad);
+    const u32x4 *src[ROWS];
+#pragma unroll
+    for (int r = 0; r < ROWS; r++) src[r] = reinterpret_cast<const u32x4 *>(w + size_t(row0 + r < width ? row0 + r : width - 1) * k_pad);
+    u32x4 cur[2][ROWS];
+    auto load = [&](uint32_t p0) {
+#pragma unroll
+        for (int u = 0; u < 2; u++) {
+            const uint32_t p = p0 + u * 64 + lane;
+#pragma unroll
+            for (int r = 0; r < ROWS; r++) cur[u][r] = src[r][p < pieces ? p : pieces - 1];
+        }
+    };
+    load(0);
+    const u32x4 zero = {0, 0, 0, 0};
+    for (uint32_t p = tid; p < padded; p += 256) act[p] = p < pieces ? reinterpret_cast<const u32x4 *>(a)[p] : zero;
+    __syncthreads();
+    // sum_i gate_i scale_i part_i: a lane's running sums by segment
+    float acc[ROWS][kMaxColSegs];
+#pragma unroll
+    for (int r = 0; r < ROWS; r++)
+#pragma unroll
+        for (uint32_t i = 0; i < kMaxColSegs; i++) acc[r][i] = 0.0f;
+    for (uint32_t p0 = 0; p0 < padded; p0 += 128) {
+        u32x4 now[2][ROWS];
+#pragma unroll
+        for (int u = 0; u < 2; u++)
+#pragma unroll
+            for (int r = 0; r < ROWS; r++) now[u][r] = cur[u][r];
+        if (p0 + 128 < padded) load(p0 + 128);
+#pragma unroll
+        for (int u = 0; u < 2; u++) {
+            const uint32_t k = (p0 + u * 64 + lane) * kPieceElems<T>;
+            const u32x4 hv = act[p0 + u * 64 + lane];
+            uint32_t seg = 0;
+#pragma unroll
+            for (uint32_t i = 0; i + 1 < kMaxColSegs; i++) seg += i + 1 < cs.n_segs && k >= cs.s[i].k_end ? 1u : 0u;
+#pragma unroll
+            for (int r = 0; r < ROWS; r++) {
+                const float d = dot_piece<T>(now[u][r], hv, 0.0f);
+#pragma unroll
+                for (uint32_t i = 0; i < kMaxColSegs; i++) acc[r][i] += seg == i ? d : 0.0f;
+            }
+        }
+    }
+#pragma unroll
+    for (int r = 0; r < ROWS; r++) {
+        const uint32_t row = row0 + r;
+        float sums[kMaxColSegs];
+#pragma unroll
+        for (uint32_t i = 0; i < kMaxColSegs; i++) sums[i] = i < cs.n_segs ? wave_sum_f32(acc[r][i]) : 0.0f;
+        if (lane != uint32_t(r) || row >= width) continue;
+        float t = 0.0f;
+#pragma unroll
+        for (uint32_t i = 0; i < kMaxColSegs; i++)
+            if (i < cs.n_segs) t = __builtin_fmaf(cs.s[i].gate ? cs.s[i].gate[row] : 1.0f, sums[i] * cs.s[i].scale, t);
+        x[row] += t;
+    }
+}
+
+// more than 64 KiB of dynamic LDS has to be asked for, once a kernel
+template <typename K>
+int allow_lds(K kernel, size_t bytes) {
+    if (bytes <= 64 * 1024) return RMI_HIP_OK;
+    RMI_HIP_CHECK(hipFuncSetAttribute(reinterpret_cast<const void *>(kernel), hipFuncAttributeMaxDynamicSharedMemorySize, kGemvLdsMax));
+    return RMI_HIP_OK;
+}
+
+template <typename T>
+int norm_gemv(const RmiDense &w, const float *x, const float *weight, float eps, uint32_t n, const RmiRowSegs &segs, hipStream_t st) {
+    const size_t lds = size_t(gemv_lds_pieces<T>(w.k_pad)) * 16;
+    if (lds > kGemvLdsMax) return rmi_fail(RMI_HIP_E_INVALID, "%u columns exceed what the GEMV holds", w.k_pad);
+    constexpr int kRows = 4;
+    int rc = allow_lds(norm_gemv_kernel<T, kRows>, lds);
+    if (rc != RMI_HIP_OK) return rc;
+    hipLaunchKernelGGL((norm_gemv_kernel<T, kRows>), dim3((w.n_rows + 4 * kRows - 1) / (4 * kRows)), dim3(256), lds, st,
+                       static_cast<const T *>(w.data), w.k_pad, x, weight, eps, n, segs);
+    RMI_HIP_CHECK(hipGetLastError());
+    return RMI_HIP_OK;
+}
+
+template <typename T>
+int gemv_residual(const RmiDense &w, const void *a, const RmiColSegs &segs, float *x, uint32_t width, hipStream_t st) {
+    const size_t lds = size_t(gemv_lds_pieces<T>(w.k_pad)) * 16;
+    if (lds > kGemvLdsMax) return rmi_fail(RMI_HIP_E_INVALID, "%u columns exceed what the GEMV holds", w.k_pad);
+    constexpr int kRows = 1;
+    int rc = allow_lds(gemv_residual_kernel<T, kRows>, lds);
+    if (rc != RMI_HIP_OK) return rc;
+    hipLaunchKernelGGL((gemv_residual_kernel<T, kRows>), dim3((width + 4 * kRows - 1) / (4 * kRows)), dim3(256), lds, st,
+                       static_cast<const T *>(w.data), w.k_pad, static_cast<const T *>(a), segs, x, width);
+    RMI_HIP_CHECK(hipGetLastError());
+    return RMI_HIP_OK;
+}
+
+}  // namespace
+
+int rmi_dense_norm(uint32_t elem_bytes, const float *x, const uint32_t *rows, const float *weight, float eps, void *h,
+                   uint32_t n_tokens, uint32_t n, uint32_t k_pad, hipStream_t st) {
+    if (n_tokens == 0) return RMI_HIP_OK;
+    if (elem_bytes == 2)
+        hipLaunchKernelGGL(norm_kernel<rmi_bf16>, dim3(n_tokens), dim3(256), 0, st, x, rows, weight, eps, static_cast<rmi_bf16 *>(h), n, k_pad);
+    else
+        hipLaunchKernelGGL(norm_kernel<float>, dim3(n_tokens), dim3(256), 0, st, x, rows, weight, eps, static_cast<float *>(h), n, k_pad);
+    RMI_HIP_CHECK(hipGetLastError());
+    return RMI_HIP_OK;
+}
+
+int rmi_dense_embed(uint32_t elem_bytes, const RmiDense &table, const uint32_t *tok, uint32_t vocab, float scale, float *x,
+                    uint32_t n_tokens, uint32_t n, hipStream_t st) {
+    if (n_tokens == 0) return RMI_HIP_OK;
+    if (elem_bytes == 2)
+        hipLaunchKernelGGL(embed_kernel<rmi_bf16>, dim3(n_tokens), dim3(256), 0, st, static_cast<const rmi_bf16 *>(table.data), table.k_pad,
+                           tok, vocab, scale, x, n);
+    else
+        hipLaunchKernelGGL(embed_kernel<float>, dim3(n_tokens), dim3(256), 0, st, static_cast<const float *>(table.data), table.k_pad, tok,
+                           vocab, scale, x, n);
+    RMI_HIP_CHECK(hipGetLastError());
+    return RMI_HIP_OK;
+}
+
+int rmi_dense_gemm(uint32_t elem_bytes, const RmiDense &w, const void *a, const RmiRowSegs &segs, uint32_t n_tokens, hipStream_t st) {
+    if (n_tokens == 0 || w.n_rows == 0) return RMI_HIP_OK;
+    if (segs.n_rows != w.n_rows || segs.n_segs == 0 || segs.n_segs > kMaxRowSegs || w.k_pad % kDenseKAlign)
+        return rmi_fail(RMI_HIP_E_INVALID, "row segments do not fit the weight");
+    return elem_bytes == 2 ? launch_gemm<rmi_bf16, false>(w, a, segs, RmiColSegs{}, nullptr, 0, n_tokens, st)
+                           : launch_gemm<float, false>(w, a, segs, RmiColSegs{}, nullptr, 0, n_tokens, st);
+}
+
+static int check_col_segs(const RmiDense &w, const RmiColSegs &segs, uint32_t width) {
+    if (segs.n_segs == 0 || segs.n_segs > kMaxColSegs || segs.s[segs.n_segs - 1].k_end != w.k_pad || w.n_rows < width)
+        return rmi_fail(RMI_HIP_E_INVALID, "column segments do not fit the weight");
+    for (uint32_t i = 0; i < segs.n_segs; i++)
+        if (segs.s[i].k_end % kDenseKAlign || segs.s[i].k_end <= (i ? segs.s[i - 1].k_end : 0u))
+            return rmi_fail(RMI_HIP_E_INVALID, "column segments do not fit the weight");
+    return RMI_HIP_OK;
+}
+
+int rmi_dense_gemm_residual(uint32_t elem_bytes, const RmiDense &w, const void *a, const RmiColSegs &segs, float *x, uint32_t width,
+                            uint32_t n_tokens, hipStream_t st) {
+    if (n_tokens == 0) return RMI_HIP_OK;
+    const int rc = check_col_segs(w, segs, width);
+    if (rc != RMI_HIP_OK) return rc;
+    return elem_bytes == 2 ? launch_gemm<rmi_bf16, true>(w, a, RmiRowSegs{}, segs, x, width, n_tokens, st)
+                           : launch_gemm<float, true>(w, a, RmiRowSegs{}, segs, x, width, n_tokens, st);
+}
+
+bool rmi_dense_gemv_fits(uint32_t elem_bytes, uint32_t k_pad) {
+    const size_t lds = size_t(elem_bytes == 2 ? gemv_lds_pieces<rmi_bf16>(k_pad) : gemv_lds_pieces<float>(k_pad)) * 16;
+    return lds <= kGemvLdsMax;
+}
+
+int rmi_dense_norm_gemv(uint32_t elem_bytes, const RmiDense &w, const float *x, const float *weight, float eps, uint32_t n,
+                        const RmiRowSegs &segs, hipStream_t st) {
+    if (segs.n_rows != w.n_rows || segs.n_segs == 0 || segs.n_segs > kMaxRowSegs || n > w.k_pad)
+        return rmi_fail(RMI_HIP_E_INVALID, "row segments do not fit the weight");
+    return elem_bytes == 2 ? norm_gemv<rmi_bf16>(w, x, weight, eps, n, segs, st) : norm_gemv<float>(w, x, weight, eps, n, segs, st);
+}
+
+int rmi_dense_gemv_residual(uint32_t elem_bytes, const RmiDense &w, const void *a, const RmiColSegs &segs, float *x, uint32_t width,
+                            hipStream_t st) {
+    const int rc = check_col_segs(w, segs, width);
+    if (rc != RMI_HIP_OK) return rc;
+    return elem_bytes == 2 ? gemv_residual<rmi_bf16>(w, a, segs, x, width, st) : gemv_residual<float>(w, a, segs, x, width, st);
+}

@@ -143,7 +143,7 @@ int rmi_device_cus();
 int rmi_device();  // the device rmi_hip_init bound, -1 before
 int rmi_batched_mode();  // RMI_HIP_BATCHED_*: what rmi_hip_set_forward_batched_mode chose
 // the device address of the no-allocation entry point's scratch array on `device`, which must be current
-int rmi_noalloc_setup(int device);
+__attribute__((weak)) int rmi_noalloc_setup(int device);
 
 // ------------------------------------------------- launchers (device ptrs)
 // repack tiles [tile0, tile0 + n_tiles) of w; src = the source rows from row tile0 * 8 on (device memory)

@@ -1,0 +1,829 @@
+// Mixers over time (seq_mixers.h): kernels for passes of several tokens and for single tokens.
+#include "seq_mixers.h"
+
+#include "device_dense.h"
+
+namespace {
+
+// Where key `k` of a block of 32 lies.  The softmax weights of keys 16t + 4g + r come out of the score product in
+// register r of lane group g, tile t; the value product's operand wants lane group g's piece contiguous: for bf16 a
+// piece is both tiles' four keys, for f32 a piece is one tile's.
+template <typename T>
+__device__ __forceinline__ uint32_t value_slot(uint32_t k) {
+    if (sizeof(T) == 4) return k;
+    return ((k >> 2) & 3) * 8 + (k >> 4) * 4 + (k & 3);
+}
+
+// ---- convolution, rotation, value norm
+struct ConvCtx {
+    const float *u, *hist, *conv;
+    uint32_t channels, taps;
+};
+// the convolved channel `c` of the pass's token t
+__device__ __forceinline__ float conv_at(const ConvCtx &x, uint32_t t, uint32_t pos0, uint32_t c) {
+    float y = 0.0f;
+    for (uint32_t j = 0; j < x.taps; j++) {
+        const uint32_t back = x.taps - 1 - j;  // position pos0 + t - back
+        float s = 0.0f;
+        if (t >= back)
+            s = x.u[size_t(t - back) * x.channels + c];
+        else if (pos0 + t >= back)
+            s = x.hist[size_t(t + j) * x.channels + c];  // row t - back + (taps - 1)
+        y = __builtin_fmaf(x.conv[c * x.taps + j], s, y);
+    }
+    return y;
+}
+// channel c's row of the history behind the pass: position pos0 + n_tokens - (taps - 1) + j, j = 0 .. taps - 2
+__device__ __forceinline__ void conv_carry(const ConvCtx &x, float *hist_out, uint32_t n_tokens, uint32_t c) {
+    for (uint32_t j = 0; j + 1 < x.taps; j++) {
+        const uint32_t at = n_tokens + j;  // row `at` of history followed by the pass's rows
+        hist_out[size_t(j) * x.channels + c] = at >= x.taps - 1 ? x.u[size_t(at - (x.taps - 1)) * x.channels + c]
+                                                                : x.hist[size_t(at) * x.channels + c];
+    }
+}
+// elements 2i, 2i + 1 of a query or key head whose channels start at c0, convolved and rotated
+__device__ __forceinline__ void conv_rotate_pair(const ConvCtx &x, const RmiAttnShape &s, const float *cos_t, const float *sin_t,
+                                                 uint32_t t, uint32_t pos0, uint32_t c0, uint32_t i, float &a, float &b) {
+    a = 2 * i < s.dim ? conv_at(x, t, pos0, c0 + 2 * i) : 0.0f;
+    b = 2 * i + 1 < s.dim ? conv_at(x, t, pos0, c0 + 2 * i + 1) : 0.0f;
+    if (2 * i < s.rot_dims) {
+        const size_t at = size_t(pos0 + t) * (s.rot_dims / 2) + i;
+        const float c = cos_t[at], sn = sin_t[at], ra = a;
+        a = __builtin_fmaf(ra, c, -(b * sn));
+        b = __builtin_fmaf(b, c, ra * sn);
+    }
+}
+template <typename T>
+__device__ __forceinline__ void store_pair(T *p, float a, float b);
+template <>
+__device__ __forceinline__ void store_pair<float>(float *p, float a, float b) {
+    p[0] = a;
+    p[1] = b;
+}
+template <>
+__device__ __forceinline__ void store_pair<rmi_bf16>(rmi_bf16 *p, float a, float b) {  // p is 4-byte aligned
+    *reinterpret_cast<uint32_t *>(p) = uint32_t(f32_to_bf16(a)) | (uint32_t(f32_to_bf16(b)) << 16);
+}
+// one wave: key head g of token t to its cache row
+template <typename T>
+__device__ __forceinline__ void key_row(const ConvCtx &x, const RmiAttnShape &s, const RmiAttnArgs &a, uint32_t t, uint32_t g, uint32_t lane) {
+    T *row = static_cast<T *>(a.k_cache) + (size_t(g) * s.capacity + a.pos0 + t) * s.dk_pad;
+    const uint32_t c0 = (s.heads + g) * s.dim;
+    for (uint32_t i = lane; i < s.dk_pad / 2; i += 64) {
+        float p, q;
+        conv_rotate_pair(x, s, a.cos_t, a.sin_t, t, a.pos0, c0, i, p, q);
+        store_pair(row + 2 * i, p, q);
+    }
+}
+// one wave: value head g of token t, over its root mean square, to its place in the value block
+template <typename T>
+__device__ __forceinline__ void value_row(const ConvCtx &x, const RmiAttnShape &s, const RmiAttnArgs &a, uint32_t t, uint32_t g, uint32_t lane) {
+    const uint32_t c0 = (s.heads + s.kv_heads) * s.dim + g * s.vdim;
+    float v[kMaxHeadDim / 64], sq = 0.0f;
+#pragma unroll
+    for (uint32_t j = 0; j < kMaxHeadDim / 64; j++) {
+        const uint32_t d = lane + j * 64;
+        v[j] = d < s.vdim ? conv_at(x, t, a.pos0, c0 + d) : 0.0f;
+        sq = __builtin_fmaf(v[j], v[j], sq);
+    }
+    const float r = 1.0f / sqrtf(wave_sum_f32(sq) / float(s.vdim) + s.eps);
+    const uint32_t pos = a.pos0 + t;
+    T *blk = static_cast<T *>(a.v_cache) + (size_t(g) * (s.capacity / kKeyBlock) + pos / kKeyBlock) * s.dv_pad * kKeyBlock +
+             value_slot<T>(pos % kKeyBlock);
+#pragma unroll
+    for (uint32_t j = 0; j < kMaxHeadDim / 64; j++) {
+        const uint32_t d = lane + j * 64;
+        if (d < s.vdim) blk[size_t(d) * kKeyBlock] = from_f32<T>(v[j] * r);
+    }
+}
+
+// a workgroup's four waves: four tokens of one head (blockIdx.x: q heads, then k, then v)
+template <typename T>
+__global__ __launch_bounds__(256) void conv_rotate_kernel(RmiAttnShape s, RmiAttnArgs a) {
+    const uint32_t lane = threadIdx.x & 63, head = blockIdx.x;
+    const uint32_t channels = (s.heads + s.kv_heads) * s.dim + s.kv_heads * s.vdim;
+    const ConvCtx x{a.u, a.hist_in, a.conv, channels, s.taps};
+    if (blockIdx.y == 0) {  // the first tokens' workgroup of a head also carries its channels' history on
+        const bool is_v = head >= s.heads + s.kv_heads;
+        const uint32_t c0 = is_v ? (s.heads + s.kv_heads) * s.dim + (head - s.heads - s.kv_heads) * s.vdim : head * s.dim;
+        for (uint32_t d = threadIdx.x; d < (is_v ? s.vdim : s.dim); d += 256) conv_carry(x, a.hist_out, a.n_tokens, c0 + d);
+    }
+    const uint32_t t = blockIdx.y * 4 + (threadIdx.x >> 6);
+    if (t >= a.n_tokens) return;
+    if (head >= s.heads + s.kv_heads) {
+        value_row<T>(x, s, a, t, head - s.heads - s.kv_heads, lane);
+    } else if (head >= s.heads) {
+        key_row<T>(x, s, a, t, head - s.heads, lane);
+    } else {
+        const uint32_t group = s.heads / s.kv_heads, g = head / group, r = head % group;
+        T *row = static_cast<T *>(a.q) + (size_t(g) * a.n_tokens * group + size_t(t) * group + r) * s.dk_pad;
+        for (uint32_t i = lane; i < s.dk_pad / 2; i += 64) {
+            float p, q;
+            conv_rotate_pair(x, s, a.cos_t, a.sin_t, t, a.pos0, head * s.dim, i, p, q);
+            store_pair(row + 2 * i, p, q);
+        }
+    }
+}
+
+// ---- attention.  The columns of a key/value head are its pass's (token, query head of the group) pairs, token by
+// token; a wave takes QT tiles of sixteen.  Scores come as K q (rows: keys, columns: queries), so a lane holds the
+// weights of one column and the running maximum and sum are a lane's own; the weights then are the operand of
+// V^T p as they lie, because the value blocks hold their keys in that order.
+template <typename T, int BUCKET, int QT>
+struct AttnWave {
+    static constexpr uint32_t kKC = BUCKET / (4 * kPieceElems<T>);  // 16-byte pieces a lane holds of a head's keys
+    static constexpr uint32_t kVT = BUCKET / 16;
+    f32x4 o[QT][kVT];
+    float m[QT], l[QT];
+    u32x4 qf[QT][kKC];
+
+    __device__ __forceinline__ void init() {
+#pragma unroll
+        for (int i = 0; i < QT; i++) {
+            m[i] = -INFINITY;
+            l[i] = 0.0f;
+#pragma unroll
+            for (uint32_t v = 0; v < kVT; v++) o[i][v] = f32x4{0.f, 0.f, 0.f, 0.f};
+        }
+    }
+    // keys [k0, k1), k0 a multiple of 32; column i sees keys up to last[i] (< k1 not required)
+    __device__ __forceinline__ void keys(const T *kc, const T *vc, const RmiAttnShape &s, uint32_t k0, uint32_t k1, const int (&last)[QT]) {
+        const uint32_t lane = threadIdx.x & 63, fr = lane & 15, g = lane >> 4;
+        const uint32_t n_kc = s.dk_pad / (4 * kPieceElems<T>), n_vt = s.dv_pad / 16;
+        const T *krow = kc + size_t(fr) * s.dk_pad + g * kPieceElems<T>;
+        for (uint32_t k = k0; k < k1; k += kKeyBlock) {
+            f32x4 sc[QT][2];
+#pragma unroll
+            for (int i = 0; i < QT; i++) sc[i][0] = sc[i][1] = f32x4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+            for (uint32_t c = 0; c < kKC; c++) {
+                if (c >= n_kc) continue;
+                const T *p = krow + size_t(k) * s.dk_pad + c * 4 * kPieceElems<T>;
+                const u32x4 f0 = *reinterpret_cast<const u32x4 *>(p);
+                const u32x4 f1 = *reinterpret_cast<const u32x4 *>(p + 16 * size_t(s.dk_pad));
+#pragma unroll
+                for (int i = 0; i < QT; i++) {
+                    sc[i][0] = mma16<T>(f0, qf[i][c], sc[i][0]);
+                    sc[i][1] = mma16<T>(f1, qf[i][c], sc[i][1]);
+                }
+            }
+            u32x4 pf[QT][2];
+#pragma unroll
+            for (int i = 0; i < QT; i++) {
+                float top = -INFINITY;
+#pragma unroll
+                for (int t = 0; t < 2; t++)
+#pragma unroll
+                    for (int r = 0; r < 4; r++) {
+                        const int key = int(k) + t * 16 + int(g) * 4 + r;
+                        sc[i][t][r] = key <= last[i] && key < int(k1) ? sc[i][t][r] * s.scale : -INFINITY;
+                        top = fmaxf(top, sc[i][t][r]);
+                    }
+                const float m_new = fmaxf(m[i], rows_max_f32(top));
+                const float ref = m_new == -INFINITY ? 0.0f : m_new;  // nothing visible yet: every weight stays zero
+                const float keep = exp_t<T>(m[i] - ref);
+                float sum = 0.0f;
+#pragma unroll
+                for (int t = 0; t < 2; t++)
+#pragma unroll
+                    for (int r = 0; r < 4; r++) {
+                        sc[i][t][r] = exp_t<T>(sc[i][t][r] - ref);
+                        sum += sc[i][t][r];
+                    }
+                m[i] = m_new;
+                l[i] = __builtin_fmaf(l[i], keep, sum);
+#pragma unroll
+                for (uint32_t v = 0; v < kVT; v++) o[i][v] *= keep;
+                if constexpr (sizeof(T) == 2) {
+                    bf16x8 b;
+#pragma unroll
+                    for (int r = 0; r < 8; r++) b[r] = static_cast<__bf16>(sc[i][r >> 2][r & 3]);
+                    pf[i][0] = __builtin_bit_cast(u32x4, b);
+                } else {
+                    pf[i][0] = __builtin_bit_cast(u32x4, sc[i][0]);
+                    pf[i][1] = __builtin_bit_cast(u32x4, sc[i][1]);
+                }
+            }
+            const T *vb = vc + size_t(k / kKeyBlock) * s.dv_pad * kKeyBlock + size_t(fr) * kKeyBlock + g * kPieceElems<T>;
+#pragma unroll
+            for (uint32_t v = 0; v < kVT; v++) {
+                if (v >= n_vt) continue;
+                const T *p = vb + size_t(v) * 16 * kKeyBlock;
+#pragma unroll
+                for (uint32_t t = 0; t < sizeof(T) / 2; t++) {
+                    const u32x4 f = *reinterpret_cast<const u32x4 *>(p + t * 16);
+#pragma unroll
+                    for (int i = 0; i < QT; i++) o[i][v] = mma16<T>(f, pf[i][t], o[i][v]);
+                }
+            }
+        }
+    }
+};
+
+// four channels d .. d + 3 of a finished column
+template <typename T>
+__device__ __forceinline__ void attn_store(const RmiAttnShape &s, const RmiAttnArgs &a, uint32_t t, uint32_t head, uint32_t d, f32x4 v) {
+    T *dst = static_cast<T *>(a.out) + size_t(t) * a.out_ld + size_t(head) * s.vdim + d;
+    if (d + 3 < s.vdim && (s.vdim & 3) == 0) {  // out_ld is a multiple of 64
+        store4(dst, v);
+    } else {
+#pragma unroll
+        for (int r = 0; r < 4; r++)
+            if (d + r < s.vdim) dst[r] = from_f32<T>(v[r]);
+    }
+}
+
+// several tokens: a workgroup is four waves of QT tiles, each over all the keys its columns see
+template <typename T, int BUCKET, int QT>
+__global__ __launch_bounds__(256) void attn_pass_kernel(RmiAttnShape s, RmiAttnArgs a) {
+    const uint32_t lane = threadIdx.x & 63, fr = lane & 15, g4 = lane >> 4;
+    const uint32_t group = s.heads / s.kv_heads, kvh = blockIdx.y, n_cols = a.n_tokens * group;
+    const uint32_t tile = (gridDim.x - 1 - blockIdx.x) * 4 + (threadIdx.x >> 6);  // the longest columns first
+    if (tile * QT * 16 >= n_cols) return;
+    AttnWave<T, BUCKET, QT> w;
+    w.init();
+    int last[QT];
+    const uint32_t n_kc = s.dk_pad / (4 * kPieceElems<T>);
+#pragma unroll
+    for (int i = 0; i < QT; i++) {
+        const uint32_t col = (tile * QT + i) * 16 + fr, cc = col < n_cols ? col : n_cols - 1;
+        last[i] = int(a.pos0 + cc / group);
+        const T *q = static_cast<const T *>(a.q) + (size_t(kvh) * n_cols + cc) * s.dk_pad + g4 * kPieceElems<T>;
+#pragma unroll
+        for (uint32_t c = 0; c < w.kKC; c++) {
+            if (c >= n_kc) continue;
+            w.qf[i][c] = *reinterpret_cast<const u32x4 *>(q + c * 4 * kPieceElems<T>);
+        }
+    }
+    const uint32_t end_col = (tile + 1) * QT * 16 < n_cols ? (tile + 1) * QT * 16 : n_cols;
+    w.keys(static_cast<const T *>(a.k_cache) + size_t(kvh) * s.capacity * s.dk_pad,
+           static_cast<const T *>(a.v_cache) + size_t(kvh) * s.capacity * s.dv_pad, s, 0, a.pos0 + (end_col - 1) / group + 1, last);
+#pragma unroll
+    for (int i = 0; i < QT; i++) {
+        const uint32_t col = (tile * QT + i) * 16 + fr;
+        const float sum = rows_sum_f32(w.l[i]);
+        if (col >= n_cols) continue;
+        const uint32_t t = col / group, head = kvh * group + col % group;
+        const float f = (a.gate ? a.gate[size_t(t) * s.heads + head] : 1.0f) / sum;
+#pragma unroll
+        for (uint32_t v = 0; v < w.kVT; v++)
+            if (v * 16 < s.dv_pad) attn_store<T>(s, a, t, head, v * 16 + g4 * 4, w.o[i][v] * f);
+    }
+}
+
+// Few columns: the keys are divided over `parts` workgroups and their four waves; each workgroup merges its waves in
+// LDS, writes its part, and the one that arrives last merges the parts.  With one token (STEP) the workgroup makes
+// its queries itself, and the workgroups of the last part the new key and value.
+__host__ __device__ inline uint32_t attn_part_floats(uint32_t dv_pad) { return 16 * (dv_pad + 2); }
+
+__device__ __forceinline__ void merge_state(float &m, float &l, float m2, float l2, float &f1, float &f2) {
+    const float top = fmaxf(m, m2), ref = top == -INFINITY ? 0.0f : top;
+    f1 = expf(m - ref);
+    f2 = expf(m2 - ref);
+    l = l * f1 + l2 * f2;
+    m = top;
+}
+
+template <typename T, int BUCKET, bool STEP>
+__device__ __forceinline__ void attn_split(const RmiAttnShape &s, const RmiAttnArgs &a, uint32_t block, uint32_t parts, uint32_t keys_per_part,
+                                           uint8_t *lds, uint32_t *flag) {
+    const uint32_t tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, fr = lane & 15, g4 = lane >> 4;
+    const uint32_t group = s.heads / s.kv_heads, n_cols = a.n_tokens * group, tiles = (n_cols + 15) / 16;
+    const uint32_t part = block % parts, ct = (block / parts) % tiles, kvh = block / parts / tiles;
+    const uint32_t n_keys = a.pos0 + a.n_tokens;
+    const uint32_t n_kc = s.dk_pad / (4 * kPieceElems<T>);
+    AttnWave<T, BUCKET, 1> w;
+    w.init();
+    const uint32_t col = ct * 16 + fr, cc = col < n_cols ? col : n_cols - 1;
+    const int last[1] = {int(a.pos0 + cc / group)};
+    if constexpr (STEP) {
+        T *q = reinterpret_cast<T *>(lds);
+        const uint32_t channels = (s.heads + s.kv_heads) * s.dim + s.kv_heads * s.vdim;
+        const ConvCtx x{a.u, a.hist_in, a.conv, channels, s.taps};
+        const uint32_t half = s.dk_pad / 2, c_end = n_cols - ct * 16 < 16 ? n_cols - ct * 16 : 16;
+        if (part == parts - 1) {
+            if (wave == 2) key_row<T>(x, s, a, 0, kvh, lane);
+            if (wave == 3) value_row<T>(x, s, a, 0, kvh, lane);
+        }
+        for (uint32_t e = tid; e < c_end * half; e += 256) {
+            const uint32_t c = e / half, i = e % half, head = kvh * group + ct * 16 + c;
+            float p, r;
+            conv_rotate_pair(x, s, a.cos_t, a.sin_t, 0, a.pos0, head * s.dim, i, p, r);
+            store_pair(q + c * s.dk_pad + 2 * i, p, r);
+        }
+        if (part == 0) {  // the history of this workgroup's channels
+            const uint32_t c0 = (kvh * group + ct * 16) * s.dim;
+            for (uint32_t d = tid; d < c_end * s.dim; d += 256) conv_carry(x, a.hist_out, 1, c0 + d);
+            if (ct == 0) {
+                for (uint32_t d = tid; d < s.dim; d += 256) conv_carry(x, a.hist_out, 1, (s.heads + kvh) * s.dim + d);
+                for (uint32_t d = tid; d < s.vdim; d += 256)
+                    conv_carry(x, a.hist_out, 1, (s.heads + s.kv_heads) * s.dim + kvh * s.vdim + d);
+            }
+        }
+        __syncthreads();
+        const uint32_t qc = fr < c_end ? fr : c_end - 1;
+#pragma unroll
+        for (uint32_t c = 0; c < w.kKC; c++) {
+            if (c >= n_kc) continue;
+            w.qf[0][c] = *reinterpret_cast<const u32x4 *>(q + qc * s.dk_pad + (c * 4 + g4) * kPieceElems<T>);
+        }
+        __syncthreads();
+    } else {
+        const T *q = static_cast<const T *>(a.q) + (size_t(kvh) * n_cols + cc) * s.dk_pad + g4 * kPieceElems<T>;
+#pragma unroll
+        for (uint32_t c = 0; c < w.kKC; c++) {
+            if (c >= n_kc) continue;
+            w.qf[0][c] = *reinterpret_cast<const u32x4 *>(q + c * 4 * kPieceElems<T>);
+        }
+    }
+    const uint32_t p0 = part * keys_per_part, p1 = p0 + keys_per_part < n_keys ? p0 + keys_per_part : n_keys;
+    const uint32_t per_wave = keys_per_part / 4;  // a multiple of the key block
+    const uint32_t k0 = p0 + wave * per_wave, k1 = k0 + per_wave < p1 ? k0 + per_wave : p1;
+    if (k0 < k1)
+        w.keys(static_cast<const T *>(a.k_cache) + size_t(kvh) * s.capacity * s.dk_pad,
+               static_cast<const T *>(a.v_cache) + size_t(kvh) * s.capacity * s.dv_pad, s, k0, k1, last);
+    float m = w.m[0], l = rows_sum_f32(w.l[0]);
+    // waves 1..3 hand their part to wave 0: [m 16][l 16][o dv_pad x 16]
+    float *mine = reinterpret_cast<float *>(lds) + (wave ? wave - 1 : 0) * attn_part_floats(s.dv_pad);
+    if (wave) {
+        if (g4 == 0) {
+            mine[fr] = m;
+            mine[16 + fr] = l;
+        }
+#pragma unroll
+        for (uint32_t v = 0; v < w.kVT; v++)
+            if (v * 16 < s.dv_pad)
+#pragma unroll
+                for (int r = 0; r < 4; r++) mine[32 + (v * 16 + g4 * 4 + r) * 16 + fr] = w.o[0][v][r];
+    }
+    __syncthreads();
+    if (wave == 0) {
+        for (uint32_t o = 0; o < 3; o++) {
+            const float *other = reinterpret_cast<const float *>(lds) + o * attn_part_floats(s.dv_pad);
+            float f1, f2;
+            merge_state(m, l, other[fr], other[16 + fr], f1, f2);
+#pragma unroll
+            for (uint32_t v = 0; v < w.kVT; v++)
+                if (v * 16 < s.dv_pad)
+#pragma unroll
+                    for (int r = 0; r < 4; r++) w.o[0][v][r] = w.o[0][v][r] * f1 + other[32 + (v * 16 + g4 * 4 + r) * 16 + fr] * f2;
+        }
+    }
+    const uint32_t slot = kvh * tiles + ct;
+    float *ws = reinterpret_cast<float *>(static_cast<uint32_t *>(a.scratch) + kAttnCounters);
+    if (parts > 1) {
+        if (wave == 0) {
+            float *dst = ws + (size_t(slot) * parts + part) * attn_part_floats(s.dv_pad);
+            if (g4 == 0) {
+                __hip_atomic_store(dst + fr, m, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
+                __hip_atomic_store(dst + 16 + fr, l, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
+            }
+#pragma unroll
+            for (uint32_t v = 0; v < w.kVT; v++)
+                if (v * 16 < s.dv_pad)
+#pragma unroll
+                    for (int r = 0; r < 4; r++)
+                        __hip_atomic_store(dst + 32 + (v * 16 + g4 * 4 + r) * 16 + fr, w.o[0][v][r], __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
+            // the storing lanes are one wave: its fence covers the stores of all of them
+            __builtin_amdgcn_fence(__ATOMIC_RELEASE, "agent");
+            if (lane == 0) {
+                uint32_t *count = static_cast<uint32_t *>(a.scratch) + slot;
+                const uint32_t n = __hip_atomic_fetch_add(count, 1u, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
+                *flag = n == parts - 1;
+                if (n == parts - 1) __hip_atomic_store(count, 0u, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);  // ready for the next launch
+            }
+        }
+        __syncthreads();
+        if (!*flag) return;
+        __builtin_amdgcn_fence(__ATOMIC_ACQUIRE, "agent");
+        // every thread: some (channel, column) pairs over all parts
+        const float *src = ws + size_t(slot) * parts * attn_part_floats(s.dv_pad);
+        const uint32_t c = tid & 15, mc = ct * 16 + c;
+        float top = -INFINITY, sum = 0.0f;
+        for (uint32_t p = 0; p < parts; p++)
+            top = fmaxf(top, __hip_atomic_load(src + size_t(p) * attn_part_floats(s.dv_pad) + c, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT));
+        for (uint32_t p = 0; p < parts; p++) {
+            const float *pp = src + size_t(p) * attn_part_floats(s.dv_pad);
+            sum += expf(__hip_atomic_load(pp + c, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT) - top) *
+                   __hip_atomic_load(pp + 16 + c, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
+        }
+        if (mc < n_cols) {
+            const uint32_t t = mc / group, head = kvh * group + mc % group;
+            const float f = (a.gate ? a.gate[size_t(t) * s.heads + head] : 1.0f) / sum;
+            for (uint32_t d = tid >> 4; d < s.vdim; d += 16) {
+                float o = 0.0f;
+                for (uint32_t p = 0; p < parts; p++) {
+                    const float *pp = src + size_t(p) * attn_part_floats(s.dv_pad);
+                    o += expf(__hip_atomic_load(pp + c, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT) - top) *
+                         __hip_atomic_load(pp + 32 + d * 16 + c, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
+                }
+                static_cast<T *>(a.out)[size_t(t) * a.out_ld + size_t(head) * s.vdim + d] = from_f32<T>(o * f);
+            }
+        }
+        return;
+    }
+    if (wave == 0 && col < n_cols) {
+        const uint32_t t = col / group, head = kvh * group + col % group;
+        const float f = (a.gate ? a.gate[size_t(t) * s.heads + head] : 1.0f) / l;
+#pragma unroll
+        for (uint32_t v = 0; v < w.kVT; v++)
+            if (v * 16 < s.dv_pad) attn_store<T>(s, a, t, head, v * 16 + g4 * 4, w.o[0][v] * f);
+    }
+}
+
+template <typename T, int BUCKET>
+__global__ __launch_bounds__(256) void attn_split_kernel(RmiAttnShape s, RmiAttnArgs a, uint32_t parts, uint32_t keys_per_part) {
+    extern __shared__ __attribute__((aligned(16))) uint8_t lds_raw[];
+    __shared__ uint32_t flag;
+    attn_split<T, BUCKET, false>(s, a, blockIdx.x, parts, keys_per_part, lds_raw, &flag);
+}
+
+// ---- gated linear recurrence
+// one token of one head: a thread takes four state columns and every (256 / (v_pad / 4))-th row
+template <typename T>
+__device__ __forceinline__ void recur_step(const RmiRecurShape &s, const RmiRecurArgs &a, uint32_t head, float *lds) {
+    const uint32_t tid = threadIdx.x, quads = s.v_pad / 4, slices = 256 / quads;
+    float *fs = lds, *qs = fs + s.d_pad, *vs = qs + s.d_pad, *part = vs + s.v_pad;  // part [slices][v_pad]
+    for (uint32_t d = tid; d < s.d_pad; d += 256) {
+        fs[d] = d < s.dim ? a.f[head * s.dim + d] : 1.0f;
+        qs[d] = d < s.dim ? a.q[head * s.dim + d] : 0.0f;
+    }
+    for (uint32_t d = tid; d < s.v_pad; d += 256) vs[d] = d < s.vdim ? a.v[head * s.vdim + d] : 0.0f;
+    __syncthreads();
+    const uint32_t c = tid % quads, sl = tid / quads;
+    f32x4 o = {0.f, 0.f, 0.f, 0.f};
+    if (sl < slices) {
+        float *st = a.state + size_t(head) * s.d_pad * s.v_pad + c * 4;
+        const f32x4 v = *reinterpret_cast<const f32x4 *>(vs + c * 4);
+        for (uint32_t d0 = sl; d0 < s.d_pad; d0 += slices * 8) {  // eight rows in flight
+            f32x4 r[8];
+#pragma unroll
+            for (uint32_t j = 0; j < 8; j++) {
+                const uint32_t d = d0 + j * slices;
+                r[j] = f32x4{0.f, 0.f, 0.f, 0.f};
+                if (a.pos0 && d < s.d_pad) r[j] = *reinterpret_cast<const f32x4 *>(st + size_t(d) * s.v_pad);
+            }
+#pragma unroll
+            for (uint32_t j = 0; j < 8; j++) {
+                const uint32_t d = d0 + j * slices;
+                if (d >= s.d_pad) break;
+                const float f = fs[d], k = 1.0f - f, q = qs[d];
+#pragma unroll
+                for (int e = 0; e < 4; e++) {
+                    r[j][e] = __builtin_fmaf(f, r[j][e], k * v[e]);
+                    o[e] = __builtin_fmaf(q, r[j][e], o[e]);
+                }
+                *reinterpret_cast<f32x4 *>(st + size_t(d) * s.v_pad) = r[j];
+            }
+        }
+        *reinterpret_cast<f32x4 *>(part + sl * s.v_pad + c * 4) = o;
+    }
+    __syncthreads();
+    float *red = fs;  // fs is read no more
+    float mine = 0.0f;
+    if (tid < s.vdim)
+        for (uint32_t i = 0; i < slices; i++) mine += part[i * s.v_pad + tid];
+    const float sq = wave_sum_f32(mine * mine);
+    if ((tid & 63) == 0) red[tid >> 6] = sq;
+    __syncthreads();
+    const float r = 1.0f / sqrtf(((red[0] + red[1]) + (red[2] + red[3])) / float(s.vdim) + s.eps);
+    if (tid < s.vdim) static_cast<T *>(a.out)[size_t(head) * s.vdim + tid] = from_f32<T>(mine * r * a.norm[tid]);
+}
+inline size_t recur_step_lds(const RmiRecurShape &s) {
+    return (2 * size_t(s.d_pad) + s.v_pad + size_t(256 / (s.v_pad / 4)) * s.v_pad) * 4;
+}
+
+template <typename T, int BUCKET>
+__global__ __launch_bounds__(256) void mixers_step_kernel(RmiAttnShape s, RmiAttnArgs a, uint32_t attn_blocks, uint32_t parts,
+                                                          uint32_t keys_per_part, RmiRecurShape rs, RmiRecurArgs ra) {
+    extern __shared__ __attribute__((aligned(16))) uint8_t lds_raw[];
+    __shared__ uint32_t flag;
+    if (blockIdx.x < attn_blocks)
+        attn_split<T, BUCKET, true>(s, a, blockIdx.x, parts, keys_per_part, lds_raw, &flag);
+    else
+        recur_step<T>(rs, ra, blockIdx.x - attn_blocks, reinterpret_cast<float *>(lds_raw));
+}
+
+// Several tokens, in chunks of sixteen.  With P_t the product of f over the chunk's tokens up to t:
+//   o_t = (q_t P_t) S_0 + sum_{s <= t} A_ts v_s,   A_ts = sum_d q_t (1 - f_s) f_{s+1} .. f_t
+//   S'  = P_15 S_0 + sum_s ((1 - f_s) f_{s+1} .. f_15) v_s
+// Every factor is a product of forget gates, at most one: nothing is divided by a decay, so channels that forget
+// at once are as exact as those that never do.  The first kernel makes the factors (all chunks at once), the
+// second walks the chunks with the state in the matrix cores' accumulators.
+constexpr uint32_t kChunk = 16;
+struct RecurScratch {
+    float *qp, *kt, *am, *pc, *o;
+};
+__host__ __device__ inline RecurScratch recur_scratch_at(float *p, const RmiRecurShape &s, uint32_t n_chunks) {
+    const size_t hc = size_t(s.heads) * n_chunks;
+    RecurScratch r;
+    r.qp = p;                               // [head][chunk][16][d_pad]
+    r.kt = r.qp + hc * kChunk * s.d_pad;    // [head][chunk][d_pad][16]
+    r.am = r.kt + hc * kChunk * s.d_pad;    // [head][chunk][16 t][16 s]
+    r.pc = r.am + hc * kChunk * kChunk;     // [head][chunk][d_pad]
+    r.o = r.pc + hc * s.d_pad;              // [head][chunk][16][v_pad]
+    return r;
+}
+
+// one chunk of one head
+__global__ __launch_bounds__(256) void recur_factors_kernel(RmiRecurShape s, RmiRecurArgs a, uint32_t n_chunks) {
+    extern __shared__ __attribute__((aligned(16))) uint8_t lds_raw[];
+    float *fl = reinterpret_cast<float *>(lds_raw);            // [16][d_pad + 4]
+    const uint32_t ld = s.d_pad + 4;
+    float *ql = fl + kChunk * ld;                              // [16][d_pad + 4]
+    float *red = ql + kChunk * ld;                             // [4][16][16]
+    const uint32_t tid = threadIdx.x, chunk = blockIdx.x, head = blockIdx.y, t0 = chunk * kChunk;
+    const RecurScratch ws = recur_scratch_at(a.scratch, s, n_chunks);
+    const size_t hc = size_t(head) * n_chunks + chunk;
+    for (uint32_t e = tid; e < kChunk * s.d_pad; e += 256) {
+        const uint32_t t = e / s.d_pad, d = e % s.d_pad;
+        const bool live = t0 + t < a.n_tokens && d < s.dim;
+        const size_t at = size_t(t0 + t) * s.heads * s.dim + size_t(head) * s.dim + d;
+        fl[t * ld + d] = live ? a.f[at] : 1.0f;  // a token past the end changes nothing
+        ql[t * ld + d] = live ? a.q[at] : 0.0f;
+    }
+    __syncthreads();
+    for (uint32_t d = tid; d < s.d_pad; d += 256) {
+        float p = 1.0f;
+#pragma unroll
+        for (uint32_t t = 0; t < kChunk; t++) {
+            p *= fl[t * ld + d];
+            ws.qp[(hc * kChunk + t) * s.d_pad + d] = ql[t * ld + d] * p;
+        }
+        ws.pc[hc * s.d_pad + d] = p;
+        float k[kChunk];
+        p = 1.0f;
+#pragma unroll
+        for (int t = kChunk - 1; t >= 0; t--) {
+            const float f = fl[t * ld + d];
+            k[t] = (1.0f - f) * p;
+            p *= f;
+        }
+#pragma unroll
+        for (uint32_t j = 0; j < kChunk / 4; j++)
+            *reinterpret_cast<f32x4 *>(ws.kt + (hc * s.d_pad + d) * kChunk + 4 * j) = f32x4{k[4 * j], k[4 * j + 1], k[4 * j + 2], k[4 * j + 3]};
+    }
+    // A: thread (column s, slice of channels)
+    const uint32_t col = tid & 15, slice = tid >> 4;
+    float acc[kChunk];
+#pragma unroll
+    for (uint32_t t = 0; t < kChunk; t++) acc[t] = 0.0f;
+    for (uint32_t d = slice; d < s.d_pad; d += 16) {
+        float w = 0.0f;
+        const float k = 1.0f - fl[col * ld + d];
+#pragma unroll
+        for (uint32_t t = 0; t < kChunk; t++) {
+            w = t == col ? k : w * fl[t * ld + d];
+            acc[t] = __builtin_fmaf(ql[t * ld + d], w, acc[t]);
+        }
+    }
+#pragma unroll
+    for (uint32_t t = 0; t < kChunk; t++) {
+        const float v = rows_sum_f32(acc[t]);  // the wave's four slices
+        if ((tid & 63) < 16) red[(tid >> 6) * 256 + t * 16 + col] = v;
+    }
+    __syncthreads();
+    ws.am[hc * 256 + tid] = (red[tid] + red[256 + tid]) + (red[512 + tid] + red[768 + tid]);
+}
+
+// One workgroup: sixteen value channels of one head over all chunks; wave w holds the state's row tiles w, w + 4, ..
+// A tile of the state in accumulator form (row 4g + r in register r) is the right operand of (q P) S as it lies.
+template <int TPW>
+__global__ __launch_bounds__(256) void recur_scan_kernel(RmiRecurShape s, RmiRecurArgs a, uint32_t n_chunks) {
+    __shared__ f32x4 part[2][4][64];
+    const uint32_t tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, fr = lane & 15, g = lane >> 4;
+    const uint32_t head = blockIdx.y, v0 = blockIdx.x * 16, n_tiles = s.d_pad / 16;
+    const RecurScratch ws = recur_scratch_at(a.scratch, s, n_chunks);
+    f32x4 st[TPW];
+    float *state = a.state + size_t(head) * s.d_pad * s.v_pad + v0 + fr;
+#pragma unroll
+    for (int i = 0; i < TPW; i++) {
+        const uint32_t tile = wave + 4 * i;
+        st[i] = f32x4{0.f, 0.f, 0.f, 0.f};
+        if (tile < n_tiles && a.pos0)
+#pragma unroll
+            for (int r = 0; r < 4; r++) st[i][r] = state[size_t(tile * 16 + g * 4 + r) * s.v_pad];
+    }
+    struct Operands {
+        f32x4 q[TPW], k[TPW], p[TPW];
+        f32x4 v;  // v of tokens 4g .. 4g + 3 at this lane's channel
+        f32x4 am;
+    };
+    auto load = [&](uint32_t chunk) {
+        Operands x;
+        const size_t hc = size_t(head) * n_chunks + chunk;
+#pragma unroll
+        for (int i = 0; i < TPW; i++) {
+            const uint32_t tile = wave + 4 * i < n_tiles ? wave + 4 * i : n_tiles - 1;
+            x.q[i] = *reinterpret_cast<const f32x4 *>(ws.qp + (hc * kChunk + fr) * s.d_pad + tile * 16 + g * 4);
+            x.k[i] = *reinterpret_cast<const f32x4 *>(ws.kt + (hc * s.d_pad + tile * 16 + fr) * kChunk + g * 4);
+            x.p[i] = *reinterpret_cast<const f32x4 *>(ws.pc + hc * s.d_pad + tile * 16 + g * 4);
+        }
+        x.am = *reinterpret_cast<const f32x4 *>(ws.am + hc * 256 + fr * 16 + g * 4);
+#pragma unroll
+        for (int r = 0; r < 4; r++) {
+            const uint32_t t = chunk * kChunk + g * 4 + r;
+            const bool live = t < a.n_tokens && v0 + fr < s.vdim;
+            const float v = a.v[live ? size_t(t) * s.heads * s.vdim + size_t(head) * s.vdim + v0 + fr : 0];
+            x.v[r] = live ? v : 0.0f;
+        }
+        return x;
+    };
+    Operands next = load(0);
+    for (uint32_t chunk = 0; chunk < n_chunks; chunk++) {
+        const Operands x = next;
+        next = load(chunk + 1 < n_chunks ? chunk + 1 : chunk);
+        f32x4 o = {0.f, 0.f, 0.f, 0.f};
+        if (wave == 0) o = mma16_f32(x.am, x.v, o);
+#pragma unroll
+        for (int i = 0; i < TPW; i++) {
+            if (wave + 4 * i >= n_tiles) break;
+            o = mma16_f32(x.q[i], st[i], o);
+#pragma unroll
+            for (int r = 0; r < 4; r++) st[i][r] *= x.p[i][r];
+            st[i] = mma16_f32(x.k[i], x.v, st[i]);
+        }
+        part[chunk & 1][wave][lane] = o;
+        __syncthreads();  // (two buffers: the next chunk's writes cannot meet this one's reads)
+        if (wave == (chunk & 3)) {
+            const f32x4 sum = (part[chunk & 1][0][lane] + part[chunk & 1][1][lane]) + (part[chunk & 1][2][lane] + part[chunk & 1][3][lane]);
+            float *dst = ws.o + ((size_t(head) * n_chunks + chunk) * kChunk + g * 4) * s.v_pad + v0 + fr;
+#pragma unroll
+            for (int r = 0; r < 4; r++) dst[size_t(r) * s.v_pad] = sum[r];
+        }
+    }
+#pragma unroll
+    for (int i = 0; i < TPW; i++) {
+        const uint32_t tile = wave + 4 * i;
+        if (tile < n_tiles)
+#pragma unroll
+            for (int r = 0; r < 4; r++) state[size_t(tile * 16 + g * 4 + r) * s.v_pad] = st[i][r];
+    }
+}
+
+// a wave: one (token, head): o over its root mean square, times the weight
+template <typename T>
+__global__ __launch_bounds__(256) void recur_norm_kernel(RmiRecurShape s, RmiRecurArgs a, uint32_t n_chunks) {
+    const uint32_t lane = threadIdx.x & 63, t = blockIdx.x * 4 + (threadIdx.x >> 6), head = blockIdx.y;
+    if (t >= a.n_tokens) return;
+    const float *o = recur_scratch_at(a.scratch, s, n_chunks).o + (size_t(head) * n_chunks * kChunk + t) * s.v_pad;
+    float v[kMaxHeadDim / 64], sq = 0.0f;
+#pragma unroll
+    for (uint32_t j = 0; j < kMaxHeadDim / 64; j++) {
+        v[j] = lane + j * 64 < s.vdim ? o[lane + j * 64] : 0.0f;
+        sq = __builtin_fmaf(v[j], v[j], sq);
+    }
+    const float r = 1.0f / sqrtf(wave_sum_f32(sq) / float(s.vdim) + s.eps);
+#pragma unroll
+    for (uint32_t j = 0; j < kMaxHeadDim / 64; j++)
+        if (lane + j * 64 < s.vdim)
+            static_cast<T *>(a.out)[size_t(t) * a.out_ld + size_t(head) * s.vdim + lane + j * 64] =
+                from_f32<T>(v[j] * r * a.norm[lane + j * 64]);
+}
+
+// ------------------------------------------------------------------ launches
+// Keys over workgroups where the columns alone would not fill the chip; at most kMaxParts parts of 128 keys or more.
+constexpr uint32_t kMaxParts = 32;
+constexpr uint32_t kSplitMaxCols = 256;  // per key/value head
+void attn_parts(const RmiAttnShape &s, uint32_t n_tokens, uint32_t n_keys, uint32_t *parts, uint32_t *keys_per_part) {
+    const uint32_t tiles = (n_tokens * (s.heads / s.kv_heads) + 15) / 16;
+    const uint32_t slots = s.kv_heads * tiles, cus = uint32_t(rmi_device_cus());
+    uint32_t p = (n_keys + 127) / 128;
+    const uint32_t fill = (cus + slots - 1) / slots;
+    if (p > fill) p = fill;
+    if (p > kMaxParts) p = kMaxParts;
+    if (slots > kAttnCounters || p < 1) p = 1;
+    const uint32_t align = 4 * kKeyBlock;  // four waves of whole value blocks
+    *keys_per_part = ((n_keys + p - 1) / p + align - 1) / align * align;
+    *parts = (n_keys + *keys_per_part - 1) / *keys_per_part;
+}
+
+int check_attn(const RmiAttnShape &s, const RmiAttnArgs &a) {
+    if (s.dim > kMaxHeadDim || s.vdim > kMaxHeadDim || s.taps == 0 || s.taps > kMaxTaps || s.heads % s.kv_heads || s.rot_dims > s.dim ||
+        s.rot_dims % 2 || s.capacity % kKeyBlock || s.dk_pad % 32 || s.dv_pad % 16 || s.dk_pad < s.dim || s.dv_pad < s.vdim ||
+        s.dk_pad > kMaxHeadDim || s.dv_pad > kMaxHeadDim || a.pos0 + a.n_tokens > s.capacity)
+        return rmi_fail(RMI_HIP_E_INVALID, "bad attention shape");
+    return RMI_HIP_OK;
+}
+uint32_t bucket_of(const RmiAttnShape &s) {
+    const uint32_t d = s.dk_pad > s.dv_pad ? s.dk_pad : s.dv_pad;
+    return d <= 64 ? 64 : d <= 128 ? 128 : 256;
+}
+size_t split_lds(uint32_t elem_bytes, const RmiAttnShape &s) {
+    const size_t q = size_t(16) * s.dk_pad * elem_bytes, merge = size_t(3) * attn_part_floats(s.dv_pad) * 4;
+    return q > merge ? q : merge;
+}
+
+template <typename T>
+int attn_pass(const RmiAttnShape &s, const RmiAttnArgs &a, hipStream_t st) {
+    const uint32_t n_heads = s.heads + 2 * s.kv_heads, group = s.heads / s.kv_heads, n_cols = a.n_tokens * group;
+    hipLaunchKernelGGL(conv_rotate_kernel<T>, dim3(n_heads, (a.n_tokens + 3) / 4), dim3(256), 0, st, s, a);
+    const uint32_t bucket = bucket_of(s);
+    if (n_cols <= kSplitMaxCols) {
+        uint32_t parts, kpp;
+        attn_parts(s, a.n_tokens, a.pos0 + a.n_tokens, &parts, &kpp);
+        const dim3 grid(s.kv_heads * ((n_cols + 15) / 16) * parts);
+        const size_t lds = split_lds(sizeof(T), s);
+        if (bucket == 64)
+            hipLaunchKernelGGL((attn_split_kernel<T, 64>), grid, dim3(256), lds, st, s, a, parts, kpp);
+        else if (bucket == 128)
+            hipLaunchKernelGGL((attn_split_kernel<T, 128>), grid, dim3(256), lds, st, s, a, parts, kpp);
+        else
+            hipLaunchKernelGGL((attn_split_kernel<T, 256>), grid, dim3(256), lds, st, s, a, parts, kpp);
+    } else {
+        auto grid = [&](uint32_t qt) { return dim3((n_cols + 64 * qt - 1) / (64 * qt), s.kv_heads); };
+        if (bucket == 64)
+            hipLaunchKernelGGL((attn_pass_kernel<T, 64, 2>), grid(2), dim3(256), 0, st, s, a);
+        else if (bucket == 128)
+            hipLaunchKernelGGL((attn_pass_kernel<T, 128, 2>), grid(2), dim3(256), 0, st, s, a);
+        else
+            hipLaunchKernelGGL((attn_pass_kernel<T, 256, 1>), grid(1), dim3(256), 0, st, s, a);
+    }
+    RMI_HIP_CHECK(hipGetLastError());
+    return RMI_HIP_OK;
+}
+
+int check_recur(const RmiRecurShape &s) {
+    if (s.heads == 0 || s.dim == 0 || s.vdim == 0 || s.dim > kMaxHeadDim || s.vdim > kMaxHeadDim || s.d_pad % 16 || s.v_pad % 16 ||
+        s.d_pad < s.dim || s.v_pad < s.vdim || s.d_pad > kMaxHeadDim || s.v_pad > kMaxHeadDim)
+        return rmi_fail(RMI_HIP_E_INVALID, "bad recurrence shape");
+    return RMI_HIP_OK;
+}
+
+template <typename T>
+int mixers_step(const RmiAttnShape *as, const RmiAttnArgs *aa, const RmiRecurShape *rs, const RmiRecurArgs *ra, hipStream_t st) {
+    const RmiAttnShape s = as ? *as : RmiAttnShape{};
+    const RmiAttnArgs a = aa ? *aa : RmiAttnArgs{};
+    const RmiRecurShape r = rs ? *rs : RmiRecurShape{};
+    const RmiRecurArgs b = ra ? *ra : RmiRecurArgs{};
+    uint32_t parts = 1, kpp = 0, blocks = 0;
+    size_t lds = 0;
+    if (as) {
+        attn_parts(s, 1, a.pos0 + 1, &parts, &kpp);
+        blocks = s.kv_heads * ((s.heads / s.kv_heads + 15) / 16) * parts;
+        lds = split_lds(sizeof(T), s);
+    }
+    if (rs && recur_step_lds(r) > lds) lds = recur_step_lds(r);
+    const dim3 grid(blocks + (rs ? r.heads : 0));
+    const uint32_t bucket = as ? bucket_of(s) : 64;
+    if (bucket == 64)
+        hipLaunchKernelGGL((mixers_step_kernel<T, 64>), grid, dim3(256), lds, st, s, a, blocks, parts, kpp, r, b);
+    else if (bucket == 128)
+        hipLaunchKernelGGL((mixers_step_kernel<T, 128>), grid, dim3(256), lds, st, s, a, blocks, parts, kpp, r, b);
+    else
+        hipLaunchKernelGGL((mixers_step_kernel<T, 256>), grid, dim3(256), lds, st, s, a, blocks, parts, kpp, r, b);
+    RMI_HIP_CHECK(hipGetLastError());
+    return RMI_HIP_OK;
+}
+
+}  // namespace
+
+size_t rmi_attn_scratch_bytes(const RmiAttnShape &s) {
+    const size_t cols = kSplitMaxCols > s.heads / s.kv_heads ? kSplitMaxCols : s.heads / s.kv_heads;
+    const size_t slots = size_t(s.kv_heads) * ((cols + 15) / 16);
+    return kAttnCounters * 4 + slots * kMaxParts * attn_part_floats(s.dv_pad) * 4;
+}
+
+size_t rmi_recur_scratch_floats(const RmiRecurShape &s, uint32_t max_tokens) {
+    const size_t hc = size_t(s.heads) * ((max_tokens + kChunk - 1) / kChunk);
+    return hc * (2 * size_t(kChunk) * s.d_pad + kChunk * kChunk + s.d_pad + size_t(kChunk) * s.v_pad);
+}
+
+int rmi_attn_pass(uint32_t elem_bytes, const RmiAttnShape &s, const RmiAttnArgs &a, hipStream_t st) {
+    if (a.n_tokens == 0) return RMI_HIP_OK;
+    const int rc = check_attn(s, a);
+    if (rc != RMI_HIP_OK) return rc;
+    return elem_bytes == 2 ? attn_pass<rmi_bf16>(s, a, st) : attn_pass<float>(s, a, st);
+}
+
+int rmi_recur_pass(uint32_t elem_bytes, const RmiRecurShape &s, const RmiRecurArgs &a, hipStream_t st) {
+    if (a.n_tokens == 0) return RMI_HIP_OK;
+    const int rc = check_recur(s);
+    if (rc != RMI_HIP_OK) return rc;
+    const uint32_t n_chunks = (a.n_tokens + kChunk - 1) / kChunk;
+    const size_t lds = (2 * size_t(kChunk) * (s.d_pad + 4) + 1024) * 4;
+    hipLaunchKernelGGL(recur_factors_kernel, dim3(n_chunks, s.heads), dim3(256), lds, st, s, a, n_chunks);
+    const dim3 grid(s.v_pad / 16, s.heads);
+    if (s.d_pad <= 64)
+        hipLaunchKernelGGL(recur_scan_kernel<1>, grid, dim3(256), 0, st, s, a, n_chunks);
+    else if (s.d_pad <= 128)
+        hipLaunchKernelGGL(recur_scan_kernel<2>, grid, dim3(256), 0, st, s, a, n_chunks);
+    else
+        hipLaunchKernelGGL(recur_scan_kernel<4>, grid, dim3(256), 0, st, s, a, n_chunks);
+    const dim3 ngrid((a.n_tokens + 3) / 4, s.heads);
+    if (elem_bytes == 2)
+        hipLaunchKernelGGL(recur_norm_kernel<rmi_bf16>, ngrid, dim3(256), 0, st, s, a, n_chunks);
+    else
+        hipLaunchKernelGGL(recur_norm_kernel<float>, ngrid, dim3(256), 0, st, s, a, n_chunks);
+    RMI_HIP_CHECK(hipGetLastError());
+    return RMI_HIP_OK;
+}
+
+int rmi_mixers_step(uint32_t elem_bytes, const RmiAttnShape *as, const RmiAttnArgs *aa, const RmiRecurShape *rs, const RmiRecurArgs *ra,
+                    hipStream_t st) {
+    if (!as && !rs) return RMI_HIP_OK;
+    int rc = as ? check_attn(*as, *aa) : RMI_HIP_OK;
+    if (rc == RMI_HIP_OK && rs) rc = check_recur(*rs);
+    if (rc != RMI_HIP_OK) return rc;
+    return elem_bytes == 2 ? mixers_step<rmi_bf16>(as, aa, rs, ra, st) : mixers_step<float>(as, aa, rs, ra, st);
+}

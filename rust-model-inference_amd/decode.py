@@ -1,6 +1,6 @@
-"""Host-side mirror of the reference's ``Qwen3Session`` (src/models/qwen3.rs:581-1158) over the
-device-resident decode entry points of the C ABI: weights go to HBM once, then whole generations
-run on the GPU with one synchronisation at the end.
+"""Decoder sessions over the device-resident entry points of the C ABI: weights go to HBM once, then whole
+generations run on the GPU with one synchronisation at the end.  ``Qwen3Session`` mirrors the reference's
+(src/models/qwen3.rs:581-1158); ``RuvenexSession`` runs a model folder of that design; ``models`` picks the class.
 """
 import ctypes as C
 
@@ -13,9 +13,58 @@ _MATMULS = (("wq", "attn_q"), ("wk", "attn_k"), ("wv", "attn_v"), ("wo", "attn_o
 _NORMS = (("attn_norm", "attn_norm"), ("ffn_norm", "ffn_norm"), ("q_norm", "attn_q_norm"), ("k_norm", "attn_k_norm"))
 
 
-class Qwen3Session:
+class _Session:
+    """What the sessions share: `_abi` names the C functions, `_h` is the handle, `vocab` the logits' width."""
+
+    _abi = None
+    _h = None
+
+    def _fn(self, name):
+        return getattr(hip.lib, f"rmi_hip_{self._abi}_{name}")
+
+    def set_stop_ids(self, ids):
+        """The tokenizer's EOS / `im_end` ids (src/models/qwen3.rs:1123-1130): generation ends before the first."""
+        ids = np.ascontiguousarray(ids, np.uint32)
+        hip.check(self._fn("set_stop_ids")(self._h, hip.ptr(ids, hip._u32p), ids.size))
+
+    def set_prompt_passes(self, enabled):
+        """Prompt positions as many to a pass as the session takes (True, the default), every position its own step
+        (False), or that many to a pass (an int above 1); same results either way (bit for bit for Qwen3, within
+        rounding for Ruvenex)."""
+        hip.check(self._fn("set_prompt_passes")(self._h, int(enabled)))
+
+    def generate(self, prompt, max_new, dump_steps=()):
+        prompt = np.ascontiguousarray(prompt, np.uint32)
+        steps = prompt.size + max_new - 1
+        gen = np.zeros(max(max_new, 1), np.uint32)
+        argmax = np.zeros(steps, np.uint32)
+        top2 = np.zeros((steps, 2), np.float32)
+        dump_steps = np.ascontiguousarray(dump_steps, np.uint32)
+        dump = np.zeros((max(dump_steps.size, 1), self.vocab), np.float32)
+        seconds = C.c_double()
+        n = self._fn("generate")(self._h, hip.ptr(prompt, hip._u32p), prompt.size, max_new, hip.ptr(gen, hip._u32p),
+                                 hip.ptr(argmax, hip._u32p), hip.ptr(top2, hip._f32p), hip.ptr(dump_steps, hip._u32p),
+                                 dump_steps.size, hip.ptr(dump, hip._f32p), C.byref(seconds))
+        if n < 0:
+            raise hip.RmiHipError(n, hip.last_error())
+        return dict(tokens=gen[:n], argmax=argmax, top2=top2, dump=dump[:dump_steps.size], seconds=seconds.value,
+                    steps=steps)
+
+    def close(self):
+        if self._h:
+            self._fn("destroy")(self._h)
+            self._h = None
+
+    def __del__(self):
+        self.close()
+
+
+class Qwen3Session(_Session):
     """`metadata` and `tensors` as a GGUF file gives them (keys of src/core/loader.rs:379-461, tensor
     names of src/models/qwen3.rs:269-349); every 2-D weight must be Q8_0 bytes, norms f32."""
+
+    _abi = "qwen3"
+    vocab = property(lambda self: self.config.vocab)
 
     def __init__(self, metadata, tensors, capacity, rounding=hip.ROUND_TIES_EVEN):
         g = lambda k: int(metadata[f"qwen3.{k}"])  # noqa: E731
@@ -72,38 +121,34 @@ class Qwen3Session:
             raise hip.RmiHipError(-1, hip.last_error())
         return self
 
-    def set_stop_ids(self, ids):
-        """The tokenizer's EOS / `im_end` ids (src/models/qwen3.rs:1123-1130): generation ends before the first."""
-        ids = np.ascontiguousarray(ids, np.uint32)
-        hip.check(hip.lib.rmi_hip_qwen3_set_stop_ids(self._h, hip.ptr(ids, hip._u32p), ids.size))
 
-    def set_prompt_passes(self, enabled):
-        """Prompt positions 128 to a pass (True, the default), every position its own step (False), or that many to a
-        pass (an int above 1, at most 128); same results either way."""
-        hip.check(hip.lib.rmi_hip_qwen3_set_prompt_passes(self._h, int(enabled)))
+class RuvenexSession(_Session):
+    """A Ruvenex model folder (config.json, model.safetensors).  dtype: hip.DTYPE_BF16 or hip.DTYPE_F32 (everything
+    true f32); capacity: most tokens of a sequence.  One sequence at a time."""
 
-    def generate(self, prompt, max_new, dump_steps=()):
-        prompt = np.ascontiguousarray(prompt, np.uint32)
-        steps = prompt.size + max_new - 1
-        gen = np.zeros(max(max_new, 1), np.uint32)
-        argmax = np.zeros(steps, np.uint32)
-        top2 = np.zeros((steps, 2), np.float32)
-        dump_steps = np.ascontiguousarray(dump_steps, np.uint32)
-        dump = np.zeros((max(dump_steps.size, 1), self.config.vocab), np.float32)
-        seconds = C.c_double()
-        n = hip.lib.rmi_hip_qwen3_generate(self._h, hip.ptr(prompt, hip._u32p), prompt.size, max_new,
-                                           hip.ptr(gen, hip._u32p), hip.ptr(argmax, hip._u32p), hip.ptr(top2, hip._f32p),
-                                           hip.ptr(dump_steps, hip._u32p), dump_steps.size, hip.ptr(dump, hip._f32p),
-                                           C.byref(seconds))
-        if n < 0:
-            raise hip.RmiHipError(n, hip.last_error())
-        return dict(tokens=gen[:n], argmax=argmax, top2=top2, dump=dump[:dump_steps.size], seconds=seconds.value,
-                    steps=steps)
+    _abi = "ruvenex"
 
-    def close(self):
-        if self._h:
-            hip.lib.rmi_hip_qwen3_destroy(self._h)
-            self._h = None
+    def __init__(self, folder, capacity, dtype=hip.DTYPE_BF16):
+        self._h = hip.lib.rmi_hip_ruvenex_open(str(folder).encode(), dtype, int(capacity))
+        if not self._h:
+            raise hip.RmiHipError(-1, hip.last_error())
+        v = [C.c_uint32() for _ in range(4)]
+        hip.check(hip.lib.rmi_hip_ruvenex_sizes(self._h, *[C.byref(x) for x in v]))
+        self.vocab, self.width, self.n_layer, self.capacity = (x.value for x in v)
 
-    def __del__(self):
-        self.close()
+    position = property(lambda self: hip.lib.rmi_hip_ruvenex_position(self._h))
+
+    def step(self, tokens, want=(), layers=False):
+        """The sequence's next tokens; logits [len(want), vocab] of the places `want` among them.  With `layers` also
+        the residual stream behind every layer, [n_layer, tokens, width]."""
+        tokens = np.ascontiguousarray(tokens, np.uint32)
+        want = np.ascontiguousarray(want, np.uint32)
+        logits = np.zeros((want.size, self.vocab), np.float32)
+        dump = np.zeros((self.n_layer, tokens.size, self.width), np.float32) if layers else None
+        hip.check(hip.lib.rmi_hip_ruvenex_step(self._h, hip.ptr(tokens, hip._u32p), tokens.size, hip.ptr(want, hip._u32p), want.size,
+                                               hip.ptr(logits, hip._f32p), hip.ptr(dump, hip._f32p) if layers else None))
+        return (logits, dump) if layers else logits
+
+    def reset(self):
+        """The sequence is over; the next step begins a new one."""
+        hip.check(hip.lib.rmi_hip_ruvenex_reset(self._h))

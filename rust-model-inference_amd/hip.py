@@ -10,7 +10,10 @@ import numpy as np
 
 _HERE = os.path.dirname(os.path.abspath(__file__))
 LIB_PATH = os.path.join(_HERE, "librmi_hip.so")
+FOLDER_LIB_PATH = os.path.join(_HERE, "librmi_folder.so")  # the model-folder sessions alone (`make folder`)
 
+DTYPE_F32 = 0
+DTYPE_BF16 = 30
 DTYPE_Q4_0 = 2
 DTYPE_Q8_0 = 8
 DTYPE_Q4_K = 12
@@ -165,6 +168,17 @@ SIGNATURES = {
     "rmi_hip_gguf_upload_stack": (_vp, [_vp, C.POINTER(C.c_char_p), C.c_int]),
     "rmi_hip_gguf_qwen3_config": (C.c_int, [_vp, _u32, C.c_int, C.POINTER(Qwen3Config)]),
     "rmi_hip_qwen3_create_from_gguf": (_vp, [_vp, _u32, C.c_int]),
+    "rmi_hip_model_folder_architecture": (C.c_int64, [C.c_char_p, C.c_char_p, _sz]),
+    "rmi_hip_ruvenex_open": (_vp, [C.c_char_p, C.c_int, _u32]),
+    "rmi_hip_ruvenex_destroy": (None, [_vp]),
+    "rmi_hip_ruvenex_sizes": (C.c_int, [_vp, _u32p, _u32p, _u32p, _u32p]),
+    "rmi_hip_ruvenex_step": (C.c_int, [_vp, _u32p, _u32, _u32p, _u32, _f32p, _f32p]),
+    "rmi_hip_ruvenex_position": (_u32, [_vp]),
+    "rmi_hip_ruvenex_reset": (C.c_int, [_vp]),
+    "rmi_hip_ruvenex_set_stop_ids": (C.c_int, [_vp, _u32p, _u32]),
+    "rmi_hip_ruvenex_set_prompt_passes": (C.c_int, [_vp, C.c_int]),
+    "rmi_hip_ruvenex_generate": (C.c_int, [_vp, _u32p, _u32, _u32, _u32p, _u32p, _f32p, _u32p, _u32, _f32p,
+                                           C.POINTER(C.c_double)]),
     "rmi_hip_gemv_group_shape": (C.c_int, [_vp, C.POINTER(_u32), C.POINTER(_u32)]),
     "rmi_hip_gemv_group_destroy": (None, [_vp]),
     "rmi_hip_gemv_group_run_dev": (C.c_int, [_vp, _vp]),
@@ -177,13 +191,26 @@ class RmiHipError(RuntimeError):
         self.code = code
 
 
+def _absent(name):
+    def call(*_):
+        raise ImportError(f"{name} is not in {os.path.basename(FOLDER_LIB_PATH)}: build the whole library "
+                          "(`python -c 'import __graft_entry__ as g; g.build()'`)")
+    return call
+
+
 def load_library():
-    if not os.path.exists(LIB_PATH):
+    path = LIB_PATH
+    if not os.path.exists(path) and os.path.exists(FOLDER_LIB_PATH):
+        path = FOLDER_LIB_PATH
+    if not os.path.exists(path):
         raise ImportError(
             f"{LIB_PATH} is missing: build it with `python -c 'import __graft_entry__ as g; g.build()'` "
             "(hipcc, gfx950); there is no CPU fallback")
-    lib = C.CDLL(LIB_PATH)
+    lib = C.CDLL(path)
     for name, (res, args) in SIGNATURES.items():
+        if path == FOLDER_LIB_PATH and not hasattr(lib, name):
+            setattr(lib, name, _absent(name))
+            continue
         fn = getattr(lib, name)  # AttributeError names a missing export
         fn.restype = res
         fn.argtypes = args

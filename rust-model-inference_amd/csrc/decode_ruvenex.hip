@@ -126,7 +126,7 @@ int rmi_hip_ruvenex::enqueue_layers(uint32_t step0, uint32_t n, hipStream_t st, 
         r.pos0 = step0;
         r.n_tokens = n;
         r.scratch = recur_scratch;
-        if (n == 1 && rmi_dense_gemv_fits(elem, k_in) && rmi_dense_gemv_fits(elem, y.w_out.k_pad)) {
+        if (n == 1 && rmi_dense_gemv_fits(elem, k_in)) {
             rc = rmi_dense_norm_gemv(elem, y.w_in, x, y.norm, eps, width, y.in, st);
             if (rc == RMI_HIP_OK) rc = rmi_mixers_step(elem, &y.attn, &a, &y.recur, &r, st);
             if (rc == RMI_HIP_OK) rc = rmi_dense_gemv_residual(elem, y.w_out, act, y.out, x, width, st);
@@ -153,6 +153,7 @@ int rmi_hip_ruvenex::enqueue_logits(const uint32_t *rows, uint32_t n_rows, hipSt
     s.n_segs = 1;
     s.n_rows = head.n_rows;
     s.s[0] = RmiRowSeg{logits, nullptr, nullptr, 0, vocab, vocab, uint16_t(kActNone), 0};
+    rmi_row_segs_done(&s);
     if (n_rows == 1 && !rows && rmi_dense_gemv_fits(elem, k_in)) return rmi_dense_norm_gemv(elem, head, x, final_norm, eps, width, s, st);
     const int rc = rmi_dense_norm(elem, x, rows, final_norm, eps, h, n_rows, width, k_in, st);
     return rc == RMI_HIP_OK ? rmi_dense_gemm(elem, head, h, s, n_rows, st) : rc;
@@ -518,6 +519,7 @@ bool rmi_hip_ruvenex::load(const RmiModelFolder &folder, uint32_t elem_bytes, ui
             n_rows += rmi_dense_pad(q1.n, kDenseRowAlign);
         }
         y.in.n_rows = n_rows;
+        rmi_row_segs_done(&y.in);
         {
             DenseBuilder b(elem, n_rows, k_in);
             for (size_t i = 0; i < parts.size() && rd.ok; i++) b.put(rd.tensor(parts[i].name, {parts[i].n, width}), y.in.s[i].row0, 0);

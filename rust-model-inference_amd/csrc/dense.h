@@ -28,9 +28,13 @@ struct RmiRowSeg {
 constexpr uint32_t kMaxRowSegs = 12;
 struct RmiRowSegs {
     RmiRowSeg s[kMaxRowSegs];
+    uint32_t start[kMaxRowSegs];  // s[i].row0, and n_rows from n_segs on: rmi_row_segs_done fills it
     uint32_t n_segs;
     uint32_t n_rows;  // padded rows of the weight
 };
+inline void rmi_row_segs_done(RmiRowSegs *r) {
+    for (uint32_t i = 0; i < kMaxRowSegs; i++) r->start[i] = i < r->n_segs ? r->s[i].row0 : r->n_rows;
+}
 
 // x[token][row] += sum over column segments i of gate_i[token][row] * scale_i * (W_i a_i)[row].  A segment's columns
 // end at k_end (padded); a null gate is one.
@@ -51,6 +55,15 @@ struct RmiDense {
     uint32_t k_pad = 0;
 };
 
+// More than 64 KiB of dynamic LDS has to be asked for (a compute unit has 160 KiB; some is left for static arrays).
+constexpr uint32_t kLdsAskedFor = 144 * 1024;
+template <typename K>
+int rmi_allow_lds(K kernel, size_t bytes) {
+    if (bytes <= 64 * 1024) return RMI_HIP_OK;
+    RMI_HIP_CHECK(hipFuncSetAttribute(reinterpret_cast<const void *>(kernel), hipFuncAttributeMaxDynamicSharedMemorySize, kLdsAskedFor));
+    return RMI_HIP_OK;
+}
+
 // elem_bytes 2: bf16, 4: f32
 // h[i][0 .. k_pad) = rms_norm(x[rows ? rows[i] : i]) * weight, zeros past n
 int rmi_dense_norm(uint32_t elem_bytes, const float *x, const uint32_t *rows, const float *weight, float eps, void *h,
@@ -62,7 +75,7 @@ int rmi_dense_embed(uint32_t elem_bytes, const RmiDense &table, const uint32_t *
 int rmi_dense_gemm(uint32_t elem_bytes, const RmiDense &w, const void *a, const RmiRowSegs &segs, uint32_t n_tokens, hipStream_t st);
 int rmi_dense_gemm_residual(uint32_t elem_bytes, const RmiDense &w, const void *a, const RmiColSegs &segs, float *x, uint32_t width,
                             uint32_t n_tokens, hipStream_t st);
-// one token: the norm in front of the product is part of the launch
+// one token: the norm in front of the product is part of the launch, for as many columns as a workgroup holds
 bool rmi_dense_gemv_fits(uint32_t elem_bytes, uint32_t k_pad);
 int rmi_dense_norm_gemv(uint32_t elem_bytes, const RmiDense &w, const float *x, const float *weight, float eps, uint32_t n,
                         const RmiRowSegs &segs, hipStream_t st);

@@ -30,14 +30,22 @@ __global__ __launch_bounds__(256) void embed_kernel(const T *__restrict__ table,
     for (uint32_t i = threadIdx.x; i < n; i += 256) x[size_t(blockIdx.x) * n + i] = to_f32(table[size_t(t) * k_pad + i]) * scale;
 }
 
+// which row segment a row lies in: the starts sit side by side (unused ones at the end of the range)
+__device__ __forceinline__ uint32_t seg_of(const RmiRowSegs &rs, uint32_t row) {
+    uint32_t si = 0;
+#pragma unroll
+    for (uint32_t i = 1; i < kMaxRowSegs; i++) si += row >= rs.start[i] ? 1u : 0u;
+    return si;
+}
+
 // ------------------------------------------------------------------ GEMM
 // One workgroup of four waves: BN weight rows x BT tokens, k in steps of 128 bytes a row through two LDS buffers; the
-// pieces of the next step are loaded into registers while this one is multiplied.  A row of a buffer is eight
+// pieces of the next PD steps are on their way to registers while one is multiplied.  A row of a buffer is eight
 // 16-byte pieces, piece p at slot p ^ (row & 7), so that the sixteen rows of a fragment spread over the banks.
 // Weights are the A operand: a lane ends with four consecutive rows of one token.
 constexpr uint32_t kStepBytes = 128;
 
-template <typename T, int BN, int BT, int WN, int WT, bool RESIDUAL>
+template <typename T, int BN, int BT, int WN, int WT, int PD, bool RESIDUAL>
 __global__ __launch_bounds__(256) void dense_gemm_kernel(const T *__restrict__ w, const T *__restrict__ a, uint32_t n_rows,
                                                          uint32_t k_pad, uint32_t n_tokens, uint32_t grid_n, uint32_t grid_t,
                                                          RmiRowSegs rs, RmiColSegs cs, float *__restrict__ x, uint32_t width) {
@@ -69,108 +77,102 @@ __global__ __launch_bounds__(256) void dense_gemm_kernel(const T *__restrict__ w
         adst[i] = BN * 8 + r * 8 + (p ^ (r & 7));
     }
     f32x4 acc[NN][NT];
-    f32x4 tot[RESIDUAL ? NN : 1][RESIDUAL ? NT : 1];
 #pragma unroll
     for (int i = 0; i < NN; i++)
 #pragma unroll
-        for (int j = 0; j < NT; j++) {
-            acc[i][j] = f32x4{0.f, 0.f, 0.f, 0.f};
-            if (RESIDUAL) tot[i][j] = f32x4{0.f, 0.f, 0.f, 0.f};
-        }
-    u32x4 rw[PW], ra[PA];
-    auto load = [&](uint32_t step) {
+        for (int j = 0; j < NT; j++) acc[i][j] = f32x4{0.f, 0.f, 0.f, 0.f};
+    constexpr uint32_t kStepElems = kStepBytes / sizeof(T);
+    const uint32_t n_steps = k_pad / kStepElems;
+    u32x4 rw[PD][PW], ra[PD][PA];
+    auto load = [&](int slot, uint32_t step) {
+        if (step >= n_steps) return;
 #pragma unroll
-        for (int i = 0; i < PW; i++) rw[i] = *reinterpret_cast<const u32x4 *>(wsrc[i] + size_t(step) * kStepBytes);
+        for (int i = 0; i < PW; i++) rw[slot][i] = *reinterpret_cast<const u32x4 *>(wsrc[i] + size_t(step) * kStepBytes);
 #pragma unroll
-        for (int i = 0; i < PA; i++) ra[i] = *reinterpret_cast<const u32x4 *>(asrc[i] + size_t(step) * kStepBytes);
+        for (int i = 0; i < PA; i++) ra[slot][i] = *reinterpret_cast<const u32x4 *>(asrc[i] + size_t(step) * kStepBytes);
     };
-    auto park = [&](uint32_t buf) {
+    auto park = [&](int slot, uint32_t buf) {
 #pragma unroll
-        for (int i = 0; i < PW; i++) lds[buf][wdst[i]] = rw[i];
+        for (int i = 0; i < PW; i++) lds[buf][wdst[i]] = rw[slot][i];
 #pragma unroll
-        for (int i = 0; i < PA; i++) lds[buf][adst[i]] = ra[i];
+        for (int i = 0; i < PA; i++) lds[buf][adst[i]] = ra[slot][i];
     };
     const uint32_t fr = lane & 15, g = lane >> 4;
-    // the gated sum of a finished column segment
+    // a finished column segment goes to the residual stream at once (each element is one thread's), so that no second
+    // set of accumulators is held
     auto fold = [&](const RmiColSeg &s) {
         if constexpr (RESIDUAL) {
+            const bool quads = (width & 3) == 0;
 #pragma unroll
             for (int j = 0; j < NT; j++) {
                 const uint32_t tok = tok0 + wt + j * 16 + fr;
-                const bool live = tok < n_tokens;
 #pragma unroll
                 for (int i = 0; i < NN; i++) {
                     const uint32_t row = row0 + wn + i * 16 + g * 4;
+                    const size_t at = size_t(tok) * width + row;
+                    if (tok < n_tokens && row < width) {
+                        if (quads) {
+                            f32x4 v = acc[i][j] * s.scale;
+                            if (s.gate) v *= *reinterpret_cast<const f32x4 *>(s.gate + at);
+                            *reinterpret_cast<f32x4 *>(x + at) += v;
+                        } else {
 #pragma unroll
-                    for (int r = 0; r < 4; r++) {
-                        const float gate = s.gate && live && row + r < width ? s.gate[size_t(tok) * width + row + r] : 1.0f;
-                        tot[i][j][r] = __builtin_fmaf(gate, acc[i][j][r] * s.scale, tot[i][j][r]);
+                            for (int r = 0; r < 4; r++)
+                                if (row + r < width) x[at + r] += acc[i][j][r] * s.scale * (s.gate ? s.gate[at + r] : 1.0f);
+                        }
                     }
                     acc[i][j] = f32x4{0.f, 0.f, 0.f, 0.f};
                 }
             }
         }
     };
-    constexpr uint32_t kStepElems = kStepBytes / sizeof(T);
-    const uint32_t n_steps = k_pad / kStepElems;
     uint32_t seg = 0;
-    load(0);
-    park(0);
+#pragma unroll
+    for (int j = 0; j < PD; j++) load(j, j);
+    park(0, 0);
+    load(0, PD);
     __syncthreads();
-    for (uint32_t step = 0; step < n_steps; step++) {
-        const uint32_t buf = step & 1;
-        if (step + 1 < n_steps) load(step + 1);
+    for (uint32_t step0 = 0; step0 < n_steps; step0 += PD) {
 #pragma unroll
-        for (int c = 0; c < 2; c++) {
-            u32x4 fw[NN], fa[NT];
+        for (int j = 0; j < PD; j++) {  // register slots by compile-time index
+            const uint32_t step = step0 + j, buf = step & 1;
+            if (step >= n_steps) break;
 #pragma unroll
-            for (int i = 0; i < NN; i++) {
-                const uint32_t r = wn + i * 16 + fr;
-                fw[i] = lds[buf][r * 8 + ((c * 4 + g) ^ (r & 7))];
+            for (int c = 0; c < 2; c++) {
+                u32x4 fw[NN], fa[NT];
+#pragma unroll
+                for (int i = 0; i < NN; i++) {
+                    const uint32_t r = wn + i * 16 + fr;
+                    fw[i] = lds[buf][r * 8 + ((c * 4 + g) ^ (r & 7))];
+                }
+#pragma unroll
+                for (int i = 0; i < NT; i++) {
+                    const uint32_t r = wt + i * 16 + fr;
+                    fa[i] = lds[buf][BN * 8 + r * 8 + ((c * 4 + g) ^ (r & 7))];
+                }
+#pragma unroll
+                for (int i = 0; i < NN; i++)
+#pragma unroll
+                    for (int i2 = 0; i2 < NT; i2++) acc[i][i2] = mma16<T>(fw[i], fa[i2], acc[i][i2]);
             }
-#pragma unroll
-            for (int j = 0; j < NT; j++) {
-                const uint32_t r = wt + j * 16 + fr;
-                fa[j] = lds[buf][BN * 8 + r * 8 + ((c * 4 + g) ^ (r & 7))];
+            if (step + 1 < n_steps) {
+                park((j + 1) % PD, buf ^ 1);
+                load((j + 1) % PD, step + 1 + PD);
             }
-#pragma unroll
-            for (int i = 0; i < NN; i++)
-#pragma unroll
-                for (int j = 0; j < NT; j++) acc[i][j] = mma16<T>(fw[i], fa[j], acc[i][j]);
+            if (RESIDUAL && (step + 1) * kStepElems == cs.s[seg].k_end) {
+                fold(cs.s[seg]);
+                seg++;
+            }
+            __syncthreads();
         }
-        if (step + 1 < n_steps) park(buf ^ 1);
-        if (RESIDUAL && (step + 1) * kStepElems == cs.s[seg].k_end) {
-            fold(cs.s[seg]);
-            seg++;
-        }
-        __syncthreads();
     }
 
-    if constexpr (RESIDUAL) {
-#pragma unroll
-        for (int j = 0; j < NT; j++) {
-            const uint32_t tok = tok0 + wt + j * 16 + fr;
-            if (tok >= n_tokens) continue;
-#pragma unroll
-            for (int i = 0; i < NN; i++) {
-                const uint32_t row = row0 + wn + i * 16 + g * 4;
-                float *dst = x + size_t(tok) * width + row;
-                if (row + 3 < width && (width & 3) == 0)
-                    *reinterpret_cast<f32x4 *>(dst) += tot[i][j];
-                else
-#pragma unroll
-                    for (int r = 0; r < 4; r++)
-                        if (row + r < width) dst[r] += tot[i][j][r];
-            }
-        }
-    } else {
+    if constexpr (!RESIDUAL) {
 #pragma unroll
         for (int i = 0; i < NN; i++) {
             const uint32_t tile_row = row0 + wn + i * 16;  // a tile of sixteen rows lies in one segment
             if (tile_row >= n_rows) continue;
-            uint32_t si = 0;
-            while (si + 1 < rs.n_segs && tile_row >= rs.s[si + 1].row0) si++;
-            const RmiRowSeg &s = rs.s[si];
+            const RmiRowSeg &s = rs.s[seg_of(rs, tile_row)];
             const uint32_t r0 = tile_row - s.row0 + g * 4;
             float bias[4], lower[4];
 #pragma unroll
@@ -215,36 +217,59 @@ int launch_gemm(const RmiDense &w, const void *a, const RmiRowSegs &rs, const Rm
         hipLaunchKernelGGL(kernel, dim3(gn * gt), dim3(256), 0, st, static_cast<const T *>(w.data), static_cast<const T *>(a), n_rows,
                            w.k_pad, n_tokens, gn, gt, rs, cs, x, width);
     };
-    const uint64_t big = uint64_t((n_rows + 127) / 128) * ((n_tokens + 127) / 128);
+    const uint64_t cus = uint64_t(rmi_device_cus());
+    auto tiles = [&](uint32_t bn, uint32_t bt) { return uint64_t((n_rows + bn - 1) / bn) * ((n_tokens + bt - 1) / bt); };
     if (n_tokens <= 16)
-        go(dense_gemm_kernel<T, 64, 16, 16, 16, RESIDUAL>, 64, 16);
-    else if (big >= uint64_t(rmi_device_cus()))
-        go(dense_gemm_kernel<T, 128, 128, 64, 64, RESIDUAL>, 128, 128);
+        go(dense_gemm_kernel<T, 64, 16, 16, 16, 4, RESIDUAL>, 64, 16);
+    else if (tiles(128, 128) >= cus)
+        go(dense_gemm_kernel<T, 128, 128, 64, 64, 3, RESIDUAL>, 128, 128);
+    else if (tiles(64, 64) >= cus)
+        go(dense_gemm_kernel<T, 64, 64, 32, 32, 4, RESIDUAL>, 64, 64);
     else
-        go(dense_gemm_kernel<T, 64, 64, 32, 32, RESIDUAL>, 64, 64);
+        go(dense_gemm_kernel<T, 64, 32, 32, 16, 4, RESIDUAL>, 64, 32);
     RMI_HIP_CHECK(hipGetLastError());
     return RMI_HIP_OK;
 }
 
 // ------------------------------------------------------------------ GEMV
-// A wave takes ROWS weight rows, its lanes the 16-byte pieces of a row; two rounds of pieces are in flight.  The
-// activation sits in LDS, zero past its end, so that a piece past the end of a row (the last one is read again)
-// counts for nothing.
-constexpr uint32_t kGemvLdsMax = 144 * 1024;
+// The activation sits in LDS, zero past its end, so that a piece past the end of a row (the last one is read again)
+// counts for nothing.  Its loads go out before the weights': memory returns in order, and everything waits for it.
+constexpr uint32_t kGemvLdsMax = kLdsAskedFor;
+constexpr uint32_t kGemvRound = 256;  // LDS activations are padded to this many pieces
 template <typename T>
 __host__ __device__ inline uint32_t gemv_lds_pieces(uint32_t k_pad) {
     const uint32_t pieces = k_pad / (16 / sizeof(T));
-    return (pieces + 127) / 128 * 128;
+    return (pieces + kGemvRound - 1) / kGemvRound * kGemvRound;
 }
 
-template <typename T, int ROWS>
+// A wave takes ROWS weight rows, its lanes the pieces of a row, two rounds of 64 in flight; R: quads of x a thread
+// keeps (n <= 1024 R).
+template <typename T, int ROWS, int R>
 __global__ __launch_bounds__(256) void norm_gemv_kernel(const T *__restrict__ w, uint32_t k_pad, const float *__restrict__ x,
                                                         const float *__restrict__ weight, float eps, uint32_t n, RmiRowSegs rs) {
     extern __shared__ u32x4 act[];
     __shared__ float red[4];
     const uint32_t tid = threadIdx.x, lane = tid & 63;
-    const uint32_t row0 = (blockIdx.x * 4 + (tid >> 6)) * ROWS;
+    const uint32_t row0 = (blockIdx.x * 4 + uint32_t(__builtin_amdgcn_readfirstlane(int(tid >> 6)))) * ROWS;
     const uint32_t pieces = k_pad / kPieceElems<T>, padded = gemv_lds_pieces<T>(k_pad);
+    f32x4 xv[R], nv[R];
+    const bool quads = (n & 3) == 0;
+#pragma unroll
+    for (int j = 0; j < R; j++) {
+        const uint32_t i = (tid + j * 256) * 4;
+        if (quads) {
+            const uint32_t ic = i < n ? i : n - 4;
+            xv[j] = *reinterpret_cast<const f32x4 *>(x + ic);
+            nv[j] = *reinterpret_cast<const f32x4 *>(weight + ic);
+        } else {
+#pragma unroll
+            for (int e = 0; e < 4; e++) {
+                const uint32_t ic = i + e < n ? i + e : n - 1;
+                xv[j][e] = x[ic];
+                nv[j][e] = weight[ic];
+            }
+        }
+    }
     const u32x4 *src[ROWS];
 #pragma unroll
     for (int r = 0; r < ROWS; r++) {
@@ -260,26 +285,39 @@ __global__ __launch_bounds__(256) void norm_gemv_kernel(const T *__restrict__ w,
             for (int r = 0; r < ROWS; r++) cur[u][r] = src[r][p < pieces ? p : pieces - 1];
         }
     };
-    load(0);  // the weights are under way while the norm is computed
+    load(0);
+    const RmiRowSeg seg = rs.s[seg_of(rs, row0)];
     float sq = 0.0f;
-    for (uint32_t i = tid; i < n; i += 256) sq = __builtin_fmaf(x[i], x[i], sq);
+#pragma unroll
+    for (int j = 0; j < R; j++)
+#pragma unroll
+        for (int e = 0; e < 4; e++) {
+            if ((tid + j * 256) * 4 + e >= n) xv[j][e] = 0.0f;
+            sq = __builtin_fmaf(xv[j][e], xv[j][e], sq);
+        }
     sq = wave_sum_f32(sq);
     if (lane == 0) red[tid >> 6] = sq;
     __syncthreads();
     const float scale = 1.0f / sqrtf(((red[0] + red[1]) + (red[2] + red[3])) / float(n) + eps);
     T *h = reinterpret_cast<T *>(act);
-    for (uint32_t i = tid; i < padded * kPieceElems<T>; i += 256) h[i] = from_f32<T>(i < n ? x[i] * scale * weight[i] : 0.0f);
+    const uint32_t h_elems = padded * kPieceElems<T>;  // a multiple of 1024
+#pragma unroll
+    for (int j = 0; j < R; j++) {
+        const uint32_t i = (tid + j * 256) * 4;
+        if (i < h_elems) store4(h + i, xv[j] * scale * nv[j]);
+    }
+    for (uint32_t i = (tid + R * 256) * 4; i < h_elems; i += 1024) store4(h + i, f32x4{0.f, 0.f, 0.f, 0.f});
     __syncthreads();
     float acc[ROWS];
 #pragma unroll
     for (int r = 0; r < ROWS; r++) acc[r] = 0.0f;
-    for (uint32_t p0 = 0; p0 < padded; p0 += 128) {
+    for (uint32_t p0 = 0; p0 < pieces; p0 += 128) {
         u32x4 now[2][ROWS];
 #pragma unroll
         for (int u = 0; u < 2; u++)
 #pragma unroll
             for (int r = 0; r < ROWS; r++) now[u][r] = cur[u][r];
-        if (p0 + 128 < padded) load(p0 + 128);
+        if (p0 + 128 < pieces) load(p0 + 128);
 #pragma unroll
         for (int u = 0; u < 2; u++) {
             const u32x4 hv = act[p0 + u * 64 + lane];
@@ -293,115 +331,106 @@ __global__ __launch_bounds__(256) void norm_gemv_kernel(const T *__restrict__ w,
         const float s = wave_sum_f32(acc[r]);
         if (lane == uint32_t(r)) mine = s;
     }
-    const uint32_t row = row0 + lane;
-    if (lane >= ROWS || row >= rs.n_rows) return;
-    uint32_t si = 0;
-    while (si + 1 < rs.n_segs && row0 >= rs.s[si + 1].row0) si++;
-    const RmiRowSeg &s = rs.s[si];
-    const uint32_t at = row - s.row0;
-    if (at >= s.n) return;
-    const float o = apply_act<T>(s.act, mine, s.bias ? s.bias[at] : 0.0f, s.lower ? s.lower[at] : 0.0f);
-    if (s.out_elem)
-        static_cast<T *>(s.y)[at] = from_f32<T>(o);
+    const uint32_t at = row0 + lane - seg.row0;
+    if (lane >= ROWS || row0 + lane >= rs.n_rows || at >= seg.n) return;
+    const float o = apply_act<T>(seg.act, mine, seg.bias ? seg.bias[at] : 0.0f, seg.lower ? seg.lower[at] : 0.0f);
+    if (seg.out_elem)
+        static_cast<T *>(seg.y)[at] = from_f32<T>(o);
     else
-        static_cast<float *>(s.y)[at] = o;
+        static_cast<float *>(seg.y)[at] = o;
 }
 
+// A workgroup takes ROWS rows, each wave a quarter of their columns, so that a long row is in flight at once; the
+// waves' sums meet in LDS.  A lane's products count with the gate and scale of the column segment its piece lies in.
 template <typename T, int ROWS>
 __global__ __launch_bounds__(256) void gemv_residual_kernel(const T *__restrict__ w, uint32_t k_pad, const T *__restrict__ a,
                                                             RmiColSegs cs, float *__restrict__ x, uint32_t width) {
-    extern __shared__ u32x4 act[];
-    const uint32_t tid = threadIdx.x, lane = tid & 63;
-    const uint32_t row0 = (blockIdx.x * 4 + (tid >> 6)) * ROWS;
-    const uint32_t pieces = k_pad / kPieceElems<T>, padded = gemv_lds_pieces<T>(k_pad);
-    const u32x4 *src[ROWS];
+    constexpr int U = 4;
+    __shared__ float part[4][ROWS];
+    const uint32_t tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
+    const uint32_t row0 = blockIdx.x * ROWS;
+    const uint32_t pieces = k_pad / kPieceElems<T>, per_wave = ((pieces + 3) / 4 + 63) / 64 * 64;
+    const uint32_t p_begin = wave * per_wave, p_end = p_begin + per_wave < pieces ? p_begin + per_wave : pieces;
+    const u32x4 *src[ROWS], *hsrc = reinterpret_cast<const u32x4 *>(a);
+    float gate[ROWS][kMaxColSegs];
 #pragma unroll
-    for (int r = 0; r < ROWS; r++) src[r] = reinterpret_cast<const u32x4 *>(w + size_t(row0 + r < width ? row0 + r : width - 1) * k_pad);
-    u32x4 cur[2][ROWS];
+    for (int r = 0; r < ROWS; r++) {
+        const uint32_t row = row0 + r < width ? row0 + r : width - 1;
+        src[r] = reinterpret_cast<const u32x4 *>(w + size_t(row) * k_pad);
+#pragma unroll
+        for (uint32_t i = 0; i < kMaxColSegs; i++) gate[r][i] = i < cs.n_segs ? (cs.s[i].gate ? cs.s[i].gate[row] : 1.0f) * cs.s[i].scale : 0.0f;
+    }
+    float acc[ROWS];
+#pragma unroll
+    for (int r = 0; r < ROWS; r++) acc[r] = 0.0f;
+    u32x4 cur[U][ROWS], hcur[U];
     auto load = [&](uint32_t p0) {
 #pragma unroll
-        for (int u = 0; u < 2; u++) {
-            const uint32_t p = p0 + u * 64 + lane;
+        for (int u = 0; u < U; u++) {
+            const uint32_t p = p0 + u * 64 + lane, pc = p < p_end ? p : pieces - 1;
+            hcur[u] = hsrc[pc];
 #pragma unroll
-            for (int r = 0; r < ROWS; r++) cur[u][r] = src[r][p < pieces ? p : pieces - 1];
+            for (int r = 0; r < ROWS; r++) cur[u][r] = src[r][pc];
         }
     };
-    load(0);
-    const u32x4 zero = {0, 0, 0, 0};
-    for (uint32_t p = tid; p < padded; p += 256) act[p] = p < pieces ? reinterpret_cast<const u32x4 *>(a)[p] : zero;
-    __syncthreads();
-    // sum_i gate_i scale_i part_i: a lane's running sums by segment
-    float acc[ROWS][kMaxColSegs];
+    if (p_begin < p_end) load(p_begin);
+    for (uint32_t p0 = p_begin; p0 < p_end; p0 += 64 * U) {
+        u32x4 now[U][ROWS], hv[U];
 #pragma unroll
-    for (int r = 0; r < ROWS; r++)
-#pragma unroll
-        for (uint32_t i = 0; i < kMaxColSegs; i++) acc[r][i] = 0.0f;
-    for (uint32_t p0 = 0; p0 < padded; p0 += 128) {
-        u32x4 now[2][ROWS];
-#pragma unroll
-        for (int u = 0; u < 2; u++)
+        for (int u = 0; u < U; u++) {
+            hv[u] = hcur[u];
 #pragma unroll
             for (int r = 0; r < ROWS; r++) now[u][r] = cur[u][r];
-        if (p0 + 128 < padded) load(p0 + 128);
+        }
+        if (p0 + 64 * U < p_end) load(p0 + 64 * U);
 #pragma unroll
-        for (int u = 0; u < 2; u++) {
-            const uint32_t k = (p0 + u * 64 + lane) * kPieceElems<T>;
-            const u32x4 hv = act[p0 + u * 64 + lane];
-            uint32_t seg = 0;
-#pragma unroll
-            for (uint32_t i = 0; i + 1 < kMaxColSegs; i++) seg += i + 1 < cs.n_segs && k >= cs.s[i].k_end ? 1u : 0u;
+        for (int u = 0; u < U; u++) {
+            const uint32_t p = p0 + u * 64 + lane, k = p * kPieceElems<T>;
+            const bool live = p < p_end;
 #pragma unroll
             for (int r = 0; r < ROWS; r++) {
-                const float d = dot_piece<T>(now[u][r], hv, 0.0f);
+                float f = gate[r][0];
 #pragma unroll
-                for (uint32_t i = 0; i < kMaxColSegs; i++) acc[r][i] += seg == i ? d : 0.0f;
+                for (uint32_t i = 0; i + 1 < kMaxColSegs; i++) f = i + 1 < cs.n_segs && k >= cs.s[i].k_end ? gate[r][i + 1] : f;
+                const float d = dot_piece<T>(now[u][r], hv[u], 0.0f);
+                acc[r] = __builtin_fmaf(f, live ? d : 0.0f, acc[r]);
             }
         }
     }
 #pragma unroll
     for (int r = 0; r < ROWS; r++) {
-        const uint32_t row = row0 + r;
-        float sums[kMaxColSegs];
-#pragma unroll
-        for (uint32_t i = 0; i < kMaxColSegs; i++) sums[i] = i < cs.n_segs ? wave_sum_f32(acc[r][i]) : 0.0f;
-        if (lane != uint32_t(r) || row >= width) continue;
-        float t = 0.0f;
-#pragma unroll
-        for (uint32_t i = 0; i < kMaxColSegs; i++)
-            if (i < cs.n_segs) t = __builtin_fmaf(cs.s[i].gate ? cs.s[i].gate[row] : 1.0f, sums[i] * cs.s[i].scale, t);
-        x[row] += t;
+        const float t = wave_sum_f32(acc[r]);
+        if (lane == 0) part[wave][r] = t;
     }
+    __syncthreads();
+    if (tid < ROWS && row0 + tid < width) x[row0 + tid] += (part[0][tid] + part[1][tid]) + (part[2][tid] + part[3][tid]);
 }
 
-// more than 64 KiB of dynamic LDS has to be asked for, once a kernel
-template <typename K>
-int allow_lds(K kernel, size_t bytes) {
-    if (bytes <= 64 * 1024) return RMI_HIP_OK;
-    RMI_HIP_CHECK(hipFuncSetAttribute(reinterpret_cast<const void *>(kernel), hipFuncAttributeMaxDynamicSharedMemorySize, kGemvLdsMax));
-    return RMI_HIP_OK;
-}
+constexpr uint32_t kNormGemvMaxN = 16384;  // what a workgroup keeps of x in registers
 
-template <typename T>
-int norm_gemv(const RmiDense &w, const float *x, const float *weight, float eps, uint32_t n, const RmiRowSegs &segs, hipStream_t st) {
+template <typename T, int R>
+int norm_gemv_r(const RmiDense &w, const float *x, const float *weight, float eps, uint32_t n, const RmiRowSegs &segs, hipStream_t st) {
     const size_t lds = size_t(gemv_lds_pieces<T>(w.k_pad)) * 16;
-    if (lds > kGemvLdsMax) return rmi_fail(RMI_HIP_E_INVALID, "%u columns exceed what the GEMV holds", w.k_pad);
     constexpr int kRows = 4;
-    int rc = allow_lds(norm_gemv_kernel<T, kRows>, lds);
+    const int rc = rmi_allow_lds(norm_gemv_kernel<T, kRows, R>, lds);
     if (rc != RMI_HIP_OK) return rc;
-    hipLaunchKernelGGL((norm_gemv_kernel<T, kRows>), dim3((w.n_rows + 4 * kRows - 1) / (4 * kRows)), dim3(256), lds, st,
+    hipLaunchKernelGGL((norm_gemv_kernel<T, kRows, R>), dim3((w.n_rows + 4 * kRows - 1) / (4 * kRows)), dim3(256), lds, st,
                        static_cast<const T *>(w.data), w.k_pad, x, weight, eps, n, segs);
     RMI_HIP_CHECK(hipGetLastError());
     return RMI_HIP_OK;
 }
+template <typename T>
+int norm_gemv(const RmiDense &w, const float *x, const float *weight, float eps, uint32_t n, const RmiRowSegs &segs, hipStream_t st) {
+    if (!rmi_dense_gemv_fits(sizeof(T), w.k_pad)) return rmi_fail(RMI_HIP_E_INVALID, "%u columns exceed what the GEMV holds", w.k_pad);
+    if (n <= 1024) return norm_gemv_r<T, 1>(w, x, weight, eps, n, segs, st);
+    if (n <= 4096) return norm_gemv_r<T, 4>(w, x, weight, eps, n, segs, st);
+    return norm_gemv_r<T, 16>(w, x, weight, eps, n, segs, st);
+}
 
 template <typename T>
 int gemv_residual(const RmiDense &w, const void *a, const RmiColSegs &segs, float *x, uint32_t width, hipStream_t st) {
-    const size_t lds = size_t(gemv_lds_pieces<T>(w.k_pad)) * 16;
-    if (lds > kGemvLdsMax) return rmi_fail(RMI_HIP_E_INVALID, "%u columns exceed what the GEMV holds", w.k_pad);
-    constexpr int kRows = 1;
-    int rc = allow_lds(gemv_residual_kernel<T, kRows>, lds);
-    if (rc != RMI_HIP_OK) return rc;
-    hipLaunchKernelGGL((gemv_residual_kernel<T, kRows>), dim3((width + 4 * kRows - 1) / (4 * kRows)), dim3(256), lds, st,
+    constexpr int kRows = 2;
+    hipLaunchKernelGGL((gemv_residual_kernel<T, kRows>), dim3((width + kRows - 1) / kRows), dim3(256), 0, st,
                        static_cast<const T *>(w.data), w.k_pad, static_cast<const T *>(a), segs, x, width);
     RMI_HIP_CHECK(hipGetLastError());
     return RMI_HIP_OK;
@@ -461,7 +490,7 @@ int rmi_dense_gemm_residual(uint32_t elem_bytes, const RmiDense &w, const void *
 
 bool rmi_dense_gemv_fits(uint32_t elem_bytes, uint32_t k_pad) {
     const size_t lds = size_t(elem_bytes == 2 ? gemv_lds_pieces<rmi_bf16>(k_pad) : gemv_lds_pieces<float>(k_pad)) * 16;
-    return lds <= kGemvLdsMax;
+    return lds <= kGemvLdsMax && k_pad <= kNormGemvMaxN;
 }
 
 int rmi_dense_norm_gemv(uint32_t elem_bytes, const RmiDense &w, const float *x, const float *weight, float eps, uint32_t n,

@@ -97,30 +97,125 @@ __device__ __forceinline__ void value_row(const ConvCtx &x, const RmiAttnShape &
     }
 }
 
-// a workgroup's four waves: four tokens of one head (blockIdx.x: q heads, then k, then v)
+// One head (blockIdx.x: q heads, then k, then v) of a run of tokens to a wave.
+constexpr uint32_t kConvRun = 8;
+__device__ __forceinline__ void conv_head_carry(const ConvCtx &x, const RmiAttnShape &s, const RmiAttnArgs &a, uint32_t head) {
+    const bool is_v = head >= s.heads + s.kv_heads;
+    const uint32_t c0 = is_v ? (s.heads + s.kv_heads) * s.dim + (head - s.heads - s.kv_heads) * s.vdim : head * s.dim;
+    for (uint32_t d = threadIdx.x; d < (is_v ? s.vdim : s.dim); d += 256) conv_carry(x, a.hist_out, a.n_tokens, c0 + d);
+}
+
+// any sizes: token by token
 template <typename T>
 __global__ __launch_bounds__(256) void conv_rotate_kernel(RmiAttnShape s, RmiAttnArgs a) {
     const uint32_t lane = threadIdx.x & 63, head = blockIdx.x;
     const uint32_t channels = (s.heads + s.kv_heads) * s.dim + s.kv_heads * s.vdim;
     const ConvCtx x{a.u, a.hist_in, a.conv, channels, s.taps};
-    if (blockIdx.y == 0) {  // the first tokens' workgroup of a head also carries its channels' history on
-        const bool is_v = head >= s.heads + s.kv_heads;
-        const uint32_t c0 = is_v ? (s.heads + s.kv_heads) * s.dim + (head - s.heads - s.kv_heads) * s.vdim : head * s.dim;
-        for (uint32_t d = threadIdx.x; d < (is_v ? s.vdim : s.dim); d += 256) conv_carry(x, a.hist_out, a.n_tokens, c0 + d);
+    if (blockIdx.y == 0) conv_head_carry(x, s, a, head);  // one workgroup of a head also carries its history on
+    const uint32_t t0 = (blockIdx.y * 4 + (threadIdx.x >> 6)) * kConvRun;
+    for (uint32_t t = t0; t < t0 + kConvRun && t < a.n_tokens; t++) {
+        if (head >= s.heads + s.kv_heads) {
+            value_row<T>(x, s, a, t, head - s.heads - s.kv_heads, lane);
+        } else if (head >= s.heads) {
+            key_row<T>(x, s, a, t, head - s.heads, lane);
+        } else {
+            const uint32_t group = s.heads / s.kv_heads, g = head / group, r = head % group;
+            T *row = static_cast<T *>(a.q) + (size_t(g) * a.n_tokens * group + size_t(t) * group + r) * s.dk_pad;
+            for (uint32_t i = lane; i < s.dk_pad / 2; i += 64) {
+                float p, q;
+                conv_rotate_pair(x, s, a.cos_t, a.sin_t, t, a.pos0, head * s.dim, i, p, q);
+                store_pair(row + 2 * i, p, q);
+            }
+        }
     }
-    const uint32_t t = blockIdx.y * 4 + (threadIdx.x >> 6);
-    if (t >= a.n_tokens) return;
-    if (head >= s.heads + s.kv_heads) {
-        value_row<T>(x, s, a, t, head - s.heads - s.kv_heads, lane);
-    } else if (head >= s.heads) {
-        key_row<T>(x, s, a, t, head - s.heads, lane);
+}
+
+// Even head sizes up to 128 and up to four taps: a lane holds one pair of channels, its taps and a sliding window of
+// the projected values; every row is read once.
+template <typename T>
+__global__ __launch_bounds__(256) void conv_rotate_pairs_kernel(RmiAttnShape s, RmiAttnArgs a) {
+    const uint32_t lane = threadIdx.x & 63, head = blockIdx.x;
+    const uint32_t channels = (s.heads + s.kv_heads) * s.dim + s.kv_heads * s.vdim;
+    const ConvCtx x{a.u, a.hist_in, a.conv, channels, s.taps};
+    if (blockIdx.y == 0) conv_head_carry(x, s, a, head);
+    const uint32_t t0 = (blockIdx.y * 4 + (threadIdx.x >> 6)) * kConvRun;
+    if (t0 >= a.n_tokens) return;
+    const bool is_v = head >= s.heads + s.kv_heads, is_q = head < s.heads;
+    const uint32_t dim = is_v ? s.vdim : s.dim;
+    const uint32_t c0 = is_v ? (s.heads + s.kv_heads) * s.dim + (head - s.heads - s.kv_heads) * s.vdim : head * s.dim;
+    const bool has = 2 * lane < dim;
+    const uint32_t c = c0 + (has ? 2 * lane : 0);
+    float w0[4], w1[4], u0[4], u1[4];  // tap and row j of four, the last one the token's own
+    const uint32_t off = 4 - s.taps;
+#pragma unroll
+    for (uint32_t j = 0; j < 4; j++) {
+        w0[j] = j >= off ? a.conv[c * s.taps + j - off] : 0.0f;
+        w1[j] = j >= off ? a.conv[(c + 1) * s.taps + j - off] : 0.0f;
+    }
+    float2 row[kConvRun];
+#pragma unroll
+    for (uint32_t i = 0; i < kConvRun; i++) {
+        const uint32_t t = t0 + i < a.n_tokens ? t0 + i : a.n_tokens - 1;
+        row[i] = *reinterpret_cast<const float2 *>(a.u + size_t(t) * channels + c);
+    }
+#pragma unroll
+    for (uint32_t j = 1; j < 4; j++) {  // the rows before the run: position pos0 + t0 - (4 - j)
+        const uint32_t back = 4 - j;
+        float2 v = make_float2(0.f, 0.f);
+        if (t0 >= back)
+            v = *reinterpret_cast<const float2 *>(a.u + size_t(t0 - back) * channels + c);
+        else if (back - t0 < s.taps && a.pos0 + t0 >= back)
+            v = *reinterpret_cast<const float2 *>(a.hist_in + size_t(t0 + s.taps - 1 - back) * channels + c);
+        u0[j] = v.x;
+        u1[j] = v.y;
+    }
+    const uint32_t group = s.heads / s.kv_heads, half = s.rot_dims / 2;
+    const bool turned = !is_v && lane < half;
+    T *out;  // of token t0; `step` further for the next
+    size_t step;
+    if (is_q) {
+        out = static_cast<T *>(a.q) + (size_t(head / group) * a.n_tokens * group + size_t(t0) * group + head % group) * s.dk_pad;
+        step = size_t(group) * s.dk_pad;
     } else {
-        const uint32_t group = s.heads / s.kv_heads, g = head / group, r = head % group;
-        T *row = static_cast<T *>(a.q) + (size_t(g) * a.n_tokens * group + size_t(t) * group + r) * s.dk_pad;
-        for (uint32_t i = lane; i < s.dk_pad / 2; i += 64) {
-            float p, q;
-            conv_rotate_pair(x, s, a.cos_t, a.sin_t, t, a.pos0, head * s.dim, i, p, q);
-            store_pair(row + 2 * i, p, q);
+        out = static_cast<T *>(a.k_cache) + (size_t(head - s.heads) * s.capacity + a.pos0 + t0) * s.dk_pad;
+        step = s.dk_pad;
+    }
+#pragma unroll
+    for (uint32_t i = 0; i < kConvRun; i++) {
+        const uint32_t t = t0 + i;
+        if (t >= a.n_tokens) break;
+#pragma unroll
+        for (uint32_t j = 0; j < 3; j++) {
+            u0[j] = u0[j + 1];
+            u1[j] = u1[j + 1];
+        }
+        u0[3] = row[i].x;
+        u1[3] = row[i].y;
+        float p = 0.0f, q = 0.0f;
+#pragma unroll
+        for (uint32_t j = 0; j < 4; j++) {
+            p = __builtin_fmaf(w0[j], u0[j], p);
+            q = __builtin_fmaf(w1[j], u1[j], q);
+        }
+        if (!has) p = q = 0.0f;
+        if (is_v) {
+            const float r = 1.0f / sqrtf(wave_sum_f32(__builtin_fmaf(p, p, q * q)) / float(dim) + s.eps);
+            const uint32_t pos = a.pos0 + t;
+            T *blk = static_cast<T *>(a.v_cache) +
+                     (size_t(head - s.heads - s.kv_heads) * (s.capacity / kKeyBlock) + pos / kKeyBlock) * s.dv_pad * kKeyBlock +
+                     value_slot<T>(pos % kKeyBlock);
+            if (has) {
+                blk[size_t(2 * lane) * kKeyBlock] = from_f32<T>(p * r);
+                blk[size_t(2 * lane + 1) * kKeyBlock] = from_f32<T>(q * r);
+            }
+        } else {
+            if (turned) {
+                const size_t at = size_t(a.pos0 + t) * half + lane;
+                const float cs = a.cos_t[at], sn = a.sin_t[at], rp = p;
+                p = __builtin_fmaf(rp, cs, -(q * sn));
+                q = __builtin_fmaf(q, cs, rp * sn);
+            }
+            if (2 * lane < s.dk_pad) store_pair(out + i * step + 2 * lane, p, q);
         }
     }
 }
@@ -151,22 +246,51 @@ struct AttnWave {
         const uint32_t lane = threadIdx.x & 63, fr = lane & 15, g = lane >> 4;
         const uint32_t n_kc = s.dk_pad / (4 * kPieceElems<T>), n_vt = s.dv_pad / 16;
         const T *krow = kc + size_t(fr) * s.dk_pad + g * kPieceElems<T>;
+        constexpr bool kAhead = BUCKET * sizeof(T) <= 256;  // a block's keys and values fit in registers beside the rest
+        u32x4 kf[2][kAhead ? kKC : 1], vf[kAhead ? kVT * (sizeof(T) / 2) : 1];
+        auto load_keys = [&](uint32_t k) {
+#pragma unroll
+            for (uint32_t c = 0; c < kKC; c++) {
+                if (c >= n_kc) continue;
+                const T *p = krow + size_t(k) * s.dk_pad + c * 4 * kPieceElems<T>;
+                kf[0][c] = *reinterpret_cast<const u32x4 *>(p);
+                kf[1][c] = *reinterpret_cast<const u32x4 *>(p + 16 * size_t(s.dk_pad));
+            }
+        };
+        if constexpr (kAhead)
+            if (k0 < k1) load_keys(k0);
         for (uint32_t k = k0; k < k1; k += kKeyBlock) {
+            const T *vb = vc + size_t(k / kKeyBlock) * s.dv_pad * kKeyBlock + size_t(fr) * kKeyBlock + g * kPieceElems<T>;
+            if constexpr (kAhead) {
+#pragma unroll
+                for (uint32_t v = 0; v < kVT; v++)
+#pragma unroll
+                    for (uint32_t t = 0; t < sizeof(T) / 2; t++)
+                        if (v < n_vt) vf[v * (sizeof(T) / 2) + t] = *reinterpret_cast<const u32x4 *>(vb + size_t(v) * 16 * kKeyBlock + t * 16);
+            }
             f32x4 sc[QT][2];
 #pragma unroll
             for (int i = 0; i < QT; i++) sc[i][0] = sc[i][1] = f32x4{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
             for (uint32_t c = 0; c < kKC; c++) {
                 if (c >= n_kc) continue;
-                const T *p = krow + size_t(k) * s.dk_pad + c * 4 * kPieceElems<T>;
-                const u32x4 f0 = *reinterpret_cast<const u32x4 *>(p);
-                const u32x4 f1 = *reinterpret_cast<const u32x4 *>(p + 16 * size_t(s.dk_pad));
+                u32x4 f0, f1;
+                if constexpr (kAhead) {
+                    f0 = kf[0][c];
+                    f1 = kf[1][c];
+                } else {
+                    const T *p = krow + size_t(k) * s.dk_pad + c * 4 * kPieceElems<T>;
+                    f0 = *reinterpret_cast<const u32x4 *>(p);
+                    f1 = *reinterpret_cast<const u32x4 *>(p + 16 * size_t(s.dk_pad));
+                }
 #pragma unroll
                 for (int i = 0; i < QT; i++) {
                     sc[i][0] = mma16<T>(f0, qf[i][c], sc[i][0]);
                     sc[i][1] = mma16<T>(f1, qf[i][c], sc[i][1]);
                 }
             }
+            if constexpr (kAhead)
+                if (k + kKeyBlock < k1) load_keys(k + kKeyBlock);
             u32x4 pf[QT][2];
 #pragma unroll
             for (int i = 0; i < QT; i++) {
@@ -204,14 +328,13 @@ struct AttnWave {
                     pf[i][1] = __builtin_bit_cast(u32x4, sc[i][1]);
                 }
             }
-            const T *vb = vc + size_t(k / kKeyBlock) * s.dv_pad * kKeyBlock + size_t(fr) * kKeyBlock + g * kPieceElems<T>;
 #pragma unroll
             for (uint32_t v = 0; v < kVT; v++) {
                 if (v >= n_vt) continue;
-                const T *p = vb + size_t(v) * 16 * kKeyBlock;
 #pragma unroll
                 for (uint32_t t = 0; t < sizeof(T) / 2; t++) {
-                    const u32x4 f = *reinterpret_cast<const u32x4 *>(p + t * 16);
+                    const u32x4 f = kAhead ? vf[kAhead ? v * (sizeof(T) / 2) + t : 0]
+                                           : *reinterpret_cast<const u32x4 *>(vb + size_t(v) * 16 * kKeyBlock + t * 16);
 #pragma unroll
                     for (int i = 0; i < QT; i++) o[i][v] = mma16<T>(f, pf[i][t], o[i][v]);
                 }
@@ -274,15 +397,9 @@ __global__ __launch_bounds__(256) void attn_pass_kernel(RmiAttnShape s, RmiAttnA
 // Few columns: the keys are divided over `parts` workgroups and their four waves; each workgroup merges its waves in
 // LDS, writes its part, and the one that arrives last merges the parts.  With one token (STEP) the workgroup makes
 // its queries itself, and the workgroups of the last part the new key and value.
+constexpr uint32_t kMaxParts = 32;
+// a part: the columns' maxima, their sums, and [column][channel]
 __host__ __device__ inline uint32_t attn_part_floats(uint32_t dv_pad) { return 16 * (dv_pad + 2); }
-
-__device__ __forceinline__ void merge_state(float &m, float &l, float m2, float l2, float &f1, float &f2) {
-    const float top = fmaxf(m, m2), ref = top == -INFINITY ? 0.0f : top;
-    f1 = expf(m - ref);
-    f2 = expf(m2 - ref);
-    l = l * f1 + l2 * f2;
-    m = top;
-}
 
 template <typename T, int BUCKET, bool STEP>
 __device__ __forceinline__ void attn_split(const RmiAttnShape &s, const RmiAttnArgs &a, uint32_t block, uint32_t parts, uint32_t keys_per_part,
@@ -342,92 +459,99 @@ __device__ __forceinline__ void attn_split(const RmiAttnShape &s, const RmiAttnA
     if (k0 < k1)
         w.keys(static_cast<const T *>(a.k_cache) + size_t(kvh) * s.capacity * s.dk_pad,
                static_cast<const T *>(a.v_cache) + size_t(kvh) * s.capacity * s.dv_pad, s, k0, k1, last);
-    float m = w.m[0], l = rows_sum_f32(w.l[0]);
-    // waves 1..3 hand their part to wave 0: [m 16][l 16][o dv_pad x 16]
-    float *mine = reinterpret_cast<float *>(lds) + (wave ? wave - 1 : 0) * attn_part_floats(s.dv_pad);
-    if (wave) {
+    // the waves' results to LDS, live columns only; then every thread merges (column, channel) pairs
+    const uint32_t live = n_cols - ct * 16 < 16 ? n_cols - ct * 16 : 16, pf = attn_part_floats(s.dv_pad);
+    float *all = reinterpret_cast<float *>(lds), *mine = all + wave * pf;
+    const float l = rows_sum_f32(w.l[0]);
+    if (fr < live) {
         if (g4 == 0) {
-            mine[fr] = m;
+            mine[fr] = w.m[0];
             mine[16 + fr] = l;
         }
 #pragma unroll
         for (uint32_t v = 0; v < w.kVT; v++)
-            if (v * 16 < s.dv_pad)
-#pragma unroll
-                for (int r = 0; r < 4; r++) mine[32 + (v * 16 + g4 * 4 + r) * 16 + fr] = w.o[0][v][r];
+            if (v * 16 < s.dv_pad) *reinterpret_cast<f32x4 *>(mine + 32 + fr * s.dv_pad + v * 16 + g4 * 4) = w.o[0][v];
     }
     __syncthreads();
-    if (wave == 0) {
-        for (uint32_t o = 0; o < 3; o++) {
-            const float *other = reinterpret_cast<const float *>(lds) + o * attn_part_floats(s.dv_pad);
-            float f1, f2;
-            merge_state(m, l, other[fr], other[16 + fr], f1, f2);
-#pragma unroll
-            for (uint32_t v = 0; v < w.kVT; v++)
-                if (v * 16 < s.dv_pad)
-#pragma unroll
-                    for (int r = 0; r < 4; r++) w.o[0][v][r] = w.o[0][v][r] * f1 + other[32 + (v * 16 + g4 * 4 + r) * 16 + fr] * f2;
-        }
-    }
     const uint32_t slot = kvh * tiles + ct;
-    float *ws = reinterpret_cast<float *>(static_cast<uint32_t *>(a.scratch) + kAttnCounters);
-    if (parts > 1) {
-        if (wave == 0) {
-            float *dst = ws + (size_t(slot) * parts + part) * attn_part_floats(s.dv_pad);
-            if (g4 == 0) {
-                __hip_atomic_store(dst + fr, m, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
-                __hip_atomic_store(dst + 16 + fr, l, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
-            }
+    float *ws = reinterpret_cast<float *>(static_cast<uint32_t *>(a.scratch) + kAttnCounters) + size_t(slot) * parts * pf;
+    const uint32_t quads = s.dv_pad / 4;
+    auto finish = [&](uint32_t c, uint32_t d, f32x4 o, float sum) {
+        const uint32_t mc = ct * 16 + c, t = mc / group, head = kvh * group + mc % group;
+        attn_store<T>(s, a, t, head, d, o * ((a.gate ? a.gate[size_t(t) * s.heads + head] : 1.0f) / sum));
+    };
+    for (uint32_t e = tid; e < live * quads; e += 256) {
+        const uint32_t c = e / quads, d = e % quads * 4;
+        float m = all[c];
 #pragma unroll
-            for (uint32_t v = 0; v < w.kVT; v++)
-                if (v * 16 < s.dv_pad)
+        for (uint32_t i = 1; i < 4; i++) m = fmaxf(m, all[i * pf + c]);
+        const float ref = m == -INFINITY ? 0.0f : m;  // a column that sees no key of this part
+        float sum = 0.0f;
+        f32x4 o = {0.f, 0.f, 0.f, 0.f};
 #pragma unroll
-                    for (int r = 0; r < 4; r++)
-                        __hip_atomic_store(dst + 32 + (v * 16 + g4 * 4 + r) * 16 + fr, w.o[0][v][r], __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
-            // the storing lanes are one wave: its fence covers the stores of all of them
-            __builtin_amdgcn_fence(__ATOMIC_RELEASE, "agent");
-            if (lane == 0) {
-                uint32_t *count = static_cast<uint32_t *>(a.scratch) + slot;
-                const uint32_t n = __hip_atomic_fetch_add(count, 1u, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
-                *flag = n == parts - 1;
-                if (n == parts - 1) __hip_atomic_store(count, 0u, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);  // ready for the next launch
+        for (uint32_t i = 0; i < 4; i++) {
+            const float f = exp_t<T>(all[i * pf + c] - ref);
+            sum = __builtin_fmaf(all[i * pf + 16 + c], f, sum);
+            o += *reinterpret_cast<const f32x4 *>(all + i * pf + 32 + c * s.dv_pad + d) * f;
+        }
+        if (parts == 1) {
+            finish(c, d, o, sum);
+        } else {
+            float *dst = ws + size_t(part) * pf;
+            if (d == 0) {
+                dst[c] = m;
+                dst[16 + c] = sum;
             }
+            *reinterpret_cast<f32x4 *>(dst + 32 + c * s.dv_pad + d) = o;
         }
-        __syncthreads();
-        if (!*flag) return;
-        __builtin_amdgcn_fence(__ATOMIC_ACQUIRE, "agent");
-        // every thread: some (channel, column) pairs over all parts
-        const float *src = ws + size_t(slot) * parts * attn_part_floats(s.dv_pad);
-        const uint32_t c = tid & 15, mc = ct * 16 + c;
-        float top = -INFINITY, sum = 0.0f;
-        for (uint32_t p = 0; p < parts; p++)
-            top = fmaxf(top, __hip_atomic_load(src + size_t(p) * attn_part_floats(s.dv_pad) + c, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT));
-        for (uint32_t p = 0; p < parts; p++) {
-            const float *pp = src + size_t(p) * attn_part_floats(s.dv_pad);
-            sum += expf(__hip_atomic_load(pp + c, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT) - top) *
-                   __hip_atomic_load(pp + 16 + c, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
-        }
-        if (mc < n_cols) {
-            const uint32_t t = mc / group, head = kvh * group + mc % group;
-            const float f = (a.gate ? a.gate[size_t(t) * s.heads + head] : 1.0f) / sum;
-            for (uint32_t d = tid >> 4; d < s.vdim; d += 16) {
-                float o = 0.0f;
-                for (uint32_t p = 0; p < parts; p++) {
-                    const float *pp = src + size_t(p) * attn_part_floats(s.dv_pad);
-                    o += expf(__hip_atomic_load(pp + c, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT) - top) *
-                         __hip_atomic_load(pp + 32 + d * 16 + c, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
-                }
-                static_cast<T *>(a.out)[size_t(t) * a.out_ld + size_t(head) * s.vdim + d] = from_f32<T>(o * f);
-            }
-        }
-        return;
     }
-    if (wave == 0 && col < n_cols) {
-        const uint32_t t = col / group, head = kvh * group + col % group;
-        const float f = (a.gate ? a.gate[size_t(t) * s.heads + head] : 1.0f) / l;
+    if (parts == 1) return;
+    // hand-over: every wave releases its own stores, then the workgroup counts once
+    __builtin_amdgcn_fence(__ATOMIC_RELEASE, "agent");
+    __syncthreads();
+    if (tid == 0) {
+        uint32_t *count = static_cast<uint32_t *>(a.scratch) + slot;
+        const uint32_t n = __hip_atomic_fetch_add(count, 1u, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
+        *flag = n == parts - 1;
+        if (n == parts - 1) __hip_atomic_store(count, 0u, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);  // ready for the next launch
+    }
+    __syncthreads();
+    if (!*flag) return;
+    __builtin_amdgcn_fence(__ATOMIC_ACQUIRE, "agent");
+    // what each part counts for: [part][column] factors in LDS, the sums behind them
+    float *fac = all, *sums = all + kMaxParts * 16;
+    if (tid < live) {
+        float ms[kMaxParts], top = -INFINITY, sum = 0.0f;
 #pragma unroll
-        for (uint32_t v = 0; v < w.kVT; v++)
-            if (v * 16 < s.dv_pad) attn_store<T>(s, a, t, head, v * 16 + g4 * 4, w.o[0][v] * f);
+        for (uint32_t p = 0; p < kMaxParts; p++) ms[p] = p < parts ? ws[size_t(p) * pf + tid] : -INFINITY;
+#pragma unroll
+        for (uint32_t p = 0; p < kMaxParts; p++) top = fmaxf(top, ms[p]);
+#pragma unroll
+        for (uint32_t p = 0; p < kMaxParts; p++) {
+            ms[p] = exp_t<T>(ms[p] - top);
+            fac[p * 16 + tid] = ms[p];
+        }
+        float ls[kMaxParts];
+#pragma unroll
+        for (uint32_t p = 0; p < kMaxParts; p++) ls[p] = p < parts ? ws[size_t(p) * pf + 16 + tid] : 0.0f;
+#pragma unroll
+        for (uint32_t p = 0; p < kMaxParts; p++) sum = __builtin_fmaf(ls[p], ms[p], sum);
+        sums[tid] = sum;
+    }
+    __syncthreads();
+    for (uint32_t e = tid; e < live * quads; e += 256) {
+        const uint32_t c = e / quads, d = e % quads * 4;
+        const float *src = ws + 32 + c * s.dv_pad + d;
+        f32x4 o = {0.f, 0.f, 0.f, 0.f};
+        for (uint32_t p0 = 0; p0 < parts; p0 += 8) {  // eight parts' loads at a time
+            f32x4 v[8];
+#pragma unroll
+            for (uint32_t j = 0; j < 8; j++) v[j] = *reinterpret_cast<const f32x4 *>(src + size_t(p0 + j < parts ? p0 + j : parts - 1) * pf);
+#pragma unroll
+            for (uint32_t j = 0; j < 8; j++)
+                if (p0 + j < parts) o += v[j] * fac[(p0 + j) * 16 + c];
+        }
+        finish(c, d, o, sums[c]);
     }
 }
 
@@ -629,27 +753,35 @@ __global__ __launch_bounds__(256) void recur_scan_kernel(RmiRecurShape s, RmiRec
         }
         return x;
     };
-    Operands next = load(0);
-    for (uint32_t chunk = 0; chunk < n_chunks; chunk++) {
-        const Operands x = next;
-        next = load(chunk + 1 < n_chunks ? chunk + 1 : chunk);
-        f32x4 o = {0.f, 0.f, 0.f, 0.f};
-        if (wave == 0) o = mma16_f32(x.am, x.v, o);
+    constexpr uint32_t kAhead = TPW <= 2 ? 4 : 2;  // chunks whose operands are on their way
+    Operands ring[kAhead];
 #pragma unroll
-        for (int i = 0; i < TPW; i++) {
-            if (wave + 4 * i >= n_tiles) break;
-            o = mma16_f32(x.q[i], st[i], o);
+    for (uint32_t j = 0; j < kAhead; j++) ring[j] = load(j < n_chunks ? j : n_chunks - 1);
+    for (uint32_t chunk0 = 0; chunk0 < n_chunks; chunk0 += kAhead) {
 #pragma unroll
-            for (int r = 0; r < 4; r++) st[i][r] *= x.p[i][r];
-            st[i] = mma16_f32(x.k[i], x.v, st[i]);
-        }
-        part[chunk & 1][wave][lane] = o;
-        __syncthreads();  // (two buffers: the next chunk's writes cannot meet this one's reads)
-        if (wave == (chunk & 3)) {
-            const f32x4 sum = (part[chunk & 1][0][lane] + part[chunk & 1][1][lane]) + (part[chunk & 1][2][lane] + part[chunk & 1][3][lane]);
-            float *dst = ws.o + ((size_t(head) * n_chunks + chunk) * kChunk + g * 4) * s.v_pad + v0 + fr;
+        for (uint32_t j = 0; j < kAhead; j++) {
+            const uint32_t chunk = chunk0 + j;
+            if (chunk >= n_chunks) break;
+            f32x4 o = {0.f, 0.f, 0.f, 0.f};
+            const Operands &x = ring[j];
+            if (wave == 0) o = mma16_f32(x.am, x.v, o);
 #pragma unroll
-            for (int r = 0; r < 4; r++) dst[size_t(r) * s.v_pad] = sum[r];
+            for (int i = 0; i < TPW; i++) {
+                if (wave + 4 * i >= n_tiles) continue;
+                o = mma16_f32(x.q[i], st[i], o);
+#pragma unroll
+                for (int r = 0; r < 4; r++) st[i][r] *= x.p[i][r];
+                st[i] = mma16_f32(x.k[i], x.v, st[i]);
+            }
+            ring[j] = load(chunk + kAhead < n_chunks ? chunk + kAhead : n_chunks - 1);
+            part[chunk & 1][wave][lane] = o;
+            __syncthreads();  // (two buffers: the next chunk's writes cannot meet this one's reads)
+            if (wave == (chunk & 3)) {
+                const f32x4 sum = (part[chunk & 1][0][lane] + part[chunk & 1][1][lane]) + (part[chunk & 1][2][lane] + part[chunk & 1][3][lane]);
+                float *dst = ws.o + ((size_t(head) * n_chunks + chunk) * kChunk + g * 4) * s.v_pad + v0 + fr;
+#pragma unroll
+                for (int r = 0; r < 4; r++) dst[size_t(r) * s.v_pad] = sum[r];
+            }
         }
     }
 #pragma unroll
@@ -683,7 +815,6 @@ __global__ __launch_bounds__(256) void recur_norm_kernel(RmiRecurShape s, RmiRec
 
 // ------------------------------------------------------------------ launches
 // Keys over workgroups where the columns alone would not fill the chip; at most kMaxParts parts of 128 keys or more.
-constexpr uint32_t kMaxParts = 32;
 constexpr uint32_t kSplitMaxCols = 256;  // per key/value head
 void attn_parts(const RmiAttnShape &s, uint32_t n_tokens, uint32_t n_keys, uint32_t *parts, uint32_t *keys_per_part) {
     const uint32_t tiles = (n_tokens * (s.heads / s.kv_heads) + 15) / 16;
@@ -710,14 +841,18 @@ uint32_t bucket_of(const RmiAttnShape &s) {
     return d <= 64 ? 64 : d <= 128 ? 128 : 256;
 }
 size_t split_lds(uint32_t elem_bytes, const RmiAttnShape &s) {
-    const size_t q = size_t(16) * s.dk_pad * elem_bytes, merge = size_t(3) * attn_part_floats(s.dv_pad) * 4;
+    const size_t q = size_t(16) * s.dk_pad * elem_bytes, merge = size_t(4) * attn_part_floats(s.dv_pad) * 4;
     return q > merge ? q : merge;
 }
 
 template <typename T>
 int attn_pass(const RmiAttnShape &s, const RmiAttnArgs &a, hipStream_t st) {
     const uint32_t n_heads = s.heads + 2 * s.kv_heads, group = s.heads / s.kv_heads, n_cols = a.n_tokens * group;
-    hipLaunchKernelGGL(conv_rotate_kernel<T>, dim3(n_heads, (a.n_tokens + 3) / 4), dim3(256), 0, st, s, a);
+    const dim3 conv_grid(n_heads, (a.n_tokens + 4 * kConvRun - 1) / (4 * kConvRun));
+    if (s.taps <= 4 && s.dim % 2 == 0 && s.vdim % 2 == 0 && s.dim <= 128 && s.vdim <= 128)
+        hipLaunchKernelGGL(conv_rotate_pairs_kernel<T>, conv_grid, dim3(256), 0, st, s, a);
+    else
+        hipLaunchKernelGGL(conv_rotate_kernel<T>, conv_grid, dim3(256), 0, st, s, a);
     const uint32_t bucket = bucket_of(s);
     if (n_cols <= kSplitMaxCols) {
         uint32_t parts, kpp;
@@ -728,8 +863,11 @@ int attn_pass(const RmiAttnShape &s, const RmiAttnArgs &a, hipStream_t st) {
             hipLaunchKernelGGL((attn_split_kernel<T, 64>), grid, dim3(256), lds, st, s, a, parts, kpp);
         else if (bucket == 128)
             hipLaunchKernelGGL((attn_split_kernel<T, 128>), grid, dim3(256), lds, st, s, a, parts, kpp);
-        else
+        else {
+            const int rc = rmi_allow_lds(attn_split_kernel<T, 256>, lds);
+            if (rc != RMI_HIP_OK) return rc;
             hipLaunchKernelGGL((attn_split_kernel<T, 256>), grid, dim3(256), lds, st, s, a, parts, kpp);
+        }
     } else {
         auto grid = [&](uint32_t qt) { return dim3((n_cols + 64 * qt - 1) / (64 * qt), s.kv_heads); };
         if (bucket == 64)
@@ -770,8 +908,11 @@ int mixers_step(const RmiAttnShape *as, const RmiAttnArgs *aa, const RmiRecurSha
         hipLaunchKernelGGL((mixers_step_kernel<T, 64>), grid, dim3(256), lds, st, s, a, blocks, parts, kpp, r, b);
     else if (bucket == 128)
         hipLaunchKernelGGL((mixers_step_kernel<T, 128>), grid, dim3(256), lds, st, s, a, blocks, parts, kpp, r, b);
-    else
+    else {
+        const int rc = rmi_allow_lds(mixers_step_kernel<T, 256>, lds);
+        if (rc != RMI_HIP_OK) return rc;
         hipLaunchKernelGGL((mixers_step_kernel<T, 256>), grid, dim3(256), lds, st, s, a, blocks, parts, kpp, r, b);
+    }
     RMI_HIP_CHECK(hipGetLastError());
     return RMI_HIP_OK;
 }

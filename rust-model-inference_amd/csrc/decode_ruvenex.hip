@@ -33,7 +33,7 @@ struct RuvenexLayer {
     float *conv = nullptr, *cos_t = nullptr, *sin_t = nullptr, *recur_norm = nullptr;
     void *k_cache = nullptr, *v_cache = nullptr;
     float *hist[2] = {nullptr, nullptr};
-    float *state = nullptr;
+    float *state[2] = {nullptr, nullptr};
     uint32_t k_attn = 0, k_recur = 0;  // where the recurrence's and the feed-forward's columns begin
 };
 
@@ -68,7 +68,7 @@ struct rmi_hip_ruvenex : RmiSession {
     float *recur_scratch = nullptr;
     uint32_t *want_rows = nullptr;
     uint32_t position = 0;         // tokens of the current sequence so far
-    int hist_now = 0;              // which of a layer's two history buffers holds the last pass's
+    int now = 0;              // which of a layer's two history and state buffers the last pass left
     uint32_t embedded = ~0u;       // the position whose embedding the last sampling launch left in x
 
     void begin_sequence() override {
@@ -101,8 +101,8 @@ int rmi_hip_ruvenex::enqueue_layers(uint32_t step0, uint32_t n, hipStream_t st, 
         const RuvenexLayer &y = layers[l];
         RmiAttnArgs a{};
         a.u = u;
-        a.hist_in = y.hist[hist_now];
-        a.hist_out = y.hist[hist_now ^ 1];
+        a.hist_in = y.hist[now];
+        a.hist_out = y.hist[now ^ 1];
         a.conv = y.conv;
         a.cos_t = y.cos_t;
         a.sin_t = y.sin_t;
@@ -119,7 +119,8 @@ int rmi_hip_ruvenex::enqueue_layers(uint32_t step0, uint32_t n, hipStream_t st, 
         r.q = rq;
         r.f = rf;
         r.v = rv;
-        r.state = y.state;
+        r.state_in = y.state[now];
+        r.state_out = y.state[now ^ 1];
         r.norm = y.recur_norm;
         r.out = static_cast<uint8_t *>(act) + size_t(y.k_attn) * elem;
         r.out_ld = y.w_out.k_pad;
@@ -142,7 +143,7 @@ int rmi_hip_ruvenex::enqueue_layers(uint32_t step0, uint32_t n, hipStream_t st, 
             RMI_HIP_CHECK(hipMemcpy(host_layers + size_t(l) * n * width, x, size_t(n) * width * 4, hipMemcpyDeviceToHost));
         }
     }
-    hist_now ^= 1;
+    now ^= 1;
     position = step0 + n;
     return rc;
 }
@@ -564,7 +565,8 @@ bool rmi_hip_ruvenex::load(const RmiModelFolder &folder, uint32_t elem_bytes, ui
         if (!y.cos_t || !y.sin_t || !(y.conv = upload(taps.data(), taps.size())) || !(y.hist[0] = alloc<float>(hist, true)) ||
             !(y.hist[1] = alloc<float>(hist, true)) || !(y.k_cache = alloc_bytes(size_t(a.kv_heads) * cap_pad * a.dk_pad * elem, true)) ||
             !(y.v_cache = alloc_bytes(size_t(a.kv_heads) * cap_pad * a.dv_pad * elem, true)) ||
-            !(y.state = alloc<float>(size_t(r.heads) * r.d_pad * r.v_pad, true)))
+            !(y.state[0] = alloc<float>(size_t(r.heads) * r.d_pad * r.v_pad, true)) ||
+            !(y.state[1] = alloc<float>(size_t(r.heads) * r.d_pad * r.v_pad, true)))
             return false;
     }
     if (hipDeviceSynchronize() != hipSuccess) {

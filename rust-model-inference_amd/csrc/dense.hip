@@ -53,7 +53,7 @@ __global__ __launch_bounds__(256) void dense_gemm_kernel(const T *__restrict__ w
     constexpr int NN = WN / 16, NT = WT / 16;
     constexpr int PW = BN * 8 / 256, PA = (BT * 8 + 255) / 256;  // pieces a thread loads per step
     __shared__ u32x4 lds[2][(BN + BT) * 8];
-    const uint32_t tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
+    const uint32_t tid = threadIdx.x, lane = tid & 63, wave = uint32_t(__builtin_amdgcn_readfirstlane(int(tid >> 6)));
     uint32_t n_tile, t_tile;
     rmi_gemm_tile_of(blockIdx.x, grid_n, grid_t, 1u, 0u, n_tile, t_tile);
     const uint32_t row0 = n_tile * BN, tok0 = t_tile * BT;
@@ -347,7 +347,7 @@ __global__ __launch_bounds__(256) void gemv_residual_kernel(const T *__restrict_
                                                             RmiColSegs cs, float *__restrict__ x, uint32_t width) {
     constexpr int U = 4;
     __shared__ float part[4][ROWS];
-    const uint32_t tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
+    const uint32_t tid = threadIdx.x, lane = tid & 63, wave = uint32_t(__builtin_amdgcn_readfirstlane(int(tid >> 6)));
     const uint32_t row0 = blockIdx.x * ROWS;
     const uint32_t pieces = k_pad / kPieceElems<T>, per_wave = ((pieces + 3) / 4 + 63) / 64 * 64;
     const uint32_t p_begin = wave * per_wave, p_end = p_begin + per_wave < pieces ? p_begin + per_wave : pieces;

@@ -45,7 +45,8 @@ struct RmiRecurShape {
 };
 struct RmiRecurArgs {
     const float *q, *f, *v;  // [n_tokens][heads * dim], f = the forget gate; [n_tokens][heads * vdim]
-    float *state;            // [head][d_pad][v_pad]; not read at pos0 == 0
+    const float *state_in;   // [head][d_pad][v_pad]; not read at pos0 == 0
+    float *state_out;        // another buffer
     const float *norm;       // [vdim]
     void *out;               // [token * out_ld + head * vdim + channel], the model's element type
     uint32_t out_ld, pos0, n_tokens;

@@ -130,8 +130,30 @@ __global__ __launch_bounds__(256) void conv_rotate_kernel(RmiAttnShape s, RmiAtt
     }
 }
 
-// Even head sizes up to 128 and up to four taps: a lane holds one pair of channels, its taps and a sliding window of
-// the projected values; every row is read once.
+// Even head sizes up to 128 and up to four taps: a lane holds one pair of channels.
+__host__ __device__ inline bool conv_pairs_fit(const RmiAttnShape &s) {
+    return s.taps <= 4 && s.dim % 2 == 0 && s.vdim % 2 == 0 && s.dim <= 128 && s.vdim <= 128;
+}
+// taps of channels c, c + 1, four each, the last one the token's own
+struct PairTaps {
+    float w0[4], w1[4];
+    __device__ __forceinline__ void load(const RmiAttnShape &s, const float *conv, uint32_t c) {
+        const uint32_t off = 4 - s.taps;
+#pragma unroll
+        for (uint32_t j = 0; j < 4; j++) {
+            w0[j] = j >= off ? conv[c * s.taps + j - off] : 0.0f;
+            w1[j] = j >= off ? conv[(c + 1) * s.taps + j - off] : 0.0f;
+        }
+    }
+};
+// the projected pair at the pass's row t - back (back <= 3), zeros before the sequence's start
+__device__ __forceinline__ float2 pair_row(const RmiAttnShape &s, const RmiAttnArgs &a, uint32_t channels, uint32_t t, uint32_t back, uint32_t c) {
+    if (t >= back) return *reinterpret_cast<const float2 *>(a.u + size_t(t - back) * channels + c);
+    if (back - t < s.taps && a.pos0 + t >= back) return *reinterpret_cast<const float2 *>(a.hist_in + size_t(t + s.taps - 1 - back) * channels + c);
+    return make_float2(0.f, 0.f);
+}
+
+// A run of tokens: the taps and a sliding window of projected values stay in registers; every row is read once.
 template <typename T>
 __global__ __launch_bounds__(256) void conv_rotate_pairs_kernel(RmiAttnShape s, RmiAttnArgs a) {
     const uint32_t lane = threadIdx.x & 63, head = blockIdx.x;
@@ -145,13 +167,9 @@ __global__ __launch_bounds__(256) void conv_rotate_pairs_kernel(RmiAttnShape s, 
     const uint32_t c0 = is_v ? (s.heads + s.kv_heads) * s.dim + (head - s.heads - s.kv_heads) * s.vdim : head * s.dim;
     const bool has = 2 * lane < dim;
     const uint32_t c = c0 + (has ? 2 * lane : 0);
-    float w0[4], w1[4], u0[4], u1[4];  // tap and row j of four, the last one the token's own
-    const uint32_t off = 4 - s.taps;
-#pragma unroll
-    for (uint32_t j = 0; j < 4; j++) {
-        w0[j] = j >= off ? a.conv[c * s.taps + j - off] : 0.0f;
-        w1[j] = j >= off ? a.conv[(c + 1) * s.taps + j - off] : 0.0f;
-    }
+    float u0[4], u1[4];  // row j of four, the last one the token's own
+    PairTaps w;
+    w.load(s, a.conv, c);
     float2 row[kConvRun];
 #pragma unroll
     for (uint32_t i = 0; i < kConvRun; i++) {
@@ -159,13 +177,8 @@ __global__ __launch_bounds__(256) void conv_rotate_pairs_kernel(RmiAttnShape s, 
         row[i] = *reinterpret_cast<const float2 *>(a.u + size_t(t) * channels + c);
     }
 #pragma unroll
-    for (uint32_t j = 1; j < 4; j++) {  // the rows before the run: position pos0 + t0 - (4 - j)
-        const uint32_t back = 4 - j;
-        float2 v = make_float2(0.f, 0.f);
-        if (t0 >= back)
-            v = *reinterpret_cast<const float2 *>(a.u + size_t(t0 - back) * channels + c);
-        else if (back - t0 < s.taps && a.pos0 + t0 >= back)
-            v = *reinterpret_cast<const float2 *>(a.hist_in + size_t(t0 + s.taps - 1 - back) * channels + c);
+    for (uint32_t j = 1; j < 4; j++) {  // the rows before the run
+        const float2 v = pair_row(s, a, channels, t0, 4 - j, c);
         u0[j] = v.x;
         u1[j] = v.y;
     }
@@ -194,8 +207,8 @@ __global__ __launch_bounds__(256) void conv_rotate_pairs_kernel(RmiAttnShape s, 
         float p = 0.0f, q = 0.0f;
 #pragma unroll
         for (uint32_t j = 0; j < 4; j++) {
-            p = __builtin_fmaf(w0[j], u0[j], p);
-            q = __builtin_fmaf(w1[j], u1[j], q);
+            p = __builtin_fmaf(w.w0[j], u0[j], p);
+            q = __builtin_fmaf(w.w1[j], u1[j], q);
         }
         if (!has) p = q = 0.0f;
         if (is_v) {
@@ -241,33 +254,45 @@ struct AttnWave {
             for (uint32_t v = 0; v < kVT; v++) o[i][v] = f32x4{0.f, 0.f, 0.f, 0.f};
         }
     }
-    // keys [k0, k1), k0 a multiple of 32; column i sees keys up to last[i] (< k1 not required)
-    __device__ __forceinline__ void keys(const T *kc, const T *vc, const RmiAttnShape &s, uint32_t k0, uint32_t k1, const int (&last)[QT]) {
+    // a block's keys and values fit in registers beside the rest: values of a block and keys of the next are under way
+    // while the block's scores and weights are computed
+    static constexpr bool kAhead = BUCKET * sizeof(T) <= 256;
+    u32x4 kf[2][kAhead ? kKC : 1], vf[kAhead ? kVT * (sizeof(T) / 2) : 1];
+
+    __device__ __forceinline__ void load_keys(const T *kc, const RmiAttnShape &s, uint32_t k) {
+        const uint32_t lane = threadIdx.x & 63, n_kc = s.dk_pad / (4 * kPieceElems<T>);
+        const T *row = kc + size_t(k + (lane & 15)) * s.dk_pad + (lane >> 4) * kPieceElems<T>;
+#pragma unroll
+        for (uint32_t c = 0; c < (kAhead ? kKC : 0); c++) {
+            if (c >= n_kc) continue;
+            kf[0][c] = *reinterpret_cast<const u32x4 *>(row + c * 4 * kPieceElems<T>);
+            kf[1][c] = *reinterpret_cast<const u32x4 *>(row + c * 4 * kPieceElems<T> + 16 * size_t(s.dk_pad));
+        }
+    }
+    __device__ __forceinline__ const T *value_at(const T *vc, const RmiAttnShape &s, uint32_t k) {
+        const uint32_t lane = threadIdx.x & 63;
+        return vc + size_t(k / kKeyBlock) * s.dv_pad * kKeyBlock + size_t(lane & 15) * kKeyBlock + (lane >> 4) * kPieceElems<T>;
+    }
+    __device__ __forceinline__ void load_values(const T *vc, const RmiAttnShape &s, uint32_t k) {
+        const T *vb = value_at(vc, s, k);
+        const uint32_t n_vt = s.dv_pad / 16;
+#pragma unroll
+        for (uint32_t v = 0; v < (kAhead ? kVT : 0); v++)
+#pragma unroll
+            for (uint32_t t = 0; t < sizeof(T) / 2; t++)
+                if (v < n_vt) vf[v * (sizeof(T) / 2) + t] = *reinterpret_cast<const u32x4 *>(vb + size_t(v) * 16 * kKeyBlock + t * 16);
+    }
+    // keys [k0, k1), k0 a multiple of 32; column i sees keys up to last[i] (< k1 not required).  loaded: the first
+    // block's keys and values are in kf and vf
+    __device__ __forceinline__ void keys(const T *kc, const T *vc, const RmiAttnShape &s, uint32_t k0, uint32_t k1, const int (&last)[QT],
+                                         bool loaded = false) {
         const uint32_t lane = threadIdx.x & 63, fr = lane & 15, g = lane >> 4;
         const uint32_t n_kc = s.dk_pad / (4 * kPieceElems<T>), n_vt = s.dv_pad / 16;
         const T *krow = kc + size_t(fr) * s.dk_pad + g * kPieceElems<T>;
-        constexpr bool kAhead = BUCKET * sizeof(T) <= 256;  // a block's keys and values fit in registers beside the rest
-        u32x4 kf[2][kAhead ? kKC : 1], vf[kAhead ? kVT * (sizeof(T) / 2) : 1];
-        auto load_keys = [&](uint32_t k) {
-#pragma unroll
-            for (uint32_t c = 0; c < kKC; c++) {
-                if (c >= n_kc) continue;
-                const T *p = krow + size_t(k) * s.dk_pad + c * 4 * kPieceElems<T>;
-                kf[0][c] = *reinterpret_cast<const u32x4 *>(p);
-                kf[1][c] = *reinterpret_cast<const u32x4 *>(p + 16 * size_t(s.dk_pad));
-            }
-        };
-        if constexpr (kAhead)
-            if (k0 < k1) load_keys(k0);
+        if (!loaded && k0 < k1) load_keys(kc, s, k0);
         for (uint32_t k = k0; k < k1; k += kKeyBlock) {
-            const T *vb = vc + size_t(k / kKeyBlock) * s.dv_pad * kKeyBlock + size_t(fr) * kKeyBlock + g * kPieceElems<T>;
-            if constexpr (kAhead) {
-#pragma unroll
-                for (uint32_t v = 0; v < kVT; v++)
-#pragma unroll
-                    for (uint32_t t = 0; t < sizeof(T) / 2; t++)
-                        if (v < n_vt) vf[v * (sizeof(T) / 2) + t] = *reinterpret_cast<const u32x4 *>(vb + size_t(v) * 16 * kKeyBlock + t * 16);
-            }
+            const T *vb = value_at(vc, s, k);
+            if (!loaded || k != k0) load_values(vc, s, k);
             f32x4 sc[QT][2];
 #pragma unroll
             for (int i = 0; i < QT; i++) sc[i][0] = sc[i][1] = f32x4{0.f, 0.f, 0.f, 0.f};
@@ -289,8 +314,7 @@ struct AttnWave {
                     sc[i][1] = mma16<T>(f1, qf[i][c], sc[i][1]);
                 }
             }
-            if constexpr (kAhead)
-                if (k + kKeyBlock < k1) load_keys(k + kKeyBlock);
+            if (k + kKeyBlock < k1) load_keys(kc, s, k + kKeyBlock);
             u32x4 pf[QT][2];
 #pragma unroll
             for (int i = 0; i < QT; i++) {
@@ -361,7 +385,7 @@ template <typename T, int BUCKET, int QT>
 __global__ __launch_bounds__(256) void attn_pass_kernel(RmiAttnShape s, RmiAttnArgs a) {
     const uint32_t lane = threadIdx.x & 63, fr = lane & 15, g4 = lane >> 4;
     const uint32_t group = s.heads / s.kv_heads, kvh = blockIdx.y, n_cols = a.n_tokens * group;
-    const uint32_t tile = (gridDim.x - 1 - blockIdx.x) * 4 + (threadIdx.x >> 6);  // the longest columns first
+    const uint32_t tile = (gridDim.x - 1 - blockIdx.x) * 4 + uint32_t(__builtin_amdgcn_readfirstlane(int(threadIdx.x >> 6)));  // the longest columns first
     if (tile * QT * 16 >= n_cols) return;
     AttnWave<T, BUCKET, QT> w;
     w.init();
@@ -398,13 +422,15 @@ __global__ __launch_bounds__(256) void attn_pass_kernel(RmiAttnShape s, RmiAttnA
 // LDS, writes its part, and the one that arrives last merges the parts.  With one token (STEP) the workgroup makes
 // its queries itself, and the workgroups of the last part the new key and value.
 constexpr uint32_t kMaxParts = 32;
+constexpr uint32_t kStepThreads = 256;  // a workgroup of the single-token launch
 // a part: the columns' maxima, their sums, and [column][channel]
 __host__ __device__ inline uint32_t attn_part_floats(uint32_t dv_pad) { return 16 * (dv_pad + 2); }
 
 template <typename T, int BUCKET, bool STEP>
 __device__ __forceinline__ void attn_split(const RmiAttnShape &s, const RmiAttnArgs &a, uint32_t block, uint32_t parts, uint32_t keys_per_part,
                                            uint8_t *lds, uint32_t *flag) {
-    const uint32_t tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, fr = lane & 15, g4 = lane >> 4;
+    constexpr uint32_t NW = 4;
+    const uint32_t tid = threadIdx.x, lane = tid & 63, wave = uint32_t(__builtin_amdgcn_readfirstlane(int(tid >> 6))), fr = lane & 15, g4 = lane >> 4;
     const uint32_t group = s.heads / s.kv_heads, n_cols = a.n_tokens * group, tiles = (n_cols + 15) / 16;
     const uint32_t part = block % parts, ct = (block / parts) % tiles, kvh = block / parts / tiles;
     const uint32_t n_keys = a.pos0 + a.n_tokens;
@@ -413,28 +439,81 @@ __device__ __forceinline__ void attn_split(const RmiAttnShape &s, const RmiAttnA
     w.init();
     const uint32_t col = ct * 16 + fr, cc = col < n_cols ? col : n_cols - 1;
     const int last[1] = {int(a.pos0 + cc / group)};
+    const T *kc = static_cast<const T *>(a.k_cache) + size_t(kvh) * s.capacity * s.dk_pad;
+    const T *vc = static_cast<const T *>(a.v_cache) + size_t(kvh) * s.capacity * s.dv_pad;
+    const uint32_t p0 = part * keys_per_part, p1 = p0 + keys_per_part < n_keys ? p0 + keys_per_part : n_keys;
+    const uint32_t per_wave = keys_per_part / NW;  // a multiple of the key block
+    const uint32_t k0 = p0 + wave * per_wave, k1 = k0 + per_wave < p1 ? k0 + per_wave : p1;
+    bool loaded = false;
     if constexpr (STEP) {
         T *q = reinterpret_cast<T *>(lds);
         const uint32_t channels = (s.heads + s.kv_heads) * s.dim + s.kv_heads * s.vdim;
         const ConvCtx x{a.u, a.hist_in, a.conv, channels, s.taps};
         const uint32_t half = s.dk_pad / 2, c_end = n_cols - ct * 16 < 16 ? n_cols - ct * 16 : 16;
-        if (part == parts - 1) {
-            if (wave == 2) key_row<T>(x, s, a, 0, kvh, lane);
-            if (wave == 3) value_row<T>(x, s, a, 0, kvh, lane);
-        }
-        for (uint32_t e = tid; e < c_end * half; e += 256) {
-            const uint32_t c = e / half, i = e % half, head = kvh * group + ct * 16 + c;
-            float p, r;
-            conv_rotate_pair(x, s, a.cos_t, a.sin_t, 0, a.pos0, head * s.dim, i, p, r);
-            store_pair(q + c * s.dk_pad + 2 * i, p, r);
-        }
-        if (part == 0) {  // the history of this workgroup's channels
-            const uint32_t c0 = (kvh * group + ct * 16) * s.dim;
-            for (uint32_t d = tid; d < c_end * s.dim; d += 256) conv_carry(x, a.hist_out, 1, c0 + d);
-            if (ct == 0) {
-                for (uint32_t d = tid; d < s.dim; d += 256) conv_carry(x, a.hist_out, 1, (s.heads + kvh) * s.dim + d);
-                for (uint32_t d = tid; d < s.vdim; d += 256)
-                    conv_carry(x, a.hist_out, 1, (s.heads + s.kv_heads) * s.dim + kvh * s.vdim + d);
+        const bool newest = part == parts - 1;  // this part holds the token's own key and value
+        // the first block of keys and values: under way behind the convolution's operands, unless it holds the new one
+        auto ahead = [&] {
+            loaded = w.kAhead && k0 < k1 && k0 + kKeyBlock < n_keys;
+            if (loaded) {
+                w.load_keys(kc, s, k0);
+                w.load_values(vc, s, k0);
+            }
+        };
+        if (conv_pairs_fit(s)) {
+            // with the new key and value to make, the last two waves make them and the others the queries
+            const uint32_t q_threads = newest ? 128 : 256, rot = s.rot_dims / 2;
+            const bool is_k = newest && wave == 2, is_v = newest && wave == 3;
+            const uint32_t n_pairs = is_v ? s.vdim / 2 : is_k ? half : c_end * half, step = is_k || is_v ? 64 : q_threads;
+            bool first = true;
+            for (uint32_t e0 = 0; e0 < n_pairs || first; e0 += step) {
+                const uint32_t e = e0 + (is_k || is_v ? lane : tid), ec = e < n_pairs ? e : 0;
+                const uint32_t c = is_k || is_v ? 0 : ec / half, i = is_k || is_v ? ec : ec % half;
+                const bool has = e < n_pairs && (is_v || 2 * i < s.dim);
+                const uint32_t c0 = is_v   ? (s.heads + s.kv_heads) * s.dim + kvh * s.vdim
+                                    : is_k ? (s.heads + kvh) * s.dim
+                                           : (kvh * group + ct * 16 + c) * s.dim;
+                const uint32_t ch = c0 + (has ? 2 * i : 0);
+                PairTaps t;
+                float2 r[4];
+#pragma unroll
+                for (uint32_t j = 0; j < 4; j++) r[j] = pair_row(s, a, channels, 0, 3 - j, ch);
+                t.load(s, a.conv, ch);
+                const bool turned = has && !is_v && i < rot;
+                const size_t at = size_t(a.pos0) * rot + (turned ? i : 0);
+                const float cs = turned ? a.cos_t[at] : 1.0f, sn = turned ? a.sin_t[at] : 0.0f;
+                if (first) ahead();
+                first = false;
+                float p = 0.0f, o = 0.0f;
+#pragma unroll
+                for (uint32_t j = 0; j < 4; j++) {
+                    p = __builtin_fmaf(t.w0[j], r[j].x, p);
+                    o = __builtin_fmaf(t.w1[j], r[j].y, o);
+                }
+                if (!has) p = o = 0.0f;
+                if (is_v) {  // (at most 64 pairs: one round)
+                    const float f = 1.0f / sqrtf(wave_sum_f32(__builtin_fmaf(p, p, o * o)) / float(s.vdim) + s.eps);
+                    T *blk = const_cast<T *>(vc) + size_t(a.pos0 / kKeyBlock) * s.dv_pad * kKeyBlock + value_slot<T>(a.pos0 % kKeyBlock);
+                    if (has) {
+                        blk[size_t(2 * i) * kKeyBlock] = from_f32<T>(p * f);
+                        blk[size_t(2 * i + 1) * kKeyBlock] = from_f32<T>(o * f);
+                    }
+                } else if (e < n_pairs) {
+                    const float rp = p;
+                    p = __builtin_fmaf(rp, cs, -(o * sn));
+                    o = __builtin_fmaf(o, cs, rp * sn);
+                    store_pair(is_k ? const_cast<T *>(kc) + size_t(a.pos0) * s.dk_pad + 2 * i : q + c * s.dk_pad + 2 * i, p, o);
+                }
+            }
+        } else {
+            if (newest) {
+                if (wave == NW - 2) key_row<T>(x, s, a, 0, kvh, lane);
+                if (wave == NW - 1) value_row<T>(x, s, a, 0, kvh, lane);
+            }
+            for (uint32_t e = tid; e < c_end * half; e += 256) {
+                const uint32_t c = e / half, i = e % half, head = kvh * group + ct * 16 + c;
+                float p, r;
+                conv_rotate_pair(x, s, a.cos_t, a.sin_t, 0, a.pos0, head * s.dim, i, p, r);
+                store_pair(q + c * s.dk_pad + 2 * i, p, r);
             }
         }
         __syncthreads();
@@ -453,15 +532,23 @@ __device__ __forceinline__ void attn_split(const RmiAttnShape &s, const RmiAttnA
             w.qf[0][c] = *reinterpret_cast<const u32x4 *>(q + c * 4 * kPieceElems<T>);
         }
     }
-    const uint32_t p0 = part * keys_per_part, p1 = p0 + keys_per_part < n_keys ? p0 + keys_per_part : n_keys;
-    const uint32_t per_wave = keys_per_part / 4;  // a multiple of the key block
-    const uint32_t k0 = p0 + wave * per_wave, k1 = k0 + per_wave < p1 ? k0 + per_wave : p1;
-    if (k0 < k1)
-        w.keys(static_cast<const T *>(a.k_cache) + size_t(kvh) * s.capacity * s.dk_pad,
-               static_cast<const T *>(a.v_cache) + size_t(kvh) * s.capacity * s.dv_pad, s, k0, k1, last);
+    if (k0 < k1) w.keys(kc, vc, s, k0, k1, last, loaded);
+    if constexpr (STEP) {
+        if (part == 0) {  // the history of this workgroup's channels
+            const uint32_t channels = (s.heads + s.kv_heads) * s.dim + s.kv_heads * s.vdim;
+            const ConvCtx x{a.u, a.hist_in, a.conv, channels, s.taps};
+            const uint32_t c_end = n_cols - ct * 16 < 16 ? n_cols - ct * 16 : 16, c0 = (kvh * group + ct * 16) * s.dim;
+            for (uint32_t d = tid; d < c_end * s.dim; d += 256) conv_carry(x, a.hist_out, 1, c0 + d);
+            if (ct == 0) {
+                for (uint32_t d = tid; d < s.dim; d += 256) conv_carry(x, a.hist_out, 1, (s.heads + kvh) * s.dim + d);
+                for (uint32_t d = tid; d < s.vdim; d += 256)
+                    conv_carry(x, a.hist_out, 1, (s.heads + s.kv_heads) * s.dim + kvh * s.vdim + d);
+            }
+        }
+    }
     // the waves' results to LDS, live columns only; then every thread merges (column, channel) pairs
-    const uint32_t live = n_cols - ct * 16 < 16 ? n_cols - ct * 16 : 16, pf = attn_part_floats(s.dv_pad);
-    float *all = reinterpret_cast<float *>(lds), *mine = all + wave * pf;
+    const uint32_t live = n_cols - ct * 16 < 16 ? n_cols - ct * 16 : 16, pf = attn_part_floats(s.dv_pad), pl = 32 + live * s.dv_pad;
+    float *all = reinterpret_cast<float *>(lds), *mine = all + wave * pl;
     const float l = rows_sum_f32(w.l[0]);
     if (fr < live) {
         if (g4 == 0) {
@@ -475,39 +562,43 @@ __device__ __forceinline__ void attn_split(const RmiAttnShape &s, const RmiAttnA
     __syncthreads();
     const uint32_t slot = kvh * tiles + ct;
     float *ws = reinterpret_cast<float *>(static_cast<uint32_t *>(a.scratch) + kAttnCounters) + size_t(slot) * parts * pf;
-    const uint32_t quads = s.dv_pad / 4;
-    auto finish = [&](uint32_t c, uint32_t d, f32x4 o, float sum) {
+    const uint32_t pairs = live * s.dv_pad;
+    auto finish = [&](uint32_t e, float o, float sum) {
+        const uint32_t c = e / s.dv_pad, d = e % s.dv_pad;
+        if (d >= s.vdim) return;
         const uint32_t mc = ct * 16 + c, t = mc / group, head = kvh * group + mc % group;
-        attn_store<T>(s, a, t, head, d, o * ((a.gate ? a.gate[size_t(t) * s.heads + head] : 1.0f) / sum));
+        static_cast<T *>(a.out)[size_t(t) * a.out_ld + size_t(head) * s.vdim + d] =
+            from_f32<T>(o * ((a.gate ? a.gate[size_t(t) * s.heads + head] : 1.0f) / sum));
     };
-    for (uint32_t e = tid; e < live * quads; e += 256) {
-        const uint32_t c = e / quads, d = e % quads * 4;
+    for (uint32_t e = tid; e < pairs; e += 256) {
+        const uint32_t c = e / s.dv_pad;
         float m = all[c];
 #pragma unroll
-        for (uint32_t i = 1; i < 4; i++) m = fmaxf(m, all[i * pf + c]);
+        for (uint32_t i = 1; i < NW; i++) m = fmaxf(m, all[i * pl + c]);
         const float ref = m == -INFINITY ? 0.0f : m;  // a column that sees no key of this part
-        float sum = 0.0f;
-        f32x4 o = {0.f, 0.f, 0.f, 0.f};
+        float sum = 0.0f, o = 0.0f;
 #pragma unroll
-        for (uint32_t i = 0; i < 4; i++) {
-            const float f = exp_t<T>(all[i * pf + c] - ref);
-            sum = __builtin_fmaf(all[i * pf + 16 + c], f, sum);
-            o += *reinterpret_cast<const f32x4 *>(all + i * pf + 32 + c * s.dv_pad + d) * f;
+        for (uint32_t i = 0; i < NW; i++) {
+            const float f = exp_t<T>(all[i * pl + c] - ref);
+            sum = __builtin_fmaf(all[i * pl + 16 + c], f, sum);
+            o = __builtin_fmaf(all[i * pl + 32 + e], f, o);
         }
         if (parts == 1) {
-            finish(c, d, o, sum);
+            finish(e, o, sum);
         } else {
             float *dst = ws + size_t(part) * pf;
-            if (d == 0) {
-                dst[c] = m;
-                dst[16 + c] = sum;
+            if (e % s.dv_pad == 0) {
+                __hip_atomic_store(dst + c, m, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
+                __hip_atomic_store(dst + 16 + c, sum, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
             }
-            *reinterpret_cast<f32x4 *>(dst + 32 + c * s.dv_pad + d) = o;
+            __hip_atomic_store(dst + 32 + e, o, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
         }
     }
     if (parts == 1) return;
-    // hand-over: every wave releases its own stores, then the workgroup counts once
-    __builtin_amdgcn_fence(__ATOMIC_RELEASE, "agent");
+    // Hand-over between workgroups.  Everything handed over is written and read by agent-scope atomics, past the caches
+    // that are not coherent; a wave's stores are complete before it arrives at the barrier, and the workgroup counts
+    // behind the barrier, so no cache has to be written back or invalidated.
+    __builtin_amdgcn_s_waitcnt(0);
     __syncthreads();
     if (tid == 0) {
         uint32_t *count = static_cast<uint32_t *>(a.scratch) + slot;
@@ -517,41 +608,34 @@ __device__ __forceinline__ void attn_split(const RmiAttnShape &s, const RmiAttnA
     }
     __syncthreads();
     if (!*flag) return;
-    __builtin_amdgcn_fence(__ATOMIC_ACQUIRE, "agent");
-    // what each part counts for: [part][column] factors in LDS, the sums behind them
-    float *fac = all, *sums = all + kMaxParts * 16;
-    if (tid < live) {
-        float ms[kMaxParts], top = -INFINITY, sum = 0.0f;
-#pragma unroll
-        for (uint32_t p = 0; p < kMaxParts; p++) ms[p] = p < parts ? ws[size_t(p) * pf + tid] : -INFINITY;
-#pragma unroll
-        for (uint32_t p = 0; p < kMaxParts; p++) top = fmaxf(top, ms[p]);
-#pragma unroll
-        for (uint32_t p = 0; p < kMaxParts; p++) {
-            ms[p] = exp_t<T>(ms[p] - top);
-            fac[p * 16 + tid] = ms[p];
-        }
-        float ls[kMaxParts];
-#pragma unroll
-        for (uint32_t p = 0; p < kMaxParts; p++) ls[p] = p < parts ? ws[size_t(p) * pf + 16 + tid] : 0.0f;
-#pragma unroll
-        for (uint32_t p = 0; p < kMaxParts; p++) sum = __builtin_fmaf(ls[p], ms[p], sum);
-        sums[tid] = sum;
-    }
-    __syncthreads();
-    for (uint32_t e = tid; e < live * quads; e += 256) {
-        const uint32_t c = e / quads, d = e % quads * 4;
-        const float *src = ws + 32 + c * s.dv_pad + d;
-        f32x4 o = {0.f, 0.f, 0.f, 0.f};
+    for (uint32_t e = tid; e < pairs; e += 256) {
+        const uint32_t c = e / s.dv_pad;
+        float m = -INFINITY, sum = 0.0f, o = 0.0f;
         for (uint32_t p0 = 0; p0 < parts; p0 += 8) {  // eight parts' loads at a time
-            f32x4 v[8];
+            float mv[8], lv[8], ov[8];
 #pragma unroll
-            for (uint32_t j = 0; j < 8; j++) v[j] = *reinterpret_cast<const f32x4 *>(src + size_t(p0 + j < parts ? p0 + j : parts - 1) * pf);
+            for (uint32_t j = 0; j < 8; j++) {
+                const float *src = ws + size_t(p0 + j < parts ? p0 + j : parts - 1) * pf;
+                mv[j] = __hip_atomic_load(src + c, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
+                lv[j] = __hip_atomic_load(src + 16 + c, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
+                ov[j] = __hip_atomic_load(src + 32 + e, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
+            }
+            float top = m;
 #pragma unroll
             for (uint32_t j = 0; j < 8; j++)
-                if (p0 + j < parts) o += v[j] * fac[(p0 + j) * 16 + c];
+                if (p0 + j < parts) top = fmaxf(top, mv[j]);
+            const float ref = top == -INFINITY ? 0.0f : top, keep = exp_t<T>(m - ref);
+            sum *= keep;
+            o *= keep;
+#pragma unroll
+            for (uint32_t j = 0; j < 8; j++) {
+                const float f = p0 + j < parts ? exp_t<T>(mv[j] - ref) : 0.0f;
+                sum = __builtin_fmaf(lv[j], f, sum);
+                o = __builtin_fmaf(ov[j], f, o);
+            }
+            m = top;
         }
-        finish(c, d, o, sums[c]);
+        finish(e, o, sum);
     }
 }
 
@@ -563,21 +647,23 @@ __global__ __launch_bounds__(256) void attn_split_kernel(RmiAttnShape s, RmiAttn
 }
 
 // ---- gated linear recurrence
-// one token of one head: a thread takes four state columns and every (256 / (v_pad / 4))-th row
+// one token of one head: a thread takes four state columns and every (kStepThreads / (v_pad / 4))-th row
 template <typename T>
 __device__ __forceinline__ void recur_step(const RmiRecurShape &s, const RmiRecurArgs &a, uint32_t head, float *lds) {
-    const uint32_t tid = threadIdx.x, quads = s.v_pad / 4, slices = 256 / quads;
+    const uint32_t tid = threadIdx.x, quads = s.v_pad / 4, slices = kStepThreads / quads;
     float *fs = lds, *qs = fs + s.d_pad, *vs = qs + s.d_pad, *part = vs + s.v_pad;  // part [slices][v_pad]
-    for (uint32_t d = tid; d < s.d_pad; d += 256) {
+    for (uint32_t d = tid; d < s.d_pad; d += kStepThreads) {
         fs[d] = d < s.dim ? a.f[head * s.dim + d] : 1.0f;
         qs[d] = d < s.dim ? a.q[head * s.dim + d] : 0.0f;
     }
-    for (uint32_t d = tid; d < s.v_pad; d += 256) vs[d] = d < s.vdim ? a.v[head * s.vdim + d] : 0.0f;
+    for (uint32_t d = tid; d < s.v_pad; d += kStepThreads) vs[d] = d < s.vdim ? a.v[head * s.vdim + d] : 0.0f;
     __syncthreads();
     const uint32_t c = tid % quads, sl = tid / quads;
     f32x4 o = {0.f, 0.f, 0.f, 0.f};
     if (sl < slices) {
-        float *st = a.state + size_t(head) * s.d_pad * s.v_pad + c * 4;
+        const size_t at = size_t(head) * s.d_pad * s.v_pad + c * 4;
+        const float *st = a.state_in + at;
+        float *st_out = a.state_out + at;
         const f32x4 v = *reinterpret_cast<const f32x4 *>(vs + c * 4);
         for (uint32_t d0 = sl; d0 < s.d_pad; d0 += slices * 8) {  // eight rows in flight
             f32x4 r[8];
@@ -597,7 +683,7 @@ __device__ __forceinline__ void recur_step(const RmiRecurShape &s, const RmiRecu
                     r[j][e] = __builtin_fmaf(f, r[j][e], k * v[e]);
                     o[e] = __builtin_fmaf(q, r[j][e], o[e]);
                 }
-                *reinterpret_cast<f32x4 *>(st + size_t(d) * s.v_pad) = r[j];
+                *reinterpret_cast<f32x4 *>(st_out + size_t(d) * s.v_pad) = r[j];
             }
         }
         *reinterpret_cast<f32x4 *>(part + sl * s.v_pad + c * 4) = o;
@@ -610,15 +696,18 @@ __device__ __forceinline__ void recur_step(const RmiRecurShape &s, const RmiRecu
     const float sq = wave_sum_f32(mine * mine);
     if ((tid & 63) == 0) red[tid >> 6] = sq;
     __syncthreads();
-    const float r = 1.0f / sqrtf(((red[0] + red[1]) + (red[2] + red[3])) / float(s.vdim) + s.eps);
+    float total = 0.0f;
+#pragma unroll
+    for (uint32_t i = 0; i < kStepThreads / 64; i++) total += red[i];
+    const float r = 1.0f / sqrtf(total / float(s.vdim) + s.eps);
     if (tid < s.vdim) static_cast<T *>(a.out)[size_t(head) * s.vdim + tid] = from_f32<T>(mine * r * a.norm[tid]);
 }
 inline size_t recur_step_lds(const RmiRecurShape &s) {
-    return (2 * size_t(s.d_pad) + s.v_pad + size_t(256 / (s.v_pad / 4)) * s.v_pad) * 4;
+    return (2 * size_t(s.d_pad) + s.v_pad + size_t(kStepThreads / (s.v_pad / 4)) * s.v_pad) * 4;
 }
 
 template <typename T, int BUCKET>
-__global__ __launch_bounds__(256) void mixers_step_kernel(RmiAttnShape s, RmiAttnArgs a, uint32_t attn_blocks, uint32_t parts,
+__global__ __launch_bounds__(kStepThreads) void mixers_step_kernel(RmiAttnShape s, RmiAttnArgs a, uint32_t attn_blocks, uint32_t parts,
                                                           uint32_t keys_per_part, RmiRecurShape rs, RmiRecurArgs ra) {
     extern __shared__ __attribute__((aligned(16))) uint8_t lds_raw[];
     __shared__ uint32_t flag;
@@ -635,8 +724,9 @@ __global__ __launch_bounds__(256) void mixers_step_kernel(RmiAttnShape s, RmiAtt
 // at once are as exact as those that never do.  The first kernel makes the factors (all chunks at once), the
 // second walks the chunks with the state in the matrix cores' accumulators.
 constexpr uint32_t kChunk = 16;
+constexpr uint32_t kMaxSegs = 8;
 struct RecurScratch {
-    float *qp, *kt, *am, *pc, *o;
+    float *qp, *kt, *am, *pc, *o, *seg_state, *seg_decay;
 };
 __host__ __device__ inline RecurScratch recur_scratch_at(float *p, const RmiRecurShape &s, uint32_t n_chunks) {
     const size_t hc = size_t(s.heads) * n_chunks;
@@ -646,6 +736,8 @@ __host__ __device__ inline RecurScratch recur_scratch_at(float *p, const RmiRecu
     r.am = r.kt + hc * kChunk * s.d_pad;    // [head][chunk][16 t][16 s]
     r.pc = r.am + hc * kChunk * kChunk;     // [head][chunk][d_pad]
     r.o = r.pc + hc * s.d_pad;              // [head][chunk][16][v_pad]
+    r.seg_state = r.o + hc * kChunk * s.v_pad;  // [segment][head][d_pad][v_pad]
+    r.seg_decay = r.seg_state + size_t(kMaxSegs) * s.heads * s.d_pad * s.v_pad;  // [segment][head][d_pad]
     return r;
 }
 
@@ -710,26 +802,38 @@ __global__ __launch_bounds__(256) void recur_factors_kernel(RmiRecurShape s, Rmi
     ws.am[hc * 256 + tid] = (red[tid] + red[256 + tid]) + (red[512 + tid] + red[768 + tid]);
 }
 
-// One workgroup: sixteen value channels of one head over all chunks; wave w holds the state's row tiles w, w + 4, ..
-// A tile of the state in accumulator form (row 4g + r in register r) is the right operand of (q P) S as it lies.
-template <int TPW>
-__global__ __launch_bounds__(256) void recur_scan_kernel(RmiRecurShape s, RmiRecurArgs a, uint32_t n_chunks) {
+// One workgroup: sixteen value channels of one head over the chunks of one segment of the pass; wave w holds the
+// state's row tiles w, w + 4, ..  A tile of the state in accumulator form (row 4g + r in register r) is the right
+// operand of (q P) S as it lies.  The segments of a long pass run side by side: a first launch (STATE_ONLY) takes every
+// segment but the last from a zero state and leaves what it adds and how much it keeps; the second puts its starting
+// state together from those before it.
+template <int TPW, bool STATE_ONLY>
+__global__ __launch_bounds__(256) void recur_scan_kernel(RmiRecurShape s, RmiRecurArgs a, uint32_t n_chunks, uint32_t seg_chunks) {
     __shared__ f32x4 part[2][4][64];
-    const uint32_t tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, fr = lane & 15, g = lane >> 4;
-    const uint32_t head = blockIdx.y, v0 = blockIdx.x * 16, n_tiles = s.d_pad / 16;
+    const uint32_t tid = threadIdx.x, lane = tid & 63, wave = uint32_t(__builtin_amdgcn_readfirstlane(int(tid >> 6))), fr = lane & 15, g = lane >> 4;
+    const uint32_t head = blockIdx.y, v0 = blockIdx.x * 16, seg = blockIdx.z, n_tiles = s.d_pad / 16;
+    const uint32_t c_begin = seg * seg_chunks, c_end = c_begin + seg_chunks < n_chunks ? c_begin + seg_chunks : n_chunks;
     const RecurScratch ws = recur_scratch_at(a.scratch, s, n_chunks);
-    f32x4 st[TPW];
-    float *state = a.state + size_t(head) * s.d_pad * s.v_pad + v0 + fr;
+    f32x4 st[TPW], kept[TPW];
+    const size_t at = size_t(head) * s.d_pad * s.v_pad + v0 + fr, head_state = size_t(s.d_pad) * s.v_pad;
 #pragma unroll
     for (int i = 0; i < TPW; i++) {
         const uint32_t tile = wave + 4 * i;
         st[i] = f32x4{0.f, 0.f, 0.f, 0.f};
-        if (tile < n_tiles && a.pos0)
+        kept[i] = f32x4{1.f, 1.f, 1.f, 1.f};
+        if (STATE_ONLY || tile >= n_tiles) continue;
+        if (a.pos0)
 #pragma unroll
-            for (int r = 0; r < 4; r++) st[i][r] = state[size_t(tile * 16 + g * 4 + r) * s.v_pad];
+            for (int r = 0; r < 4; r++) st[i][r] = a.state_in[at + size_t(tile * 16 + g * 4 + r) * s.v_pad];
+        for (uint32_t before = 0; before < seg; before++) {
+            const float *u = ws.seg_state + size_t(before) * s.heads * head_state + at;
+            const f32x4 keep = *reinterpret_cast<const f32x4 *>(ws.seg_decay + (size_t(before) * s.heads + head) * s.d_pad + tile * 16 + g * 4);
+#pragma unroll
+            for (int r = 0; r < 4; r++) st[i][r] = __builtin_fmaf(st[i][r], keep[r], u[size_t(tile * 16 + g * 4 + r) * s.v_pad]);
+        }
     }
     struct Operands {
-        f32x4 q[TPW], k[TPW], p[TPW];
+        f32x4 q[STATE_ONLY ? 1 : TPW], k[TPW], p[TPW];
         f32x4 v;  // v of tokens 4g .. 4g + 3 at this lane's channel
         f32x4 am;
     };
@@ -739,11 +843,11 @@ __global__ __launch_bounds__(256) void recur_scan_kernel(RmiRecurShape s, RmiRec
 #pragma unroll
         for (int i = 0; i < TPW; i++) {
             const uint32_t tile = wave + 4 * i < n_tiles ? wave + 4 * i : n_tiles - 1;
-            x.q[i] = *reinterpret_cast<const f32x4 *>(ws.qp + (hc * kChunk + fr) * s.d_pad + tile * 16 + g * 4);
+            if (!STATE_ONLY) x.q[STATE_ONLY ? 0 : i] = *reinterpret_cast<const f32x4 *>(ws.qp + (hc * kChunk + fr) * s.d_pad + tile * 16 + g * 4);
             x.k[i] = *reinterpret_cast<const f32x4 *>(ws.kt + (hc * s.d_pad + tile * 16 + fr) * kChunk + g * 4);
             x.p[i] = *reinterpret_cast<const f32x4 *>(ws.pc + hc * s.d_pad + tile * 16 + g * 4);
         }
-        x.am = *reinterpret_cast<const f32x4 *>(ws.am + hc * 256 + fr * 16 + g * 4);
+        if (!STATE_ONLY) x.am = *reinterpret_cast<const f32x4 *>(ws.am + hc * 256 + fr * 16 + g * 4);
 #pragma unroll
         for (int r = 0; r < 4; r++) {
             const uint32_t t = chunk * kChunk + g * 4 + r;
@@ -756,25 +860,26 @@ __global__ __launch_bounds__(256) void recur_scan_kernel(RmiRecurShape s, RmiRec
     constexpr uint32_t kAhead = TPW <= 2 ? 4 : 2;  // chunks whose operands are on their way
     Operands ring[kAhead];
 #pragma unroll
-    for (uint32_t j = 0; j < kAhead; j++) ring[j] = load(j < n_chunks ? j : n_chunks - 1);
-    for (uint32_t chunk0 = 0; chunk0 < n_chunks; chunk0 += kAhead) {
+    for (uint32_t j = 0; j < kAhead; j++) ring[j] = load(c_begin + j < c_end ? c_begin + j : c_end - 1);
+    for (uint32_t chunk0 = c_begin; chunk0 < c_end; chunk0 += kAhead) {
 #pragma unroll
         for (uint32_t j = 0; j < kAhead; j++) {
             const uint32_t chunk = chunk0 + j;
-            if (chunk >= n_chunks) break;
-            f32x4 o = {0.f, 0.f, 0.f, 0.f};
+            if (chunk >= c_end) break;
             const Operands &x = ring[j];
-            if (wave == 0) o = mma16_f32(x.am, x.v, o);
+            f32x4 o[2] = {{0.f, 0.f, 0.f, 0.f}, {0.f, 0.f, 0.f, 0.f}};  // two chains
+            if (!STATE_ONLY && wave == 3) o[0] = mma16_f32(x.am, x.v, o[0]);
 #pragma unroll
             for (int i = 0; i < TPW; i++) {
                 if (wave + 4 * i >= n_tiles) continue;
-                o = mma16_f32(x.q[i], st[i], o);
-#pragma unroll
-                for (int r = 0; r < 4; r++) st[i][r] *= x.p[i][r];
+                if (!STATE_ONLY) o[(i + 1) & 1] = mma16_f32(x.q[STATE_ONLY ? 0 : i], st[i], o[(i + 1) & 1]);
+                st[i] *= x.p[i];
+                if (STATE_ONLY) kept[i] *= x.p[i];
                 st[i] = mma16_f32(x.k[i], x.v, st[i]);
             }
-            ring[j] = load(chunk + kAhead < n_chunks ? chunk + kAhead : n_chunks - 1);
-            part[chunk & 1][wave][lane] = o;
+            ring[j] = load(chunk + kAhead < c_end ? chunk + kAhead : c_end - 1);
+            if (STATE_ONLY) continue;
+            part[chunk & 1][wave][lane] = o[0] + o[1];
             __syncthreads();  // (two buffers: the next chunk's writes cannot meet this one's reads)
             if (wave == (chunk & 3)) {
                 const f32x4 sum = (part[chunk & 1][0][lane] + part[chunk & 1][1][lane]) + (part[chunk & 1][2][lane] + part[chunk & 1][3][lane]);
@@ -784,12 +889,16 @@ __global__ __launch_bounds__(256) void recur_scan_kernel(RmiRecurShape s, RmiRec
             }
         }
     }
+    if (!STATE_ONLY && c_end != n_chunks) return;  // the last segment ends with the pass's state
+    float *out = STATE_ONLY ? ws.seg_state + size_t(seg) * s.heads * head_state + at : a.state_out + at;
 #pragma unroll
     for (int i = 0; i < TPW; i++) {
         const uint32_t tile = wave + 4 * i;
-        if (tile < n_tiles)
+        if (tile >= n_tiles) continue;
 #pragma unroll
-            for (int r = 0; r < 4; r++) state[size_t(tile * 16 + g * 4 + r) * s.v_pad] = st[i][r];
+        for (int r = 0; r < 4; r++) out[size_t(tile * 16 + g * 4 + r) * s.v_pad] = st[i][r];
+        if (STATE_ONLY && blockIdx.x == 0 && fr == 0)
+            *reinterpret_cast<f32x4 *>(ws.seg_decay + (size_t(seg) * s.heads + head) * s.d_pad + tile * 16 + g * 4) = kept[i];
     }
 }
 
@@ -824,7 +933,7 @@ void attn_parts(const RmiAttnShape &s, uint32_t n_tokens, uint32_t n_keys, uint3
     if (p > fill) p = fill;
     if (p > kMaxParts) p = kMaxParts;
     if (slots > kAttnCounters || p < 1) p = 1;
-    const uint32_t align = 4 * kKeyBlock;  // four waves of whole value blocks
+    const uint32_t align = 4 * kKeyBlock;  // each wave whole value blocks
     *keys_per_part = ((n_keys + p - 1) / p + align - 1) / align * align;
     *parts = (n_keys + *keys_per_part - 1) / *keys_per_part;
 }
@@ -840,8 +949,9 @@ uint32_t bucket_of(const RmiAttnShape &s) {
     const uint32_t d = s.dk_pad > s.dv_pad ? s.dk_pad : s.dv_pad;
     return d <= 64 ? 64 : d <= 128 ? 128 : 256;
 }
-size_t split_lds(uint32_t elem_bytes, const RmiAttnShape &s) {
-    const size_t q = size_t(16) * s.dk_pad * elem_bytes, merge = size_t(4) * attn_part_floats(s.dv_pad) * 4;
+size_t split_lds(uint32_t elem_bytes, const RmiAttnShape &s, uint32_t n_tokens) {
+    const uint32_t cols = n_tokens * (s.heads / s.kv_heads), live = cols < 16 ? cols : 16;
+    const size_t q = size_t(16) * s.dk_pad * elem_bytes, merge = size_t(4) * (32 + live * s.dv_pad) * 4;
     return q > merge ? q : merge;
 }
 
@@ -849,7 +959,7 @@ template <typename T>
 int attn_pass(const RmiAttnShape &s, const RmiAttnArgs &a, hipStream_t st) {
     const uint32_t n_heads = s.heads + 2 * s.kv_heads, group = s.heads / s.kv_heads, n_cols = a.n_tokens * group;
     const dim3 conv_grid(n_heads, (a.n_tokens + 4 * kConvRun - 1) / (4 * kConvRun));
-    if (s.taps <= 4 && s.dim % 2 == 0 && s.vdim % 2 == 0 && s.dim <= 128 && s.vdim <= 128)
+    if (conv_pairs_fit(s))
         hipLaunchKernelGGL(conv_rotate_pairs_kernel<T>, conv_grid, dim3(256), 0, st, s, a);
     else
         hipLaunchKernelGGL(conv_rotate_kernel<T>, conv_grid, dim3(256), 0, st, s, a);
@@ -858,16 +968,14 @@ int attn_pass(const RmiAttnShape &s, const RmiAttnArgs &a, hipStream_t st) {
         uint32_t parts, kpp;
         attn_parts(s, a.n_tokens, a.pos0 + a.n_tokens, &parts, &kpp);
         const dim3 grid(s.kv_heads * ((n_cols + 15) / 16) * parts);
-        const size_t lds = split_lds(sizeof(T), s);
-        if (bucket == 64)
-            hipLaunchKernelGGL((attn_split_kernel<T, 64>), grid, dim3(256), lds, st, s, a, parts, kpp);
-        else if (bucket == 128)
-            hipLaunchKernelGGL((attn_split_kernel<T, 128>), grid, dim3(256), lds, st, s, a, parts, kpp);
-        else {
-            const int rc = rmi_allow_lds(attn_split_kernel<T, 256>, lds);
-            if (rc != RMI_HIP_OK) return rc;
-            hipLaunchKernelGGL((attn_split_kernel<T, 256>), grid, dim3(256), lds, st, s, a, parts, kpp);
-        }
+        const size_t lds = split_lds(sizeof(T), s, a.n_tokens);
+        auto go = [&](auto kernel) {
+            const int rc = rmi_allow_lds(kernel, lds);
+            if (rc == RMI_HIP_OK) hipLaunchKernelGGL(kernel, grid, dim3(256), lds, st, s, a, parts, kpp);
+            return rc;
+        };
+        const int rc = bucket == 64 ? go(attn_split_kernel<T, 64>) : bucket == 128 ? go(attn_split_kernel<T, 128>) : go(attn_split_kernel<T, 256>);
+        if (rc != RMI_HIP_OK) return rc;
     } else {
         auto grid = [&](uint32_t qt) { return dim3((n_cols + 64 * qt - 1) / (64 * qt), s.kv_heads); };
         if (bucket == 64)
@@ -899,20 +1007,18 @@ int mixers_step(const RmiAttnShape *as, const RmiAttnArgs *aa, const RmiRecurSha
     if (as) {
         attn_parts(s, 1, a.pos0 + 1, &parts, &kpp);
         blocks = s.kv_heads * ((s.heads / s.kv_heads + 15) / 16) * parts;
-        lds = split_lds(sizeof(T), s);
+        lds = split_lds(sizeof(T), s, 1);
     }
     if (rs && recur_step_lds(r) > lds) lds = recur_step_lds(r);
     const dim3 grid(blocks + (rs ? r.heads : 0));
     const uint32_t bucket = as ? bucket_of(s) : 64;
-    if (bucket == 64)
-        hipLaunchKernelGGL((mixers_step_kernel<T, 64>), grid, dim3(256), lds, st, s, a, blocks, parts, kpp, r, b);
-    else if (bucket == 128)
-        hipLaunchKernelGGL((mixers_step_kernel<T, 128>), grid, dim3(256), lds, st, s, a, blocks, parts, kpp, r, b);
-    else {
-        const int rc = rmi_allow_lds(mixers_step_kernel<T, 256>, lds);
-        if (rc != RMI_HIP_OK) return rc;
-        hipLaunchKernelGGL((mixers_step_kernel<T, 256>), grid, dim3(256), lds, st, s, a, blocks, parts, kpp, r, b);
-    }
+    auto go = [&](auto kernel) {
+        const int rc = rmi_allow_lds(kernel, lds);
+        if (rc == RMI_HIP_OK) hipLaunchKernelGGL(kernel, grid, dim3(kStepThreads), lds, st, s, a, blocks, parts, kpp, r, b);
+        return rc;
+    };
+    const int rc = bucket == 64 ? go(mixers_step_kernel<T, 64>) : bucket == 128 ? go(mixers_step_kernel<T, 128>) : go(mixers_step_kernel<T, 256>);
+    if (rc != RMI_HIP_OK) return rc;
     RMI_HIP_CHECK(hipGetLastError());
     return RMI_HIP_OK;
 }
@@ -927,7 +1033,8 @@ size_t rmi_attn_scratch_bytes(const RmiAttnShape &s) {
 
 size_t rmi_recur_scratch_floats(const RmiRecurShape &s, uint32_t max_tokens) {
     const size_t hc = size_t(s.heads) * ((max_tokens + kChunk - 1) / kChunk);
-    return hc * (2 * size_t(kChunk) * s.d_pad + kChunk * kChunk + s.d_pad + size_t(kChunk) * s.v_pad);
+    return hc * (2 * size_t(kChunk) * s.d_pad + kChunk * kChunk + s.d_pad + size_t(kChunk) * s.v_pad) +
+           size_t(kMaxSegs) * s.heads * s.d_pad * (s.v_pad + 1);
 }
 
 int rmi_attn_pass(uint32_t elem_bytes, const RmiAttnShape &s, const RmiAttnArgs &a, hipStream_t st) {
@@ -944,13 +1051,24 @@ int rmi_recur_pass(uint32_t elem_bytes, const RmiRecurShape &s, const RmiRecurAr
     const uint32_t n_chunks = (a.n_tokens + kChunk - 1) / kChunk;
     const size_t lds = (2 * size_t(kChunk) * (s.d_pad + 4) + 1024) * 4;
     hipLaunchKernelGGL(recur_factors_kernel, dim3(n_chunks, s.heads), dim3(256), lds, st, s, a, n_chunks);
-    const dim3 grid(s.v_pad / 16, s.heads);
+    // segments of eight chunks or more, as many as still find an idle compute unit
+    const uint32_t columns = s.heads * (s.v_pad / 16);
+    uint32_t segs = (2 * uint32_t(rmi_device_cus()) + columns - 1) / columns;
+    if (segs > n_chunks / 8) segs = n_chunks / 8;
+    if (segs > kMaxSegs) segs = kMaxSegs;
+    if (segs < 1) segs = 1;
+    const uint32_t seg_chunks = (n_chunks + segs - 1) / segs;
+    segs = (n_chunks + seg_chunks - 1) / seg_chunks;
+    auto scan = [&](auto state_only, auto whole) {
+        if (segs > 1) hipLaunchKernelGGL(state_only, dim3(s.v_pad / 16, s.heads, segs - 1), dim3(256), 0, st, s, a, n_chunks, seg_chunks);
+        hipLaunchKernelGGL(whole, dim3(s.v_pad / 16, s.heads, segs), dim3(256), 0, st, s, a, n_chunks, seg_chunks);
+    };
     if (s.d_pad <= 64)
-        hipLaunchKernelGGL(recur_scan_kernel<1>, grid, dim3(256), 0, st, s, a, n_chunks);
+        scan(recur_scan_kernel<1, true>, recur_scan_kernel<1, false>);
     else if (s.d_pad <= 128)
-        hipLaunchKernelGGL(recur_scan_kernel<2>, grid, dim3(256), 0, st, s, a, n_chunks);
+        scan(recur_scan_kernel<2, true>, recur_scan_kernel<2, false>);
     else
-        hipLaunchKernelGGL(recur_scan_kernel<4>, grid, dim3(256), 0, st, s, a, n_chunks);
+        scan(recur_scan_kernel<4, true>, recur_scan_kernel<4, false>);
     const dim3 ngrid((a.n_tokens + 3) / 4, s.heads);
     if (elem_bytes == 2)
         hipLaunchKernelGGL(recur_norm_kernel<rmi_bf16>, ngrid, dim3(256), 0, st, s, a, n_chunks);

@@ -41,13 +41,13 @@ struct RuvenexLayer {
 template <typename T>
 struct EmbedDense {
     const T *table;
-    uint32_t k_pad, vocab;
+    uint32_t ld, vocab;
     float scale;
     float *x;
     uint32_t n;
     __device__ __forceinline__ void operator()(uint32_t token) const {
         if (token >= vocab) token = vocab - 1;
-        for (uint32_t i = threadIdx.x; i < n; i += 256) x[i] = to_f32(table[size_t(token) * k_pad + i]) * scale;
+        for (uint32_t i = threadIdx.x; i < n; i += 256) x[i] = to_f32(table[size_t(token) * ld + i]) * scale;
     }
 };
 
@@ -111,7 +111,7 @@ int rmi_hip_ruvenex::enqueue_layers(uint32_t step0, uint32_t n, hipStream_t st, 
         a.v_cache = y.v_cache;
         a.gate = gate;
         a.out = act;
-        a.out_ld = y.w_out.k_pad;
+        a.out_ld = y.w_out.ld;
         a.pos0 = step0;
         a.n_tokens = n;
         a.scratch = attn_scratch;
@@ -123,7 +123,7 @@ int rmi_hip_ruvenex::enqueue_layers(uint32_t step0, uint32_t n, hipStream_t st, 
         r.state_out = y.state[now ^ 1];
         r.norm = y.recur_norm;
         r.out = static_cast<uint8_t *>(act) + size_t(y.k_attn) * elem;
-        r.out_ld = y.w_out.k_pad;
+        r.out_ld = y.w_out.ld;
         r.pos0 = step0;
         r.n_tokens = n;
         r.scratch = recur_scratch;
@@ -168,9 +168,9 @@ int rmi_hip_ruvenex::enqueue_sample(uint32_t step0, const uint32_t *rows, uint32
                            step_top2, nonfinite, embed_next);
     };
     if (elem == 2)
-        finish(EmbedDense<rmi_bf16>{static_cast<const rmi_bf16 *>(embed.data), embed.k_pad, vocab, embed_scale, x, width});
+        finish(EmbedDense<rmi_bf16>{static_cast<const rmi_bf16 *>(embed.data), embed.ld, vocab, embed_scale, x, width});
     else
-        finish(EmbedDense<float>{static_cast<const float *>(embed.data), embed.k_pad, vocab, embed_scale, x, width});
+        finish(EmbedDense<float>{static_cast<const float *>(embed.data), embed.ld, vocab, embed_scale, x, width});
     RMI_HIP_CHECK(hipGetLastError());
     return RMI_HIP_OK;
 }
@@ -314,14 +314,15 @@ void f32_to_bf16_host(const RmiTensor &t, uint64_t at, uint64_t n, uint16_t *dst
 
 // A dense weight put together on the host from blocks of tensors, then uploaded.
 struct DenseBuilder {
-    uint32_t elem, n_rows, k_pad;
+    uint32_t elem, n_rows, k_pad, ld;
     std::vector<uint8_t> bytes;
-    DenseBuilder(uint32_t e, uint32_t rows, uint32_t k) : elem(e), n_rows(rows), k_pad(k), bytes(size_t(rows) * k * e, 0) {}
+    DenseBuilder(uint32_t e, uint32_t rows, uint32_t k)
+        : elem(e), n_rows(rows), k_pad(k), ld(rmi_dense_ld(k, e)), bytes(size_t(rows) * ld * e, 0) {}
     void put(const RmiTensor *t, uint32_t row0, uint32_t col0) {
         if (!t) return;
         const uint64_t rows = t->shape[0], cols = t->shape[1];
         for (uint64_t r = 0; r < rows; r++) {
-            uint8_t *dst = bytes.data() + (size_t(row0 + r) * k_pad + col0) * elem;
+            uint8_t *dst = bytes.data() + (size_t(row0 + r) * ld + col0) * elem;
             if (elem == 2)
                 f32_to_bf16_host(*t, r * cols, cols, reinterpret_cast<uint16_t *>(dst));
             else
@@ -335,6 +336,7 @@ struct DenseBuilder {
         out->data = s->alloc_bytes(bytes.size(), false);
         out->n_rows = n_rows;
         out->k_pad = k_pad;
+        out->ld = ld;
         if (!out->data) return false;
         if (hipMemcpy(out->data, bytes.data(), bytes.size(), hipMemcpyHostToDevice) != hipSuccess) {
             rmi_set_error("weight upload failed");
@@ -395,7 +397,7 @@ bool rmi_hip_ruvenex::load(const RmiModelFolder &folder, uint32_t elem_bytes, ui
     };
     std::vector<Sizes> sizes(n_layer);
     layers.resize(n_layer);
-    uint32_t max_channels = 1, max_heads = 1, max_rq = 1, max_rv = 1, max_k = kDenseKAlign;
+    uint32_t max_channels = 1, max_heads = 1, max_rq = 1, max_rv = 1, max_ld = kDenseKAlign;
     size_t max_q = 1, max_attn_scratch = 0, max_recur_scratch = 1;
     for (uint32_t l = 0; l < n_layer; l++) {
         const RmiJson *e = &ls->items[l], *type = e->get("type");
@@ -455,7 +457,7 @@ bool rmi_hip_ruvenex::load(const RmiModelFolder &folder, uint32_t elem_bytes, ui
         grow(max_heads, a.heads);
         grow(max_rq, z.n_recur);
         grow(max_rv, z.n_recur_v);
-        grow(max_k, y.w_out.k_pad);
+        grow(max_ld, rmi_dense_ld(y.w_out.k_pad, elem));
         grow(max_q, size_t(pass_rows) * a.heads * a.dk_pad * elem);
         grow(max_attn_scratch, rmi_attn_scratch_bytes(a));
         grow(max_recur_scratch, rmi_recur_scratch_floats(r, pass_rows));
@@ -465,7 +467,7 @@ bool rmi_hip_ruvenex::load(const RmiModelFolder &folder, uint32_t elem_bytes, ui
     if (!alloc_sampling() || !(x = alloc<float>(rows * width, true)) || !(u = alloc<float>(rows * max_channels, true)) ||
         !(gate = alloc<float>(rows * max_heads, true)) || !(rq = alloc<float>(rows * max_rq, true)) || !(rf = alloc<float>(rows * max_rq, true)) ||
         !(rv = alloc<float>(rows * max_rv, true)) || !(rg1 = alloc<float>(rows * width, true)) || !(rg2 = alloc<float>(rows * width, true)) ||
-        !(h = alloc_bytes(rows * k_in * elem, true)) || !(act = alloc_bytes(rows * max_k * elem, true)) || !(q = alloc_bytes(max_q, true)) ||
+        !(h = alloc_bytes(rows * rmi_dense_ld(k_in, elem) * elem, true)) || !(act = alloc_bytes(rows * max_ld * elem, true)) || !(q = alloc_bytes(max_q, true)) ||
         !(logits = alloc<float>(size_t(logit_rows) * vocab, true)) || !(attn_scratch = alloc_bytes(max_attn_scratch + 16, true)) ||
         !(recur_scratch = alloc<float>(max_recur_scratch, true)) || !(want_rows = alloc<uint32_t>(kLogitRows, true)) ||
         !(partial = alloc_bytes(size_t(logit_rows) * kArgmaxGroups * kTopBytes, false)))
@@ -504,7 +506,7 @@ bool rmi_hip_ruvenex::load(const RmiModelFolder &folder, uint32_t elem_bytes, ui
         };
         if (z.ff) {
             parts.push_back({p + "rg2", width, width, rg2, kActSigmoid, 0, b2, nullptr});
-            parts.push_back({p + "mlp.up", z.ff, y.w_out.k_pad, static_cast<uint8_t *>(act) + size_t(y.k_recur) * elem, kActGeluTanh, 1, nullptr, nullptr});
+            parts.push_back({p + "mlp.up", z.ff, rmi_dense_ld(y.w_out.k_pad, elem), static_cast<uint8_t *>(act) + size_t(y.k_recur) * elem, kActGeluTanh, 1, nullptr, nullptr});
         }
         uint32_t n_rows = 0;
         for (const Part &q1 : parts) {

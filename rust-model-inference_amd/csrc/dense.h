@@ -1,7 +1,7 @@
 // Dense (bf16 or f32) weights and the products on them: the launch interface that decoder sessions use.
 //
 // A weight is row-major, rows of k_pad elements (the sum of its column segments, each padded with zeros to
-// kDenseKAlign elements), its row segments each padded with zero rows to kDenseRowAlign.  Both element types share
+// kDenseKAlign elements) that lie rmi_dense_ld apart, as do those of an activation; its row segments each padded with zero rows to kDenseRowAlign.  Both element types share
 // every kernel: the code works on 16-byte pieces.  Accumulation is f32; the residual stream and everything a product
 // writes is f32 unless its segment says otherwise.
 #pragma once
@@ -13,6 +13,12 @@ typedef uint16_t rmi_bf16;  // bits
 constexpr uint32_t kDenseKAlign = 64;
 constexpr uint32_t kDenseRowAlign = 16;
 inline uint32_t rmi_dense_pad(uint32_t n, uint32_t to) { return (n + to - 1) / to * to; }
+
+// Elements from row to row: an odd multiple of 128 bytes.  Rows a multiple of 256 bytes apart would put the same
+// columns of many rows into few of the L2's channels, and a tile reads just that.
+inline uint32_t rmi_dense_ld(uint32_t k_pad, uint32_t elem_bytes) {
+    return k_pad + (size_t(k_pad) * elem_bytes % 256 == 0 ? 128 / elem_bytes : 0);
+}
 
 enum RmiAct : uint32_t { kActNone, kActSigmoid, kActSilu, kActGeluTanh, kActForgetGate };
 
@@ -53,6 +59,7 @@ struct RmiDense {
     void *data = nullptr;
     uint32_t n_rows = 0;  // padded
     uint32_t k_pad = 0;
+    uint32_t ld = 0;  // rmi_dense_ld(k_pad)
 };
 
 // More than 64 KiB of dynamic LDS has to be asked for (a compute unit has 160 KiB; some is left for static arrays).
@@ -65,13 +72,13 @@ int rmi_allow_lds(K kernel, size_t bytes) {
 }
 
 // elem_bytes 2: bf16, 4: f32
-// h[i][0 .. k_pad) = rms_norm(x[rows ? rows[i] : i]) * weight, zeros past n
+// h[i][0 .. k_pad) (rows rmi_dense_ld apart) = rms_norm(x[rows ? rows[i] : i]) * weight, zeros past n
 int rmi_dense_norm(uint32_t elem_bytes, const float *x, const uint32_t *rows, const float *weight, float eps, void *h,
                    uint32_t n_tokens, uint32_t n, uint32_t k_pad, hipStream_t st);
-// x[i] = table[tok[i]] * scale (table: rows of k_pad elements)
+// x[i] = table[tok[i]] * scale (table: a dense weight)
 int rmi_dense_embed(uint32_t elem_bytes, const RmiDense &table, const uint32_t *tok, uint32_t vocab, float scale, float *x,
                     uint32_t n_tokens, uint32_t n, hipStream_t st);
-// several tokens: matrix cores; a = [n_tokens][k_pad]
+// several tokens: matrix cores; a = [n_tokens] rows of k_pad elements, rmi_dense_ld apart
 int rmi_dense_gemm(uint32_t elem_bytes, const RmiDense &w, const void *a, const RmiRowSegs &segs, uint32_t n_tokens, hipStream_t st);
 int rmi_dense_gemm_residual(uint32_t elem_bytes, const RmiDense &w, const void *a, const RmiColSegs &segs, float *x, uint32_t width,
                             uint32_t n_tokens, hipStream_t st);

@@ -8,11 +8,11 @@ namespace {
 template <typename T>
 __global__ __launch_bounds__(256) void norm_kernel(const float *__restrict__ x, const uint32_t *__restrict__ rows,
                                                    const float *__restrict__ weight, float eps, T *__restrict__ h, uint32_t n,
-                                                   uint32_t k_pad) {
+                                                   uint32_t k_pad, uint32_t ld) {
     __shared__ float red[4];
     const uint32_t tid = threadIdx.x;
     x += size_t(rows ? rows[blockIdx.x] : blockIdx.x) * n;
-    h += size_t(blockIdx.x) * k_pad;
+    h += size_t(blockIdx.x) * ld;
     float sq = 0.0f;
     for (uint32_t i = tid; i < n; i += 256) sq = __builtin_fmaf(x[i], x[i], sq);
     sq = wave_sum_f32(sq);
@@ -23,11 +23,11 @@ __global__ __launch_bounds__(256) void norm_kernel(const float *__restrict__ x, 
 }
 
 template <typename T>
-__global__ __launch_bounds__(256) void embed_kernel(const T *__restrict__ table, uint32_t k_pad, const uint32_t *__restrict__ tok,
+__global__ __launch_bounds__(256) void embed_kernel(const T *__restrict__ table, uint32_t ld, const uint32_t *__restrict__ tok,
                                                     uint32_t vocab, float scale, float *__restrict__ x, uint32_t n) {
     uint32_t t = tok[blockIdx.x];
     if (t >= vocab) t = vocab - 1;  // ids are validated on the host; never read outside the table
-    for (uint32_t i = threadIdx.x; i < n; i += 256) x[size_t(blockIdx.x) * n + i] = to_f32(table[size_t(t) * k_pad + i]) * scale;
+    for (uint32_t i = threadIdx.x; i < n; i += 256) x[size_t(blockIdx.x) * n + i] = to_f32(table[size_t(t) * ld + i]) * scale;
 }
 
 // which row segment a row lies in: the starts sit side by side (unused ones at the end of the range)
@@ -40,25 +40,26 @@ __device__ __forceinline__ uint32_t seg_of(const RmiRowSegs &rs, uint32_t row) {
 
 // ------------------------------------------------------------------ GEMM
 // One workgroup of four waves: BN weight rows x BT tokens, k in steps of 128 bytes a row through two LDS buffers; the
-// pieces of the next PD steps are on their way to registers while one is multiplied.  A row of a buffer is eight
+// pieces of the next PD steps are on their way to registers while one is multiplied.  The largest tile keeps one LDS
+// buffer (NB = 1), so that three workgroups share a compute unit.  A row of a buffer is eight
 // 16-byte pieces, piece p at slot p ^ (row & 7), so that the sixteen rows of a fragment spread over the banks.
 // Weights are the A operand: a lane ends with four consecutive rows of one token.
 constexpr uint32_t kStepBytes = 128;
 
-template <typename T, int BN, int BT, int WN, int WT, int PD, bool RESIDUAL>
-__global__ __launch_bounds__(256) void dense_gemm_kernel(const T *__restrict__ w, const T *__restrict__ a, uint32_t n_rows,
-                                                         uint32_t k_pad, uint32_t n_tokens, uint32_t grid_n, uint32_t grid_t,
+template <typename T, int BN, int BT, int WN, int WT, int PD, int NB, int WPS, bool RESIDUAL>
+__global__ __launch_bounds__(256, WPS) void dense_gemm_kernel(const T *__restrict__ w, const T *__restrict__ a, uint32_t n_rows,
+                                                              uint32_t k_pad, uint32_t ld, uint32_t n_tokens, uint32_t grid_n, uint32_t grid_t, uint32_t xcd_split,
                                                          RmiRowSegs rs, RmiColSegs cs, float *__restrict__ x, uint32_t width) {
     static_assert((BN / WN) * (BT / WT) == 4, "four waves");
     constexpr int NN = WN / 16, NT = WT / 16;
     constexpr int PW = BN * 8 / 256, PA = (BT * 8 + 255) / 256;  // pieces a thread loads per step
-    __shared__ u32x4 lds[2][(BN + BT) * 8];
+    __shared__ u32x4 lds[NB][(BN + BT) * 8];
     const uint32_t tid = threadIdx.x, lane = tid & 63, wave = uint32_t(__builtin_amdgcn_readfirstlane(int(tid >> 6)));
     uint32_t n_tile, t_tile;
-    rmi_gemm_tile_of(blockIdx.x, grid_n, grid_t, 1u, 0u, n_tile, t_tile);
+    rmi_gemm_tile_of(blockIdx.x, grid_n, grid_t, 1u, xcd_split, n_tile, t_tile);
     const uint32_t row0 = n_tile * BN, tok0 = t_tile * BT;
     const uint32_t wn = (wave % (BN / WN)) * WN, wt = (wave / (BN / WN)) * WT;
-    const size_t stride = size_t(k_pad) * sizeof(T);
+    const size_t stride = size_t(ld) * sizeof(T);
 
     const uint8_t *wsrc[PW], *asrc[PA];
     uint32_t wdst[PW], adst[PA];
@@ -135,7 +136,7 @@ __global__ __launch_bounds__(256) void dense_gemm_kernel(const T *__restrict__ w
     for (uint32_t step0 = 0; step0 < n_steps; step0 += PD) {
 #pragma unroll
         for (int j = 0; j < PD; j++) {  // register slots by compile-time index
-            const uint32_t step = step0 + j, buf = step & 1;
+            const uint32_t step = step0 + j, buf = step & (NB - 1);
             if (step >= n_steps) break;
 #pragma unroll
             for (int c = 0; c < 2; c++) {
@@ -156,7 +157,8 @@ __global__ __launch_bounds__(256) void dense_gemm_kernel(const T *__restrict__ w
                     for (int i2 = 0; i2 < NT; i2++) acc[i][i2] = mma16<T>(fw[i], fa[i2], acc[i][i2]);
             }
             if (step + 1 < n_steps) {
-                park((j + 1) % PD, buf ^ 1);
+                if (NB == 1) __syncthreads();
+                park((j + 1) % PD, buf ^ (NB - 1));
                 load((j + 1) % PD, step + 1 + PD);
             }
             if (RESIDUAL && (step + 1) * kStepElems == cs.s[seg].k_end) {
@@ -214,19 +216,20 @@ int launch_gemm(const RmiDense &w, const void *a, const RmiRowSegs &rs, const Rm
     const uint32_t n_rows = RESIDUAL ? width : w.n_rows;
     auto go = [&](auto kernel, uint32_t bn, uint32_t bt) {
         const uint32_t gn = (n_rows + bn - 1) / bn, gt = (n_tokens + bt - 1) / bt;
+        const uint32_t split = rmi_gemm_xcd_split(gn, gt, double(n_rows) * w.k_pad, double(n_tokens) * w.k_pad);
         hipLaunchKernelGGL(kernel, dim3(gn * gt), dim3(256), 0, st, static_cast<const T *>(w.data), static_cast<const T *>(a), n_rows,
-                           w.k_pad, n_tokens, gn, gt, rs, cs, x, width);
+                           w.k_pad, w.ld, n_tokens, gn, gt, split, rs, cs, x, width);
     };
     const uint64_t cus = uint64_t(rmi_device_cus());
     auto tiles = [&](uint32_t bn, uint32_t bt) { return uint64_t((n_rows + bn - 1) / bn) * ((n_tokens + bt - 1) / bt); };
     if (n_tokens <= 16)
-        go(dense_gemm_kernel<T, 64, 16, 16, 16, 4, RESIDUAL>, 64, 16);
+        go(dense_gemm_kernel<T, 64, 16, 16, 16, 4, 2, 4, RESIDUAL>, 64, 16);
     else if (tiles(128, 128) >= cus)
-        go(dense_gemm_kernel<T, 128, 128, 64, 64, 3, RESIDUAL>, 128, 128);
+        go(dense_gemm_kernel<T, 128, 128, 64, 64, 1, 1, 3, RESIDUAL>, 128, 128);
     else if (tiles(64, 64) >= cus)
-        go(dense_gemm_kernel<T, 64, 64, 32, 32, 4, RESIDUAL>, 64, 64);
+        go(dense_gemm_kernel<T, 64, 64, 32, 32, 4, 2, 4, RESIDUAL>, 64, 64);
     else
-        go(dense_gemm_kernel<T, 64, 32, 32, 16, 4, RESIDUAL>, 64, 32);
+        go(dense_gemm_kernel<T, 64, 32, 32, 16, 4, 2, 4, RESIDUAL>, 64, 32);
     RMI_HIP_CHECK(hipGetLastError());
     return RMI_HIP_OK;
 }
@@ -245,7 +248,7 @@ __host__ __device__ inline uint32_t gemv_lds_pieces(uint32_t k_pad) {
 // A wave takes ROWS weight rows, its lanes the pieces of a row, two rounds of 64 in flight; R: quads of x a thread
 // keeps (n <= 1024 R).
 template <typename T, int ROWS, int R>
-__global__ __launch_bounds__(256) void norm_gemv_kernel(const T *__restrict__ w, uint32_t k_pad, const float *__restrict__ x,
+__global__ __launch_bounds__(256) void norm_gemv_kernel(const T *__restrict__ w, uint32_t k_pad, uint32_t ld, const float *__restrict__ x,
                                                         const float *__restrict__ weight, float eps, uint32_t n, RmiRowSegs rs) {
     extern __shared__ u32x4 act[];
     __shared__ float red[4];
@@ -274,7 +277,7 @@ __global__ __launch_bounds__(256) void norm_gemv_kernel(const T *__restrict__ w,
 #pragma unroll
     for (int r = 0; r < ROWS; r++) {
         const uint32_t row = row0 + r < rs.n_rows ? row0 + r : rs.n_rows - 1;
-        src[r] = reinterpret_cast<const u32x4 *>(w + size_t(row) * k_pad);
+        src[r] = reinterpret_cast<const u32x4 *>(w + size_t(row) * ld);
     }
     u32x4 cur[2][ROWS];
     auto load = [&](uint32_t p0) {
@@ -343,7 +346,7 @@ __global__ __launch_bounds__(256) void norm_gemv_kernel(const T *__restrict__ w,
 // A workgroup takes ROWS rows, each wave a quarter of their columns, so that a long row is in flight at once; the
 // waves' sums meet in LDS.  A lane's products count with the gate and scale of the column segment its piece lies in.
 template <typename T, int ROWS>
-__global__ __launch_bounds__(256) void gemv_residual_kernel(const T *__restrict__ w, uint32_t k_pad, const T *__restrict__ a,
+__global__ __launch_bounds__(256) void gemv_residual_kernel(const T *__restrict__ w, uint32_t k_pad, uint32_t ld, const T *__restrict__ a,
                                                             RmiColSegs cs, float *__restrict__ x, uint32_t width) {
     constexpr int U = 4;
     __shared__ float part[4][ROWS];
@@ -356,7 +359,7 @@ __global__ __launch_bounds__(256) void gemv_residual_kernel(const T *__restrict_
 #pragma unroll
     for (int r = 0; r < ROWS; r++) {
         const uint32_t row = row0 + r < width ? row0 + r : width - 1;
-        src[r] = reinterpret_cast<const u32x4 *>(w + size_t(row) * k_pad);
+        src[r] = reinterpret_cast<const u32x4 *>(w + size_t(row) * ld);
 #pragma unroll
         for (uint32_t i = 0; i < kMaxColSegs; i++) gate[r][i] = i < cs.n_segs ? (cs.s[i].gate ? cs.s[i].gate[row] : 1.0f) * cs.s[i].scale : 0.0f;
     }
@@ -415,7 +418,7 @@ int norm_gemv_r(const RmiDense &w, const float *x, const float *weight, float ep
     const int rc = rmi_allow_lds(norm_gemv_kernel<T, kRows, R>, lds);
     if (rc != RMI_HIP_OK) return rc;
     hipLaunchKernelGGL((norm_gemv_kernel<T, kRows, R>), dim3((w.n_rows + 4 * kRows - 1) / (4 * kRows)), dim3(256), lds, st,
-                       static_cast<const T *>(w.data), w.k_pad, x, weight, eps, n, segs);
+                       static_cast<const T *>(w.data), w.k_pad, w.ld, x, weight, eps, n, segs);
     RMI_HIP_CHECK(hipGetLastError());
     return RMI_HIP_OK;
 }
@@ -431,7 +434,7 @@ template <typename T>
 int gemv_residual(const RmiDense &w, const void *a, const RmiColSegs &segs, float *x, uint32_t width, hipStream_t st) {
     constexpr int kRows = 2;
     hipLaunchKernelGGL((gemv_residual_kernel<T, kRows>), dim3((width + kRows - 1) / kRows), dim3(256), 0, st,
-                       static_cast<const T *>(w.data), w.k_pad, static_cast<const T *>(a), segs, x, width);
+                       static_cast<const T *>(w.data), w.k_pad, w.ld, static_cast<const T *>(a), segs, x, width);
     RMI_HIP_CHECK(hipGetLastError());
     return RMI_HIP_OK;
 }
@@ -442,9 +445,9 @@ int rmi_dense_norm(uint32_t elem_bytes, const float *x, const uint32_t *rows, co
                    uint32_t n_tokens, uint32_t n, uint32_t k_pad, hipStream_t st) {
     if (n_tokens == 0) return RMI_HIP_OK;
     if (elem_bytes == 2)
-        hipLaunchKernelGGL(norm_kernel<rmi_bf16>, dim3(n_tokens), dim3(256), 0, st, x, rows, weight, eps, static_cast<rmi_bf16 *>(h), n, k_pad);
+        hipLaunchKernelGGL(norm_kernel<rmi_bf16>, dim3(n_tokens), dim3(256), 0, st, x, rows, weight, eps, static_cast<rmi_bf16 *>(h), n, k_pad, rmi_dense_ld(k_pad, 2));
     else
-        hipLaunchKernelGGL(norm_kernel<float>, dim3(n_tokens), dim3(256), 0, st, x, rows, weight, eps, static_cast<float *>(h), n, k_pad);
+        hipLaunchKernelGGL(norm_kernel<float>, dim3(n_tokens), dim3(256), 0, st, x, rows, weight, eps, static_cast<float *>(h), n, k_pad, rmi_dense_ld(k_pad, 4));
     RMI_HIP_CHECK(hipGetLastError());
     return RMI_HIP_OK;
 }
@@ -453,10 +456,10 @@ int rmi_dense_embed(uint32_t elem_bytes, const RmiDense &table, const uint32_t *
                     uint32_t n_tokens, uint32_t n, hipStream_t st) {
     if (n_tokens == 0) return RMI_HIP_OK;
     if (elem_bytes == 2)
-        hipLaunchKernelGGL(embed_kernel<rmi_bf16>, dim3(n_tokens), dim3(256), 0, st, static_cast<const rmi_bf16 *>(table.data), table.k_pad,
+        hipLaunchKernelGGL(embed_kernel<rmi_bf16>, dim3(n_tokens), dim3(256), 0, st, static_cast<const rmi_bf16 *>(table.data), table.ld,
                            tok, vocab, scale, x, n);
     else
-        hipLaunchKernelGGL(embed_kernel<float>, dim3(n_tokens), dim3(256), 0, st, static_cast<const float *>(table.data), table.k_pad, tok,
+        hipLaunchKernelGGL(embed_kernel<float>, dim3(n_tokens), dim3(256), 0, st, static_cast<const float *>(table.data), table.ld, tok,
                            vocab, scale, x, n);
     RMI_HIP_CHECK(hipGetLastError());
     return RMI_HIP_OK;
@@ -464,14 +467,14 @@ int rmi_dense_embed(uint32_t elem_bytes, const RmiDense &table, const uint32_t *
 
 int rmi_dense_gemm(uint32_t elem_bytes, const RmiDense &w, const void *a, const RmiRowSegs &segs, uint32_t n_tokens, hipStream_t st) {
     if (n_tokens == 0 || w.n_rows == 0) return RMI_HIP_OK;
-    if (segs.n_rows != w.n_rows || segs.n_segs == 0 || segs.n_segs > kMaxRowSegs || w.k_pad % kDenseKAlign)
+    if (segs.n_rows != w.n_rows || segs.n_segs == 0 || segs.n_segs > kMaxRowSegs || w.k_pad % kDenseKAlign || w.ld != rmi_dense_ld(w.k_pad, elem_bytes))
         return rmi_fail(RMI_HIP_E_INVALID, "row segments do not fit the weight");
     return elem_bytes == 2 ? launch_gemm<rmi_bf16, false>(w, a, segs, RmiColSegs{}, nullptr, 0, n_tokens, st)
                            : launch_gemm<float, false>(w, a, segs, RmiColSegs{}, nullptr, 0, n_tokens, st);
 }
 
-static int check_col_segs(const RmiDense &w, const RmiColSegs &segs, uint32_t width) {
-    if (segs.n_segs == 0 || segs.n_segs > kMaxColSegs || segs.s[segs.n_segs - 1].k_end != w.k_pad || w.n_rows < width)
+static int check_col_segs(uint32_t elem_bytes, const RmiDense &w, const RmiColSegs &segs, uint32_t width) {
+    if (w.ld != rmi_dense_ld(w.k_pad, elem_bytes) || segs.n_segs == 0 || segs.n_segs > kMaxColSegs || segs.s[segs.n_segs - 1].k_end != w.k_pad || w.n_rows < width)
         return rmi_fail(RMI_HIP_E_INVALID, "column segments do not fit the weight");
     for (uint32_t i = 0; i < segs.n_segs; i++)
         if (segs.s[i].k_end % kDenseKAlign || segs.s[i].k_end <= (i ? segs.s[i - 1].k_end : 0u))
@@ -482,7 +485,7 @@ static int check_col_segs(const RmiDense &w, const RmiColSegs &segs, uint32_t wi
 int rmi_dense_gemm_residual(uint32_t elem_bytes, const RmiDense &w, const void *a, const RmiColSegs &segs, float *x, uint32_t width,
                             uint32_t n_tokens, hipStream_t st) {
     if (n_tokens == 0) return RMI_HIP_OK;
-    const int rc = check_col_segs(w, segs, width);
+    const int rc = check_col_segs(elem_bytes, w, segs, width);
     if (rc != RMI_HIP_OK) return rc;
     return elem_bytes == 2 ? launch_gemm<rmi_bf16, true>(w, a, RmiRowSegs{}, segs, x, width, n_tokens, st)
                            : launch_gemm<float, true>(w, a, RmiRowSegs{}, segs, x, width, n_tokens, st);
@@ -502,7 +505,7 @@ int rmi_dense_norm_gemv(uint32_t elem_bytes, const RmiDense &w, const float *x, 
 
 int rmi_dense_gemv_residual(uint32_t elem_bytes, const RmiDense &w, const void *a, const RmiColSegs &segs, float *x, uint32_t width,
                             hipStream_t st) {
-    const int rc = check_col_segs(w, segs, width);
+    const int rc = check_col_segs(elem_bytes, w, segs, width);
     if (rc != RMI_HIP_OK) return rc;
     return elem_bytes == 2 ? gemv_residual<rmi_bf16>(w, a, segs, x, width, st) : gemv_residual<float>(w, a, segs, x, width, st);
 }

@@ -10,7 +10,7 @@
 
 typedef uint16_t rmi_bf16;  // bits
 
-constexpr uint32_t kDenseKAlign = 64;
+constexpr uint32_t kDenseKAlign = 256;
 constexpr uint32_t kDenseRowAlign = 16;
 inline uint32_t rmi_dense_pad(uint32_t n, uint32_t to) { return (n + to - 1) / to * to; }
 

@@ -51,6 +51,7 @@ __global__ __launch_bounds__(256, WPS) void dense_gemm_kernel(const T *__restric
                                                               uint32_t k_pad, uint32_t ld, uint32_t n_tokens, uint32_t grid_n, uint32_t grid_t, uint32_t xcd_split,
                                                          RmiRowSegs rs, RmiColSegs cs, float *__restrict__ x, uint32_t width) {
     static_assert((BN / WN) * (BT / WT) == 4, "four waves");
+    static_assert(kDenseKAlign * sizeof(T) % (kStepBytes * PD) == 0, "whole rounds of the register slots");
     constexpr int NN = WN / 16, NT = WT / 16;
     constexpr int PW = BN * 8 / 256, PA = (BT * 8 + 255) / 256;  // pieces a thread loads per step
     __shared__ u32x4 lds[NB][(BN + BT) * 8];
@@ -86,7 +87,9 @@ __global__ __launch_bounds__(256, WPS) void dense_gemm_kernel(const T *__restric
     const uint32_t n_steps = k_pad / kStepElems;
     u32x4 rw[PD][PW], ra[PD][PA];
     auto load = [&](int slot, uint32_t step) {
-        if (step >= n_steps) return;
+        // always issued (past the end the last step again): the waits count loads, and a skipped one would make every
+        // wait a wait for all
+        step = step < n_steps ? step : n_steps - 1;
 #pragma unroll
         for (int i = 0; i < PW; i++) rw[slot][i] = *reinterpret_cast<const u32x4 *>(wsrc[i] + size_t(step) * kStepBytes);
 #pragma unroll
@@ -127,46 +130,48 @@ __global__ __launch_bounds__(256, WPS) void dense_gemm_kernel(const T *__restric
             }
         }
     };
-    uint32_t seg = 0;
 #pragma unroll
-    for (int j = 0; j < PD; j++) load(j, j);
+    for (int j = 0; j < PD; j++) {
+        load(j, j);
+        asm volatile("" ::: "memory");  // in this order, and here: the waits in the loop count on it
+    }
     park(0, 0);
     load(0, PD);
+    asm volatile("" ::: "memory");
     __syncthreads();
-    for (uint32_t step0 = 0; step0 < n_steps; step0 += PD) {
+    uint32_t step = 0;
+    for (uint32_t seg = 0; seg < (RESIDUAL ? cs.n_segs : 1u); seg++) {
+        // segments end at multiples of kDenseKAlign, whole rounds of the register slots
+        const uint32_t seg_end = RESIDUAL ? cs.s[seg].k_end / kStepElems : n_steps;
+        for (; step < seg_end; step += PD) {
 #pragma unroll
-        for (int j = 0; j < PD; j++) {  // register slots by compile-time index
-            const uint32_t step = step0 + j, buf = step & (NB - 1);
-            if (step >= n_steps) break;
+            for (int j = 0; j < PD; j++) {  // register slots by compile-time index
+                const uint32_t buf = (step + j) & (NB - 1);
 #pragma unroll
-            for (int c = 0; c < 2; c++) {
-                u32x4 fw[NN], fa[NT];
+                for (int c = 0; c < 2; c++) {
+                    u32x4 fw[NN], fa[NT];
 #pragma unroll
-                for (int i = 0; i < NN; i++) {
-                    const uint32_t r = wn + i * 16 + fr;
-                    fw[i] = lds[buf][r * 8 + ((c * 4 + g) ^ (r & 7))];
+                    for (int i = 0; i < NN; i++) {
+                        const uint32_t r = wn + i * 16 + fr;
+                        fw[i] = lds[buf][r * 8 + ((c * 4 + g) ^ (r & 7))];
+                    }
+#pragma unroll
+                    for (int i = 0; i < NT; i++) {
+                        const uint32_t r = wt + i * 16 + fr;
+                        fa[i] = lds[buf][BN * 8 + r * 8 + ((c * 4 + g) ^ (r & 7))];
+                    }
+#pragma unroll
+                    for (int i = 0; i < NN; i++)
+#pragma unroll
+                        for (int i2 = 0; i2 < NT; i2++) acc[i][i2] = mma16<T>(fw[i], fa[i2], acc[i][i2]);
                 }
-#pragma unroll
-                for (int i = 0; i < NT; i++) {
-                    const uint32_t r = wt + i * 16 + fr;
-                    fa[i] = lds[buf][BN * 8 + r * 8 + ((c * 4 + g) ^ (r & 7))];
-                }
-#pragma unroll
-                for (int i = 0; i < NN; i++)
-#pragma unroll
-                    for (int i2 = 0; i2 < NT; i2++) acc[i][i2] = mma16<T>(fw[i], fa[i2], acc[i][i2]);
-            }
-            if (step + 1 < n_steps) {
                 if (NB == 1) __syncthreads();
-                park((j + 1) % PD, buf ^ (NB - 1));
-                load((j + 1) % PD, step + 1 + PD);
+                park((j + 1) % PD, buf ^ (NB - 1));  // (behind the last step: that step again, read by nobody)
+                load((j + 1) % PD, step + j + 1 + PD);
+                __syncthreads();
             }
-            if (RESIDUAL && (step + 1) * kStepElems == cs.s[seg].k_end) {
-                fold(cs.s[seg]);
-                seg++;
-            }
-            __syncthreads();
         }
+        if (RESIDUAL) fold(cs.s[seg]);
     }
 
     if constexpr (!RESIDUAL) {

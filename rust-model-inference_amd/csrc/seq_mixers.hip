@@ -160,8 +160,11 @@ __global__ __launch_bounds__(256) void conv_rotate_pairs_kernel(RmiAttnShape s, 
     const uint32_t channels = (s.heads + s.kv_heads) * s.dim + s.kv_heads * s.vdim;
     const ConvCtx x{a.u, a.hist_in, a.conv, channels, s.taps};
     if (blockIdx.y == 0) conv_head_carry(x, s, a, head);
-    const uint32_t t0 = (blockIdx.y * 4 + (threadIdx.x >> 6)) * kConvRun;
-    if (t0 >= a.n_tokens) return;
+    // runs end at multiples of kConvRun positions: a value block takes four keys of a channel in one store
+    const uint32_t p_run = a.pos0 / kConvRun * kConvRun + (blockIdx.y * 4 + uint32_t(__builtin_amdgcn_readfirstlane(int(threadIdx.x >> 6)))) * kConvRun;
+    if (p_run >= a.pos0 + a.n_tokens) return;
+    const uint32_t skip = p_run < a.pos0 ? a.pos0 - p_run : 0;  // positions of the first run that came before
+    const uint32_t t0 = p_run + skip - a.pos0;
     const bool is_v = head >= s.heads + s.kv_heads, is_q = head < s.heads;
     const uint32_t dim = is_v ? s.vdim : s.dim;
     const uint32_t c0 = is_v ? (s.heads + s.kv_heads) * s.dim + (head - s.heads - s.kv_heads) * s.vdim : head * s.dim;
@@ -173,7 +176,7 @@ __global__ __launch_bounds__(256) void conv_rotate_pairs_kernel(RmiAttnShape s, 
     float2 row[kConvRun];
 #pragma unroll
     for (uint32_t i = 0; i < kConvRun; i++) {
-        const uint32_t t = t0 + i < a.n_tokens ? t0 + i : a.n_tokens - 1;
+        const uint32_t ti = i < skip ? 0 : p_run + i - a.pos0, t = ti < a.n_tokens ? ti : a.n_tokens - 1;
         row[i] = *reinterpret_cast<const float2 *>(a.u + size_t(t) * channels + c);
     }
 #pragma unroll
@@ -184,7 +187,7 @@ __global__ __launch_bounds__(256) void conv_rotate_pairs_kernel(RmiAttnShape s, 
     }
     const uint32_t group = s.heads / s.kv_heads, half = s.rot_dims / 2;
     const bool turned = !is_v && lane < half;
-    T *out;  // of token t0; `step` further for the next
+    T *out;  // of the first live token; `step` further for the next
     size_t step;
     if (is_q) {
         out = static_cast<T *>(a.q) + (size_t(head / group) * a.n_tokens * group + size_t(t0) * group + head % group) * s.dk_pad;
@@ -193,10 +196,13 @@ __global__ __launch_bounds__(256) void conv_rotate_pairs_kernel(RmiAttnShape s, 
         out = static_cast<T *>(a.k_cache) + (size_t(head - s.heads) * s.capacity + a.pos0 + t0) * s.dk_pad;
         step = s.dk_pad;
     }
+    float v0[kConvRun], v1[kConvRun];
+    uint32_t n_live = skip;  // one past the last live place of the run
 #pragma unroll
     for (uint32_t i = 0; i < kConvRun; i++) {
-        const uint32_t t = t0 + i;
-        if (t >= a.n_tokens) break;
+        v0[i] = v1[i] = 0.0f;
+        if (i < skip || p_run + i >= a.pos0 + a.n_tokens) continue;
+        n_live = i + 1;
 #pragma unroll
         for (uint32_t j = 0; j < 3; j++) {
             u0[j] = u0[j + 1];
@@ -213,22 +219,35 @@ __global__ __launch_bounds__(256) void conv_rotate_pairs_kernel(RmiAttnShape s, 
         if (!has) p = q = 0.0f;
         if (is_v) {
             const float r = 1.0f / sqrtf(wave_sum_f32(__builtin_fmaf(p, p, q * q)) / float(dim) + s.eps);
-            const uint32_t pos = a.pos0 + t;
-            T *blk = static_cast<T *>(a.v_cache) +
-                     (size_t(head - s.heads - s.kv_heads) * (s.capacity / kKeyBlock) + pos / kKeyBlock) * s.dv_pad * kKeyBlock +
-                     value_slot<T>(pos % kKeyBlock);
-            if (has) {
-                blk[size_t(2 * lane) * kKeyBlock] = from_f32<T>(p * r);
-                blk[size_t(2 * lane + 1) * kKeyBlock] = from_f32<T>(q * r);
-            }
+            v0[i] = p * r;
+            v1[i] = q * r;
         } else {
             if (turned) {
-                const size_t at = size_t(a.pos0 + t) * half + lane;
+                const size_t at = size_t(p_run + i) * half + lane;
                 const float cs = a.cos_t[at], sn = a.sin_t[at], rp = p;
                 p = __builtin_fmaf(rp, cs, -(q * sn));
                 q = __builtin_fmaf(q, cs, rp * sn);
             }
-            if (2 * lane < s.dk_pad) store_pair(out + i * step + 2 * lane, p, q);
+            if (2 * lane < s.dk_pad) store_pair(out + (i - skip) * step + 2 * lane, p, q);
+        }
+    }
+    if (is_v && has) {
+        T *blk = static_cast<T *>(a.v_cache) +
+                 (size_t(head - s.heads - s.kv_heads) * (s.capacity / kKeyBlock) + p_run / kKeyBlock) * s.dv_pad * kKeyBlock + size_t(2 * lane) * kKeyBlock;
+#pragma unroll
+        for (uint32_t g = 0; g < kConvRun; g += 4) {  // four keys lie side by side
+            T *dst = blk + value_slot<T>((p_run + g) % kKeyBlock);
+            if (g >= skip && g + 4 <= n_live) {
+                store4(dst, f32x4{v0[g], v0[g + 1], v0[g + 2], v0[g + 3]});
+                store4(dst + kKeyBlock, f32x4{v1[g], v1[g + 1], v1[g + 2], v1[g + 3]});
+            } else {
+#pragma unroll
+                for (uint32_t i = g; i < g + 4; i++)
+                    if (i >= skip && i < n_live) {
+                        dst[i - g] = from_f32<T>(v0[i]);
+                        dst[kKeyBlock + i - g] = from_f32<T>(v1[i]);
+                    }
+            }
         }
     }
 }
@@ -380,13 +399,13 @@ __device__ __forceinline__ void attn_store(const RmiAttnShape &s, const RmiAttnA
     }
 }
 
-// several tokens: a workgroup is four waves of QT tiles, each over all the keys its columns see
+// several tokens: a workgroup takes QT tiles, each of its four waves a quarter of the keys they see; merged in LDS
 template <typename T, int BUCKET, int QT>
 __global__ __launch_bounds__(256) void attn_pass_kernel(RmiAttnShape s, RmiAttnArgs a) {
-    const uint32_t lane = threadIdx.x & 63, fr = lane & 15, g4 = lane >> 4;
-    const uint32_t group = s.heads / s.kv_heads, kvh = blockIdx.y, n_cols = a.n_tokens * group;
-    const uint32_t tile = (gridDim.x - 1 - blockIdx.x) * 4 + uint32_t(__builtin_amdgcn_readfirstlane(int(threadIdx.x >> 6)));  // the longest columns first
-    if (tile * QT * 16 >= n_cols) return;
+    extern __shared__ __attribute__((aligned(16))) uint8_t lds_raw[];
+    const uint32_t tid = threadIdx.x, lane = tid & 63, wave = uint32_t(__builtin_amdgcn_readfirstlane(int(tid >> 6))), fr = lane & 15, g4 = lane >> 4;
+    const uint32_t group = s.heads / s.kv_heads, kvh = blockIdx.x % s.kv_heads, n_cols = a.n_tokens * group;
+    const uint32_t tile = gridDim.x / s.kv_heads - 1 - blockIdx.x / s.kv_heads;  // the longest columns first
     AttnWave<T, BUCKET, QT> w;
     w.init();
     int last[QT];
@@ -402,19 +421,44 @@ __global__ __launch_bounds__(256) void attn_pass_kernel(RmiAttnShape s, RmiAttnA
             w.qf[i][c] = *reinterpret_cast<const u32x4 *>(q + c * 4 * kPieceElems<T>);
         }
     }
-    const uint32_t end_col = (tile + 1) * QT * 16 < n_cols ? (tile + 1) * QT * 16 : n_cols;
-    w.keys(static_cast<const T *>(a.k_cache) + size_t(kvh) * s.capacity * s.dk_pad,
-           static_cast<const T *>(a.v_cache) + size_t(kvh) * s.capacity * s.dv_pad, s, 0, a.pos0 + (end_col - 1) / group + 1, last);
+    const uint32_t first_col = tile * QT * 16, live = n_cols - first_col < QT * 16 ? n_cols - first_col : QT * 16;
+    const uint32_t n_keys = a.pos0 + (first_col + live - 1) / group + 1;
+    const uint32_t per_wave = (n_keys + 4 * kKeyBlock - 1) / (4 * kKeyBlock) * kKeyBlock;
+    const uint32_t k0 = wave * per_wave, k1 = k0 + per_wave < n_keys ? k0 + per_wave : n_keys;
+    if (k0 < k1)
+        w.keys(static_cast<const T *>(a.k_cache) + size_t(kvh) * s.capacity * s.dk_pad,
+               static_cast<const T *>(a.v_cache) + size_t(kvh) * s.capacity * s.dv_pad, s, k0, k1, last);
+    // [wave][maxima, sums, column x channel (rows a float4 apart more than they hold)]
+    const uint32_t row = s.dv_pad + 4, pl = QT * 16 * (row + 2);
+    float *all = reinterpret_cast<float *>(lds_raw), *mine = all + wave * pl;
 #pragma unroll
     for (int i = 0; i < QT; i++) {
-        const uint32_t col = (tile * QT + i) * 16 + fr;
-        const float sum = rows_sum_f32(w.l[i]);
-        if (col >= n_cols) continue;
-        const uint32_t t = col / group, head = kvh * group + col % group;
-        const float f = (a.gate ? a.gate[size_t(t) * s.heads + head] : 1.0f) / sum;
+        const float l = rows_sum_f32(w.l[i]);
+        if (g4 == 0) {
+            mine[i * 16 + fr] = w.m[i];
+            mine[QT * 16 + i * 16 + fr] = l;
+        }
 #pragma unroll
         for (uint32_t v = 0; v < w.kVT; v++)
-            if (v * 16 < s.dv_pad) attn_store<T>(s, a, t, head, v * 16 + g4 * 4, w.o[i][v] * f);
+            if (v * 16 < s.dv_pad) *reinterpret_cast<f32x4 *>(mine + QT * 32 + (i * 16 + fr) * row + v * 16 + g4 * 4) = w.o[i][v];
+    }
+    __syncthreads();
+    const uint32_t quads = s.dv_pad / 4;
+    for (uint32_t e = tid; e < live * quads; e += 256) {
+        const uint32_t c = e / quads, d = e % quads * 4;
+        float m = all[c];
+#pragma unroll
+        for (uint32_t i = 1; i < 4; i++) m = fmaxf(m, all[i * pl + c]);
+        float sum = 0.0f;  // (every column sees key 0: m is finite)
+        f32x4 o = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+        for (uint32_t i = 0; i < 4; i++) {
+            const float f = exp_t<T>(all[i * pl + c] - m);
+            sum = __builtin_fmaf(all[i * pl + QT * 16 + c], f, sum);
+            o += *reinterpret_cast<const f32x4 *>(all + i * pl + QT * 32 + c * row + d) * f;
+        }
+        const uint32_t mc = first_col + c, t = mc / group, head = kvh * group + mc % group;
+        attn_store<T>(s, a, t, head, d, o * ((a.gate ? a.gate[size_t(t) * s.heads + head] : 1.0f) / sum));
     }
 }
 
@@ -958,7 +1002,7 @@ size_t split_lds(uint32_t elem_bytes, const RmiAttnShape &s, uint32_t n_tokens) 
 template <typename T>
 int attn_pass(const RmiAttnShape &s, const RmiAttnArgs &a, hipStream_t st) {
     const uint32_t n_heads = s.heads + 2 * s.kv_heads, group = s.heads / s.kv_heads, n_cols = a.n_tokens * group;
-    const dim3 conv_grid(n_heads, (a.n_tokens + 4 * kConvRun - 1) / (4 * kConvRun));
+    const dim3 conv_grid(n_heads, (a.pos0 % kConvRun + a.n_tokens + 4 * kConvRun - 1) / (4 * kConvRun));
     if (conv_pairs_fit(s))
         hipLaunchKernelGGL(conv_rotate_pairs_kernel<T>, conv_grid, dim3(256), 0, st, s, a);
     else
@@ -977,13 +1021,17 @@ int attn_pass(const RmiAttnShape &s, const RmiAttnArgs &a, hipStream_t st) {
         const int rc = bucket == 64 ? go(attn_split_kernel<T, 64>) : bucket == 128 ? go(attn_split_kernel<T, 128>) : go(attn_split_kernel<T, 256>);
         if (rc != RMI_HIP_OK) return rc;
     } else {
-        auto grid = [&](uint32_t qt) { return dim3((n_cols + 64 * qt - 1) / (64 * qt), s.kv_heads); };
-        if (bucket == 64)
-            hipLaunchKernelGGL((attn_pass_kernel<T, 64, 2>), grid(2), dim3(256), 0, st, s, a);
-        else if (bucket == 128)
-            hipLaunchKernelGGL((attn_pass_kernel<T, 128, 2>), grid(2), dim3(256), 0, st, s, a);
-        else
-            hipLaunchKernelGGL((attn_pass_kernel<T, 256, 1>), grid(1), dim3(256), 0, st, s, a);
+        auto go = [&](auto kernel, uint32_t qt) {
+            const size_t lds = size_t(4) * qt * 16 * (s.dv_pad + 6) * 4;
+            const int rc = rmi_allow_lds(kernel, lds);
+            if (rc == RMI_HIP_OK)
+                hipLaunchKernelGGL(kernel, dim3((n_cols + 16 * qt - 1) / (16 * qt) * s.kv_heads), dim3(256), lds, st, s, a);
+            return rc;
+        };
+        const int rc = bucket == 64    ? go(attn_pass_kernel<T, 64, 2>, 2)
+                       : bucket == 128 ? go(attn_pass_kernel<T, 128, 2>, 2)
+                                       : go(attn_pass_kernel<T, 256, 1>, 1);
+        if (rc != RMI_HIP_OK) return rc;
     }
     RMI_HIP_CHECK(hipGetLastError());
     return RMI_HIP_OK;

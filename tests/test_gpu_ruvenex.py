@@ -351,3 +351,20 @@ def test_trace_run(open_model, tmp_path):
     for step, rows in ((0, [0, 4]), (2, [11]), (3, [2])):
         assert rel(np.fromfile(out / f"{step}.f32", "<f4").reshape(-1, 60), ref[rows]) < TOL[F32]
     assert not (out / "1.f32").exists()
+
+
+def test_command_line_generates(hip, tmp_path, capsys):
+    """`python -m rust-model-inference_amd` on a model folder and on a GGUF file: the sessions' own tokens."""
+    import importlib
+
+    cli = importlib.import_module("rust-model-inference_amd.__main__")
+    cfg = G.config([G.layer_config()])
+    folder = G.write_folder(tmp_path / "m", cfg, G.weights(cfg))
+    gguf = str(tmp_path / "q.gguf")
+    hip.gguf.write_synthetic_qwen3(gguf, 3, n_layer=1, n_embd=64, n_head=2, n_head_kv=1, head_dim=32, n_ff=64, vocab=96)
+    for path, args in ((folder, ["--dtype", F32]), (gguf, [])):
+        s = hip.models.open_session(path, 32, F32)
+        want = s.generate([5, 17, 3], 9)["tokens"].tolist()
+        s.close()
+        assert cli.main(["--model", path, "--tokens", "5,17,3", "--max-new", "9", *args]) == 0
+        assert [int(t) for t in capsys.readouterr().out.strip().split(",")] == want

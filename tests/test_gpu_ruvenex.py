@@ -309,6 +309,17 @@ def test_generation_in_bf16_follows_its_own_logits(open_model):
     assert logits.argmax(-1).tolist() == out
 
 
+def test_generation_repeats_bit_for_bit(open_model):
+    """Keys divided over workgroups that hand their parts to whichever arrives last: the order of arrival does not show."""
+    cfg = G.config([G.layer_config(heads=4, kv_heads=2, dim=64, vdim=64, rot_dims=16)] * 3, vocab=150)
+    s, _ = open_model(cfg, None, BF16, 1300)
+    prompt = G.tokens(cfg, 900)
+    runs = [s.generate(prompt, 300) for _ in range(4)]
+    for r in runs[1:]:
+        assert np.array_equal(r["tokens"], runs[0]["tokens"])
+        assert np.array_equal(r["top2"][899:].view(np.uint32), runs[0]["top2"][899:].view(np.uint32))
+
+
 def test_errors_are_reported(hip, open_model, tmp_path):
     cfg = G.config([G.layer_config()])
     s, w = open_model(cfg, None, F32, 8)

@@ -229,7 +229,7 @@ int launch_gemm(const RmiDense &w, const void *a, const RmiRowSegs &rs, const Rm
     auto tiles = [&](uint32_t bn, uint32_t bt) { return uint64_t((n_rows + bn - 1) / bn) * ((n_tokens + bt - 1) / bt); };
     if (n_tokens <= 16)
         go(dense_gemm_kernel<T, 64, 16, 16, 16, 4, 2, 4, RESIDUAL>, 64, 16);
-    else if (tiles(128, 128) >= cus)
+    else if (tiles(128, 128) >= 2 * cus)
         go(dense_gemm_kernel<T, 128, 128, 64, 64, 1, 1, 3, RESIDUAL>, 128, 128);
     else if (tiles(64, 64) >= cus)
         go(dense_gemm_kernel<T, 64, 64, 32, 32, 4, 2, 4, RESIDUAL>, 64, 64);

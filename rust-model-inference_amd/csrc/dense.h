@@ -1,9 +1,9 @@
 // Dense (bf16 or f32) weights and the products on them: the launch interface that decoder sessions use.
 //
 // A weight is row-major, rows of k_pad elements (the sum of its column segments, each padded with zeros to
-// kDenseKAlign elements) that lie rmi_dense_ld apart, as do those of an activation; its row segments each padded with zero rows to kDenseRowAlign.  Both element types share
-// every kernel: the code works on 16-byte pieces.  Accumulation is f32; the residual stream and everything a product
-// writes is f32 unless its segment says otherwise.
+// kDenseKAlign elements) that lie rmi_dense_ld apart, as do those of an activation; its row segments are each padded
+// with zero rows to kDenseRowAlign.  Both element types share every kernel: the code works on 16-byte pieces.
+// Accumulation is f32; the residual stream and everything a product writes is f32 unless its segment says otherwise.
 #pragma once
 
 #include "rmi_internal.h"

@@ -1,4 +1,4 @@
-// Model folders: config.json and model.safetensors (an 8-byte little-endian length, that many bytes of JSON naming
+// Model folders: config.json and model.safetensors (a 64-bit length and a JSON header of that size, naming
 // each tensor's dtype, shape and byte range, then the data).  Host code only; the file stays mapped while a session
 // uploads from it.
 #include "model_folder.h"

@@ -146,7 +146,7 @@ struct PairTaps {
         }
     }
 };
-// the projected pair at the pass's row t - back (back <= 3), zeros before the sequence's start
+// the projected pair at the pass's row t - back (back <= 3); a position below zero reads as zero
 __device__ __forceinline__ float2 pair_row(const RmiAttnShape &s, const RmiAttnArgs &a, uint32_t channels, uint32_t t, uint32_t back, uint32_t c) {
     if (t >= back) return *reinterpret_cast<const float2 *>(a.u + size_t(t - back) * channels + c);
     if (back - t < s.taps && a.pos0 + t >= back) return *reinterpret_cast<const float2 *>(a.hist_in + size_t(t + s.taps - 1 - back) * channels + c);

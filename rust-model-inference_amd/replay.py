@@ -1,12 +1,9 @@
-"""Replays a trace: given token ids through a model's session, step by step, the wanted logits to files.
+"""Replays recorded traffic through a model's session and writes the logits asked for.
 
-Steps are read as JSON objects, one a line:
-
-    {"step": 0, "entries": [{"id": "a", "tokens": [5, 17, 3], "want": [0, 2]}], "end": ["a"]}
-
-For a step in which something is wanted OUT/<step>.f32 gets the logits of the wanted places, little-endian f32,
-[wanted, vocab]; then "done <step>" is printed.  A request keeps its cache and state between steps; `end` gives them
-back.  The session holds one sequence, so requests come one after the other.
+Every input line is a JSON object: ``step`` (a number), ``entries`` (each the ``id`` of a sequence, its next
+``tokens``, and ``want``, indices into them) and ``end`` (ids of sequences that are over).  The wanted rows of a step
+go to OUT/<step>.f32 as little-endian f32, in order, and "done <step>" follows on standard output.  A sequence keeps
+its cache and state from step to step until `end` names it; the session holds one, so the next begins after that.
 """
 import json
 import os

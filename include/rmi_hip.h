@@ -527,29 +527,50 @@ rmi_hip_qwen3 *rmi_hip_qwen3_create_from_gguf(const rmi_hip_gguf *g, uint32_t ca
  * names decides the session: its length, and the name in buf (up to cap - 1 bytes and a terminator); -1 on error. */
 int64_t rmi_hip_model_folder_architecture(const char *dir, char *buf, size_t cap);
 
-/* ------------------------------------------------------------------ Ruvenex decoder
- * Parallel layers: one RMS norm read by a softmax-attention mixer (short causal convolution, partial interleaved
- * rotation, value norm, per-head output gate), an HGRN2 mixer beside it (gated linear recurrence) and a gelu
- * feed-forward, each sublayer's result gated element by element.  Sizes, constants and the order of layers come
- * from config.json.  No counterpart in the reference.
+/* Sessions over such folders.  Designs (none has a counterpart in the reference):
  *
- * dtype: RMI_HIP_DTYPE_BF16 (matrix operands, keys and values in bf16, f32 accumulation; residual, norms, scores,
- * gates and recurrent state f32) or RMI_HIP_DTYPE_F32 (everything true f32).  capacity: most tokens of a sequence.
- * A session holds one sequence at a time. */
-typedef struct rmi_hip_ruvenex rmi_hip_ruvenex;
-rmi_hip_ruvenex *rmi_hip_ruvenex_open(const char *dir, int dtype, uint32_t capacity); /* NULL on error */
-void rmi_hip_ruvenex_destroy(rmi_hip_ruvenex *s);
-int rmi_hip_ruvenex_sizes(const rmi_hip_ruvenex *s, uint32_t *vocab, uint32_t *width, uint32_t *n_layer, uint32_t *capacity);
+ * Ruvenex: parallel layers; one RMS norm read by a softmax-attention mixer (short causal convolution, partial
+ * interleaved rotation, value norm, per-head output gate), an HGRN2 mixer beside it (gated linear recurrence) and a
+ * gelu feed-forward, each sublayer's result gated element by element.
+ * Vogizen: sequential layers with layer norms and layer scales, each a mixer (sliding-window latent attention, or the
+ * gated delta rule behind short convolutions), an optional relu-gated feed-forward and a per-layer input looked up by
+ * the token; sinusoidal positions, tied embedding, a run of layers looped with the same weights.
+ *
+ * Sizes, constants and the order of layers come from config.json.
+ *
+ * architecture: what config.json must name, NULL: any of these.  dtype: RMI_HIP_DTYPE_BF16 (matrix operands, keys and
+ * values in bf16, f32 accumulation; residual, norms, scores, gates and recurrent state f32) or RMI_HIP_DTYPE_F32
+ * (everything true f32).  capacity: most tokens of a sequence.  A session holds one sequence at a time. */
+typedef struct rmi_hip_folder_session rmi_hip_folder_session;
+rmi_hip_folder_session *rmi_hip_folder_open(const char *dir, const char *architecture, int dtype, uint32_t capacity); /* NULL on error */
+void rmi_hip_folder_destroy(rmi_hip_folder_session *s);
+/* n_layer: layers that a token runs through; one of a loop counts each time */
+int rmi_hip_folder_sizes(const rmi_hip_folder_session *s, uint32_t *vocab, uint32_t *width, uint32_t *n_layer, uint32_t *capacity);
 /* The next tokens of the sequence from the cache and state the earlier ones left; any portions give the same
  * result within rounding.  logits[i * vocab ..] = those of place want[i] among these tokens.  layers (NULL, or
  * [n_layer][n_tokens][width]): the residual stream behind every layer, for comparisons. */
+int rmi_hip_folder_step(rmi_hip_folder_session *s, const uint32_t *tokens, uint32_t n_tokens, const uint32_t *want, uint32_t n_want,
+                        float *logits, float *layers);
+uint32_t rmi_hip_folder_position(const rmi_hip_folder_session *s); /* tokens of the sequence so far */
+int rmi_hip_folder_reset(rmi_hip_folder_session *s);               /* the sequence is over; a new one begins */
+/* As the rmi_hip_qwen3_* calls of the same names (greedy; a new sequence).  A prompt pass takes up to 2048 positions
+ * and computes logits only where they are read: step_argmax and step_top2 of a prompt position that is neither the
+ * prompt's last nor listed in dump_steps are left as they were, unless prompt passes are off. */
+int rmi_hip_folder_set_stop_ids(rmi_hip_folder_session *s, const uint32_t *ids, uint32_t n_ids);
+int rmi_hip_folder_set_prompt_passes(rmi_hip_folder_session *s, int enabled);
+int rmi_hip_folder_generate(rmi_hip_folder_session *s, const uint32_t *prompt, uint32_t n_prompt, uint32_t max_new,
+                            uint32_t *generated, uint32_t *step_argmax, float *step_top2, const uint32_t *dump_steps,
+                            uint32_t n_dump, float *dump_logits, double *seconds);
+
+/* The same calls under the names they had when Ruvenex was the only design; open takes no other. */
+typedef rmi_hip_folder_session rmi_hip_ruvenex;
+rmi_hip_ruvenex *rmi_hip_ruvenex_open(const char *dir, int dtype, uint32_t capacity); /* NULL on error */
+void rmi_hip_ruvenex_destroy(rmi_hip_ruvenex *s);
+int rmi_hip_ruvenex_sizes(const rmi_hip_ruvenex *s, uint32_t *vocab, uint32_t *width, uint32_t *n_layer, uint32_t *capacity);
 int rmi_hip_ruvenex_step(rmi_hip_ruvenex *s, const uint32_t *tokens, uint32_t n_tokens, const uint32_t *want, uint32_t n_want,
                          float *logits, float *layers);
 uint32_t rmi_hip_ruvenex_position(const rmi_hip_ruvenex *s); /* tokens of the sequence so far */
 int rmi_hip_ruvenex_reset(rmi_hip_ruvenex *s);               /* the sequence is over; a new one begins */
-/* As the rmi_hip_qwen3_* calls of the same names (greedy; a new sequence).  A prompt pass takes up to 2048 positions
- * and computes logits only where they are read: step_argmax and step_top2 of a prompt position that is neither the
- * prompt's last nor listed in dump_steps are left as they were, unless prompt passes are off. */
 int rmi_hip_ruvenex_set_stop_ids(rmi_hip_ruvenex *s, const uint32_t *ids, uint32_t n_ids);
 int rmi_hip_ruvenex_set_prompt_passes(rmi_hip_ruvenex *s, int enabled);
 int rmi_hip_ruvenex_generate(rmi_hip_ruvenex *s, const uint32_t *prompt, uint32_t n_prompt, uint32_t max_new,

@@ -20,13 +20,21 @@ inline uint32_t rmi_dense_ld(uint32_t k_pad, uint32_t elem_bytes) {
     return k_pad + (size_t(k_pad) * elem_bytes % 256 == 0 ? 128 / elem_bytes : 0);
 }
 
-enum RmiAct : uint32_t { kActNone, kActSigmoid, kActSilu, kActGeluTanh, kActForgetGate };
+// kActForgetGate: lower + (1 - lower) sigmoid(z + bias) in full f32 (without either array a plain sigmoid);
+// kActDecay: exp(-lower softplus(z + bias)) in full f32; kActReluGlu: rows come in pairs (gate, up) and
+// y[row / 2] = relu(gate) * up.
+enum RmiAct : uint32_t { kActNone, kActSigmoid, kActSilu, kActGeluTanh, kActForgetGate, kActDecay, kActReluGlu };
 
 // Rows [row0, row0 + n) of a product: y[token * ld + row - row0] = act(result), f32 or the model's element type.
+// mul (nullptr = none): the activation's result times mul[mul_tok[token] * mul_ld + row - row0], a table of the
+// model's element type with mul_rows rows, looked up by the token's id.
 struct RmiRowSeg {
     void *y;
-    const float *bias;   // kActSigmoid (nullptr = none), kActForgetGate
-    const float *lower;  // kActForgetGate
+    const float *bias;   // kActSigmoid, kActForgetGate, kActDecay; nullptr = 0
+    const float *lower;  // kActForgetGate (nullptr = 0), kActDecay
+    const void *mul;
+    const uint32_t *mul_tok;
+    uint32_t mul_ld, mul_rows;
     uint32_t row0, n, ld;
     uint16_t act;
     uint16_t out_elem;  // 1: the model's element type, 0: f32
@@ -45,7 +53,8 @@ inline void rmi_row_segs_done(RmiRowSegs *r) {
 // x[token][row] += sum over column segments i of gate_i[token][row] * scale_i * (W_i a_i)[row].  A segment's columns
 // end at k_end (padded); a null gate is one.
 struct RmiColSeg {
-    const float *gate;  // [token][width]
+    const float *gate;  // rows gate_ld apart: width, or 0 for one row that all tokens share (a layer scale)
+    uint32_t gate_ld;
     float scale;
     uint32_t k_end;
 };
@@ -71,20 +80,51 @@ int rmi_allow_lds(K kernel, size_t bytes) {
     return RMI_HIP_OK;
 }
 
+// What a product reads of the f32 residual stream, n values a token:
+//   v = x                                        y == nullptr
+//   v = x + y / sqrt(mean(y^2) + y_eps) * y_weight   otherwise: a sublayer's result that only now joins the stream
+// v goes to x_out where that is given (in a product of one token never x itself: its workgroups all read x), and
+// norm(v) is the product's operand; with a second part (x2, n2 values, kNormNone only) [v ; x2], the second one from
+// column k2 on.
+enum RmiNorm : uint32_t { kNormNone, kNormRms, kNormLayer };
+struct RmiInput {
+    const float *x = nullptr;
+    uint32_t n = 0;
+    RmiNorm norm = kNormNone;
+    const float *weight = nullptr;
+    float eps = 0, y_eps = 0;
+    const float *y = nullptr, *y_weight = nullptr;
+    float *x_out = nullptr;
+    const float *x2 = nullptr;
+    uint32_t n2 = 0, k2 = 0;
+};
+constexpr uint32_t kInputMax = 16384;    // most values of an input: a workgroup keeps a row in registers
+constexpr uint32_t kGemvAddMax = 4096;   // most with y in a product of one token
+
 // elem_bytes 2: bf16, 4: f32
-// h[i][0 .. k_pad) (rows rmi_dense_ld apart) = rms_norm(x[rows ? rows[i] : i]) * weight, zeros past n
-int rmi_dense_norm(uint32_t elem_bytes, const float *x, const uint32_t *rows, const float *weight, float eps, void *h,
-                   uint32_t n_tokens, uint32_t n, uint32_t k_pad, hipStream_t st);
-// x[i] = table[tok[i]] * scale (table: a dense weight)
-int rmi_dense_embed(uint32_t elem_bytes, const RmiDense &table, const uint32_t *tok, uint32_t vocab, float scale, float *x,
-                    uint32_t n_tokens, uint32_t n, hipStream_t st);
+// h[i][0 .. k_pad) (rows rmi_dense_ld apart) = the operand of token rows ? rows[i] : i, zeros elsewhere; h may be
+// nullptr where x_out is all that is wanted.  Here x_out may be x.
+int rmi_dense_input(uint32_t elem_bytes, const RmiInput &in, const uint32_t *rows, void *h, uint32_t n_tokens, uint32_t k_pad,
+                    hipStream_t st);
+// x[i] = table[tok[i]] * scale (table: a dense weight), with `turns` plus the sinusoidal vector of position pos0 + i:
+// sin and cos in turn, of 2 pi turns[c / 2] a position; x_also: a second copy
+struct RmiEmbed {
+    const void *table;
+    uint32_t ld, vocab, n;
+    float scale;
+    const double *turns;
+    float *x, *x_also;
+};
+int rmi_dense_embed(uint32_t elem_bytes, const RmiEmbed &e, const uint32_t *tok, uint32_t pos0, uint32_t n_tokens, hipStream_t st);
 // several tokens: matrix cores; a = [n_tokens] rows of k_pad elements, rmi_dense_ld apart
 int rmi_dense_gemm(uint32_t elem_bytes, const RmiDense &w, const void *a, const RmiRowSegs &segs, uint32_t n_tokens, hipStream_t st);
 int rmi_dense_gemm_residual(uint32_t elem_bytes, const RmiDense &w, const void *a, const RmiColSegs &segs, float *x, uint32_t width,
                             uint32_t n_tokens, hipStream_t st);
-// one token: the norm in front of the product is part of the launch, for as many columns as a workgroup holds
+// one token: the input in front of the product is part of the launch, for as many columns as a workgroup holds; the
+// second form computes two products with inputs of their own side by side
 bool rmi_dense_gemv_fits(uint32_t elem_bytes, uint32_t k_pad);
-int rmi_dense_norm_gemv(uint32_t elem_bytes, const RmiDense &w, const float *x, const float *weight, float eps, uint32_t n,
-                        const RmiRowSegs &segs, hipStream_t st);
+int rmi_dense_gemv(uint32_t elem_bytes, const RmiDense &w, const RmiInput &in, const RmiRowSegs &segs, hipStream_t st);
+int rmi_dense_gemv_pair(uint32_t elem_bytes, const RmiDense &w0, const RmiInput &in0, const RmiRowSegs &segs0, const RmiDense &w1,
+                        const RmiInput &in1, const RmiRowSegs &segs1, hipStream_t st);
 int rmi_dense_gemv_residual(uint32_t elem_bytes, const RmiDense &w, const void *a, const RmiColSegs &segs, float *x, uint32_t width,
                             hipStream_t st);

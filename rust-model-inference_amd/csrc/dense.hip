@@ -1,41 +1,28 @@
-// Products on dense bf16 / f32 weights: a tiled matrix-core GEMM for several tokens, a GEMV for one, each with the
-// layer's elementwise work in its epilogue (activations, forget gates, gated residual) and, in the GEMV, the RMS
-// norm in its prologue.
-#include "device_dense.h"
+// Products of several tokens on dense bf16 / f32 weights: the inputs (norms) in front of them, a tiled matrix-core
+// GEMM with the layer's elementwise work in its epilogue (activations, gates, gated residual), and the embedding.
+#include "dense_launch.h"
 
 namespace {
 
-template <typename T>
-__global__ __launch_bounds__(256) void norm_kernel(const float *__restrict__ x, const uint32_t *__restrict__ rows,
-                                                   const float *__restrict__ weight, float eps, T *__restrict__ h, uint32_t n,
-                                                   uint32_t k_pad, uint32_t ld) {
-    __shared__ float red[4];
-    const uint32_t tid = threadIdx.x;
-    x += size_t(rows ? rows[blockIdx.x] : blockIdx.x) * n;
-    h += size_t(blockIdx.x) * ld;
-    float sq = 0.0f;
-    for (uint32_t i = tid; i < n; i += 256) sq = __builtin_fmaf(x[i], x[i], sq);
-    sq = wave_sum_f32(sq);
-    if ((tid & 63) == 0) red[tid >> 6] = sq;
-    __syncthreads();
-    const float r = 1.0f / sqrtf(((red[0] + red[1]) + (red[2] + red[3])) / float(n) + eps);
-    for (uint32_t i = tid; i < k_pad; i += 256) h[i] = from_f32<T>(i < n ? x[i] * r * weight[i] : 0.0f);
+template <typename T, int NORM, bool ADD, int R>
+__global__ __launch_bounds__(256) void input_kernel(RmiInput in, const uint32_t *__restrict__ rows, T *__restrict__ h, uint32_t k_pad,
+                                                    uint32_t ld) {
+    __shared__ float red[12];
+    InputRow<NORM, ADD, R> r;
+    const uint32_t row = rows ? rows[blockIdx.x] : blockIdx.x;
+    r.load(in, row);
+    r.finish(in, row, in.x_out != nullptr, red);
+    if (h) r.store(in, row, h + size_t(blockIdx.x) * ld, k_pad);
 }
 
 template <typename T>
-__global__ __launch_bounds__(256) void embed_kernel(const T *__restrict__ table, uint32_t ld, const uint32_t *__restrict__ tok,
-                                                    uint32_t vocab, float scale, float *__restrict__ x, uint32_t n) {
-    uint32_t t = tok[blockIdx.x];
-    if (t >= vocab) t = vocab - 1;  // ids are validated on the host; never read outside the table
-    for (uint32_t i = threadIdx.x; i < n; i += 256) x[size_t(blockIdx.x) * n + i] = to_f32(table[size_t(t) * ld + i]) * scale;
-}
-
-// which row segment a row lies in: the starts sit side by side (unused ones at the end of the range)
-__device__ __forceinline__ uint32_t seg_of(const RmiRowSegs &rs, uint32_t row) {
-    uint32_t si = 0;
-#pragma unroll
-    for (uint32_t i = 1; i < kMaxRowSegs; i++) si += row >= rs.start[i] ? 1u : 0u;
-    return si;
+__global__ __launch_bounds__(256) void embed_kernel(RmiEmbed e, const uint32_t *__restrict__ tok, uint32_t pos0) {
+    const uint32_t t = blockIdx.x, id = tok[t];
+    for (uint32_t i = threadIdx.x; i < e.n; i += 256) {
+        const float v = embed_value<T>(e, id, pos0 + t, i);
+        e.x[size_t(t) * e.n + i] = v;
+        if (e.x_also) e.x_also[size_t(t) * e.n + i] = v;
+    }
 }
 
 // ------------------------------------------------------------------ GEMM
@@ -117,12 +104,12 @@ __global__ __launch_bounds__(256, WPS) void dense_gemm_kernel(const T *__restric
                     if (tok < n_tokens && row < width) {
                         if (quads) {
                             f32x4 v = acc[i][j] * s.scale;
-                            if (s.gate) v *= *reinterpret_cast<const f32x4 *>(s.gate + at);
+                            if (s.gate) v *= *reinterpret_cast<const f32x4 *>(s.gate + size_t(tok) * s.gate_ld + row);
                             *reinterpret_cast<f32x4 *>(x + at) += v;
                         } else {
 #pragma unroll
                             for (int r = 0; r < 4; r++)
-                                if (row + r < width) x[at + r] += acc[i][j][r] * s.scale * (s.gate ? s.gate[at + r] : 1.0f);
+                                if (row + r < width) x[at + r] += acc[i][j][r] * s.scale * (s.gate ? s.gate[size_t(tok) * s.gate_ld + row + r] : 1.0f);
                         }
                     }
                     acc[i][j] = f32x4{0.f, 0.f, 0.f, 0.f};
@@ -190,10 +177,30 @@ __global__ __launch_bounds__(256, WPS) void dense_gemm_kernel(const T *__restric
 #pragma unroll
             for (int j = 0; j < NT; j++) {
                 const uint32_t tok = tok0 + wt + j * 16 + fr;
+                if (tok >= n_tokens) continue;
+                if (s.act == kActReluGlu) {  // (gate, up) pairs: two results
+#pragma unroll
+                    for (uint32_t r = 0; r < 2; r++) {
+                        const float v = fmaxf(acc[i][j][2 * r], 0.0f) * acc[i][j][2 * r + 1];
+                        const size_t at = size_t(tok) * s.ld + r0 / 2 + r;
+                        if (r0 + 2 * r < s.n) {
+                            if (s.out_elem)
+                                static_cast<T *>(s.y)[at] = from_f32<T>(v);
+                            else
+                                static_cast<float *>(s.y)[at] = v;
+                        }
+                    }
+                    continue;
+                }
                 f32x4 o;
 #pragma unroll
                 for (int r = 0; r < 4; r++) o[r] = apply_act<T>(s.act, acc[i][j][r], bias[r], lower[r]);
-                if (tok >= n_tokens) continue;
+                if (s.mul) {
+                    const T *m = mul_row<T>(s, tok) + r0;
+#pragma unroll
+                    for (uint32_t r = 0; r < 4; r++)
+                        if (r0 + r < s.n) o[r] *= to_f32(m[r]);
+                }
                 const size_t at = size_t(tok) * s.ld + r0;
                 if (r0 + 3 < s.n && (s.ld & 3) == 0) {
                     if (s.out_elem)
@@ -239,278 +246,49 @@ int launch_gemm(const RmiDense &w, const void *a, const RmiRowSegs &rs, const Rm
     return RMI_HIP_OK;
 }
 
-// ------------------------------------------------------------------ GEMV
-// The activation sits in LDS, zero past its end, so that a piece past the end of a row (the last one is read again)
-// counts for nothing.  Its loads go out before the weights': memory returns in order, and everything waits for it.
-constexpr uint32_t kGemvLdsMax = kLdsAskedFor;
-constexpr uint32_t kGemvRound = 256;  // LDS activations are padded to this many pieces
-template <typename T>
-__host__ __device__ inline uint32_t gemv_lds_pieces(uint32_t k_pad) {
-    const uint32_t pieces = k_pad / (16 / sizeof(T));
-    return (pieces + kGemvRound - 1) / kGemvRound * kGemvRound;
-}
-
-// A wave takes ROWS weight rows, its lanes the pieces of a row, two rounds of 64 in flight; R: quads of x a thread
-// keeps (n <= 1024 R).
-template <typename T, int ROWS, int R>
-__global__ __launch_bounds__(256) void norm_gemv_kernel(const T *__restrict__ w, uint32_t k_pad, uint32_t ld, const float *__restrict__ x,
-                                                        const float *__restrict__ weight, float eps, uint32_t n, RmiRowSegs rs) {
-    extern __shared__ u32x4 act[];
-    __shared__ float red[4];
-    const uint32_t tid = threadIdx.x, lane = tid & 63;
-    const uint32_t row0 = (blockIdx.x * 4 + uint32_t(__builtin_amdgcn_readfirstlane(int(tid >> 6)))) * ROWS;
-    const uint32_t pieces = k_pad / kPieceElems<T>, padded = gemv_lds_pieces<T>(k_pad);
-    f32x4 xv[R], nv[R];
-    const bool quads = (n & 3) == 0;
-#pragma unroll
-    for (int j = 0; j < R; j++) {
-        const uint32_t i = (tid + j * 256) * 4;
-        if (quads) {
-            const uint32_t ic = i < n ? i : n - 4;
-            xv[j] = *reinterpret_cast<const f32x4 *>(x + ic);
-            nv[j] = *reinterpret_cast<const f32x4 *>(weight + ic);
-        } else {
-#pragma unroll
-            for (int e = 0; e < 4; e++) {
-                const uint32_t ic = i + e < n ? i + e : n - 1;
-                xv[j][e] = x[ic];
-                nv[j][e] = weight[ic];
-            }
-        }
-    }
-    const u32x4 *src[ROWS];
-#pragma unroll
-    for (int r = 0; r < ROWS; r++) {
-        const uint32_t row = row0 + r < rs.n_rows ? row0 + r : rs.n_rows - 1;
-        src[r] = reinterpret_cast<const u32x4 *>(w + size_t(row) * ld);
-    }
-    u32x4 cur[2][ROWS];
-    auto load = [&](uint32_t p0) {
-#pragma unroll
-        for (int u = 0; u < 2; u++) {
-            const uint32_t p = p0 + u * 64 + lane;
-#pragma unroll
-            for (int r = 0; r < ROWS; r++) cur[u][r] = src[r][p < pieces ? p : pieces - 1];
-        }
-    };
-    load(0);
-    const RmiRowSeg seg = rs.s[seg_of(rs, row0)];
-    float sq = 0.0f;
-#pragma unroll
-    for (int j = 0; j < R; j++)
-#pragma unroll
-        for (int e = 0; e < 4; e++) {
-            if ((tid + j * 256) * 4 + e >= n) xv[j][e] = 0.0f;
-            sq = __builtin_fmaf(xv[j][e], xv[j][e], sq);
-        }
-    sq = wave_sum_f32(sq);
-    if (lane == 0) red[tid >> 6] = sq;
-    __syncthreads();
-    const float scale = 1.0f / sqrtf(((red[0] + red[1]) + (red[2] + red[3])) / float(n) + eps);
-    T *h = reinterpret_cast<T *>(act);
-    const uint32_t h_elems = padded * kPieceElems<T>;  // a multiple of 1024
-#pragma unroll
-    for (int j = 0; j < R; j++) {
-        const uint32_t i = (tid + j * 256) * 4;
-        if (i < h_elems) store4(h + i, xv[j] * scale * nv[j]);
-    }
-    for (uint32_t i = (tid + R * 256) * 4; i < h_elems; i += 1024) store4(h + i, f32x4{0.f, 0.f, 0.f, 0.f});
-    __syncthreads();
-    float acc[ROWS];
-#pragma unroll
-    for (int r = 0; r < ROWS; r++) acc[r] = 0.0f;
-    for (uint32_t p0 = 0; p0 < pieces; p0 += 128) {
-        u32x4 now[2][ROWS];
-#pragma unroll
-        for (int u = 0; u < 2; u++)
-#pragma unroll
-            for (int r = 0; r < ROWS; r++) now[u][r] = cur[u][r];
-        if (p0 + 128 < pieces) load(p0 + 128);
-#pragma unroll
-        for (int u = 0; u < 2; u++) {
-            const u32x4 hv = act[p0 + u * 64 + lane];
-#pragma unroll
-            for (int r = 0; r < ROWS; r++) acc[r] = dot_piece<T>(now[u][r], hv, acc[r]);
-        }
-    }
-    float mine = 0.0f;
-#pragma unroll
-    for (int r = 0; r < ROWS; r++) {
-        const float s = wave_sum_f32(acc[r]);
-        if (lane == uint32_t(r)) mine = s;
-    }
-    const uint32_t at = row0 + lane - seg.row0;
-    if (lane >= ROWS || row0 + lane >= rs.n_rows || at >= seg.n) return;
-    const float o = apply_act<T>(seg.act, mine, seg.bias ? seg.bias[at] : 0.0f, seg.lower ? seg.lower[at] : 0.0f);
-    if (seg.out_elem)
-        static_cast<T *>(seg.y)[at] = from_f32<T>(o);
-    else
-        static_cast<float *>(seg.y)[at] = o;
-}
-
-// A workgroup takes ROWS rows, each wave a quarter of their columns, so that a long row is in flight at once; the
-// waves' sums meet in LDS.  A lane's products count with the gate and scale of the column segment its piece lies in.
-template <typename T, int ROWS>
-__global__ __launch_bounds__(256) void gemv_residual_kernel(const T *__restrict__ w, uint32_t k_pad, uint32_t ld, const T *__restrict__ a,
-                                                            RmiColSegs cs, float *__restrict__ x, uint32_t width) {
-    constexpr int U = 4;
-    __shared__ float part[4][ROWS];
-    const uint32_t tid = threadIdx.x, lane = tid & 63, wave = uint32_t(__builtin_amdgcn_readfirstlane(int(tid >> 6)));
-    const uint32_t row0 = blockIdx.x * ROWS;
-    const uint32_t pieces = k_pad / kPieceElems<T>, per_wave = ((pieces + 3) / 4 + 63) / 64 * 64;
-    const uint32_t p_begin = wave * per_wave, p_end = p_begin + per_wave < pieces ? p_begin + per_wave : pieces;
-    const u32x4 *src[ROWS], *hsrc = reinterpret_cast<const u32x4 *>(a);
-    float gate[ROWS][kMaxColSegs];
-#pragma unroll
-    for (int r = 0; r < ROWS; r++) {
-        const uint32_t row = row0 + r < width ? row0 + r : width - 1;
-        src[r] = reinterpret_cast<const u32x4 *>(w + size_t(row) * ld);
-#pragma unroll
-        for (uint32_t i = 0; i < kMaxColSegs; i++) gate[r][i] = i < cs.n_segs ? (cs.s[i].gate ? cs.s[i].gate[row] : 1.0f) * cs.s[i].scale : 0.0f;
-    }
-    float acc[ROWS];
-#pragma unroll
-    for (int r = 0; r < ROWS; r++) acc[r] = 0.0f;
-    u32x4 cur[U][ROWS], hcur[U];
-    auto load = [&](uint32_t p0) {
-#pragma unroll
-        for (int u = 0; u < U; u++) {
-            const uint32_t p = p0 + u * 64 + lane, pc = p < p_end ? p : pieces - 1;
-            hcur[u] = hsrc[pc];
-#pragma unroll
-            for (int r = 0; r < ROWS; r++) cur[u][r] = src[r][pc];
-        }
-    };
-    if (p_begin < p_end) load(p_begin);
-    for (uint32_t p0 = p_begin; p0 < p_end; p0 += 64 * U) {
-        u32x4 now[U][ROWS], hv[U];
-#pragma unroll
-        for (int u = 0; u < U; u++) {
-            hv[u] = hcur[u];
-#pragma unroll
-            for (int r = 0; r < ROWS; r++) now[u][r] = cur[u][r];
-        }
-        if (p0 + 64 * U < p_end) load(p0 + 64 * U);
-#pragma unroll
-        for (int u = 0; u < U; u++) {
-            const uint32_t p = p0 + u * 64 + lane, k = p * kPieceElems<T>;
-            const bool live = p < p_end;
-#pragma unroll
-            for (int r = 0; r < ROWS; r++) {
-                float f = gate[r][0];
-#pragma unroll
-                for (uint32_t i = 0; i + 1 < kMaxColSegs; i++) f = i + 1 < cs.n_segs && k >= cs.s[i].k_end ? gate[r][i + 1] : f;
-                const float d = dot_piece<T>(now[u][r], hv[u], 0.0f);
-                acc[r] = __builtin_fmaf(f, live ? d : 0.0f, acc[r]);
-            }
-        }
-    }
-#pragma unroll
-    for (int r = 0; r < ROWS; r++) {
-        const float t = wave_sum_f32(acc[r]);
-        if (lane == 0) part[wave][r] = t;
-    }
-    __syncthreads();
-    if (tid < ROWS && row0 + tid < width) x[row0 + tid] += (part[0][tid] + part[1][tid]) + (part[2][tid] + part[3][tid]);
-}
-
-constexpr uint32_t kNormGemvMaxN = 16384;  // what a workgroup keeps of x in registers
-
-template <typename T, int R>
-int norm_gemv_r(const RmiDense &w, const float *x, const float *weight, float eps, uint32_t n, const RmiRowSegs &segs, hipStream_t st) {
-    const size_t lds = size_t(gemv_lds_pieces<T>(w.k_pad)) * 16;
-    constexpr int kRows = 4;
-    const int rc = rmi_allow_lds(norm_gemv_kernel<T, kRows, R>, lds);
-    if (rc != RMI_HIP_OK) return rc;
-    hipLaunchKernelGGL((norm_gemv_kernel<T, kRows, R>), dim3((w.n_rows + 4 * kRows - 1) / (4 * kRows)), dim3(256), lds, st,
-                       static_cast<const T *>(w.data), w.k_pad, w.ld, x, weight, eps, n, segs);
-    RMI_HIP_CHECK(hipGetLastError());
-    return RMI_HIP_OK;
-}
-template <typename T>
-int norm_gemv(const RmiDense &w, const float *x, const float *weight, float eps, uint32_t n, const RmiRowSegs &segs, hipStream_t st) {
-    if (!rmi_dense_gemv_fits(sizeof(T), w.k_pad)) return rmi_fail(RMI_HIP_E_INVALID, "%u columns exceed what the GEMV holds", w.k_pad);
-    if (n <= 1024) return norm_gemv_r<T, 1>(w, x, weight, eps, n, segs, st);
-    if (n <= 4096) return norm_gemv_r<T, 4>(w, x, weight, eps, n, segs, st);
-    return norm_gemv_r<T, 16>(w, x, weight, eps, n, segs, st);
-}
-
-template <typename T>
-int gemv_residual(const RmiDense &w, const void *a, const RmiColSegs &segs, float *x, uint32_t width, hipStream_t st) {
-    constexpr int kRows = 2;
-    hipLaunchKernelGGL((gemv_residual_kernel<T, kRows>), dim3((width + kRows - 1) / kRows), dim3(256), 0, st,
-                       static_cast<const T *>(w.data), w.k_pad, w.ld, static_cast<const T *>(a), segs, x, width);
-    RMI_HIP_CHECK(hipGetLastError());
-    return RMI_HIP_OK;
-}
-
 }  // namespace
 
-int rmi_dense_norm(uint32_t elem_bytes, const float *x, const uint32_t *rows, const float *weight, float eps, void *h,
-                   uint32_t n_tokens, uint32_t n, uint32_t k_pad, hipStream_t st) {
+int rmi_dense_input(uint32_t elem_bytes, const RmiInput &in, const uint32_t *rows, void *h, uint32_t n_tokens, uint32_t k_pad,
+                    hipStream_t st) {
     if (n_tokens == 0) return RMI_HIP_OK;
-    if (elem_bytes == 2)
-        hipLaunchKernelGGL(norm_kernel<rmi_bf16>, dim3(n_tokens), dim3(256), 0, st, x, rows, weight, eps, static_cast<rmi_bf16 *>(h), n, k_pad, rmi_dense_ld(k_pad, 2));
-    else
-        hipLaunchKernelGGL(norm_kernel<float>, dim3(n_tokens), dim3(256), 0, st, x, rows, weight, eps, static_cast<float *>(h), n, k_pad, rmi_dense_ld(k_pad, 4));
+    int rc = rmi_check_input(in, k_pad, h == nullptr);
+    if (rc != RMI_HIP_OK) return rc;
+    auto go = [&](auto type) {
+        using T = decltype(type);
+        return rmi_input_dispatch(in, [&](auto norm, auto add, auto r) {
+            hipLaunchKernelGGL((input_kernel<T, norm.value, add.value, r.value>), dim3(n_tokens), dim3(256), 0, st, in, rows, static_cast<T *>(h),
+                               k_pad, rmi_dense_ld(k_pad, sizeof(T)));
+            return RMI_HIP_OK;
+        });
+    };
+    rc = elem_bytes == 2 ? go(rmi_bf16()) : go(float());
     RMI_HIP_CHECK(hipGetLastError());
-    return RMI_HIP_OK;
+    return rc;
 }
 
-int rmi_dense_embed(uint32_t elem_bytes, const RmiDense &table, const uint32_t *tok, uint32_t vocab, float scale, float *x,
-                    uint32_t n_tokens, uint32_t n, hipStream_t st) {
+int rmi_dense_embed(uint32_t elem_bytes, const RmiEmbed &e, const uint32_t *tok, uint32_t pos0, uint32_t n_tokens, hipStream_t st) {
     if (n_tokens == 0) return RMI_HIP_OK;
     if (elem_bytes == 2)
-        hipLaunchKernelGGL(embed_kernel<rmi_bf16>, dim3(n_tokens), dim3(256), 0, st, static_cast<const rmi_bf16 *>(table.data), table.ld,
-                           tok, vocab, scale, x, n);
+        hipLaunchKernelGGL(embed_kernel<rmi_bf16>, dim3(n_tokens), dim3(256), 0, st, e, tok, pos0);
     else
-        hipLaunchKernelGGL(embed_kernel<float>, dim3(n_tokens), dim3(256), 0, st, static_cast<const float *>(table.data), table.ld, tok,
-                           vocab, scale, x, n);
+        hipLaunchKernelGGL(embed_kernel<float>, dim3(n_tokens), dim3(256), 0, st, e, tok, pos0);
     RMI_HIP_CHECK(hipGetLastError());
     return RMI_HIP_OK;
 }
 
 int rmi_dense_gemm(uint32_t elem_bytes, const RmiDense &w, const void *a, const RmiRowSegs &segs, uint32_t n_tokens, hipStream_t st) {
     if (n_tokens == 0 || w.n_rows == 0) return RMI_HIP_OK;
-    if (segs.n_rows != w.n_rows || segs.n_segs == 0 || segs.n_segs > kMaxRowSegs || w.k_pad % kDenseKAlign || w.ld != rmi_dense_ld(w.k_pad, elem_bytes))
-        return rmi_fail(RMI_HIP_E_INVALID, "row segments do not fit the weight");
+    const int rc = rmi_check_row_segs(elem_bytes, w, segs);
+    if (rc != RMI_HIP_OK) return rc;
     return elem_bytes == 2 ? launch_gemm<rmi_bf16, false>(w, a, segs, RmiColSegs{}, nullptr, 0, n_tokens, st)
                            : launch_gemm<float, false>(w, a, segs, RmiColSegs{}, nullptr, 0, n_tokens, st);
-}
-
-static int check_col_segs(uint32_t elem_bytes, const RmiDense &w, const RmiColSegs &segs, uint32_t width) {
-    if (w.ld != rmi_dense_ld(w.k_pad, elem_bytes) || segs.n_segs == 0 || segs.n_segs > kMaxColSegs || segs.s[segs.n_segs - 1].k_end != w.k_pad || w.n_rows < width)
-        return rmi_fail(RMI_HIP_E_INVALID, "column segments do not fit the weight");
-    for (uint32_t i = 0; i < segs.n_segs; i++)
-        if (segs.s[i].k_end % kDenseKAlign || segs.s[i].k_end <= (i ? segs.s[i - 1].k_end : 0u))
-            return rmi_fail(RMI_HIP_E_INVALID, "column segments do not fit the weight");
-    return RMI_HIP_OK;
 }
 
 int rmi_dense_gemm_residual(uint32_t elem_bytes, const RmiDense &w, const void *a, const RmiColSegs &segs, float *x, uint32_t width,
                             uint32_t n_tokens, hipStream_t st) {
     if (n_tokens == 0) return RMI_HIP_OK;
-    const int rc = check_col_segs(elem_bytes, w, segs, width);
+    const int rc = rmi_check_col_segs(elem_bytes, w, segs, width);
     if (rc != RMI_HIP_OK) return rc;
     return elem_bytes == 2 ? launch_gemm<rmi_bf16, true>(w, a, RmiRowSegs{}, segs, x, width, n_tokens, st)
                            : launch_gemm<float, true>(w, a, RmiRowSegs{}, segs, x, width, n_tokens, st);
-}
-
-bool rmi_dense_gemv_fits(uint32_t elem_bytes, uint32_t k_pad) {
-    const size_t lds = size_t(elem_bytes == 2 ? gemv_lds_pieces<rmi_bf16>(k_pad) : gemv_lds_pieces<float>(k_pad)) * 16;
-    return lds <= kGemvLdsMax && k_pad <= kNormGemvMaxN;
-}
-
-int rmi_dense_norm_gemv(uint32_t elem_bytes, const RmiDense &w, const float *x, const float *weight, float eps, uint32_t n,
-                        const RmiRowSegs &segs, hipStream_t st) {
-    if (segs.n_rows != w.n_rows || segs.n_segs == 0 || segs.n_segs > kMaxRowSegs || n > w.k_pad)
-        return rmi_fail(RMI_HIP_E_INVALID, "row segments do not fit the weight");
-    return elem_bytes == 2 ? norm_gemv<rmi_bf16>(w, x, weight, eps, n, segs, st) : norm_gemv<float>(w, x, weight, eps, n, segs, st);
-}
-
-int rmi_dense_gemv_residual(uint32_t elem_bytes, const RmiDense &w, const void *a, const RmiColSegs &segs, float *x, uint32_t width,
-                            hipStream_t st) {
-    const int rc = check_col_segs(elem_bytes, w, segs, width);
-    if (rc != RMI_HIP_OK) return rc;
-    return elem_bytes == 2 ? gemv_residual<rmi_bf16>(w, a, segs, x, width, st) : gemv_residual<float>(w, a, segs, x, width, st);
 }

@@ -114,7 +114,10 @@ __device__ __forceinline__ float rcp_t<rmi_bf16>(float z) { return __builtin_amd
 template <typename T>
 __device__ __forceinline__ float sigmoid_t(float z) { return rcp_t<T>(1.0f + exp_t<T>(-z)); }
 
-// What a row segment of a product does with its result z.
+// log(1 + e^z) in full f32
+__device__ __forceinline__ float softplus_f32(float z) { return fmaxf(z, 0.0f) + log1pf(expf(-fabsf(z))); }
+
+// What a row segment of a product does with its result z (kActReluGlu: its two rows, in the epilogues themselves).
 template <typename T>
 __device__ __forceinline__ float apply_act(uint32_t act, float z, float bias, float lower) {
     switch (act) {
@@ -123,8 +126,148 @@ __device__ __forceinline__ float apply_act(uint32_t act, float z, float bias, fl
         case kActGeluTanh:  // z/2 (1 + tanh u) = z sigmoid(2u)
             return z * sigmoid_t<T>(1.59576912160573071176f * __builtin_fmaf(0.044715f * z * z, z, z));
         case kActForgetGate: return __builtin_fmaf(1.0f - lower, sigmoid_t<float>(z + bias), lower);
+        case kActDecay: return expf(-lower * softplus_f32(z + bias));
         default: return z;
     }
 }
+
+// which row segment a row lies in: the starts sit side by side (unused ones at the end of the range)
+__device__ __forceinline__ uint32_t seg_of(const RmiRowSegs &rs, uint32_t row) {
+    uint32_t si = 0;
+#pragma unroll
+    for (uint32_t i = 1; i < kMaxRowSegs; i++) si += row >= rs.start[i] ? 1u : 0u;
+    return si;
+}
+
+// the row of a segment's table that token t of the pass picks (ids past the end read the last row)
+template <typename T>
+__device__ __forceinline__ const T *mul_row(const RmiRowSeg &s, uint32_t t) {
+    const uint32_t id = s.mul_tok[t];
+    return static_cast<const T *>(s.mul) + size_t(id < s.mul_rows ? id : s.mul_rows - 1) * s.mul_ld;
+}
+
+// channel c of a token's embedding at position p (RmiEmbed)
+template <typename T>
+__device__ __forceinline__ float embed_value(const RmiEmbed &e, uint32_t token, uint32_t p, uint32_t c) {
+    if (token >= e.vocab) token = e.vocab - 1;  // ids are validated on the host; never read outside the table
+    float v = to_f32(static_cast<const T *>(e.table)[size_t(token) * e.ld + c]) * e.scale;
+    if (e.turns) {
+        double r = double(p) * e.turns[c >> 1];
+        r -= rint(r);  // the whole turns leave in f64, what stays is exact enough for f32
+        const float a = float(r * 6.283185307179586476925286766559);
+        v += c & 1 ? cosf(a) : sinf(a);
+    }
+    return v;
+}
+
+// ---- a product's input (RmiInput) in the registers of a workgroup of 256: R quads of values a thread, quad j of
+// thread t at 4 (t + 256 j)
+__device__ __forceinline__ float block_sum_f32(float v, float *red) {  // red: four floats of this sum's own
+    v = wave_sum_f32(v);
+    if ((threadIdx.x & 63) == 0) red[threadIdx.x >> 6] = v;
+    __syncthreads();
+    return (red[0] + red[1]) + (red[2] + red[3]);
+}
+template <int NORM, bool ADD, int R>
+struct InputRow {
+    f32x4 v[R];
+    f32x4 w[NORM != kNormNone ? R : 1], y[ADD ? R : 1], yw[ADD ? R : 1];
+
+    static __device__ __forceinline__ f32x4 quad(const float *p, uint32_t i, uint32_t n, bool quads) {
+        if (quads) return *reinterpret_cast<const f32x4 *>(p + (i < n ? i : n - 4));
+        f32x4 r;
+#pragma unroll
+        for (uint32_t e = 0; e < 4; e++) r[e] = p[i + e < n ? i + e : n - 1];
+        return r;
+    }
+    // all loads, none waited for
+    __device__ __forceinline__ void load(const RmiInput &in, uint32_t row) {
+        const bool quads = (in.n & 3) == 0;
+#pragma unroll
+        for (int j = 0; j < R; j++) {
+            const uint32_t i = (threadIdx.x + j * 256) * 4;
+            v[j] = quad(in.x + size_t(row) * in.n, i, in.n, quads);
+            if constexpr (ADD) {
+                y[j] = quad(in.y + size_t(row) * in.n, i, in.n, quads);
+                yw[j] = quad(in.y_weight, i, in.n, quads);
+            }
+            if constexpr (NORM != kNormNone) w[j] = quad(in.weight, i, in.n, quads);
+        }
+    }
+    // v = the operand, zero past its end; write: v before the norm goes to x_out.  red: twelve floats of LDS
+    __device__ __forceinline__ void finish(const RmiInput &in, uint32_t row, bool write, float *red) {
+        const float n = float(in.n);
+        if constexpr (ADD) {
+            float sq = 0.0f;
+#pragma unroll
+            for (int j = 0; j < R; j++)
+#pragma unroll
+                for (int e = 0; e < 4; e++)
+                    if ((threadIdx.x + j * 256) * 4 + e < in.n) sq = __builtin_fmaf(y[j][e], y[j][e], sq);
+            const float r = 1.0f / sqrtf(block_sum_f32(sq, red) / n + in.y_eps);
+#pragma unroll
+            for (int j = 0; j < R; j++)
+#pragma unroll
+                for (int e = 0; e < 4; e++) v[j][e] = __builtin_fmaf(y[j][e] * r, yw[j][e], v[j][e]);
+        }
+#pragma unroll
+        for (int j = 0; j < R; j++) {
+            const uint32_t i = (threadIdx.x + j * 256) * 4;
+            if (ADD && write) {
+                float *dst = in.x_out + size_t(row) * in.n + i;
+                if ((in.n & 3) == 0) {
+                    if (i < in.n) *reinterpret_cast<f32x4 *>(dst) = v[j];
+                } else {
+#pragma unroll
+                    for (uint32_t e = 0; e < 4; e++)
+                        if (i + e < in.n) dst[e] = v[j][e];
+                }
+            }
+#pragma unroll
+            for (uint32_t e = 0; e < 4; e++)
+                if (i + e >= in.n) v[j][e] = 0.0f;
+        }
+        if constexpr (NORM == kNormLayer) {
+            float sum = 0.0f;
+#pragma unroll
+            for (int j = 0; j < R; j++) sum += (v[j][0] + v[j][1]) + (v[j][2] + v[j][3]);
+            const float mean = block_sum_f32(sum, red + 4) / n;
+#pragma unroll
+            for (int j = 0; j < R; j++)
+#pragma unroll
+                for (uint32_t e = 0; e < 4; e++) v[j][e] = (threadIdx.x + j * 256) * 4 + e < in.n ? v[j][e] - mean : 0.0f;
+        }
+        if constexpr (NORM != kNormNone) {
+            float sq = 0.0f;
+#pragma unroll
+            for (int j = 0; j < R; j++)
+#pragma unroll
+                for (int e = 0; e < 4; e++) sq = __builtin_fmaf(v[j][e], v[j][e], sq);
+            const float r = 1.0f / sqrtf(block_sum_f32(sq, red + 8) / n + in.eps);
+#pragma unroll
+            for (int j = 0; j < R; j++) v[j] = v[j] * r * w[j];
+        }
+    }
+    // the operand as T to dst[0 .. k), k a multiple of 256
+    template <typename T>
+    __device__ __forceinline__ void store(const RmiInput &in, uint32_t row, T *dst, uint32_t k) {
+        const uint32_t k1 = in.x2 ? in.k2 : k;
+#pragma unroll
+        for (int j = 0; j < R; j++) {
+            const uint32_t i = (threadIdx.x + j * 256) * 4;
+            if (i < k1) store4(dst + i, v[j]);
+        }
+        for (uint32_t i = (threadIdx.x + R * 256) * 4; i < k1; i += 1024) store4(dst + i, f32x4{0.f, 0.f, 0.f, 0.f});
+        if (!in.x2) return;
+        const float *x2 = in.x2 + size_t(row) * in.n2;
+        for (uint32_t i = threadIdx.x * 4; i < k - k1; i += 1024) {
+            f32x4 b = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+            for (uint32_t e = 0; e < 4; e++)
+                if (i + e < in.n2) b[e] = x2[i + e];
+            store4(dst + k1 + i, b);
+        }
+    }
+};
 
 #endif  // RMI_DEVICE_DENSE_H

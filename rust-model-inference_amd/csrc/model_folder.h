@@ -37,3 +37,5 @@ struct RmiModelFolder {
 bool rmi_read_config(const char *dir, RmiJson *out);
 // element i of a bf16 / f16 / f32 tensor's data as f32
 float rmi_tensor_f32(const RmiTensor &t, uint64_t i);
+// elements at .. at + n - 1 as bf16, to nearest even
+void rmi_tensor_bf16(const RmiTensor &t, uint64_t at, uint64_t n, uint16_t *dst);

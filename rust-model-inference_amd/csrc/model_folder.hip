@@ -130,6 +130,19 @@ float rmi_tensor_f32(const RmiTensor &t, uint64_t i) {
     }
 }
 
+void rmi_tensor_bf16(const RmiTensor &t, uint64_t at, uint64_t n, uint16_t *dst) {
+    if (t.dtype == RmiTensor::kBf16) {
+        memcpy(dst, t.data + 2 * at, 2 * n);
+        return;
+    }
+    for (uint64_t i = 0; i < n; i++) {
+        const float v = rmi_tensor_f32(t, at + i);
+        uint32_t b;
+        memcpy(&b, &v, 4);
+        dst[i] = uint16_t((b + 0x7fff + ((b >> 16) & 1)) >> 16);
+    }
+}
+
 extern "C" int64_t rmi_hip_model_folder_architecture(const char *dir, char *buf, size_t cap) {
     RmiJson c;
     if (!dir || !rmi_read_config(dir, &c)) return -1;

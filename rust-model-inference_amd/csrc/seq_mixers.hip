@@ -1,6 +1,7 @@
 // Mixers over time (seq_mixers.h): kernels for passes of several tokens and for single tokens.
 #include "seq_mixers.h"
 
+#include "device_conv.h"
 #include "device_dense.h"
 
 namespace {
@@ -15,32 +16,6 @@ __device__ __forceinline__ uint32_t value_slot(uint32_t k) {
 }
 
 // ---- convolution, rotation, value norm
-struct ConvCtx {
-    const float *u, *hist, *conv;
-    uint32_t channels, taps;
-};
-// the convolved channel `c` of the pass's token t
-__device__ __forceinline__ float conv_at(const ConvCtx &x, uint32_t t, uint32_t pos0, uint32_t c) {
-    float y = 0.0f;
-    for (uint32_t j = 0; j < x.taps; j++) {
-        const uint32_t back = x.taps - 1 - j;  // position pos0 + t - back
-        float s = 0.0f;
-        if (t >= back)
-            s = x.u[size_t(t - back) * x.channels + c];
-        else if (pos0 + t >= back)
-            s = x.hist[size_t(t + j) * x.channels + c];  // row t - back + (taps - 1)
-        y = __builtin_fmaf(x.conv[c * x.taps + j], s, y);
-    }
-    return y;
-}
-// channel c's row of the history behind the pass: position pos0 + n_tokens - (taps - 1) + j, j = 0 .. taps - 2
-__device__ __forceinline__ void conv_carry(const ConvCtx &x, float *hist_out, uint32_t n_tokens, uint32_t c) {
-    for (uint32_t j = 0; j + 1 < x.taps; j++) {
-        const uint32_t at = n_tokens + j;  // row `at` of history followed by the pass's rows
-        hist_out[size_t(j) * x.channels + c] = at >= x.taps - 1 ? x.u[size_t(at - (x.taps - 1)) * x.channels + c]
-                                                                : x.hist[size_t(at) * x.channels + c];
-    }
-}
 // elements 2i, 2i + 1 of a query or key head whose channels start at c0, convolved and rotated
 __device__ __forceinline__ void conv_rotate_pair(const ConvCtx &x, const RmiAttnShape &s, const float *cos_t, const float *sin_t,
                                                  uint32_t t, uint32_t pos0, uint32_t c0, uint32_t i, float &a, float &b) {
@@ -67,7 +42,7 @@ __device__ __forceinline__ void store_pair<rmi_bf16>(rmi_bf16 *p, float a, float
 // one wave: key head g of token t to its cache row
 template <typename T>
 __device__ __forceinline__ void key_row(const ConvCtx &x, const RmiAttnShape &s, const RmiAttnArgs &a, uint32_t t, uint32_t g, uint32_t lane) {
-    T *row = static_cast<T *>(a.k_cache) + (size_t(g) * s.capacity + a.pos0 + t) * s.dk_pad;
+    T *row = static_cast<T *>(a.k_cache) + (size_t(g) * s.capacity + (a.pos0 + t) % s.capacity) * s.dk_pad;
     const uint32_t c0 = (s.heads + g) * s.dim;
     for (uint32_t i = lane; i < s.dk_pad / 2; i += 64) {
         float p, q;
@@ -86,8 +61,8 @@ __device__ __forceinline__ void value_row(const ConvCtx &x, const RmiAttnShape &
         v[j] = d < s.vdim ? conv_at(x, t, a.pos0, c0 + d) : 0.0f;
         sq = __builtin_fmaf(v[j], v[j], sq);
     }
-    const float r = 1.0f / sqrtf(wave_sum_f32(sq) / float(s.vdim) + s.eps);
-    const uint32_t pos = a.pos0 + t;
+    const float r = s.v_norm ? 1.0f / sqrtf(wave_sum_f32(sq) / float(s.vdim) + s.eps) : 1.0f;
+    const uint32_t pos = (a.pos0 + t) % s.capacity;
     T *blk = static_cast<T *>(a.v_cache) + (size_t(g) * (s.capacity / kKeyBlock) + pos / kKeyBlock) * s.dv_pad * kKeyBlock +
              value_slot<T>(pos % kKeyBlock);
 #pragma unroll
@@ -193,7 +168,7 @@ __global__ __launch_bounds__(256) void conv_rotate_pairs_kernel(RmiAttnShape s, 
         out = static_cast<T *>(a.q) + (size_t(head / group) * a.n_tokens * group + size_t(t0) * group + head % group) * s.dk_pad;
         step = size_t(group) * s.dk_pad;
     } else {
-        out = static_cast<T *>(a.k_cache) + (size_t(head - s.heads) * s.capacity + a.pos0 + t0) * s.dk_pad;
+        out = static_cast<T *>(a.k_cache) + (size_t(head - s.heads) * s.capacity + (a.pos0 + t0) % s.capacity) * s.dk_pad;  // (a run does not wrap)
         step = s.dk_pad;
     }
     float v0[kConvRun], v1[kConvRun];
@@ -218,7 +193,7 @@ __global__ __launch_bounds__(256) void conv_rotate_pairs_kernel(RmiAttnShape s, 
         }
         if (!has) p = q = 0.0f;
         if (is_v) {
-            const float r = 1.0f / sqrtf(wave_sum_f32(__builtin_fmaf(p, p, q * q)) / float(dim) + s.eps);
+            const float r = s.v_norm ? 1.0f / sqrtf(wave_sum_f32(__builtin_fmaf(p, p, q * q)) / float(dim) + s.eps) : 1.0f;
             v0[i] = p * r;
             v1[i] = q * r;
         } else {
@@ -233,7 +208,8 @@ __global__ __launch_bounds__(256) void conv_rotate_pairs_kernel(RmiAttnShape s, 
     }
     if (is_v && has) {
         T *blk = static_cast<T *>(a.v_cache) +
-                 (size_t(head - s.heads - s.kv_heads) * (s.capacity / kKeyBlock) + p_run / kKeyBlock) * s.dv_pad * kKeyBlock + size_t(2 * lane) * kKeyBlock;
+                 (size_t(head - s.heads - s.kv_heads) * (s.capacity / kKeyBlock) + p_run % s.capacity / kKeyBlock) * s.dv_pad * kKeyBlock +
+                 size_t(2 * lane) * kKeyBlock;
 #pragma unroll
         for (uint32_t g = 0; g < kConvRun; g += 4) {  // four keys lie side by side
             T *dst = blk + value_slot<T>((p_run + g) % kKeyBlock);
@@ -301,17 +277,19 @@ struct AttnWave {
             for (uint32_t t = 0; t < sizeof(T) / 2; t++)
                 if (v < n_vt) vf[v * (sizeof(T) / 2) + t] = *reinterpret_cast<const u32x4 *>(vb + size_t(v) * 16 * kKeyBlock + t * 16);
     }
-    // keys [k0, k1), k0 a multiple of 32; column i sees keys up to last[i] (< k1 not required).  loaded: the first
-    // block's keys and values are in kf and vf
+    // keys [k0, k1), k0 a multiple of 32; column i sees keys up to last[i] (< k1 not required) and, with a window, from
+    // last[i] - window + 1 on.  loaded: the first block's keys and values are in kf and vf
     __device__ __forceinline__ void keys(const T *kc, const T *vc, const RmiAttnShape &s, uint32_t k0, uint32_t k1, const int (&last)[QT],
                                          bool loaded = false) {
         const uint32_t lane = threadIdx.x & 63, fr = lane & 15, g = lane >> 4;
         const uint32_t n_kc = s.dk_pad / (4 * kPieceElems<T>), n_vt = s.dv_pad / 16;
         const T *krow = kc + size_t(fr) * s.dk_pad + g * kPieceElems<T>;
-        if (!loaded && k0 < k1) load_keys(kc, s, k0);
+        uint32_t row = k0 % s.capacity;  // where the block lies
+        if (!loaded && k0 < k1) load_keys(kc, s, row);
         for (uint32_t k = k0; k < k1; k += kKeyBlock) {
-            const T *vb = value_at(vc, s, k);
-            if (!loaded || k != k0) load_values(vc, s, k);
+            const T *vb = value_at(vc, s, row);
+            if (!loaded || k != k0) load_values(vc, s, row);
+            const uint32_t next = row + kKeyBlock < s.capacity ? row + kKeyBlock : 0;
             f32x4 sc[QT][2];
 #pragma unroll
             for (int i = 0; i < QT; i++) sc[i][0] = sc[i][1] = f32x4{0.f, 0.f, 0.f, 0.f};
@@ -323,7 +301,7 @@ struct AttnWave {
                     f0 = kf[0][c];
                     f1 = kf[1][c];
                 } else {
-                    const T *p = krow + size_t(k) * s.dk_pad + c * 4 * kPieceElems<T>;
+                    const T *p = krow + size_t(row) * s.dk_pad + c * 4 * kPieceElems<T>;
                     f0 = *reinterpret_cast<const u32x4 *>(p);
                     f1 = *reinterpret_cast<const u32x4 *>(p + 16 * size_t(s.dk_pad));
                 }
@@ -333,17 +311,19 @@ struct AttnWave {
                     sc[i][1] = mma16<T>(f1, qf[i][c], sc[i][1]);
                 }
             }
-            if (k + kKeyBlock < k1) load_keys(kc, s, k + kKeyBlock);
+            if (k + kKeyBlock < k1) load_keys(kc, s, next);
+            row = next;
             u32x4 pf[QT][2];
 #pragma unroll
             for (int i = 0; i < QT; i++) {
                 float top = -INFINITY;
+                const int first = s.window ? last[i] - int(s.window) + 1 : 0;
 #pragma unroll
                 for (int t = 0; t < 2; t++)
 #pragma unroll
                     for (int r = 0; r < 4; r++) {
                         const int key = int(k) + t * 16 + int(g) * 4 + r;
-                        sc[i][t][r] = key <= last[i] && key < int(k1) ? sc[i][t][r] * s.scale : -INFINITY;
+                        sc[i][t][r] = key >= first && key <= last[i] && key < int(k1) ? sc[i][t][r] * s.scale : -INFINITY;
                         top = fmaxf(top, sc[i][t][r]);
                     }
                 const float m_new = fmaxf(m[i], rows_max_f32(top));
@@ -386,6 +366,11 @@ struct AttnWave {
     }
 };
 
+// the block in which the first key lies that position p sees
+__device__ __forceinline__ uint32_t first_block(const RmiAttnShape &s, uint32_t p) {
+    return s.window && p + 1 > s.window ? (p + 1 - s.window) / kKeyBlock * kKeyBlock : 0;
+}
+
 // four channels d .. d + 3 of a finished column
 template <typename T>
 __device__ __forceinline__ void attn_store(const RmiAttnShape &s, const RmiAttnArgs &a, uint32_t t, uint32_t head, uint32_t d, f32x4 v) {
@@ -422,9 +407,9 @@ __global__ __launch_bounds__(256) void attn_pass_kernel(RmiAttnShape s, RmiAttnA
         }
     }
     const uint32_t first_col = tile * QT * 16, live = n_cols - first_col < QT * 16 ? n_cols - first_col : QT * 16;
-    const uint32_t n_keys = a.pos0 + (first_col + live - 1) / group + 1;
-    const uint32_t per_wave = (n_keys + 4 * kKeyBlock - 1) / (4 * kKeyBlock) * kKeyBlock;
-    const uint32_t k0 = wave * per_wave, k1 = k0 + per_wave < n_keys ? k0 + per_wave : n_keys;
+    const uint32_t n_keys = a.pos0 + (first_col + live - 1) / group + 1, begin = first_block(s, a.pos0 + first_col / group);
+    const uint32_t per_wave = (n_keys - begin + 4 * kKeyBlock - 1) / (4 * kKeyBlock) * kKeyBlock;
+    const uint32_t k0 = begin + wave * per_wave, k1 = k0 + per_wave < n_keys ? k0 + per_wave : n_keys;
     if (k0 < k1)
         w.keys(static_cast<const T *>(a.k_cache) + size_t(kvh) * s.capacity * s.dk_pad,
                static_cast<const T *>(a.v_cache) + size_t(kvh) * s.capacity * s.dv_pad, s, k0, k1, last);
@@ -449,7 +434,7 @@ __global__ __launch_bounds__(256) void attn_pass_kernel(RmiAttnShape s, RmiAttnA
         float m = all[c];
 #pragma unroll
         for (uint32_t i = 1; i < 4; i++) m = fmaxf(m, all[i * pl + c]);
-        float sum = 0.0f;  // (every column sees key 0: m is finite)
+        float sum = 0.0f;  // (every column sees its own key: m is finite)
         f32x4 o = {0.f, 0.f, 0.f, 0.f};
 #pragma unroll
         for (uint32_t i = 0; i < 4; i++) {
@@ -477,7 +462,8 @@ __device__ __forceinline__ void attn_split(const RmiAttnShape &s, const RmiAttnA
     const uint32_t tid = threadIdx.x, lane = tid & 63, wave = uint32_t(__builtin_amdgcn_readfirstlane(int(tid >> 6))), fr = lane & 15, g4 = lane >> 4;
     const uint32_t group = s.heads / s.kv_heads, n_cols = a.n_tokens * group, tiles = (n_cols + 15) / 16;
     const uint32_t part = block % parts, ct = (block / parts) % tiles, kvh = block / parts / tiles;
-    const uint32_t n_keys = a.pos0 + a.n_tokens;
+    const uint32_t last_col = ct * 16 + 15 < n_cols ? ct * 16 + 15 : n_cols - 1;
+    const uint32_t begin = first_block(s, a.pos0 + ct * 16 / group), n_keys = a.pos0 + last_col / group + 1;  // what the tile sees
     const uint32_t n_kc = s.dk_pad / (4 * kPieceElems<T>);
     AttnWave<T, BUCKET, 1> w;
     w.init();
@@ -485,7 +471,7 @@ __device__ __forceinline__ void attn_split(const RmiAttnShape &s, const RmiAttnA
     const int last[1] = {int(a.pos0 + cc / group)};
     const T *kc = static_cast<const T *>(a.k_cache) + size_t(kvh) * s.capacity * s.dk_pad;
     const T *vc = static_cast<const T *>(a.v_cache) + size_t(kvh) * s.capacity * s.dv_pad;
-    const uint32_t p0 = part * keys_per_part, p1 = p0 + keys_per_part < n_keys ? p0 + keys_per_part : n_keys;
+    const uint32_t p0 = begin + part * keys_per_part, p1 = p0 + keys_per_part < n_keys ? p0 + keys_per_part : n_keys;
     const uint32_t per_wave = keys_per_part / NW;  // a multiple of the key block
     const uint32_t k0 = p0 + wave * per_wave, k1 = k0 + per_wave < p1 ? k0 + per_wave : p1;
     bool loaded = false;
@@ -494,13 +480,14 @@ __device__ __forceinline__ void attn_split(const RmiAttnShape &s, const RmiAttnA
         const uint32_t channels = (s.heads + s.kv_heads) * s.dim + s.kv_heads * s.vdim;
         const ConvCtx x{a.u, a.hist_in, a.conv, channels, s.taps};
         const uint32_t half = s.dk_pad / 2, c_end = n_cols - ct * 16 < 16 ? n_cols - ct * 16 : 16;
-        const bool newest = part == parts - 1;  // this part holds the token's own key and value
+        const uint32_t own = a.pos0 % s.capacity;
+        const bool newest = a.pos0 - p0 < keys_per_part;  // this part holds the token's own key and value
         // the first block of keys and values: under way behind the convolution's operands, unless it holds the new one
         auto ahead = [&] {
             loaded = w.kAhead && k0 < k1 && k0 + kKeyBlock < n_keys;
             if (loaded) {
-                w.load_keys(kc, s, k0);
-                w.load_values(vc, s, k0);
+                w.load_keys(kc, s, k0 % s.capacity);
+                w.load_values(vc, s, k0 % s.capacity);
             }
         };
         if (conv_pairs_fit(s)) {
@@ -535,8 +522,8 @@ __device__ __forceinline__ void attn_split(const RmiAttnShape &s, const RmiAttnA
                 }
                 if (!has) p = o = 0.0f;
                 if (is_v) {  // (at most 64 pairs: one round)
-                    const float f = 1.0f / sqrtf(wave_sum_f32(__builtin_fmaf(p, p, o * o)) / float(s.vdim) + s.eps);
-                    T *blk = const_cast<T *>(vc) + size_t(a.pos0 / kKeyBlock) * s.dv_pad * kKeyBlock + value_slot<T>(a.pos0 % kKeyBlock);
+                    const float f = s.v_norm ? 1.0f / sqrtf(wave_sum_f32(__builtin_fmaf(p, p, o * o)) / float(s.vdim) + s.eps) : 1.0f;
+                    T *blk = const_cast<T *>(vc) + size_t(own / kKeyBlock) * s.dv_pad * kKeyBlock + value_slot<T>(own % kKeyBlock);
                     if (has) {
                         blk[size_t(2 * i) * kKeyBlock] = from_f32<T>(p * f);
                         blk[size_t(2 * i + 1) * kKeyBlock] = from_f32<T>(o * f);
@@ -545,7 +532,7 @@ __device__ __forceinline__ void attn_split(const RmiAttnShape &s, const RmiAttnA
                     const float rp = p;
                     p = __builtin_fmaf(rp, cs, -(o * sn));
                     o = __builtin_fmaf(o, cs, rp * sn);
-                    store_pair(is_k ? const_cast<T *>(kc) + size_t(a.pos0) * s.dk_pad + 2 * i : q + c * s.dk_pad + 2 * i, p, o);
+                    store_pair(is_k ? const_cast<T *>(kc) + size_t(own) * s.dk_pad + 2 * i : q + c * s.dk_pad + 2 * i, p, o);
                 }
             }
         } else {
@@ -970,7 +957,10 @@ __global__ __launch_bounds__(256) void recur_norm_kernel(RmiRecurShape s, RmiRec
 // Keys over workgroups where the columns alone would not fill the chip; at most kMaxParts parts of 128 keys or more.
 constexpr uint32_t kSplitMaxCols = 256;  // per key/value head
 void attn_parts(const RmiAttnShape &s, uint32_t n_tokens, uint32_t n_keys, uint32_t *parts, uint32_t *keys_per_part) {
-    const uint32_t tiles = (n_tokens * (s.heads / s.kv_heads) + 15) / 16;
+    const uint32_t group = s.heads / s.kv_heads, tiles = (n_tokens * group + 15) / 16;
+    // the most that a tile of sixteen columns sees, from a block's edge on
+    const uint64_t seen = s.window ? uint64_t(s.window) + 15 / group + 1 + kKeyBlock : n_keys;
+    if (seen < n_keys) n_keys = uint32_t(seen);
     const uint32_t slots = s.kv_heads * tiles, cus = uint32_t(rmi_device_cus());
     uint32_t p = (n_keys + 127) / 128;
     const uint32_t fill = (cus + slots - 1) / slots;
@@ -985,7 +975,8 @@ void attn_parts(const RmiAttnShape &s, uint32_t n_tokens, uint32_t n_keys, uint3
 int check_attn(const RmiAttnShape &s, const RmiAttnArgs &a) {
     if (s.dim > kMaxHeadDim || s.vdim > kMaxHeadDim || s.taps == 0 || s.taps > kMaxTaps || s.heads % s.kv_heads || s.rot_dims > s.dim ||
         s.rot_dims % 2 || s.capacity % kKeyBlock || s.dk_pad % 32 || s.dv_pad % 16 || s.dk_pad < s.dim || s.dv_pad < s.vdim ||
-        s.dk_pad > kMaxHeadDim || s.dv_pad > kMaxHeadDim || a.pos0 + a.n_tokens > s.capacity)
+        s.dk_pad > kMaxHeadDim || s.dv_pad > kMaxHeadDim || s.capacity == 0 ||
+        (uint64_t(a.pos0) + a.n_tokens > s.capacity && (s.window == 0 || uint64_t(s.window) - 1 + a.n_tokens > s.capacity)))
         return rmi_fail(RMI_HIP_E_INVALID, "bad attention shape");
     return RMI_HIP_OK;
 }

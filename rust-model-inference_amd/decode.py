@@ -1,6 +1,6 @@
 """Decoder sessions over the device-resident entry points of the C ABI: weights go to HBM once, then whole
 generations run on the GPU with one synchronisation at the end.  ``Qwen3Session`` mirrors the reference's
-(src/models/qwen3.rs:581-1158); ``RuvenexSession`` runs a model folder of that design; ``models`` picks the class.
+(src/models/qwen3.rs:581-1158); the ``FolderSession`` classes run model folders; ``models`` picks the class.
 """
 import ctypes as C
 
@@ -30,7 +30,7 @@ class _Session:
     def set_prompt_passes(self, enabled):
         """Prompt positions as many to a pass as the session takes (True, the default), every position its own step
         (False), or that many to a pass (an int above 1); same results either way (bit for bit for Qwen3, within
-        rounding for Ruvenex)."""
+        rounding for model folders)."""
         hip.check(self._fn("set_prompt_passes")(self._h, int(enabled)))
 
     def generate(self, prompt, max_new, dump_steps=()):
@@ -122,33 +122,47 @@ class Qwen3Session(_Session):
         return self
 
 
-class RuvenexSession(_Session):
-    """A Ruvenex model folder (config.json, model.safetensors).  dtype: hip.DTYPE_BF16 or hip.DTYPE_F32 (everything
-    true f32); capacity: most tokens of a sequence.  One sequence at a time."""
+class FolderSession(_Session):
+    """A model folder (config.json, model.safetensors) of any design the library knows.  dtype: hip.DTYPE_BF16 or
+    hip.DTYPE_F32 (everything true f32); capacity: most tokens of a sequence.  One sequence at a time."""
 
-    _abi = "ruvenex"
+    _abi = "folder"
+    architecture = None  # the one that config.json has to name
 
     def __init__(self, folder, capacity, dtype=hip.DTYPE_BF16):
-        self._h = hip.lib.rmi_hip_ruvenex_open(str(folder).encode(), dtype, int(capacity))
+        arch = self.architecture.encode() if self.architecture else None
+        self._h = hip.lib.rmi_hip_folder_open(str(folder).encode(), arch, dtype, int(capacity))
         if not self._h:
             raise hip.RmiHipError(-1, hip.last_error())
         v = [C.c_uint32() for _ in range(4)]
-        hip.check(hip.lib.rmi_hip_ruvenex_sizes(self._h, *[C.byref(x) for x in v]))
+        hip.check(hip.lib.rmi_hip_folder_sizes(self._h, *[C.byref(x) for x in v]))
         self.vocab, self.width, self.n_layer, self.capacity = (x.value for x in v)
 
-    position = property(lambda self: hip.lib.rmi_hip_ruvenex_position(self._h))
+    position = property(lambda self: hip.lib.rmi_hip_folder_position(self._h))
 
     def step(self, tokens, want=(), layers=False):
         """The sequence's next tokens; logits [len(want), vocab] of the places `want` among them.  With `layers` also
-        the residual stream behind every layer, [n_layer, tokens, width]."""
+        the residual stream behind every layer, [n_layer, tokens, width] (a looped layer counts each time)."""
         tokens = np.ascontiguousarray(tokens, np.uint32)
         want = np.ascontiguousarray(want, np.uint32)
         logits = np.zeros((want.size, self.vocab), np.float32)
         dump = np.zeros((self.n_layer, tokens.size, self.width), np.float32) if layers else None
-        hip.check(hip.lib.rmi_hip_ruvenex_step(self._h, hip.ptr(tokens, hip._u32p), tokens.size, hip.ptr(want, hip._u32p), want.size,
+        hip.check(hip.lib.rmi_hip_folder_step(self._h, hip.ptr(tokens, hip._u32p), tokens.size, hip.ptr(want, hip._u32p), want.size,
                                                hip.ptr(logits, hip._f32p), hip.ptr(dump, hip._f32p) if layers else None))
         return (logits, dump) if layers else logits
 
     def reset(self):
         """The sequence is over; the next step begins a new one."""
-        hip.check(hip.lib.rmi_hip_ruvenex_reset(self._h))
+        hip.check(hip.lib.rmi_hip_folder_reset(self._h))
+
+
+class RuvenexSession(FolderSession):
+    """Parallel layers of softmax attention, an HGRN2 recurrence and a gelu feed-forward."""
+
+    architecture = "Ruvenex"
+
+
+class VogizenSession(FolderSession):
+    """Layers of sliding-window latent attention or the gated delta rule, a token-side input, a looped run of layers."""
+
+    architecture = "Vogizen"

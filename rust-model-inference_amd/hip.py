@@ -169,6 +169,16 @@ SIGNATURES = {
     "rmi_hip_gguf_qwen3_config": (C.c_int, [_vp, _u32, C.c_int, C.POINTER(Qwen3Config)]),
     "rmi_hip_qwen3_create_from_gguf": (_vp, [_vp, _u32, C.c_int]),
     "rmi_hip_model_folder_architecture": (C.c_int64, [C.c_char_p, C.c_char_p, _sz]),
+    "rmi_hip_folder_open": (_vp, [C.c_char_p, C.c_char_p, C.c_int, _u32]),
+    "rmi_hip_folder_destroy": (None, [_vp]),
+    "rmi_hip_folder_sizes": (C.c_int, [_vp, _u32p, _u32p, _u32p, _u32p]),
+    "rmi_hip_folder_step": (C.c_int, [_vp, _u32p, _u32, _u32p, _u32, _f32p, _f32p]),
+    "rmi_hip_folder_position": (_u32, [_vp]),
+    "rmi_hip_folder_reset": (C.c_int, [_vp]),
+    "rmi_hip_folder_set_stop_ids": (C.c_int, [_vp, _u32p, _u32]),
+    "rmi_hip_folder_set_prompt_passes": (C.c_int, [_vp, C.c_int]),
+    "rmi_hip_folder_generate": (C.c_int, [_vp, _u32p, _u32, _u32, _u32p, _u32p, _f32p, _u32p, _u32, _f32p,
+                                           C.POINTER(C.c_double)]),
     "rmi_hip_ruvenex_open": (_vp, [C.c_char_p, C.c_int, _u32]),
     "rmi_hip_ruvenex_destroy": (None, [_vp]),
     "rmi_hip_ruvenex_sizes": (C.c_int, [_vp, _u32p, _u32p, _u32p, _u32p]),

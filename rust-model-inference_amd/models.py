@@ -8,7 +8,7 @@ import os
 from . import hip
 
 # architecture of a model folder -> name of its session class in ``decode``
-FOLDER_SESSIONS = {"Ruvenex": "RuvenexSession"}
+FOLDER_SESSIONS = {"Ruvenex": "RuvenexSession", "Vogizen": "VogizenSession"}
 
 DTYPES = {"bfloat16": hip.DTYPE_BF16, "float32": hip.DTYPE_F32}
 

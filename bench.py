@@ -1124,19 +1124,81 @@ def ruvenex_work(z):
     return weights, weights + 2 * nr * z["rdim"]
 
 
-def run_ruvenex(args, pkg, ev):
-    """Prefill and decode throughput of a random Ruvenex model at a few sizes of layers, and of the Qwen3 session at the
-    same width, feed-forward, heads and layer count.  One bench step = one generation at the first size: a 2048-token
-    prompt and 128 greedy tokens."""
+# Sizes of --workload vogizen: the same widths, feed-forwards, heads and numbers of layer runs; three delta-rule layers
+# to one of latent attention; at 0.6b and 1.7b a looped run of four layers makes up the number.
+VOGIZEN_SIZES = {
+    "0.6b": dict(layers="ddda" * 6, loop=(0, 4, 2), width=1024, ff=3072, heads=16, dim=128, q_rank=768, kv_rank=256, window=1024, rheads=16,
+                 rkv_heads=8, rdim=128, side=64, vocab=151936),
+    "1.7b": dict(layers="ddda", loop=(0, 4, 2), width=2048, ff=6144, heads=16, dim=128, q_rank=1024, kv_rank=512, window=1024, rheads=16,
+                 rkv_heads=8, rdim=128, side=128, vocab=32768),
+    "8b": dict(layers="ddda", loop=(0, 4, 1), width=4096, ff=12288, heads=32, dim=128, q_rank=1536, kv_rank=512, window=1024, rheads=32,
+               rkv_heads=16, rdim=128, side=256, vocab=32768),
+}
+
+
+class RuvenexWork:
+    """What a token costs: weight elements read, multiply-adds outside attention, those of a prompt's attention, bytes of
+    cache and state that a token behind n positions reads and writes."""
+
+    def __init__(self, z):
+        self.z = z
+        layer, macs = ruvenex_work(z)
+        self.weights = layer * z["n_layer"] + z["vocab"] * z["width"]
+        self.macs = macs * z["n_layer"]
+
+    def attention_macs(self, n):
+        return self.z["n_layer"] * self.z["heads"] * self.z["dim"] * n * n
+
+    def cache_bytes(self, n, elem):
+        z = self.z
+        return elem * 2.0 * z["n_layer"] * z["kv_heads"] * z["dim"] * n + 8.0 * z["n_layer"] * z["rheads"] * z["rdim"]**2
+
+
+class VogizenWork:
+    def __init__(self, z):
+        self.z = z
+        W, nk, nr, rk = z["width"], z["heads"] * z["dim"], z["rheads"] * z["rdim"], z["rkv_heads"] * z["rdim"]
+        rest = 3 * W * z["ff"] + 2 * W * z["side"]
+        delta = W * (2 * rk + 3 * nr + 2 * z["rheads"]) + rest
+        latent = W * (z["q_rank"] + z["kv_rank"] + nk) + nk * z["q_rank"] + 2 * nk * z["kv_rank"] + rest
+        a, b, times = z["loop"]
+        runs = z["layers"][:a] + z["layers"][a:b] * times + z["layers"][b:]
+        self.n_delta, self.n_latent = runs.count("d"), runs.count("a")
+        self.macs = self.n_delta * (delta + 3 * nr * z["rdim"]) + self.n_latent * latent + 2 * W * W * times
+        self.weights = self.n_delta * delta + self.n_latent * latent + 2 * W * W * times + z["vocab"] * W
+
+    def attention_macs(self, n):  # a position sees min(n, window) keys
+        w = min(n, self.z["window"])
+        return 2 * self.n_latent * self.z["heads"] * self.z["dim"] * (n * w - w * w / 2)
+
+    def cache_bytes(self, n, elem):
+        z = self.z
+        return elem * 2.0 * self.n_latent * z["heads"] * z["dim"] * min(n, z["window"]) + 8.0 * self.n_delta * z["rheads"] * z["rdim"]**2
+
+
+FOLDER_DESIGNS = {"ruvenex": (RUVENEX_SIZES, RuvenexWork), "vogizen": (VOGIZEN_SIZES, VogizenWork)}
+
+
+def run_folder(args, pkg, ev):
+    """Prefill and decode throughput of a random Ruvenex or Vogizen model at a few sizes of layers, beside the closest
+    other session at the same width, feed-forward, heads and number of layer runs: Qwen3 for the first, Ruvenex for the
+    second.  One bench step = one generation at the first size: a 2048-token prompt and 128 greedy tokens."""
     import shutil
     import tempfile
     H = pkg.hip
     dev_name, cus, hbm = H.device_info()
     n_prompt, n_new, long_prompt = 512, 128, 2048
-    dtype = pkg.models.DTYPES[args.dtype]
     elem = 4 if args.dtype == "float32" else 2
     flop_peak = 157.3e12 if elem == 4 else 2.5e15
-    records, first_wall = {}, None
+    design = args.workload
+
+    def session(write, file=""):
+        tmp = tempfile.mkdtemp(prefix="rmi_bench_")
+        try:
+            write(os.path.join(tmp, file) if file else tmp)
+            return pkg.models.open_session(os.path.join(tmp, file) if file else tmp, long_prompt + n_new, args.dtype)
+        finally:
+            shutil.rmtree(tmp)
 
     def phases(sess, prompt):
         """(prompt seconds, seconds a generated token), each the best of three"""
@@ -1144,19 +1206,32 @@ def run_ruvenex(args, pkg, ev):
         t2 = min(sess.generate(prompt, n_new)["seconds"] for _ in range(3))
         return t1, (t2 - t1) / (n_new - 1)
 
+    def measure(sess, work, prompts):
+        rec = {}
+        for p in prompts:
+            t_prompt, t_tok = phases(sess, p)
+            rec[f"prompt_{p.size}"] = r = {
+                "prompt_tokens_per_s": round(p.size / t_prompt, 1), "prompt_ms": round(t_prompt * 1e3, 3),
+                "generated_tokens_per_s": round(1 / t_tok, 1), "generated_ms_per_token": round(t_tok * 1e3, 4)}
+            if work:
+                flop = 2.0 * (work.macs * p.size + work.attention_macs(p.size))
+                read = elem * work.weights + work.cache_bytes(p.size + n_new / 2, elem)
+                r.update({"prompt_tflops": round(flop / t_prompt / 1e12, 1), "prompt_frac_of_peak": round(flop / t_prompt / flop_peak, 4),
+                          "generated_gb_per_s": round(read / t_tok / 1e9, 1), "generated_frac_of_hbm": round(read / t_tok / 1e9 / HBM_PEAK_GBS, 4)})
+        return rec
+
+    def folder_session(name, size):
+        write = getattr(pkg.folder, f"write_synthetic_{name}")
+        return session(lambda path: write(path, 4, **FOLDER_DESIGNS[name][0][size]))
+
+    records, first_wall = {}, None
+    sizes, work = FOLDER_DESIGNS[design]
     for name in args.size.split(","):
-        z = RUVENEX_SIZES[name]
+        z = sizes[name]
         rng = np.random.default_rng(11)
         prompts = [rng.integers(0, z["vocab"], n, dtype=np.uint32) for n in (n_prompt, long_prompt)]
-        tmp = tempfile.mkdtemp(prefix="rmi_bench_")
-        try:
-            pkg.folder.write_synthetic_ruvenex(tmp, 4, **z)
-            sess = pkg.decode.RuvenexSession(tmp, long_prompt + n_new, dtype)
-        finally:
-            shutil.rmtree(tmp)
-        log(f"[bench] ruvenex {name}: model ready")
-        weights, macs = ruvenex_work(z)
-        rec = {"sizes": z}
+        sess = folder_session(design, name)
+        log(f"[bench] {design} {name}: model ready")
         if first_wall is None:
             for _ in range(args.warmup):
                 sess.generate(prompts[1], n_new)
@@ -1165,38 +1240,21 @@ def run_ruvenex(args, pkg, ev):
             for _ in range(args.steps):
                 sess.generate(prompts[1], n_new)  # ends with its own synchronisation
             first_wall = (time.perf_counter() - t0) / args.steps
-        for p in prompts:
-            t_prompt, t_tok = phases(sess, p)
-            flop = 2.0 * macs * z["n_layer"] * p.size + 2.0 * z["n_layer"] * z["heads"] * z["dim"] * p.size * p.size
-            read = elem * (weights * z["n_layer"] + z["vocab"] * z["width"]) + \
-                elem * 2.0 * z["n_layer"] * z["kv_heads"] * z["dim"] * (p.size + n_new / 2) + \
-                8.0 * z["n_layer"] * z["rheads"] * z["rdim"]**2
-            rec[f"prompt_{p.size}"] = {
-                "prompt_tokens_per_s": round(p.size / t_prompt, 1), "prompt_ms": round(t_prompt * 1e3, 3),
-                "prompt_tflops": round(flop / t_prompt / 1e12, 1), "prompt_frac_of_peak": round(flop / t_prompt / flop_peak, 4),
-                "generated_tokens_per_s": round(1 / t_tok, 1), "generated_ms_per_token": round(t_tok * 1e3, 4),
-                "generated_gb_per_s": round(read / t_tok / 1e9, 1), "generated_frac_of_hbm": round(read / t_tok / 1e9 / HBM_PEAK_GBS, 4)}
+        rec = {"sizes": z, **measure(sess, work(z), prompts)}
         sess.close()
-        if not args.no_qwen3:
-            tmp = tempfile.mkdtemp(prefix="rmi_bench_")
-            path = os.path.join(tmp, "qwen3.gguf")
-            try:
-                pkg.gguf.write_synthetic_qwen3(path, seed=4, n_layer=z["n_layer"], n_embd=z["width"], n_head=z["heads"],
-                                               n_head_kv=z["kv_heads"], head_dim=z["dim"], n_ff=z["ff"], vocab=z["vocab"])
-                sess = pkg.models.open_session(path, long_prompt + n_new)
-            finally:
-                shutil.rmtree(tmp)
-            q = {}
-            for p in prompts:
-                t_prompt, t_tok = phases(sess, p)
-                q[f"prompt_{p.size}"] = {
-                    "prompt_tokens_per_s": round(p.size / t_prompt, 1), "prompt_ms": round(t_prompt * 1e3, 3),
-                    "generated_tokens_per_s": round(1 / t_tok, 1), "generated_ms_per_token": round(t_tok * 1e3, 4)}
-            rec["qwen3_q8_0_same_size"] = q
+        if not args.alone and design == "ruvenex":
+            sess = session(lambda path: pkg.gguf.write_synthetic_qwen3(path, seed=4, n_layer=z["n_layer"], n_embd=z["width"], n_head=z["heads"],
+                                                                       n_head_kv=z["kv_heads"], head_dim=z["dim"], n_ff=z["ff"],
+                                                                       vocab=z["vocab"]), "qwen3.gguf")
+            rec["qwen3_q8_0_same_size"] = measure(sess, None, prompts)
+            sess.close()
+        elif not args.alone:
+            sess = folder_session("ruvenex", name)
+            rec["ruvenex_same_size"] = measure(sess, RuvenexWork(RUVENEX_SIZES[name]), prompts)
             sess.close()
         records[name] = rec
-        log(f"[bench] ruvenex {name}: {json.dumps(rec)}")
-    result = base_result(args, "tokens/s, Ruvenex, 2048 prompt + 128 greedy tokens, 1 GPU", "tok/s",
+        log(f"[bench] {design} {name}: {json.dumps(rec)}")
+    result = base_result(args, f"tokens/s, {design.capitalize()}, 2048 prompt + 128 greedy tokens, 1 GPU", "tok/s",
                          round((long_prompt + n_new - 1) / first_wall, 1), first_wall, args.dtype,
                          {"workload": f"device-resident greedy generation, random weights, sizes {args.size}",
                           "device": dev_name.strip(), "compute_units": cus})
@@ -1214,11 +1272,11 @@ def main():
                     help="untimed steps before (default 10; 100 for q4_0 / q4k / q6k).  Left at its default, the compute-bound "
                          "workloads (GEMM, Q4_K GEMM, batches of two and more) add untimed steps until the clocks have "
                          "settled and report the total as `warmup`; given, it is exactly the number asked for")
-    ap.add_argument("--workload", choices=["projection_set", "single_gemv", "gemm", "q4_0", "q4k", "q6k", "q4k_gemm", "qlinear", "attention", "decode", "ruvenex"], default="projection_set",
+    ap.add_argument("--workload", choices=["projection_set", "single_gemv", "gemm", "q4_0", "q4k", "q6k", "q4k_gemm", "qlinear", "attention", "decode", "ruvenex", "vogizen"], default="projection_set",
                     help="projection_set: the headline Q8_0 decode GEMV workload (default); gemm: Q8_0 prefill GEMM; "
                          "q4_0: Q4_0 x Q8_0 decode GEMV; q4k / q6k: Q4_K / Q6_K x Q8_K decode GEMV; q4k_gemm: Q4_K prefill GEMM (M = --tokens); qlinear: QuantizedLinear::forward (Q4_K dequantise-and-dot, f32 activation); decode: end-to-end device-resident greedy decode "
-                         "(one step = one 639-token-step generation); ruvenex: prefill and decode of a random Ruvenex model "
-                         "beside the Qwen3 session at equal sizes")
+                         "(one step = one 639-token-step generation); ruvenex, vogizen: prefill and decode of a random model "
+                         "of that design beside the closest other session at equal sizes")
     ap.add_argument("--batch", type=int, default=1, help="decode batch (1..8 tokens; 1..64 with --order neon)")
     ap.add_argument("--order", choices=["avx2", "neon"], default="avx2",
                     help="projection_set: accumulation order of the reference's x86-64 kernel (GEMV, the default) or of "
@@ -1228,9 +1286,10 @@ def main():
                     help="gemm: 'fast' lets the library split the blocks of a row over the waves of a workgroup where the "
                          "tile grid is smaller than the chip (outputs within the reference's tolerance); 'exact' keeps the "
                          "aarch64 kernel's single f32 chain per output, bit for bit")
-    ap.add_argument("--size", default="0.6b", help="ruvenex: one or more of %s, separated by commas" % ", ".join(RUVENEX_SIZES))
-    ap.add_argument("--dtype", choices=["bfloat16", "float32"], default="bfloat16", help="ruvenex: what the session computes in")
-    ap.add_argument("--no-qwen3", action="store_true", help="ruvenex: leave out the Qwen3 session of the same sizes")
+    ap.add_argument("--size", default="0.6b", help="ruvenex, vogizen: one or more of %s, separated by commas" % ", ".join(RUVENEX_SIZES))
+    ap.add_argument("--dtype", choices=["bfloat16", "float32"], default="bfloat16", help="ruvenex, vogizen: what the session computes in")
+    ap.add_argument("--alone", "--no-qwen3", action="store_true",
+                    help="ruvenex, vogizen: leave out the other session of the same sizes (Qwen3 beside Ruvenex, Ruvenex beside Vogizen)")
     ap.add_argument("--keys", type=int, default=4096, help="cached positions for --workload attention")
     ap.add_argument("--mode", choices=["grouped", "per_matmul", "layer"], default="grouped")
     ap.add_argument("--no-cpu-baseline", action="store_true")
@@ -1254,7 +1313,7 @@ def main():
     # exactly the W asked for)
     args.settle_ms = SETTLE_MS if args.warmup is None else 0.0
     long_run = args.workload in ("q4_0", "q4k", "q6k")
-    if args.workload == "ruvenex":  # a step is a whole generation
+    if args.workload in FOLDER_DESIGNS:  # a step is a whole generation
         args.steps, args.warmup = 5 if args.steps is None else args.steps, 2 if args.warmup is None else args.warmup
     if args.steps is None:
         args.steps = 500 if long_run else 50
@@ -1268,7 +1327,7 @@ def main():
     pkg.init(int(os.environ.get("LOCAL_RANK", "0")))
     ev = HipEvents()
     run = {"projection_set": run_projection_set, "single_gemv": run_single_gemv, "gemm": run_gemm, "q4_0": run_q4_0, "q4k": run_q4k, "q6k": run_q6k, "q4k_gemm": run_q4k_gemm, "qlinear": run_qlinear,
-           "attention": run_attention, "decode": run_decode, "ruvenex": run_ruvenex}[args.workload]
+           "attention": run_attention, "decode": run_decode, "ruvenex": run_folder, "vogizen": run_folder}[args.workload]
     result = run(args, pkg, ev)
     if args.workload == "projection_set" and not args.no_decode and args.batch == 1:
         # the second half of the headline metric: end-to-end decode tok/s of the same model shape, measured

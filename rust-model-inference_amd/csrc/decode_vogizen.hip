@@ -32,7 +32,7 @@ struct VogizenLayer {
     float *dq_norm = nullptr, *dkv_norm = nullptr, *ones = nullptr;
     // the delta rule
     RmiDeltaShape rule{};
-    float *conv = nullptr, *head_norm = nullptr;
+    float *conv = nullptr, *head_norm = nullptr, *rate = nullptr, *bias = nullptr;
 };
 
 // A layer as often as a token runs through it, each time with a cache or state of its own.
@@ -170,8 +170,10 @@ int VogizenSession::mixer(const VogizenLayer &l, const VogizenRun &r, uint32_t s
         a.hist_in = r.hist[now];
         a.hist_out = r.hist[now ^ 1];
         a.conv = l.conv;
-        a.beta = beta;
-        a.g = decay;
+        a.b = beta;
+        a.a = decay;
+        a.rate = l.rate;
+        a.bias = l.bias;
         a.gate = gate;
         a.norm = l.head_norm;
         a.state_in = r.state[now];
@@ -248,14 +250,12 @@ int VogizenSession::enqueue_layers(uint32_t step0, uint32_t n, hipStream_t st, f
 
 // ------------------------------------------------------------------ loading
 
-RmiRowSeg segment(void *y, uint32_t n, uint32_t ld, RmiAct act, const float *bias = nullptr, const float *lower = nullptr) {
+RmiRowSeg segment(void *y, uint32_t n, uint32_t ld, RmiAct act) {
     RmiRowSeg s{};
     s.y = y;
     s.n = n;
     s.ld = ld;
     s.act = uint16_t(act);
-    s.bias = bias;
-    s.lower = lower;
     return s;
 }
 
@@ -305,14 +305,13 @@ bool VogizenSession::load_delta(RmiFolderReader &rd, VogizenLayer &l, const std:
     if (!a_log) return false;
     std::vector<float> rate(s.heads);
     for (uint32_t i = 0; i < s.heads; i++) rate[i] = float(std::exp(double(rmi_tensor_f32(*a_log, i))));
-    const float *rates = upload(rate.data(), rate.size()), *bias = upload_vector(rd.tensor(m + "dt_bias", {s.heads}));
-    if (!rates || !bias) return false;
+    if (!(l.rate = upload(rate.data(), rate.size())) || !(l.bias = upload_vector(rd.tensor(m + "dt_bias", {s.heads})))) return false;
     if (!stack(rd, &l.w_in, &l.in,
                {{m + "q", segment(u, nk, ld, kActNone)},
                 {m + "k", segment(u + nk, nk, ld, kActNone)},
                 {m + "v", segment(u + 2 * nk, nv, ld, kActNone)},
-                {m + "b", segment(beta, s.heads, s.heads, kActForgetGate)},
-                {m + "a", segment(decay, s.heads, s.heads, kActDecay, bias, rates)},
+                {m + "b", segment(beta, s.heads, s.heads, kActNone)},
+                {m + "a", segment(decay, s.heads, s.heads, kActNone)},
                 {m + "g", segment(gate, nv, nv, kActSilu)}},
                width) ||
         !output(rd, &l.w_out, &l.out, m + "o", p + "ls1", nv))

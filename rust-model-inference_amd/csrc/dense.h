@@ -20,18 +20,17 @@ inline uint32_t rmi_dense_ld(uint32_t k_pad, uint32_t elem_bytes) {
     return k_pad + (size_t(k_pad) * elem_bytes % 256 == 0 ? 128 / elem_bytes : 0);
 }
 
-// kActForgetGate: lower + (1 - lower) sigmoid(z + bias) in full f32 (without either array a plain sigmoid);
-// kActDecay: exp(-lower softplus(z + bias)) in full f32; kActReluGlu: rows come in pairs (gate, up) and
-// y[row / 2] = relu(gate) * up.
-enum RmiAct : uint32_t { kActNone, kActSigmoid, kActSilu, kActGeluTanh, kActForgetGate, kActDecay, kActReluGlu };
+// kActForgetGate: lower + (1 - lower) sigmoid(z + bias) in full f32; kActReluGlu: rows come in pairs (gate, up) and
+// y[row / 2] = relu(gate) * up (of all segments of a product or of none).
+enum RmiAct : uint32_t { kActNone, kActSigmoid, kActSilu, kActGeluTanh, kActForgetGate, kActReluGlu };
 
 // Rows [row0, row0 + n) of a product: y[token * ld + row - row0] = act(result), f32 or the model's element type.
 // mul (nullptr = none): the activation's result times mul[mul_tok[token] * mul_ld + row - row0], a table of the
 // model's element type with mul_rows rows, looked up by the token's id.
 struct RmiRowSeg {
     void *y;
-    const float *bias;   // kActSigmoid, kActForgetGate, kActDecay; nullptr = 0
-    const float *lower;  // kActForgetGate (nullptr = 0), kActDecay
+    const float *bias;   // kActSigmoid, kActForgetGate; nullptr = 0
+    const float *lower;  // kActForgetGate
     const void *mul;
     const uint32_t *mul_tok;
     uint32_t mul_ld, mul_rows;

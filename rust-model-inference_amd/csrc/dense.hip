@@ -32,11 +32,13 @@ __global__ __launch_bounds__(256) void embed_kernel(RmiEmbed e, const uint32_t *
 // 16-byte pieces, piece p at slot p ^ (row & 7), so that the sixteen rows of a fragment spread over the banks.
 // Weights are the A operand: a lane ends with four consecutive rows of one token.
 constexpr uint32_t kStepBytes = 128;
+constexpr int kResidual = -1;  // the epilogue that adds to the residual stream; the others are RmiEpilogue's
 
-template <typename T, int BN, int BT, int WN, int WT, int PD, int NB, int WPS, bool RESIDUAL>
+template <typename T, int BN, int BT, int WN, int WT, int PD, int NB, int WPS, int EPI>
 __global__ __launch_bounds__(256, WPS) void dense_gemm_kernel(const T *__restrict__ w, const T *__restrict__ a, uint32_t n_rows,
                                                               uint32_t k_pad, uint32_t ld, uint32_t n_tokens, uint32_t grid_n, uint32_t grid_t, uint32_t xcd_split,
                                                          RmiRowSegs rs, RmiColSegs cs, float *__restrict__ x, uint32_t width) {
+    constexpr bool RESIDUAL = EPI == kResidual;
     static_assert((BN / WN) * (BT / WT) == 4, "four waves");
     static_assert(kDenseKAlign * sizeof(T) % (kStepBytes * PD) == 0, "whole rounds of the register slots");
     constexpr int NN = WN / 16, NT = WT / 16;
@@ -169,16 +171,18 @@ __global__ __launch_bounds__(256, WPS) void dense_gemm_kernel(const T *__restric
             const RmiRowSeg &s = rs.s[seg_of(rs, tile_row)];
             const uint32_t r0 = tile_row - s.row0 + g * 4;
             float bias[4], lower[4];
+            if constexpr (EPI == kRowsActed || EPI == kRowsTimesTable) {
 #pragma unroll
-            for (int r = 0; r < 4; r++) {
-                bias[r] = s.bias && r0 + r < s.n ? s.bias[r0 + r] : 0.0f;
-                lower[r] = s.lower && r0 + r < s.n ? s.lower[r0 + r] : 0.0f;
+                for (int r = 0; r < 4; r++) {
+                    bias[r] = s.bias && r0 + r < s.n ? s.bias[r0 + r] : 0.0f;
+                    lower[r] = s.lower && r0 + r < s.n ? s.lower[r0 + r] : 0.0f;
+                }
             }
 #pragma unroll
             for (int j = 0; j < NT; j++) {
                 const uint32_t tok = tok0 + wt + j * 16 + fr;
-                if (tok >= n_tokens) continue;
-                if (s.act == kActReluGlu) {  // (gate, up) pairs: two results
+                if constexpr (EPI == kRowsPaired) {  // (gate, up) twice: two results
+                    if (tok >= n_tokens) continue;
 #pragma unroll
                     for (uint32_t r = 0; r < 2; r++) {
                         const float v = fmaxf(acc[i][j][2 * r], 0.0f) * acc[i][j][2 * r + 1];
@@ -192,14 +196,19 @@ __global__ __launch_bounds__(256, WPS) void dense_gemm_kernel(const T *__restric
                     }
                     continue;
                 }
-                f32x4 o;
+                f32x4 o = acc[i][j];
+                if constexpr (EPI == kRowsActed || EPI == kRowsTimesTable) {
 #pragma unroll
-                for (int r = 0; r < 4; r++) o[r] = apply_act<T>(s.act, acc[i][j][r], bias[r], lower[r]);
-                if (s.mul) {
-                    const T *m = mul_row<T>(s, tok) + r0;
+                    for (int r = 0; r < 4; r++) o[r] = apply_act<T>(s.act, o[r], bias[r], lower[r]);
+                }
+                if (tok >= n_tokens) continue;
+                if constexpr (EPI == kRowsTimesTable) {
+                    if (s.mul) {
+                        const T *m = mul_row<T>(s, tok) + r0;
 #pragma unroll
-                    for (uint32_t r = 0; r < 4; r++)
-                        if (r0 + r < s.n) o[r] *= to_f32(m[r]);
+                        for (uint32_t r = 0; r < 4; r++)
+                            if (r0 + r < s.n) o[r] *= to_f32(m[r]);
+                    }
                 }
                 const size_t at = size_t(tok) * s.ld + r0;
                 if (r0 + 3 < s.n && (s.ld & 3) == 0) {
@@ -222,10 +231,10 @@ __global__ __launch_bounds__(256, WPS) void dense_gemm_kernel(const T *__restric
     }
 }
 
-template <typename T, bool RESIDUAL>
+template <typename T, int EPI>
 int launch_gemm(const RmiDense &w, const void *a, const RmiRowSegs &rs, const RmiColSegs &cs, float *x, uint32_t width,
                 uint32_t n_tokens, hipStream_t st) {
-    const uint32_t n_rows = RESIDUAL ? width : w.n_rows;
+    const uint32_t n_rows = EPI == kResidual ? width : w.n_rows;
     auto go = [&](auto kernel, uint32_t bn, uint32_t bt) {
         const uint32_t gn = (n_rows + bn - 1) / bn, gt = (n_tokens + bt - 1) / bt;
         const uint32_t split = rmi_gemm_xcd_split(gn, gt, double(n_rows) * w.k_pad, double(n_tokens) * w.k_pad);
@@ -235,13 +244,13 @@ int launch_gemm(const RmiDense &w, const void *a, const RmiRowSegs &rs, const Rm
     const uint64_t cus = uint64_t(rmi_device_cus());
     auto tiles = [&](uint32_t bn, uint32_t bt) { return uint64_t((n_rows + bn - 1) / bn) * ((n_tokens + bt - 1) / bt); };
     if (n_tokens <= 16)
-        go(dense_gemm_kernel<T, 64, 16, 16, 16, 4, 2, 4, RESIDUAL>, 64, 16);
+        go(dense_gemm_kernel<T, 64, 16, 16, 16, 4, 2, 4, EPI>, 64, 16);
     else if (tiles(128, 128) >= 2 * cus)
-        go(dense_gemm_kernel<T, 128, 128, 64, 64, 1, 1, 3, RESIDUAL>, 128, 128);
+        go(dense_gemm_kernel<T, 128, 128, 64, 64, 1, 1, 3, EPI>, 128, 128);
     else if (tiles(64, 64) >= cus)
-        go(dense_gemm_kernel<T, 64, 64, 32, 32, 4, 2, 4, RESIDUAL>, 64, 64);
+        go(dense_gemm_kernel<T, 64, 64, 32, 32, 4, 2, 4, EPI>, 64, 64);
     else
-        go(dense_gemm_kernel<T, 64, 32, 32, 16, 4, 2, 4, RESIDUAL>, 64, 32);
+        go(dense_gemm_kernel<T, 64, 32, 32, 16, 4, 2, 4, EPI>, 64, 32);
     RMI_HIP_CHECK(hipGetLastError());
     return RMI_HIP_OK;
 }
@@ -280,8 +289,16 @@ int rmi_dense_gemm(uint32_t elem_bytes, const RmiDense &w, const void *a, const 
     if (n_tokens == 0 || w.n_rows == 0) return RMI_HIP_OK;
     const int rc = rmi_check_row_segs(elem_bytes, w, segs);
     if (rc != RMI_HIP_OK) return rc;
-    return elem_bytes == 2 ? launch_gemm<rmi_bf16, false>(w, a, segs, RmiColSegs{}, nullptr, 0, n_tokens, st)
-                           : launch_gemm<float, false>(w, a, segs, RmiColSegs{}, nullptr, 0, n_tokens, st);
+    auto go = [&](auto type) {
+        using T = decltype(type);
+        switch (rmi_epilogue_of(segs)) {
+            case kRowsActed: return launch_gemm<T, kRowsActed>(w, a, segs, RmiColSegs{}, nullptr, 0, n_tokens, st);
+            case kRowsPaired: return launch_gemm<T, kRowsPaired>(w, a, segs, RmiColSegs{}, nullptr, 0, n_tokens, st);
+            case kRowsTimesTable: return launch_gemm<T, kRowsTimesTable>(w, a, segs, RmiColSegs{}, nullptr, 0, n_tokens, st);
+            default: return launch_gemm<T, kRowsPlain>(w, a, segs, RmiColSegs{}, nullptr, 0, n_tokens, st);
+        }
+    };
+    return elem_bytes == 2 ? go(rmi_bf16()) : go(float());
 }
 
 int rmi_dense_gemm_residual(uint32_t elem_bytes, const RmiDense &w, const void *a, const RmiColSegs &segs, float *x, uint32_t width,
@@ -289,6 +306,6 @@ int rmi_dense_gemm_residual(uint32_t elem_bytes, const RmiDense &w, const void *
     if (n_tokens == 0) return RMI_HIP_OK;
     const int rc = rmi_check_col_segs(elem_bytes, w, segs, width);
     if (rc != RMI_HIP_OK) return rc;
-    return elem_bytes == 2 ? launch_gemm<rmi_bf16, true>(w, a, RmiRowSegs{}, segs, x, width, n_tokens, st)
-                           : launch_gemm<float, true>(w, a, RmiRowSegs{}, segs, x, width, n_tokens, st);
+    return elem_bytes == 2 ? launch_gemm<rmi_bf16, kResidual>(w, a, RmiRowSegs{}, segs, x, width, n_tokens, st)
+                           : launch_gemm<float, kResidual>(w, a, RmiRowSegs{}, segs, x, width, n_tokens, st);
 }

@@ -183,16 +183,11 @@ constexpr uint32_t kFewRows = 1024;  // up to here a wave takes one row: four wo
 GemvProblem problem_of(const RmiDense &w, const RmiInput &in, const RmiRowSegs &segs, uint32_t rows) {
     return GemvProblem{w.data, w.k_pad, w.ld, (w.n_rows + 4 * rows - 1) / (4 * rows), in, segs};
 }
-bool has_pairs(const RmiRowSegs &segs) {
-    for (uint32_t i = 0; i < segs.n_segs; i++)
-        if (segs.s[i].act == kActReluGlu) return true;
-    return false;
-}
 
 template <typename T>
 int gemv(const RmiDense &w, const RmiInput &in, const RmiRowSegs &segs, hipStream_t st) {
     const size_t lds = size_t(gemv_lds_pieces<T>(w.k_pad)) * 16;
-    const bool few = w.n_rows <= kFewRows && in.norm == kNormNone && !in.y && !has_pairs(segs);
+    const bool few = w.n_rows <= kFewRows && in.norm == kNormNone && !in.y && rmi_epilogue_of(segs) != kRowsPaired;
     const GemvProblem p = problem_of(w, in, segs, few ? 1 : 4);
     auto go = [&](auto kernel) {
         const int rc = rmi_allow_lds(kernel, lds);

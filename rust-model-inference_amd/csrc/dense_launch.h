@@ -18,7 +18,7 @@ inline int rmi_check_row_segs(uint32_t elem_bytes, const RmiDense &w, const RmiR
     bool ok = segs.n_rows == w.n_rows && segs.n_segs > 0 && segs.n_segs <= kMaxRowSegs && w.k_pad % kDenseKAlign == 0 &&
               w.ld == rmi_dense_ld(w.k_pad, elem_bytes);
     for (uint32_t i = 0; ok && i < segs.n_segs; i++)
-        ok = (segs.s[i].act != kActDecay || segs.s[i].lower) && (segs.s[i].act != kActReluGlu || (segs.s[i].n % 2 == 0 && !segs.s[i].mul)) &&
+        ok = (segs.s[i].act == kActReluGlu) == (segs.s[0].act == kActReluGlu) && (segs.s[i].act != kActReluGlu || (segs.s[i].n % 2 == 0 && !segs.s[i].mul)) &&
              (!segs.s[i].mul || (segs.s[i].mul_tok && segs.s[i].mul_rows));
     return ok ? RMI_HIP_OK : rmi_fail(RMI_HIP_E_INVALID, "row segments do not fit the weight");
 }
@@ -30,6 +30,18 @@ inline int rmi_check_col_segs(uint32_t elem_bytes, const RmiDense &w, const RmiC
         if (segs.s[i].k_end % kDenseKAlign || segs.s[i].k_end <= (i ? segs.s[i - 1].k_end : 0u))
             return rmi_fail(RMI_HIP_E_INVALID, "column segments do not fit the weight");
     return RMI_HIP_OK;
+}
+
+// What a product's row segments ask of its epilogue: each kind is a kernel of its own, so that the plain one stays small.
+enum RmiEpilogue : int { kRowsPlain, kRowsActed, kRowsPaired, kRowsTimesTable };
+inline RmiEpilogue rmi_epilogue_of(const RmiRowSegs &segs) {
+    RmiEpilogue e = kRowsPlain;
+    for (uint32_t i = 0; i < segs.n_segs; i++) {
+        if (segs.s[i].act == kActReluGlu) return kRowsPaired;
+        if (segs.s[i].mul) return kRowsTimesTable;
+        if (segs.s[i].act != kActNone) e = kRowsActed;
+    }
+    return e;
 }
 
 // go(norm, add, quads a thread) with the three as compile-time constants

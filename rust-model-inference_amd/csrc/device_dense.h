@@ -126,7 +126,6 @@ __device__ __forceinline__ float apply_act(uint32_t act, float z, float bias, fl
         case kActGeluTanh:  // z/2 (1 + tanh u) = z sigmoid(2u)
             return z * sigmoid_t<T>(1.59576912160573071176f * __builtin_fmaf(0.044715f * z * z, z, z));
         case kActForgetGate: return __builtin_fmaf(1.0f - lower, sigmoid_t<float>(z + bias), lower);
-        case kActDecay: return expf(-lower * softplus_f32(z + bias));
         default: return z;
     }
 }

@@ -13,6 +13,13 @@ __device__ __forceinline__ uint32_t q_channel(const RmiDeltaShape &s, uint32_t g
 __device__ __forceinline__ uint32_t k_channel(const RmiDeltaShape &s, uint32_t g) { return (s.kv_heads + g) * s.dim; }
 __device__ __forceinline__ uint32_t v_channel(const RmiDeltaShape &s, uint32_t h) { return 2 * s.kv_heads * s.dim + h * s.vdim; }
 
+__device__ __forceinline__ float delta_beta(const RmiDeltaShape &s, const RmiDeltaArgs &a, uint32_t t, uint32_t h) {
+    return sigmoid_t<float>(a.b[size_t(t) * s.heads + h]);
+}
+__device__ __forceinline__ float delta_decay(const RmiDeltaShape &s, const RmiDeltaArgs &a, uint32_t t, uint32_t h) {
+    return expf(-a.rate[h] * softplus_f32(a.a[size_t(t) * s.heads + h] + a.bias[h]));
+}
+
 // the history that head h passes on: its values' channels, and as the first of its group the queries' and keys'
 __device__ __forceinline__ void delta_carry(const RmiDeltaShape &s, const RmiDeltaArgs &a, const ConvCtx &x, uint32_t h, uint32_t threads) {
     const uint32_t group = s.heads / s.kv_heads, g = h / group;
@@ -57,7 +64,7 @@ __global__ __launch_bounds__(kStepThreads) void delta_step_kernel(RmiDeltaShape 
             }
         }
     }
-    const float decay = a.g[h], beta = a.beta[h];
+    const float decay = delta_decay(s, a, 0, h), beta = delta_beta(s, a, 0, h);
     const uint32_t quads = s.v_pad / 4, slices = kStepThreads / quads, col = tid % quads, sl = tid / quads;
     const size_t at = size_t(h) * s.d_pad * s.v_pad + col * 4;
     f32x4 r[NR];
@@ -214,7 +221,7 @@ __global__ __launch_bounds__(256) void delta_factors_kernel(RmiDeltaShape s, Rmi
     extern __shared__ __attribute__((aligned(16))) uint8_t lds_raw[];
     const uint32_t ld = s.d_pad + 4;
     float *ql = reinterpret_cast<float *>(lds_raw), *kl = ql + kChunk * ld;  // [16][d_pad + 4]
-    __shared__ float dm[kChunk][kChunk], am[kChunk][kChunk + 1], beta[kChunk];
+    __shared__ float dm[kChunk][kChunk], am[kChunk][kChunk + 1], beta[kChunk], decay[kChunk];
     const uint32_t tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, chunk = blockIdx.x, h = blockIdx.y, t0 = chunk * kChunk;
     const uint32_t group = s.heads / s.kv_heads, g = h / group;
     const bool first = h % group == 0;
@@ -242,23 +249,29 @@ __global__ __launch_bounds__(256) void delta_factors_kernel(RmiDeltaShape s, Rmi
             for (uint32_t t = 0; t < kChunk; t++) dst[t * ld] = y[t];
         }
     }
-    if (tid < kChunk) {  // column s of D, and G as the column before the first
+    if (tid >= 128 && tid < 128 + kChunk) {
+        const uint32_t t = tid - 128;
+        const bool live = t0 + t < a.n_tokens;  // a token past the end changes nothing
+        decay[t] = live ? delta_decay(s, a, t0 + t, h) : 1.0f;
+        beta[t] = live ? delta_beta(s, a, t0 + t, h) : 0.0f;
+    }
+    __syncthreads();
+    if (tid < kChunk) {  // column s of D
         float w = 1.0f;
+#pragma unroll
         for (uint32_t t = 0; t < kChunk; t++) {
-            const float gt = t0 + t < a.n_tokens ? a.g[size_t(t0 + t) * s.heads + h] : 1.0f;
-            if (t > tid) w *= gt;
+            if (t > tid) w *= decay[t];
             dm[t][tid] = t < tid ? 0.0f : w;
         }
         ws.gd[hc * 2 * kChunk + kChunk + tid] = w;
-        beta[tid] = t0 + tid < a.n_tokens ? a.beta[size_t(t0 + tid) * s.heads + h] : 0.0f;
     } else if (tid == 64) {
         float w = 1.0f;
+#pragma unroll
         for (uint32_t t = 0; t < kChunk; t++) {
-            if (t0 + t < a.n_tokens) w *= a.g[size_t(t0 + t) * s.heads + h];
+            w *= decay[t];
             ws.gd[hc * 2 * kChunk + t] = w;
         }
     }
-    __syncthreads();
     // unit length: four tokens a wave
     for (uint32_t t = wave; t < kChunk; t += 4) {
         float qq = 0.0f, kk = 0.0f;

@@ -66,7 +66,7 @@ size_t rmi_recur_scratch_floats(const RmiRecurShape &s, uint32_t max_tokens);
 // Gated delta rule.  q, k (kv_heads of dim) and v (heads of vdim) pass a short causal convolution and silu; q and k
 // become unit vectors, q also over sqrt(dim).  Per head, with the key head h / (heads / kv_heads):
 //   S <- g S;  u = beta (v - S^T k);  S <- S + k u^T;  o = S^T q
-// then o over its root mean square times norm, times gate.
+// with beta = sigmoid(b) and the decay g = exp(-rate softplus(a + bias)), then o over its root mean square times norm, times gate.
 struct RmiDeltaShape {
     uint32_t heads, kv_heads, dim, vdim, d_pad, v_pad;  // padded to 16
     uint32_t taps;
@@ -77,7 +77,8 @@ struct RmiDeltaArgs {
     const float *hist_in;    // the taps - 1 rows before it; rows of positions below zero are never read
     float *hist_out;         // another buffer: the taps - 1 rows before the next pass's first
     const float *conv;       // [channels][taps], the last tap is the token's own
-    const float *beta, *g;   // [n_tokens][heads]
+    const float *b, *a;      // [n_tokens][heads]
+    const float *rate, *bias;  // [heads]
     const float *gate;       // [n_tokens][heads * vdim]
     const float *norm;       // [vdim]
     const float *state_in;   // [head][d_pad][v_pad]; not read at pos0 == 0

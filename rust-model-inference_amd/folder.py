@@ -1,4 +1,4 @@
-"""Writes model folders (config.json and model.safetensors): the synthetic Ruvenex models of the benchmark."""
+"""Writes model folders (config.json and model.safetensors): the synthetic models of the benchmark."""
 import json
 import os
 import struct
@@ -24,6 +24,14 @@ def write_safetensors(path, tensors):
         f.write(struct.pack("<Q", len(text)) + text)
         for _, a in tensors:
             f.write(a.tobytes())
+
+
+def _write(path, cfg, tensors):
+    os.makedirs(path, exist_ok=True)
+    with open(os.path.join(path, "config.json"), "w") as f:
+        json.dump(cfg, f)
+    write_safetensors(os.path.join(path, "model.safetensors"), tensors)
+    return cfg
 
 
 def synthetic_ruvenex_config(n_layer, width, ff, heads, kv_heads, dim, rheads, rdim, vocab):
@@ -62,8 +70,56 @@ def write_synthetic_ruvenex(path, seed, **sizes):
     tensors = [("embed", mat(V, W)), ("final.norm", vec(W, 1, 0.1)), ("head", mat(V, W))]
     for i in range(len(cfg["layers"])):
         tensors += [(f"l{i}.{n}", t) for n, t in layer.items()]
-    os.makedirs(path, exist_ok=True)
-    with open(os.path.join(path, "config.json"), "w") as f:
-        json.dump(cfg, f)
-    write_safetensors(os.path.join(path, "model.safetensors"), tensors)
-    return cfg
+    return _write(path, cfg, tensors)
+
+
+def synthetic_vogizen_config(layers, width, ff, heads, dim, q_rank, kv_rank, window, rheads, rkv_heads, rdim, side, vocab, loop):
+    """layers: "d" (delta rule) or "a" (latent attention) each; loop: (start, stop, times)."""
+    kinds = {"d": ("delta", {"heads": rheads, "kv_heads": rkv_heads, "dim": rdim, "vdim": rdim, "conv": 4}),
+             "a": ("latent_attention", {"heads": heads, "dim": dim, "vdim": dim, "q_rank": q_rank, "kv_rank": kv_rank,
+                                        "scale": dim**-0.5, "mask": {"size": window}})}
+    entries = [{"type": kinds[k][0], "mixer": kinds[k][1], "mlp": {"kind": "dense", "ff": ff}} for k in layers]
+    return {"architecture": "Vogizen", "embedding": {"scale": 1.0}, "layers": entries, "loop": dict(zip(("start", "stop", "times"), loop)),
+            "norm": {"eps": 1e-6}, "token_side": {"dim": side}, "vocab": vocab, "width": width}
+
+
+def write_synthetic_vogizen(path, seed, **sizes):
+    """A random model of those sizes.  One layer's weights of either kind are drawn and stored once for every such layer
+    (each layer's copy has its own place in the file and in HBM)."""
+    cfg = synthetic_vogizen_config(**sizes)
+    rng = np.random.default_rng(seed)
+    W, V, side = cfg["width"], cfg["vocab"], cfg["token_side"]["dim"]
+
+    def mat(out, inp):
+        return bf16_bits(rng.standard_normal((out, inp), dtype=np.float32) / np.sqrt(inp))
+
+    def vec(n, mean, spread):
+        return bf16_bits(mean + spread * rng.standard_normal(n))
+
+    def layer(entry):
+        m, ff = entry["mixer"], entry["mlp"]["ff"]
+        t = {"norm1": vec(W, 1, 0.1), "norm2": vec(W, 1, 0.1), "ls1": vec(W, 0.5, 0.1), "ls2": vec(W, 0.5, 0.1), "mlp.gate": mat(ff, W),
+             "mlp.up": mat(ff, W), "mlp.down": mat(W, ff), "side.gate": mat(side, W), "side.proj": mat(W, side), "side.norm": vec(W, 0.3, 0.1),
+             "mix.o": mat(W, m["heads"] * m["vdim"])}
+        if entry["type"] == "delta":
+            nk, nv = m["kv_heads"] * m["dim"], m["heads"] * m["vdim"]
+            for n, size in (("q", nk), ("k", nk), ("v", nv)):
+                t[f"mix.{n}"] = mat(size, W)
+                t[f"mix.{n}.conv"] = bf16_bits(0.3 * rng.standard_normal((size, m["conv"])) + (np.arange(m["conv"]) == m["conv"] - 1))
+            t.update({"mix.b": mat(m["heads"], W), "mix.a": mat(m["heads"], W), "mix.A_log": vec(m["heads"], 0, 0.5),
+                      "mix.dt_bias": vec(m["heads"], -2, 1), "mix.g": mat(nv, W), "mix.norm": vec(m["vdim"], 1, 0.1)})
+        else:
+            nk, nv, rq, rk = m["heads"] * m["dim"], m["heads"] * m["vdim"], m["q_rank"], m["kv_rank"]
+            t.update({"mix.dq": mat(rq, W), "mix.dq.norm": vec(rq, 1, 0.1), "mix.uq": mat(nk, rq), "mix.dkv": mat(rk, W),
+                      "mix.dkv.norm": vec(rk, 1, 0.1), "mix.uk": mat(nk, rk), "mix.uv": mat(nv, rk)})
+        return t
+
+    kinds = {}
+    for entry in cfg["layers"]:
+        if entry["type"] not in kinds:
+            kinds[entry["type"]] = layer(entry)
+    tensors = [("embed", mat(V, W)), ("final.norm", vec(W, 1, 0.1)), ("loop.in", mat(W, 2 * W)),
+               ("side.embed", np.tile(mat(V, side), (1, len(cfg["layers"]))))]
+    for i, entry in enumerate(cfg["layers"]):
+        tensors += [(f"l{i}.{n}", t) for n, t in kinds[entry["type"]].items()]
+    return _write(path, cfg, tensors)

@@ -17,12 +17,7 @@ __global__ __launch_bounds__(256) void input_kernel(RmiInput in, const uint32_t 
 
 template <typename T>
 __global__ __launch_bounds__(256) void embed_kernel(RmiEmbed e, const uint32_t *__restrict__ tok, uint32_t pos0) {
-    const uint32_t t = blockIdx.x, id = tok[t];
-    for (uint32_t i = threadIdx.x; i < e.n; i += 256) {
-        const float v = embed_value<T>(e, id, pos0 + t, i);
-        e.x[size_t(t) * e.n + i] = v;
-        if (e.x_also) e.x_also[size_t(t) * e.n + i] = v;
-    }
+    embed_row<T>(e, tok[blockIdx.x], pos0 + blockIdx.x, blockIdx.x);
 }
 
 // ------------------------------------------------------------------ GEMM

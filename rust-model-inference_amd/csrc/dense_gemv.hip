@@ -178,8 +178,6 @@ __global__ __launch_bounds__(256) void gemv_residual_kernel(const T *__restrict_
     if (tid < ROWS && row0 + tid < width) x[row0 + tid] += (part[0][tid] + part[1][tid]) + (part[2][tid] + part[3][tid]);
 }
 
-constexpr uint32_t kFewRows = 1024;  // up to here a wave takes one row: four would leave most of the chip idle
-
 GemvProblem problem_of(const RmiDense &w, const RmiInput &in, const RmiRowSegs &segs, uint32_t rows) {
     return GemvProblem{w.data, w.k_pad, w.ld, (w.n_rows + 4 * rows - 1) / (4 * rows), in, segs};
 }
@@ -187,7 +185,9 @@ GemvProblem problem_of(const RmiDense &w, const RmiInput &in, const RmiRowSegs &
 template <typename T>
 int gemv(const RmiDense &w, const RmiInput &in, const RmiRowSegs &segs, hipStream_t st) {
     const size_t lds = size_t(gemv_lds_pieces<T>(w.k_pad)) * 16;
-    const bool few = w.n_rows <= kFewRows && in.norm == kNormNone && !in.y && rmi_epilogue_of(segs) != kRowsPaired;
+    // a wave takes four rows, and with no norm in front (whose work every workgroup repeats) one where four would leave
+    // compute units idle
+    const bool few = w.n_rows <= 16u * 2 * uint32_t(rmi_device_cus()) && in.norm == kNormNone && rmi_epilogue_of(segs) != kRowsPaired;
     const GemvProblem p = problem_of(w, in, segs, few ? 1 : 4);
     auto go = [&](auto kernel) {
         const int rc = rmi_allow_lds(kernel, lds);
@@ -195,7 +195,7 @@ int gemv(const RmiDense &w, const RmiInput &in, const RmiRowSegs &segs, hipStrea
         return rc;
     };
     const int rc = rmi_input_dispatch(in, [&](auto norm, auto add, auto r) {
-        if constexpr (norm.value == kNormNone && !add.value)
+        if constexpr (norm.value == kNormNone && (!add.value || r.value <= 4))
             if (few) return go(input_gemv_kernel<T, norm.value, add.value, 1, r.value>);
         if constexpr (!add.value || r.value <= 4)
             return go(input_gemv_kernel<T, norm.value, add.value, 4, r.value>);

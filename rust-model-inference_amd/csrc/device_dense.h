@@ -145,18 +145,53 @@ __device__ __forceinline__ const T *mul_row(const RmiRowSeg &s, uint32_t t) {
     return static_cast<const T *>(s.mul) + size_t(id < s.mul_rows ? id : s.mul_rows - 1) * s.mul_ld;
 }
 
+// sin(2 pi r), or with `cosine` cos(2 pi r), for |r| <= 1/2: the nearest quarter turn apart, then the Taylor polynomials on
+// an eighth of a turn to either side (their remainders are below 2e-9)
+__device__ __forceinline__ float sin_turns(double r, bool cosine) {
+    const double quarter = rint(r * 4.0);
+    const float z = float((r - quarter * 0.25) * 6.283185307179586476925286766559), z2 = z * z;
+    const int q = int(quarter) + (cosine ? 1 : 0);
+    float s = 2.75573192e-6f, c = -2.75573192e-7f;
+    s = __builtin_fmaf(s, z2, -1.98412698e-4f);
+    s = __builtin_fmaf(s, z2, 8.33333333e-3f);
+    s = __builtin_fmaf(s, z2, -1.66666667e-1f);
+    s = __builtin_fmaf(s * z2, z, z);
+    c = __builtin_fmaf(c, z2, 2.48015873e-5f);
+    c = __builtin_fmaf(c, z2, -1.38888889e-3f);
+    c = __builtin_fmaf(c, z2, 4.16666667e-2f);
+    c = __builtin_fmaf(c, z2, -0.5f);
+    c = __builtin_fmaf(c, z2, 1.0f);
+    const float v = q & 1 ? c : s;  // sin(a + q pi/2): s, c, -s, -c
+    return q & 2 ? -v : v;
+}
+
 // channel c of a token's embedding at position p (RmiEmbed)
 template <typename T>
 __device__ __forceinline__ float embed_value(const RmiEmbed &e, uint32_t token, uint32_t p, uint32_t c) {
     if (token >= e.vocab) token = e.vocab - 1;  // ids are validated on the host; never read outside the table
     float v = to_f32(static_cast<const T *>(e.table)[size_t(token) * e.ld + c]) * e.scale;
     if (e.turns) {
-        double r = double(p) * e.turns[c >> 1];
-        r -= rint(r);  // the whole turns leave in f64, what stays is exact enough for f32
-        const float a = float(r * 6.283185307179586476925286766559);
-        v += c & 1 ? cosf(a) : sinf(a);
+        const double r = double(p) * e.turns[c >> 1];
+        v += sin_turns(r - rint(r), c & 1);  // the whole turns leave in f64
     }
     return v;
+}
+
+// a workgroup of 256: row t of the stream, four channels of a thread under way at a time
+template <typename T>
+__device__ __forceinline__ void embed_row(const RmiEmbed &e, uint32_t token, uint32_t p, uint32_t t) {
+    for (uint32_t i0 = threadIdx.x; i0 < e.n; i0 += 1024) {
+        float v[4];
+#pragma unroll
+        for (uint32_t j = 0; j < 4; j++) v[j] = embed_value<T>(e, token, p, i0 + j * 256 < e.n ? i0 + j * 256 : i0);
+#pragma unroll
+        for (uint32_t j = 0; j < 4; j++) {
+            const uint32_t i = i0 + j * 256;
+            if (i >= e.n) break;
+            e.x[size_t(t) * e.n + i] = v[j];
+            if (e.x_also) e.x_also[size_t(t) * e.n + i] = v[j];
+        }
+    }
 }
 
 // ---- a product's input (RmiInput) in the registers of a workgroup of 256: R quads of values a thread, quad j of

@@ -11,13 +11,7 @@ template <typename T>
 struct EmbedNext {
     RmiEmbed e;
     uint32_t pos;
-    __device__ __forceinline__ void operator()(uint32_t token) const {
-        for (uint32_t i = threadIdx.x; i < e.n; i += 256) {
-            const float v = embed_value<T>(e, token, pos, i);
-            e.x[i] = v;
-            if (e.x_also) e.x_also[i] = v;
-        }
-    }
+    __device__ __forceinline__ void operator()(uint32_t token) const { embed_row<T>(e, token, pos, 0); }
 };
 
 struct Architecture {

@@ -51,16 +51,19 @@ __global__ __launch_bounds__(kStepThreads) void delta_step_kernel(RmiDeltaShape 
     };
     // the convolution's operands first, the state's behind them: everything waits for the former
     float row[2][kRunTaps], tap[2][kRunTaps];
+    uint32_t ch[2];
     const bool run = s.taps <= kRunTaps;
     if (run) {
 #pragma unroll
         for (uint32_t i = 0; i < 2; i++) {
-            const uint32_t e = tid + i * kStepThreads, c = channel(e < n_ch ? e : 0);
+            const uint32_t e = tid + i * kStepThreads;
+            ch[i] = channel(e < n_ch ? e : 0);
 #pragma unroll
-            for (uint32_t back = 0; back < kRunTaps; back++) {
-                const bool live = back < s.taps && a.pos0 >= back;
-                row[i][back] = !live ? 0.0f : back == 0 ? a.u[c] : a.hist_in[size_t(s.taps - 1 - back) * x.channels + c];
-                tap[i][back] = back < s.taps ? a.conv[c * s.taps + s.taps - 1 - back] : 0.0f;
+            for (uint32_t back = 0; back < kRunTaps; back++) {  // (every load is issued; what does not count is cleared below)
+                const uint32_t b = back < s.taps ? back : s.taps - 1;
+                const float *src = back == 0 || b == 0 ? a.u : a.hist_in + size_t(s.taps - 1 - b) * x.channels;
+                row[i][back] = src[ch[i]];
+                tap[i][back] = a.conv[ch[i] * s.taps + s.taps - 1 - b];
             }
         }
     }
@@ -71,8 +74,7 @@ __global__ __launch_bounds__(kStepThreads) void delta_step_kernel(RmiDeltaShape 
 #pragma unroll
     for (uint32_t j = 0; j < NR; j++) {
         const uint32_t d = sl + j * slices;
-        r[j] = f32x4{0.f, 0.f, 0.f, 0.f};
-        if (a.pos0 && sl < slices && d < s.d_pad) r[j] = *reinterpret_cast<const f32x4 *>(a.state_in + at + size_t(d) * s.v_pad);
+        r[j] = *reinterpret_cast<const f32x4 *>(a.state_in + at + size_t(d < s.d_pad ? d : 0) * s.v_pad);
     }
     const float gate = tid < s.vdim ? a.gate[size_t(h) * s.vdim + tid] : 0.0f, weight = tid < s.vdim ? a.norm[tid] : 0.0f;
     if (run) {
@@ -81,11 +83,17 @@ __global__ __launch_bounds__(kStepThreads) void delta_step_kernel(RmiDeltaShape 
             const uint32_t e = tid + i * kStepThreads;
             float z = 0.0f;
 #pragma unroll
-            for (uint32_t back = kRunTaps; back-- > 0;) z = __builtin_fmaf(tap[i][back], row[i][back], z);
+            for (uint32_t back = kRunTaps; back-- > 0;) z = __builtin_fmaf(tap[i][back], back < s.taps && a.pos0 >= back ? row[i][back] : 0.0f, z);
             if (e < n_ch) put(e, z);
+            if (e < n_ch && (e >= 2 * s.dim || h % group == 0)) {  // the rows that the next token looks back on
+#pragma unroll
+                for (uint32_t back = 0; back + 1 < kRunTaps; back++)
+                    if (back + 1 < s.taps) a.hist_out[size_t(s.taps - 2 - back) * x.channels + ch[i]] = row[i][back];
+            }
         }
     } else {
         for (uint32_t e = tid; e < n_ch; e += kStepThreads) put(e, conv_at(x, 0, a.pos0, channel(e)));
+        delta_carry(s, a, x, h, kStepThreads);
     }
     for (uint32_t d = s.dim + tid; d < s.d_pad; d += kStepThreads) qs[d] = ks[d] = 0.0f;
     for (uint32_t d = s.vdim + tid; d < s.v_pad; d += kStepThreads) vs[d] = 0.0f;
@@ -103,8 +111,10 @@ __global__ __launch_bounds__(kStepThreads) void delta_step_kernel(RmiDeltaShape 
         f32x4 pk = {0.f, 0.f, 0.f, 0.f}, pq = {0.f, 0.f, 0.f, 0.f};
 #pragma unroll
         for (uint32_t j = 0; j < NR; j++) {
-            const uint32_t d = sl + j * slices < s.d_pad ? sl + j * slices : 0;  // (past the end r is zero)
-            const float k = ks[d], q = qs[d];
+            const uint32_t d = sl + j * slices;
+            const bool live = d < s.d_pad && a.pos0;
+            const float k = ks[live ? d : 0], q = qs[live ? d : 0];
+            if (!live) r[j] = f32x4{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
             for (int e = 0; e < 4; e++) {
                 pk[e] = __builtin_fmaf(r[j][e], k, pk[e]);
@@ -147,7 +157,6 @@ __global__ __launch_bounds__(kStepThreads) void delta_step_kernel(RmiDeltaShape 
     for (uint32_t i = 0; i < kStepThreads / 64; i++) total += red[i];
     const float norm = 1.0f / sqrtf(total / float(s.vdim) + s.eps);
     if (tid < s.vdim) static_cast<T *>(a.out)[size_t(h) * s.vdim + tid] = from_f32<T>(o * norm * weight * gate);
-    delta_carry(s, a, x, h, kStepThreads);
 }
 
 // ---- several tokens, in chunks of sixteen.  With G_t the product of g over the chunk's tokens up to t and

@@ -10,42 +10,16 @@ import pytest
 import ruvenex_gen as G
 import ruvenex_plain as P
 from conftest import ROOT
+from folder_helpers import BF16, F32, TOL, Opener, feed, rel
 
 pytestmark = pytest.mark.gpu
-F32, BF16 = "float32", "bfloat16"
-TOL = {F32: 3e-5, BF16: 4e-2}
-
-
-def rel(got, want):
-    """Largest row error: root mean square over the row's, against the typical row's size."""
-    d = np.asarray(got, np.float64) - want
-    return float(np.sqrt((d * d).mean(-1)).max() / np.sqrt((want * want).mean()))
-
-
-def feed(s, tokens, sizes):
-    """Logits of every position, the tokens cut into portions of the given sizes (the last one repeats)."""
-    out, at, i = [], 0, 0
-    while at < len(tokens):
-        n = min(sizes[min(i, len(sizes) - 1)], len(tokens) - at)
-        out.append(s.step(tokens[at: at + n], range(n)))
-        at += n
-        i += 1
-    return np.concatenate(out)
 
 
 @pytest.fixture
 def open_model(hip, tmp_path):
-    opened = []
-
-    def go(cfg, w=None, dtype=F32, capacity=256):
-        w = G.weights(cfg) if w is None else w
-        s = hip.models.open_session(G.write_folder(tmp_path / f"m{len(opened)}", cfg, w), capacity, dtype)
-        opened.append(s)
-        return s, w
-
-    yield go
-    for s in opened:
-        s.close()
+    o = Opener(hip, tmp_path, G)
+    yield o
+    o.close()
 
 
 def only(w, keep):

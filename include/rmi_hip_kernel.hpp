@@ -394,30 +394,31 @@ class Qwen3Session {
     rmi_hip_qwen3 *h_;
 };
 
-// A Ruvenex model folder (config.json, model.safetensors); one sequence at a time.
-class RuvenexSession {
+// A model folder (config.json, model.safetensors) of any design the library knows, or of the one that `architecture`
+// names; one sequence at a time.
+class FolderSession {
   public:
-    RuvenexSession(const std::string &folder, uint32_t capacity, int dtype = RMI_HIP_DTYPE_BF16)
-        : h_(rmi_hip_ruvenex_open(folder.c_str(), dtype, capacity)) {
+    FolderSession(const std::string &folder, uint32_t capacity, int dtype = RMI_HIP_DTYPE_BF16, const char *architecture = nullptr)
+        : h_(rmi_hip_folder_open(folder.c_str(), architecture, dtype, capacity)) {
         if (!h_) throw HipError(RMI_HIP_E_RUNTIME, rmi_hip_last_error());
-        check(rmi_hip_ruvenex_sizes(h_, &vocab_, nullptr, nullptr, nullptr));
+        check(rmi_hip_folder_sizes(h_, &vocab_, nullptr, nullptr, nullptr));
     }
-    ~RuvenexSession() { rmi_hip_ruvenex_destroy(h_); }
-    RuvenexSession(const RuvenexSession &) = delete;
-    RuvenexSession &operator=(const RuvenexSession &) = delete;
+    ~FolderSession() { rmi_hip_folder_destroy(h_); }
+    FolderSession(const FolderSession &) = delete;
+    FolderSession &operator=(const FolderSession &) = delete;
     uint32_t vocab() const { return vocab_; }
-    uint32_t position() const { return rmi_hip_ruvenex_position(h_); }
-    void reset() { check(rmi_hip_ruvenex_reset(h_)); }
+    uint32_t position() const { return rmi_hip_folder_position(h_); }
+    void reset() { check(rmi_hip_folder_reset(h_)); }
     // the sequence's next tokens; logits [want.size()][vocab] of the places `want` among them
     std::vector<float> step(const std::vector<uint32_t> &tokens, const std::vector<uint32_t> &want) {
         std::vector<float> logits(want.size() * size_t(vocab_));
-        check(rmi_hip_ruvenex_step(h_, tokens.data(), uint32_t(tokens.size()), want.data(), uint32_t(want.size()), logits.data(), nullptr));
+        check(rmi_hip_folder_step(h_, tokens.data(), uint32_t(tokens.size()), want.data(), uint32_t(want.size()), logits.data(), nullptr));
         return logits;
     }
     // greedy generation of a new sequence
     std::vector<uint32_t> generate(const std::vector<uint32_t> &prompt, uint32_t max_new, double *seconds = nullptr) {
         std::vector<uint32_t> out(max_new);
-        const int n = rmi_hip_ruvenex_generate(h_, prompt.data(), uint32_t(prompt.size()), max_new, out.data(), nullptr, nullptr, nullptr,
+        const int n = rmi_hip_folder_generate(h_, prompt.data(), uint32_t(prompt.size()), max_new, out.data(), nullptr, nullptr, nullptr,
                                                0, nullptr, seconds);
         check(n < 0 ? n : 0);
         out.resize(size_t(n));
@@ -425,8 +426,20 @@ class RuvenexSession {
     }
 
   private:
-    rmi_hip_ruvenex *h_;
+    rmi_hip_folder_session *h_;
     uint32_t vocab_ = 0;
+};
+
+class RuvenexSession : public FolderSession {
+  public:
+    RuvenexSession(const std::string &folder, uint32_t capacity, int dtype = RMI_HIP_DTYPE_BF16)
+        : FolderSession(folder, capacity, dtype, "Ruvenex") {}
+};
+
+class VogizenSession : public FolderSession {
+  public:
+    VogizenSession(const std::string &folder, uint32_t capacity, int dtype = RMI_HIP_DTYPE_BF16)
+        : FolderSession(folder, capacity, dtype, "Vogizen") {}
 };
 
 }  // namespace rmi

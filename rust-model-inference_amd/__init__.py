@@ -1,11 +1,11 @@
 """MI355X (gfx950) back end for rust-model-inference's quantized matrix products.
 
 ``synth``  seeded synthetic tensors of the benchmark shapes (numpy only)
-``folder`` model folders: safetensors writer, synthetic Ruvenex models (numpy only)
+``folder`` model folders: safetensors writer, synthetic Ruvenex and Vogizen models (numpy only)
 ``gguf``   minimal GGUF v3 writer / mmap reader (synthetic Qwen3 file)
 ``hip``    ctypes binding of librmi_hip.so, the C ABI of include/rmi_hip.h
 ``kernel`` mirror of the reference's Kernel / Layer interface over that ABI
-``decode`` decoder sessions (Qwen3, Ruvenex) over the device-resident decode entry points
+``decode`` decoder sessions (Qwen3, Ruvenex, Vogizen) over the device-resident decode entry points
 ``models`` registry: the session class of a model file or folder
 ``replay`` token ids through a session, step by step, logits to files (bin/trace_run)
 ``loader`` mirror of GGUFLoader over the library's parser; file -> HBM uploads

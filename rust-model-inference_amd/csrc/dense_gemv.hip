@@ -185,18 +185,21 @@ GemvProblem problem_of(const RmiDense &w, const RmiInput &in, const RmiRowSegs &
 template <typename T>
 int gemv(const RmiDense &w, const RmiInput &in, const RmiRowSegs &segs, hipStream_t st) {
     const size_t lds = size_t(gemv_lds_pieces<T>(w.k_pad)) * 16;
-    // a wave takes four rows, and with no norm in front (whose work every workgroup repeats) one where four would leave
-    // compute units idle
-    const bool few = w.n_rows <= 16u * 2 * uint32_t(rmi_device_cus()) && in.norm == kNormNone && rmi_epilogue_of(segs) != kRowsPaired;
-    const GemvProblem p = problem_of(w, in, segs, few ? 1 : 4);
+    // A wave takes four rows; fewer where that would leave compute units with little to do (the prologue, which every
+    // workgroup repeats, then weighs less than the wait for memory).  Pairs of rows stay together.
+    const uint32_t cus = uint32_t(rmi_device_cus()), pairs = rmi_epilogue_of(segs) == kRowsPaired ? 2 : 1;
+    const uint32_t rows = in.norm == kNormRms || w.n_rows > 64 * cus ? 4 : w.n_rows > 4 * cus ? 2 : pairs;
+    const GemvProblem p = problem_of(w, in, segs, rows);
     auto go = [&](auto kernel) {
         const int rc = rmi_allow_lds(kernel, lds);
         if (rc == RMI_HIP_OK) hipLaunchKernelGGL(kernel, dim3(p.blocks), dim3(256), lds, st, p);
         return rc;
     };
     const int rc = rmi_input_dispatch(in, [&](auto norm, auto add, auto r) {
-        if constexpr (norm.value == kNormNone && (!add.value || r.value <= 4))
-            if (few) return go(input_gemv_kernel<T, norm.value, add.value, 1, r.value>);
+        if constexpr (norm.value != kNormRms && (!add.value || r.value <= 4)) {
+            if (rows == 1) return go(input_gemv_kernel<T, norm.value, add.value, 1, r.value>);
+            if (rows == 2) return go(input_gemv_kernel<T, norm.value, add.value, 2, r.value>);
+        }
         if constexpr (!add.value || r.value <= 4)
             return go(input_gemv_kernel<T, norm.value, add.value, 4, r.value>);
         else

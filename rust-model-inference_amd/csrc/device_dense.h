@@ -145,12 +145,12 @@ __device__ __forceinline__ const T *mul_row(const RmiRowSeg &s, uint32_t t) {
     return static_cast<const T *>(s.mul) + size_t(id < s.mul_rows ? id : s.mul_rows - 1) * s.mul_ld;
 }
 
-// sin(2 pi r), or with `cosine` cos(2 pi r), for |r| <= 1/2: the nearest quarter turn apart, then the Taylor polynomials on
-// an eighth of a turn to either side (their remainders are below 2e-9)
-__device__ __forceinline__ float sin_turns(double r, bool cosine) {
+// sin and cos of 2 pi r, |r| <= 1/2: the nearest quarter turn apart, then the Taylor polynomials on an eighth of a turn to
+// either side (their remainders are below 2e-9)
+__device__ __forceinline__ float2 sin_cos_turns(double r) {
     const double quarter = rint(r * 4.0);
     const float z = float((r - quarter * 0.25) * 6.283185307179586476925286766559), z2 = z * z;
-    const int q = int(quarter) + (cosine ? 1 : 0);
+    const int q = int(quarter);
     float s = 2.75573192e-6f, c = -2.75573192e-7f;
     s = __builtin_fmaf(s, z2, -1.98412698e-4f);
     s = __builtin_fmaf(s, z2, 8.33333333e-3f);
@@ -161,35 +161,45 @@ __device__ __forceinline__ float sin_turns(double r, bool cosine) {
     c = __builtin_fmaf(c, z2, 4.16666667e-2f);
     c = __builtin_fmaf(c, z2, -0.5f);
     c = __builtin_fmaf(c, z2, 1.0f);
-    const float v = q & 1 ? c : s;  // sin(a + q pi/2): s, c, -s, -c
-    return q & 2 ? -v : v;
+    const float a = q & 1 ? c : s, b = q & 1 ? s : c;  // sin(z + q pi/2) = s, c, -s, -c; cos = c, -s, -c, s
+    return make_float2(q & 2 ? -a : a, (q + 1) & 2 ? -b : b);
 }
 
-// channel c of a token's embedding at position p (RmiEmbed)
-template <typename T>
-__device__ __forceinline__ float embed_value(const RmiEmbed &e, uint32_t token, uint32_t p, uint32_t c) {
-    if (token >= e.vocab) token = e.vocab - 1;  // ids are validated on the host; never read outside the table
-    float v = to_f32(static_cast<const T *>(e.table)[size_t(token) * e.ld + c]) * e.scale;
-    if (e.turns) {
-        const double r = double(p) * e.turns[c >> 1];
-        v += sin_turns(r - rint(r), c & 1);  // the whole turns leave in f64
-    }
-    return v;
-}
-
-// a workgroup of 256: row t of the stream, four channels of a thread under way at a time
+// A workgroup of 256: row t of the stream, a token's embedding at position p.  A thread takes pairs of channels, eight at
+// a time, all their loads under way together.
 template <typename T>
 __device__ __forceinline__ void embed_row(const RmiEmbed &e, uint32_t token, uint32_t p, uint32_t t) {
-    for (uint32_t i0 = threadIdx.x; i0 < e.n; i0 += 1024) {
-        float v[4];
+    if (token >= e.vocab) token = e.vocab - 1;  // ids are validated on the host; never read outside the table
+    const T *row = static_cast<const T *>(e.table) + size_t(token) * e.ld;
+    const uint32_t pairs = (e.n + 1) / 2;
+    for (uint32_t i0 = threadIdx.x; i0 < pairs; i0 += 8 * 256) {
+        double turns[8];
+        float2 v[8];
 #pragma unroll
-        for (uint32_t j = 0; j < 4; j++) v[j] = embed_value<T>(e, token, p, i0 + j * 256 < e.n ? i0 + j * 256 : i0);
+        for (uint32_t j = 0; j < 8; j++) {
+            const uint32_t i = i0 + j * 256 < pairs ? i0 + j * 256 : i0;
+            turns[j] = e.turns ? e.turns[i] : 0.0;
+            v[j] = make_float2(to_f32(row[2 * i]), to_f32(row[2 * i + 1 < e.n ? 2 * i + 1 : 2 * i]));
+        }
 #pragma unroll
-        for (uint32_t j = 0; j < 4; j++) {
+        for (uint32_t j = 0; j < 8; j++) {
             const uint32_t i = i0 + j * 256;
-            if (i >= e.n) break;
-            e.x[size_t(t) * e.n + i] = v[j];
-            if (e.x_also) e.x_also[size_t(t) * e.n + i] = v[j];
+            if (i >= pairs) break;
+            v[j].x *= e.scale;
+            v[j].y *= e.scale;
+            if (e.turns) {
+                const double r = double(p) * turns[j];
+                const float2 sc = sin_cos_turns(r - rint(r));  // the whole turns leave in f64
+                v[j].x += sc.x;
+                v[j].y += sc.y;
+            }
+            float *dst = e.x + size_t(t) * e.n + 2 * i, *also = e.x_also ? e.x_also + size_t(t) * e.n + 2 * i : nullptr;
+            dst[0] = v[j].x;
+            if (also) also[0] = v[j].x;
+            if (2 * i + 1 < e.n) {
+                dst[1] = v[j].y;
+                if (also) also[1] = v[j].y;
+            }
         }
     }
 }

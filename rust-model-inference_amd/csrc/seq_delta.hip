@@ -37,7 +37,7 @@ __device__ __forceinline__ void delta_carry(const RmiDeltaShape &s, const RmiDel
 constexpr uint32_t kStepThreads = 512;
 template <typename T, int NR>
 __global__ __launch_bounds__(kStepThreads) void delta_step_kernel(RmiDeltaShape s, RmiDeltaArgs a) {
-    __shared__ float ks[kMaxHeadDim], qs[kMaxHeadDim], vs[kMaxHeadDim], us[kMaxHeadDim], red[8];
+    __shared__ __attribute__((aligned(16))) float ks[kMaxHeadDim], qs[kMaxHeadDim], vs[kMaxHeadDim], us[kMaxHeadDim], red[8];
     __shared__ __attribute__((aligned(16))) float part[2][4 * kStepThreads];  // [S^T k, S^T q][slice][column]
     const uint32_t tid = threadIdx.x, lane = tid & 63, h = blockIdx.x, group = s.heads / s.kv_heads, g = h / group;
     const ConvCtx x{a.u, a.hist_in, a.conv, delta_channels(s), s.taps};
